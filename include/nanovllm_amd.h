@@ -38,6 +38,9 @@ enum nva_status {
     NVA_ERR_SCRATCH_TOO_SMALL = 9     /* problem exceeds the library's built-in scratch array */
 };
 
+/* Element type of the entry points that take bf16 or fp32 tensors. */
+enum nva_dtype { NVA_DTYPE_BF16 = 0, NVA_DTYPE_F32 = 1 };
+
 /* Library version, (major << 16) | minor. */
 int nva_version(void);
 
@@ -288,6 +291,80 @@ int nva_silu_and_mul(const void *x, int64_t x_row_stride, void *out,
 int nva_stage_decode_inputs(void *dst, const void *src_host, int64_t nbytes, int64_t ids_offset,
                             int64_t index_offset, int32_t n, const int64_t *prev_tokens, int32_t n_prev,
                             void *stream);
+
+/*
+ * ---- layered models: mixers and the steps around them -----------------------------------
+ * bf16 or fp32 tensors (dtype: enum nva_dtype), fp32 residual stream, no counterpart in the reference.
+ * A step's rows are either portions of sequences (cu_seqlens_q [n_seqs + 1]: row bounds; seq_lens: tokens
+ * of each sequence once these rows are in; token_seq [n_tokens]: sequence of every row) or single tokens
+ * (cu_seqlens_q NULL: row i is the newest token of sequence i, at position seq_lens[i] - 1; a row with
+ * seq_lens[i] <= 0 is padding: its result is zero and nothing is stored).  Recurrent state and carried
+ * rows live in slots; a sequence whose rows begin at position 0 starts from zeros whatever its slot
+ * holds, and slots outside [0, num_state_slots) are neither read nor written.  Sizes that are multiples
+ * of 8 with 16-byte aligned tensors take the vector paths; any other size runs too.
+ */
+
+/* residual[r] = table[ids[r]] * scale (fp32); out[r] = layer_norm(residual[r]) * weight + bias.
+ * ids are clamped to [0, vocab).  Variance is the mean of the squared deviations, eps inside the root. */
+int nva_embed_norm(const int64_t *ids, const void *table, float scale, const void *weight, const void *bias,
+                   float *residual, void *out, int32_t rows, int32_t width, int32_t vocab, float eps,
+                   int32_t dtype, void *stream);
+
+/* residual[r] += layer_norm(y[r]) * post_weight + post_bias, in place, fp32;
+ * out[r] = layer_norm(residual[r]) * next_weight + next_bias.
+ * rows_of (int32 [rows], may be NULL): out[r] is computed from row rows_of[r] of y and residual
+ * (clamped to [0, src_rows)) and residual is not written; without it rows == src_rows. */
+int nva_post_add_norm(const void *y, int64_t y_row_stride, float *residual, const void *post_weight,
+                      const void *post_bias, const void *next_weight, const void *next_bias, void *out,
+                      const int32_t *rows_of, int32_t rows, int32_t src_rows, int32_t width, float eps,
+                      int32_t dtype, void *stream);
+
+/* x: [rows, 2 * inter] (gate | up, row stride in elements).  g = min(gate, limit), u = clamp(up, -limit, limit),
+ * out = g * sigmoid(alpha * g) * (u + 1). */
+int nva_clamped_gate(const void *x, int64_t x_row_stride, void *out, int32_t rows, int32_t inter, float limit,
+                     float alpha, int32_t dtype, void *stream);
+
+/* q, k and v of an attention layer: causal convolution over time on every channel, rotary embedding of
+ * the first rot_dims elements of each q and k head (pairs i, i + rot_dims / 2), q to q_out, k and v to
+ * their cache slots.
+ * qkv: [n_tokens, channels], channels = (num_heads + num_kv_heads) * qk_dim + num_kv_heads * v_dim.
+ * conv_weight: [taps, channels], tap taps - 1 meets the row itself; 1 <= taps <= 8.
+ * conv_state: [num_state_slots, taps - 1, channels], the last projected rows of every sequence, oldest
+ * first; read for rows before a portion, updated by the call.
+ * rope_cache: fp32 [max_position, rot_dims], cos in the first half of a row, sin in the second. */
+int nva_conv_rope_store(const void *qkv, int64_t qkv_row_stride, const void *conv_weight, void *conv_state,
+                        const int32_t *state_slots_of_seq, const int32_t *cu_seqlens_q, const int32_t *seq_lens,
+                        const int32_t *token_seq, const int64_t *positions, const float *rope_cache,
+                        void *q_out, void *k_cache, void *v_cache, const int32_t *slot_mapping,
+                        int64_t num_slots, int32_t n_tokens, int32_t n_seqs, int32_t num_heads,
+                        int32_t num_kv_heads, int32_t qk_dim, int32_t v_dim, int32_t rot_dims, int32_t taps,
+                        int32_t max_position, int32_t num_state_slots, int32_t dtype, void *stream);
+
+/* Softmax attention inside position chunks: the query at position p sees keys [p / chunk * chunk, p] of
+ * its sequence, all of them read from the paged cache (this step's rows must be stored already).
+ * score = (q . k) * scale, then softcap * tanh(score / softcap) where softcap > 0.
+ * q: [n_tokens, num_heads, qk_dim] (row stride in elements), caches [num_blocks, block_size, num_kv_heads,
+ * qk_dim or v_dim], block_tables int32 [n_seqs, >= max_blocks]; out: [n_tokens, num_heads, v_dim] dense.
+ * A key behind a table entry outside [0, num_blocks) is not seen. */
+int nva_chunk_attn(const void *q, int64_t q_row_stride, const void *k_cache, const void *v_cache,
+                   const int32_t *block_tables, int64_t bt_row_stride, int32_t max_blocks,
+                   const int32_t *cu_seqlens_q, const int32_t *seq_lens, const int32_t *token_seq, void *out,
+                   int32_t n_tokens, int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads,
+                   int32_t num_kv_heads, int32_t qk_dim, int32_t v_dim, int32_t block_size,
+                   int32_t num_blocks, int32_t chunk, float scale, float softcap, int32_t dtype,
+                   void *stream);
+
+/* Retention: S_t = decay S_{t-1} + k_t v_t^T, o_t = S_t^T q_t per head, with rotary q and k, k scaled by
+ * k_scale; out = o / rms(o) * silu(gate).
+ * qkvg: [n_tokens, 2 * num_heads * (qk_dim + v_dim)] (q | k | v | gate, row stride in elements);
+ * state: fp32 [num_state_slots, num_heads, qk_dim, v_dim], carried across calls; log2_decay: fp32
+ * [num_heads], log2 of every head's decay; rope_cache as above; out: [n_tokens, num_heads * v_dim] dense. */
+int nva_retention(const void *qkvg, int64_t row_stride, float *state, const int32_t *state_slots_of_seq,
+                  const int32_t *cu_seqlens_q, const int32_t *seq_lens, const int64_t *positions,
+                  const float *rope_cache, const float *log2_decay, void *out, int32_t n_tokens, int32_t n_seqs,
+                  int32_t max_seqlen_q, int32_t num_heads, int32_t qk_dim, int32_t v_dim, int32_t rot_dims,
+                  int32_t max_position, int32_t num_state_slots, float k_scale, float eps, int32_t dtype,
+                  void *stream);
 
 /*
  * Calibration, no counterpart in the reference: streams nbytes from src with the access discipline of

@@ -23,6 +23,9 @@ ERR_LAUNCH_FAILED = 7
 ERR_NO_DEVICE = 8
 ERR_SCRATCH_TOO_SMALL = 9
 
+# element types of enum nva_dtype
+DTYPE_BF16, DTYPE_F32 = 0, 1
+
 _vp, _i32, _i64, _u64, _f32, _sz = C.c_void_p, C.c_int32, C.c_int64, C.c_uint64, C.c_float, C.c_size_t
 
 # name -> (restype, argtypes); must list every symbol the header declares
@@ -48,6 +51,15 @@ SIGNATURES = {
     "nva_stage_decode_inputs": (C.c_int, [_vp, _vp, _i64, _i64, _i64, _i32, _vp, _i32, _vp]),
     "nva_sample": (C.c_int, [_vp, _i64, _vp, _vp, _i64, _u64, _u64, _vp, _vp, _sz, _i32, _i32, _vp]),
     "nva_sample_static": (C.c_int, [_vp, _i64, _vp, _vp, _i64, _u64, _u64, _vp, _i32, _i32, _vp]),
+    "nva_embed_norm": (C.c_int, [_vp, _vp, _f32, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _f32, _i32, _vp]),
+    "nva_post_add_norm": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _f32, _i32, _vp]),
+    "nva_clamped_gate": (C.c_int, [_vp, _i64, _vp, _i32, _i32, _f32, _f32, _i32, _vp]),
+    "nva_conv_rope_store": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp,
+                                      _i64, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _vp]),
+    "nva_chunk_attn": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _i64, _i32, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _i32,
+                                 _i32, _i32, _i32, _i32, _i32, _i32, _f32, _f32, _i32, _vp]),
+    "nva_retention": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _i32, _i32,
+                                _i32, _i32, _i32, _i32, _f32, _f32, _i32, _vp]),
     "nva_probe_stream_read": (C.c_int, [_vp, _i64, _vp, _vp]),
 }
 

@@ -8,8 +8,8 @@ defaults and the positional order of ``set_context`` are the reference's
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
-from typing import Optional
+from dataclasses import dataclass, field
+from typing import List, Optional
 
 import torch
 
@@ -35,6 +35,23 @@ class DecodePlan:
 
 
 @dataclass
+class RowGroup:
+    """Consecutive rows of a step that run through the same kernels: single tokens (``cu`` is None,
+    row i is the newest token of sequence i) or portions of sequences.  Index tensors are int32 on the
+    device; ``seq_lens`` counts a sequence's tokens once these rows are in."""
+    first: int                                   # first row of the group
+    count: int                                   # rows
+    num_seqs: int
+    seq_lens: torch.Tensor                       # [num_seqs]; <= 0 marks a padded row
+    slot_mapping: torch.Tensor                   # [count] cache slot of every row
+    block_tables: torch.Tensor                   # [num_seqs, max_blocks]
+    state_slots: torch.Tensor                    # [num_seqs] slot of recurrent state and carried rows
+    cu: Optional[torch.Tensor] = None            # [num_seqs + 1] row bounds, relative to ``first``
+    token_seq: Optional[torch.Tensor] = None     # [count] sequence of every row
+    max_q: int = 1                               # longest portion
+
+
+@dataclass
 class Context:
     """Tensors describing the batch being run.  Index tensors are int32 on the device.
 
@@ -53,6 +70,13 @@ class Context:
     decode_plan: Optional[DecodePlan] = None     # not in the reference: see DecodePlan
 
 
+@dataclass
+class SpanContext(Context):
+    """Context of a step of a model that takes portions: single tokens and portions as row groups."""
+    groups: List[RowGroup] = field(default_factory=list)
+    logit_rows: Optional[torch.Tensor] = None    # int32: rows whose logits are asked for (None: all)
+
+
 class _Holder:
     current = Context()
 
@@ -65,6 +89,10 @@ def set_context(is_prefill, cu_seqlens_q=None, cu_seqlens_k=None, max_seqlen_q=0
                 slot_mapping=None, context_lens=None, block_tables=None, decode_plan=None) -> None:
     _Holder.current = Context(is_prefill, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen_k,
                               slot_mapping, context_lens, block_tables, decode_plan)
+
+
+def set_row_groups(groups, logit_rows=None) -> None:
+    _Holder.current = SpanContext(any(g.cu is not None for g in groups), groups=groups, logit_rows=logit_rows)
 
 
 def reset_context() -> None:

@@ -6,6 +6,10 @@ covers the hash of block i-1 followed by the block's ids as little-endian int64,
 ``compute_hash`` does at :36-41) so that two prompts sharing a prefix share physical blocks.
 Blocks keep their hash after they are freed: a later prompt can revive them as long as the
 block has not been handed out again.
+
+Models with recurrent state also hold one state slot per sequence (``num_state_slots``), handed out and
+given back together with the blocks.  A prefix of cached keys is of no use to them without the state
+that goes with it, so they run with ``prefix_cache=False``.
 """
 from __future__ import annotations
 
@@ -32,8 +36,11 @@ class _Block:
 
 class BlockManager:
 
-    def __init__(self, num_blocks: int, block_size: int = 256):
+    def __init__(self, num_blocks: int, block_size: int = 256, prefix_cache: bool = True, num_state_slots: int = 0):
         self.block_size = block_size
+        self.prefix_cache = prefix_cache
+        self.num_state_slots = num_state_slots
+        self.free_state_slots: Deque[int] = deque(range(num_state_slots))
         self.blocks = [_Block(i) for i in range(num_blocks)]
         self.hash_to_block_id: Dict[int, int] = {}
         self.free_block_ids: Deque[int] = deque(range(num_blocks))
@@ -65,12 +72,19 @@ class BlockManager:
 
     # ---- prefill -------------------------------------------------------------------------
     def can_allocate(self, seq: Sequence) -> bool:
+        if self.num_state_slots and not self.free_state_slots:
+            return False
         return len(self.free_block_ids) >= seq.num_blocks
 
     def allocate(self, seq: Sequence) -> None:
         """Give ``seq`` a block table; leading blocks whose content hash is known are shared
         and counted in ``seq.num_cached_tokens``.  After the first miss every block is fresh."""
         assert not seq.block_table
+        if self.num_state_slots:
+            seq.state_slot = self.free_state_slots.popleft()
+        if not self.prefix_cache:
+            self.extend(seq)
+            return
         h = NO_HASH
         missed = False
         for i in range(seq.num_blocks):
@@ -94,7 +108,19 @@ class BlockManager:
                 self.hash_to_block_id[h] = blk.block_id
             seq.block_table.append(blk.block_id)
 
+    def extend(self, seq: Sequence) -> None:
+        """Fresh blocks until the table covers every token of ``seq`` (no prefix cache)."""
+        assert not self.prefix_cache
+        need = seq.num_blocks - len(seq.block_table)
+        if need > len(self.free_block_ids):
+            raise RuntimeError("the KV cache has no free block left")
+        for _ in range(need):
+            seq.block_table.append(self._take(self.free_block_ids[0]).block_id)
+
     def deallocate(self, seq: Sequence) -> None:
+        if seq.state_slot >= 0:
+            self.free_state_slots.append(seq.state_slot)
+            seq.state_slot = -1
         for block_id in reversed(seq.block_table):
             blk = self.blocks[block_id]
             blk.ref_count -= 1
@@ -109,6 +135,9 @@ class BlockManager:
         return len(self.free_block_ids) >= (1 if len(seq) % self.block_size == 1 else 0)
 
     def may_append(self, seq: Sequence) -> None:
+        if not self.prefix_cache:
+            self.extend(seq)
+            return
         table = seq.block_table
         last = self.blocks[table[-1]]
         fill = len(seq) % self.block_size
@@ -127,6 +156,8 @@ class BlockManager:
         runs ahead of the sampled tokens the block's last id is not known at that moment, and the
         loop seals the block once the token has been read back (``table``: the block table the
         sequence had, if it has been deallocated since)."""
+        if not self.prefix_cache:
+            return
         table = seq.block_table if table is None else table
         blk = self.blocks[table[index]]
         if blk.hash != NO_HASH:

@@ -11,6 +11,8 @@ import os
 from dataclasses import dataclass, field
 from typing import Optional
 
+from . import registry
+
 
 @dataclass
 class ModelConfig:
@@ -27,10 +29,16 @@ class ModelConfig:
     tie_word_embeddings: bool = True
     name: str = "qwen3"
 
+    portions = False                                      # class attributes: see registry.py
+    dtypes = ("bfloat16",)
+
     @classmethod
     def from_json(cls, path: str) -> "ModelConfig":
         with open(path) as f:
-            raw = json.load(f)
+            return cls.from_raw(json.load(f))
+
+    @classmethod
+    def from_raw(cls, raw: dict) -> "ModelConfig":
         keys = {f_.name for f_ in cls.__dataclass_fields__.values()}
         cfg = cls(**{k: v for k, v in raw.items() if k in keys})
         if "head_dim" not in raw:
@@ -57,30 +65,41 @@ def qwen3_8b() -> ModelConfig:
 
 @dataclass
 class EngineConfig:
-    model: object = field(default_factory=qwen3_0_6b)     # ModelConfig, or a directory holding config.json
+    model: object = field(default_factory=qwen3_0_6b)     # a family's configuration, or a directory holding config.json
     max_num_batched_tokens: int = 16384
     max_num_seqs: int = 512
     max_model_len: int = 4096
     gpu_memory_utilization: float = 0.9
     tensor_parallel_size: int = 1
     enforce_eager: bool = False
-    hf_config: Optional[ModelConfig] = None
+    hf_config: Optional[object] = None                    # the family's configuration object
     eos: int = -1
     kvcache_block_size: int = 256
     num_kvcache_blocks: int = -1
     seed: int = 0
     decode_lookahead: bool = True                        # launch decode steps one step ahead of their tokens
+    dtype: str = "bfloat16"                              # element type of weights, activations and cache ("float32" where the family runs in it)
     graph_bucket_step: int = 16                          # decode graphs are captured for batch sizes 1, 2, 4, 8 and every multiple of this
 
     def __post_init__(self):
-        if isinstance(self.model, ModelConfig):
+        if registry.is_config(self.model):
             self.hf_config = self.model
         else:
             assert os.path.isdir(self.model), f"{self.model} is not a directory"
-            self.hf_config = ModelConfig.from_json(os.path.join(self.model, "config.json"))
+            self.hf_config = registry.load_config(self.model)
+        if self.dtype not in self.hf_config.dtypes:
+            raise ValueError(f"{self.hf_config.name} runs in {' or '.join(self.hf_config.dtypes)}, not {self.dtype}")
         assert self.kvcache_block_size % 256 == 0
         assert self.kvcache_block_size == 256, "this engine keeps Sequence.block_size = 256 like nanovllm/engine/sequence.py:15 (the kernels take 256 * 2^k)"
         assert self.tensor_parallel_size == 1, "this build runs on one GPU"
         assert self.graph_bucket_step >= 1
         self.max_model_len = min(self.max_model_len, self.hf_config.max_position_embeddings)
-        assert self.max_num_batched_tokens >= self.max_model_len
+        if self.hf_config.portions:                       # prompts are cut into portions that fit a step
+            assert self.max_num_batched_tokens >= self.max_num_seqs
+        else:
+            assert self.max_num_batched_tokens >= self.max_model_len
+
+    @property
+    def torch_dtype(self):
+        import torch
+        return {"bfloat16": torch.bfloat16, "float32": torch.float32}[self.dtype]

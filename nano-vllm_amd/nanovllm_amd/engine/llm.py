@@ -51,7 +51,7 @@ class LLMEngine:
         sch, runner = self.scheduler, self.model_runner
         finished = []
         # admission (prefix hashes, recompute of preempted sequences) needs every token in place
-        if self._inflight is not None and (sch.waiting or not sch.running):
+        if self._inflight is not None and sch.needs_tokens():
             finished += self._commit_inflight()
         if sch.is_finished():
             return self._report(finished), 0
@@ -68,7 +68,10 @@ class LLMEngine:
             token_ids = runner.run(seqs, is_prefill)
             sch.postprocess(seqs, token_ids)
             finished += [s for s in seqs if s.is_finished]
-        num_tokens = sum(len(s) for s in seqs) if is_prefill else -len(seqs)
+        if is_prefill:
+            num_tokens = sum(s.num_scheduled_tokens for s in seqs) if sch.portions else sum(len(s) for s in seqs)
+        else:
+            num_tokens = -len(seqs)
         kind = "prefill" if is_prefill else "decode"
         self.stats[kind + "_steps"] += 1
         self.stats[kind + "_tokens"] += abs(num_tokens)

@@ -5,6 +5,10 @@ Single-GPU counterpart of nanovllm/engine/model_runner.py: ``prepare_prefill`` /
 its cache layout ``[2, layers, num_blocks, 256, Hkv, Dh]`` (:100-117) and ``capture_graphs``
 its static-buffer graph replay per batch-size bucket (:215-250).  Host tensors are built
 with numpy into pinned staging buffers instead of Python lists.
+
+Models that take portions (``config.hf_config.portions``) are run through ``run_spans``: any mix of
+single tokens and portions of prompts in one batch, each span from the cache and state its sequence
+left behind; their pure decode steps replay the same graphs as the others'.
 """
 from __future__ import annotations
 
@@ -15,10 +19,10 @@ import numpy as np
 import torch
 
 from .. import _lib
-from ..context import DecodePlan, get_context, reset_context, set_context
+from ..context import DecodePlan, RowGroup, get_context, reset_context, set_context, set_row_groups
 from ..sampler import Sampler
+from . import registry
 from .config import EngineConfig
-from .model import Qwen3ForCausalLM
 from .sequence import PENDING_TOKEN, Sequence
 
 
@@ -37,6 +41,48 @@ class DecodeHandle:
     def tokens(self) -> List[int]:
         self.ready.synchronize()
         return self.tokens_host[: len(self.seqs)].tolist()
+
+
+@dataclass
+class Span:
+    """The tokens ``[start, start + count)`` of a sequence, to be run in one step; ``want`` lists the places
+    among them whose logits are asked for."""
+    seq: Sequence
+    start: int
+    count: int
+    want: List[int]
+
+
+def build_span_inputs(spans: List[Span], block_size: int) -> dict:
+    """Host-side inputs of a step of spans.  Single tokens take the first rows, portions the rest;
+    ``logit_rows`` names the wanted rows in the order of ``spans`` and their ``want``."""
+    singles = [i for i, s in enumerate(spans) if s.count == 1]
+    portions = [i for i, s in enumerate(spans) if s.count != 1]
+    order = [spans[i] for i in singles + portions]
+    first_row = np.zeros(len(spans), dtype=np.int64)
+    first_row[singles + portions] = np.cumsum([0] + [s.count for s in order])[:-1]
+    ids, pos, slots = [], [], []
+    for s in order:
+        assert s.count >= 1 and 0 <= s.start and s.start + s.count <= len(s.seq)
+        ids.append(np.asarray(s.seq.token_ids[s.start: s.start + s.count], dtype=np.int64))
+        p = np.arange(s.start, s.start + s.count, dtype=np.int64)
+        pos.append(p)
+        table = np.asarray(s.seq.block_table, dtype=np.int64)
+        slots.append(table[p // block_size] * block_size + p % block_size)
+
+    def group(members: List[Span]) -> Optional[dict]:
+        if not members:
+            return None
+        counts = np.asarray([s.count for s in members], dtype=np.int32)
+        return dict(seq_lens=np.asarray([s.start + s.count for s in members], dtype=np.int32),
+                    block_tables=build_block_tables([s.seq for s in members]),
+                    state_slots=np.asarray([s.seq.state_slot for s in members], dtype=np.int32),
+                    cu=np.concatenate([[0], np.cumsum(counts)]).astype(np.int32),
+                    token_seq=np.repeat(np.arange(len(members), dtype=np.int32), counts), max_q=int(counts.max()))
+
+    return dict(input_ids=np.concatenate(ids), positions=np.concatenate(pos), slot_mapping=np.concatenate(slots).astype(np.int32),
+                singles=group([spans[i] for i in singles]), portions=group([spans[i] for i in portions]),
+                logit_rows=np.asarray([first_row[i] + w for i, s in enumerate(spans) for w in s.want], dtype=np.int32))
 
 
 def build_block_tables(seqs: List[Sequence]) -> np.ndarray:
@@ -99,14 +145,17 @@ class ModelRunner:
         self.enforce_eager = config.enforce_eager
         self.device = torch.device(device)
         torch.cuda.set_device(self.device)
+        self.portions = self.cfg.portions
         prev = torch.get_default_dtype()
-        torch.set_default_dtype(torch.bfloat16)
+        torch.set_default_dtype(config.torch_dtype)
         try:
             with torch.device(self.device):
-                self.model = Qwen3ForCausalLM(self.cfg, config.max_model_len, self.device, config.seed)
+                self.model = registry.model_class(self.cfg)(self.cfg, config.max_model_len, self.device, config.seed)
         finally:
             torch.set_default_dtype(prev)
         self.model.eval()
+        if isinstance(config.model, str) and hasattr(self.model, "load_weights"):
+            self.model.load_weights(config.model)
         self.sampler = Sampler(seed=config.seed)
         self.max_table_width = -(-config.max_model_len // self.block_size)
         self.graphs = {}
@@ -127,8 +176,11 @@ class ModelRunner:
                 one = one + 1
             _capture_anchor.append((probe, one))
         with torch.inference_mode():
-            self.warmup_model()
-            self.allocate_kv_cache()
+            if self.portions:
+                self.bind_model_cache()
+            else:
+                self.warmup_model()
+                self.allocate_kv_cache()
             if not self.enforce_eager:
                 self.capture_graphs()
 
@@ -165,6 +217,38 @@ class ModelRunner:
                 layer_id += 1
         assert layer_id == m.num_hidden_layers
 
+    def bind_model_cache(self) -> None:
+        """Cache and state of a model that keeps its own per layer.  Without a given number of blocks the
+        largest step is run once in a cache that just holds it, and what memory is then left over is
+        divided into blocks."""
+        cfg, bs = self.config, self.block_size
+        slots = cfg.max_num_seqs
+        if cfg.num_kvcache_blocks <= 0:
+            num_seqs = max(1, min(cfg.max_num_batched_tokens // cfg.max_model_len, slots))
+            length = min(cfg.max_model_len, cfg.max_num_batched_tokens)
+            per_seq = -(-length // bs)
+            self.model.bind_cache(num_seqs * per_seq, bs, num_seqs)
+            torch.cuda.empty_cache()
+            torch.cuda.reset_peak_memory_stats()
+            held = torch.cuda.memory_stats()["allocated_bytes.all.current"]
+            spans = []
+            for i in range(num_seqs):
+                seq = Sequence([0] * length)
+                seq.block_table, seq.state_slot = list(range(i * per_seq, (i + 1) * per_seq)), i
+                spans.append(Span(seq, 0, length, [length - 1]))
+            self.run_spans(spans)
+            torch.cuda.synchronize()
+            activations = torch.cuda.memory_stats()["allocated_bytes.all.peak"] - held
+            self.model.unbind_cache()
+            torch.cuda.empty_cache()
+            free, total = torch.cuda.mem_get_info()
+            budget = int(total * cfg.gpu_memory_utilization) - (total - free) - activations - slots * self.model.state_bytes_per_slot()
+            cfg.num_kvcache_blocks = budget // max(self.model.kv_bytes_per_token() * bs, 1)
+            if self.model.kv_bytes_per_token() == 0:          # no layer keeps keys: blocks only count tokens
+                cfg.num_kvcache_blocks = slots * self.max_table_width
+        assert cfg.num_kvcache_blocks > 0, "no memory left for the KV cache"
+        self.model.bind_cache(cfg.num_kvcache_blocks, bs, slots)
+
     # ---- host -> device inputs -----------------------------------------------------------------
     def _to_device(self, array: np.ndarray, dtype: torch.dtype) -> torch.Tensor:
         t = torch.from_numpy(np.ascontiguousarray(array)).to(dtype)
@@ -181,6 +265,8 @@ class ModelRunner:
         cfg = self.config
         tokens, seqs = cfg.max_num_batched_tokens, cfg.max_num_seqs
         total = tokens * (8 + 8 + 4) + 2 * (seqs + 1) * 4 + seqs * self.max_table_width * 4 + seqs * 4 + 8 * 256
+        if self.portions:                                 # sequence and wanted row of every token, lengths and state slots, finer padding
+            total += tokens * (4 + 4) + 4 * seqs * 4 + 16 * 256
         self._pf_host = [torch.zeros(total, dtype=torch.uint8).pin_memory() for _ in range(2)]
         self._pf_dev = torch.zeros(total, dtype=torch.uint8, device=self.device)
         self._pf_turn = 0
@@ -228,6 +314,61 @@ class ModelRunner:
         return self._to_device(np.fromiter((s.temperature for s in seqs), dtype=np.float32, count=len(seqs)),
                                torch.float32)
 
+    def prepare_spans(self, spans: List[Span]):
+        """Stages a step of spans and installs its row groups; returns (ids, positions)."""
+        h = build_span_inputs(spans, self.block_size)
+        fields = [(h["input_ids"], torch.int64), (h["positions"], torch.int64), (h["slot_mapping"], torch.int32),
+                  (h["logit_rows"] if h["logit_rows"].size else None, torch.int32)]
+        for name in ("singles", "portions"):
+            g = h[name]
+            fields += [(None if g is None else g[k], torch.int32) for k in ("seq_lens", "block_tables", "state_slots", "cu", "token_seq")]
+        ids, pos, slots, rows, *rest = self._stage_prefill(fields)
+        groups, first = [], 0
+        for name, (lens, tables, state, cu, token_seq) in (("singles", rest[:5]), ("portions", rest[5:])):
+            if h[name] is None:
+                continue
+            single, n = name == "singles", h[name]["token_seq"].size
+            groups.append(RowGroup(first, n, len(h[name]["seq_lens"]), lens, slots[first: first + n], tables, state,
+                                   None if single else cu, None if single else token_seq, h[name]["max_q"]))
+            first += n
+        set_row_groups(groups, torch.empty(0, dtype=torch.int32, device=self.device) if rows is None else rows)
+        return ids, pos
+
+    @torch.inference_mode()
+    def run_spans(self, spans: List[Span]) -> Optional[torch.Tensor]:
+        """Runs the spans as one batch; logits of the wanted places (rows in the order of ``spans`` and their
+        ``want``), None when nothing is wanted.  A step of single tokens at the end of their sequences replays
+        the decode graphs."""
+        if self.graph_bs and len(spans) <= self.graph_bs[-1] and all(s.count == 1 and s.start == len(s.seq) - 1 for s in spans):
+            logits = self._run_decode_graph([s.seq for s in spans])
+            wanted = [i for i, s in enumerate(spans) for _ in s.want]
+            if wanted != list(range(len(spans))):
+                logits = logits[torch.tensor(wanted, dtype=torch.int64, device=self.device)] if wanted else None
+            return logits
+        ids, pos = self.prepare_spans(spans)
+        hidden = self.model(ids, pos)
+        reset_context()
+        return self.model.compute_logits(hidden) if hidden.shape[0] else None
+
+    def _run_scheduled(self, seqs: List[Sequence]) -> List[int]:
+        """A scheduled step of single tokens and portions; the token of every sequence that reached its
+        end, PENDING_TOKEN for the others."""
+        spans = []
+        for s in seqs:
+            start = len(s) - 1 if s.is_prefilled else s.num_cached_tokens
+            end = start + s.num_scheduled_tokens
+            spans.append(Span(s, start, s.num_scheduled_tokens, [end - start - 1] if end == len(s) else []))
+        done = [i for i, s in enumerate(spans) if s.want]
+        self.kv_tokens_attended += sum(len(s) for s in seqs)
+        logits = self.run_spans(spans)
+        tokens = [PENDING_TOKEN] * len(seqs)
+        if done:
+            for i, tok in zip(done, self.sampler(logits, self.prepare_sample([seqs[i] for i in done])).tolist()):
+                tokens[i] = tok
+        else:
+            torch.cuda.synchronize()                       # the staging buffers are filled again in two steps' time
+        return tokens
+
     # ---- execution -----------------------------------------------------------------------------
     def _init_decode_staging(self, max_bs: int) -> None:
         """Pinned host buffers and one device buffer holding every per-step decode input; the
@@ -240,6 +381,8 @@ class ModelRunner:
                   ("slot_mapping", np.int32, (max_bs,)), ("context_lens", np.int32, (max_bs,)),
                   ("temperatures", np.float32, (max_bs,)), ("token_src", np.int32, (max_bs,)),
                   ("block_tables", np.int32, (max_bs, self.max_table_width))]
+        if self.portions:
+            fields.append(("state_slots", np.int32, (max_bs,)))
         offsets, total = {}, 0
         for name, dt, shape in fields:
             nbytes = int(np.prod(shape)) * np.dtype(dt).itemsize
@@ -282,6 +425,9 @@ class ModelRunner:
         st["slot_mapping"][bs:bucket] = -1                        # padded rows store nothing ...
         st["context_lens"][:bs] = h["context_lens"]
         st["context_lens"][bs:bucket] = 0                         # ... and attend over nothing
+        if self.portions:
+            st["state_slots"][:bs] = np.fromiter((s.state_slot for s in seqs), dtype=np.int32, count=bs)
+            st["state_slots"][bs:bucket] = -1
         st["temperatures"][:bs] = np.fromiter((s.temperature for s in seqs), dtype=np.float32, count=bs)
         st["block_tables"][:bs, : h["block_tables"].shape[1]] = h["block_tables"]   # stale columns stay: never read
         # one kernel reads the pinned buffer and writes the device buffer; pending input ids come
@@ -339,6 +485,8 @@ class ModelRunner:
             self.decode_step_events.append((started, ev))
 
     def run(self, seqs: List[Sequence], is_prefill: bool) -> List[int]:
+        if self.portions and (is_prefill or not self.can_launch_ahead(len(seqs))):
+            return self._run_scheduled(seqs)
         with torch.inference_mode():
             started = None if is_prefill else self._step_started()
             if not is_prefill and self.graph_bs and len(seqs) <= self.graph_bs[-1]:
@@ -367,7 +515,7 @@ class ModelRunner:
         gv = self.graph_vars
         input_ids, positions, slot_mapping = gv["input_ids"], gv["positions"], gv["slot_mapping"]
         context_lens, block_tables = gv["context_lens"], gv["block_tables"]
-        outputs = torch.zeros(max_bs, self.cfg.hidden_size, dtype=torch.bfloat16, device=self.device)
+        outputs = torch.zeros(max_bs, self.cfg.hidden_size, dtype=cfg.torch_dtype, device=self.device)
         step = cfg.graph_bucket_step                      # the reference captures 1, 2, 4, 8 and every 16th size (model_runner.py:227)
         self.graph_bs = [b for b in (1, 2, 4, 8) if b <= max_bs and b < step] + list(range(step, max_bs + 1, step))
         if self.graph_bs[-1] != max_bs:
@@ -380,8 +528,12 @@ class ModelRunner:
         cuts = sorted({round(i * n_layers / self.graph_segments) for i in range(self.graph_segments + 1)})
         pool = None
         for bs in reversed(self.graph_bs):
-            set_context(False, slot_mapping=slot_mapping[:bs], context_lens=context_lens[:bs],
-                        block_tables=block_tables[:bs])
+            if self.portions:
+                set_row_groups([RowGroup(0, bs, bs, context_lens[:bs], slot_mapping[:bs], block_tables[:bs],
+                                         gv["state_slots"][:bs])])
+            else:
+                set_context(False, slot_mapping=slot_mapping[:bs], context_lens=context_lens[:bs],
+                            block_tables=block_tables[:bs])
             outputs[:bs] = self.model(input_ids[:bs], positions[:bs])        # eager warm-up (sizes workspaces)
             # the captured layers share one work split of the decode kernel: the first layer derives
             # it at every replay, the others take it from the workspace

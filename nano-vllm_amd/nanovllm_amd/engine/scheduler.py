@@ -4,6 +4,10 @@
 free KV blocks allow and returns them as one prefill batch; only when nothing can be
 admitted does it return a decode batch of the running sequences, preempting from the back
 of the queue when a sequence needs a block and none is free.
+
+Models that take portions (``config.hf_config.portions``) get mixed steps instead: every running
+sequence contributes its next token, and the rest of the token budget goes to portions of prompts,
+in order of arrival.
 """
 from __future__ import annotations
 
@@ -21,7 +25,10 @@ class Scheduler:
         self.max_num_seqs = config.max_num_seqs
         self.max_num_batched_tokens = config.max_num_batched_tokens
         self.eos = config.eos
-        self.block_manager = BlockManager(config.num_kvcache_blocks, config.kvcache_block_size)
+        self.portions = config.hf_config.portions
+        self.block_manager = BlockManager(config.num_kvcache_blocks, config.kvcache_block_size,
+                                          prefix_cache=not self.portions,
+                                          num_state_slots=config.max_num_seqs if self.portions else 0)
         self.waiting: Deque[Sequence] = deque()
         self.running: Deque[Sequence] = deque()
 
@@ -31,7 +38,28 @@ class Scheduler:
     def add(self, seq: Sequence) -> None:
         self.waiting.append(seq)
 
+    # ---- sequences whose tokens come from a caller instead of the sampler ---------------------------
+    def hold(self, seq: Sequence) -> None:
+        """Blocks (and, the first time, a state slot) for every token ``seq`` has now."""
+        if not seq.block_table:
+            if not self.block_manager.can_allocate(seq):
+                raise RuntimeError("no cache blocks or state slot left for the sequence")
+            self.block_manager.allocate(seq)
+            seq.status = SequenceStatus.RUNNING
+        else:
+            self.block_manager.extend(seq)
+
+    def release(self, seq: Sequence) -> None:
+        self.block_manager.deallocate(seq)
+        seq.status = SequenceStatus.FINISHED
+
+    def needs_tokens(self) -> bool:
+        """Whether the next step reads token ids of every sequence on the host (it is not a pure decode step)."""
+        return bool(self.waiting) or not self.running or any(not s.is_prefilled for s in self.running)
+
     def schedule(self) -> Tuple[List[Sequence], bool]:
+        if self.portions:
+            return self._schedule_mixed()
         batch: List[Sequence] = []
         tokens = 0
         while self.waiting and len(batch) < self.max_num_seqs:
@@ -64,6 +92,51 @@ class Scheduler:
         self.running.extendleft(reversed(batch))
         return batch, False
 
+    def _schedule_mixed(self) -> Tuple[List[Sequence], bool]:
+        """Next tokens of the running sequences first, then portions.  Every sequence returned carries
+        ``num_scheduled_tokens``; the flag is False for a pure decode step."""
+        decode: List[Sequence] = []
+        portions: List[Sequence] = []
+        idle: List[Sequence] = []
+        # every running sequence past its prompt is sure of its token
+        budget = self.max_num_batched_tokens - sum(s.is_prefilled for s in self.running)
+        while self.running:
+            seq = self.running.popleft()
+            if not seq.is_prefilled:
+                take = min(budget, seq.prefill_target - seq.num_cached_tokens)
+                seq.num_scheduled_tokens = take
+                (portions if take else idle).append(seq)
+                budget -= take
+                continue
+            evicted_self = False
+            while not self.block_manager.can_append(seq):
+                if self.running:
+                    self.preempt(self.running.pop())
+                else:
+                    self.preempt(seq)
+                    evicted_self = True
+                    break
+            if not evicted_self:
+                self.block_manager.may_append(seq)
+                seq.num_scheduled_tokens = 1
+                decode.append(seq)
+        held = len(decode) + len(portions) + len(idle)
+        while self.waiting and budget > 0 and held < self.max_num_seqs:
+            seq = self.waiting[0]
+            if not self.block_manager.can_allocate(seq):
+                break
+            self.block_manager.allocate(seq)
+            self.waiting.popleft()
+            seq.status = SequenceStatus.RUNNING
+            seq.prefill_target = len(seq)
+            seq.num_scheduled_tokens = min(budget, len(seq))
+            budget -= seq.num_scheduled_tokens
+            portions.append(seq)
+            held += 1
+        assert decode or portions, "nothing schedulable: the KV cache is too small for a single sequence"
+        self.running.extend(decode + portions + idle)
+        return decode + portions, bool(portions)
+
     def preempt(self, seq: Sequence) -> None:
         seq.status = SequenceStatus.WAITING
         self.block_manager.deallocate(seq)
@@ -71,6 +144,10 @@ class Scheduler:
 
     def postprocess(self, seqs: List[Sequence], token_ids: List[int]) -> None:
         for seq, tok in zip(seqs, token_ids):
+            if self.portions and not seq.is_prefilled:
+                seq.num_cached_tokens += seq.num_scheduled_tokens
+                if not seq.is_prefilled:               # more of the prompt to come: nothing was sampled
+                    continue
             seq.append_token(tok)
             hit_eos = (not seq.ignore_eos) and tok == self.eos
             if hit_eos or seq.num_completion_tokens == seq.max_tokens:

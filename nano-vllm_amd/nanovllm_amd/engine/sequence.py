@@ -34,6 +34,9 @@ class Sequence:
         self.num_prompt_tokens = len(self.token_ids)
         self.num_cached_tokens = 0                 # leading tokens whose KV is already in the cache
         self.block_table: List[int] = []
+        self.state_slot = -1                       # slot of recurrent state, for models that have one
+        self.prefill_target = 0                    # tokens to run before the sequence decodes (set at admission)
+        self.num_scheduled_tokens = 0              # tokens of the step being run (models that take portions)
         self.temperature = sampling_params.temperature
         self.max_tokens = sampling_params.max_tokens
         self.ignore_eos = sampling_params.ignore_eos
@@ -71,6 +74,11 @@ class Sequence:
     @property
     def num_cached_blocks(self) -> int:
         return self.num_cached_tokens // self.block_size
+
+    @property
+    def is_prefilled(self) -> bool:
+        """Every token it was admitted with has been run: its next token is decoded."""
+        return self.num_cached_tokens >= self.prefill_target
 
     @property
     def num_blocks(self) -> int:

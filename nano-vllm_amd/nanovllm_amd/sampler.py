@@ -69,7 +69,7 @@ class Sampler(nn.Module):
     Each call advances a Philox offset, so successive calls draw afresh while a run
     with the same ``seed`` is reproducible.  The chunk records go to the library's built-in
     scratch array (a module's calls are ordered on one stream), so a step allocates only its
-    output tokens.
+    output tokens.  fp32 logits (an engine in fp32) are accepted too.
     """
 
     def __init__(self, seed: int = 0, static_scratch: bool = True):
@@ -80,4 +80,8 @@ class Sampler(nn.Module):
 
     def forward(self, logits: torch.Tensor, temperatures: torch.Tensor) -> torch.Tensor:
         self.calls += 1
+        if logits.dtype == torch.float32:
+            # greedy rows from the fp32 logits themselves; drawn rows from the same logits rounded once
+            drawn = sample(logits.to(torch.bfloat16), temperatures, None, self.seed, self.calls, self.static_scratch)
+            return torch.where(temperatures == 0, logits.argmax(-1), drawn)
         return sample(logits, temperatures, None, self.seed, self.calls, self.static_scratch)
