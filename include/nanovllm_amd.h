@@ -345,10 +345,15 @@ int nva_conv_rope_store(const void *qkv, int64_t qkv_row_stride, const void *con
  * score = (q . k) * scale, then softcap * tanh(score / softcap) where softcap > 0.
  * q: [n_tokens, num_heads, qk_dim] (row stride in elements), caches [num_blocks, block_size, num_kv_heads,
  * qk_dim or v_dim], block_tables int32 [n_seqs, >= max_blocks]; out: [n_tokens, num_heads, v_dim] dense.
- * A key behind a table entry outside [0, num_blocks) is not seen. */
+ * A key behind a table entry outside [0, num_blocks) is not seen.
+ * workspace: partial results of single-token rows, nva_chunk_attn_workspace_bytes() bytes, 16-byte aligned
+ * (NULL where that is 0, and for portions); needs no initialisation.  max_seqlen_q: longest portion. */
+size_t nva_chunk_attn_workspace_bytes(int32_t n_tokens, int32_t num_heads, int32_t num_kv_heads, int32_t v_dim,
+                                      int32_t max_blocks, int32_t block_size, int32_t chunk);
 int nva_chunk_attn(const void *q, int64_t q_row_stride, const void *k_cache, const void *v_cache,
                    const int32_t *block_tables, int64_t bt_row_stride, int32_t max_blocks,
                    const int32_t *cu_seqlens_q, const int32_t *seq_lens, const int32_t *token_seq, void *out,
+                   void *workspace, size_t workspace_bytes,
                    int32_t n_tokens, int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads,
                    int32_t num_kv_heads, int32_t qk_dim, int32_t v_dim, int32_t block_size,
                    int32_t num_blocks, int32_t chunk, float scale, float softcap, int32_t dtype,
@@ -358,10 +363,16 @@ int nva_chunk_attn(const void *q, int64_t q_row_stride, const void *k_cache, con
  * k_scale; out = o / rms(o) * silu(gate).
  * qkvg: [n_tokens, 2 * num_heads * (qk_dim + v_dim)] (q | k | v | gate, row stride in elements);
  * state: fp32 [num_state_slots, num_heads, qk_dim, v_dim], carried across calls; log2_decay: fp32
- * [num_heads], log2 of every head's decay; rope_cache as above; out: [n_tokens, num_heads * v_dim] dense. */
+ * [num_heads], log2 of every head's decay; rope_cache as above; out: [n_tokens, num_heads * v_dim] dense.
+ * workspace: states between the segments of long portions, nva_retention_workspace_bytes() bytes, 16-byte
+ * aligned (NULL where that is 0, and for single tokens); needs no initialisation.  max_seqlen_q: longest
+ * portion. */
+size_t nva_retention_workspace_bytes(int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads, int32_t qk_dim,
+                                     int32_t v_dim, int32_t rot_dims, int32_t dtype);
 int nva_retention(const void *qkvg, int64_t row_stride, float *state, const int32_t *state_slots_of_seq,
                   const int32_t *cu_seqlens_q, const int32_t *seq_lens, const int64_t *positions,
-                  const float *rope_cache, const float *log2_decay, void *out, int32_t n_tokens, int32_t n_seqs,
+                  const float *rope_cache, const float *log2_decay, void *out, void *workspace,
+                  size_t workspace_bytes, int32_t n_tokens, int32_t n_seqs,
                   int32_t max_seqlen_q, int32_t num_heads, int32_t qk_dim, int32_t v_dim, int32_t rot_dims,
                   int32_t max_position, int32_t num_state_slots, float k_scale, float eps, int32_t dtype,
                   void *stream);

@@ -2,8 +2,12 @@
 // sees the keys [floor(p / chunk) * chunk, p] of its own sequence.  Scores may be capped
 // (cap * tanh(s / cap)); query/key and value sizes may differ; scores, weights and sums are fp32.
 #include "nva_elem.h"
+#include "nva_matrix.h"
 
 #include <math.h>
+
+#include <algorithm>
+#include <type_traits>
 
 namespace nva {
 
@@ -96,6 +100,518 @@ __global__ __launch_bounds__(256) void chunk_attn_any_kernel(ChunkAttnArgs a) {
         if (i * 64 + lane < a.vdim) out[i * 64 + lane] = Elem<T>::from_f32(acc[i] * inv);
 }
 
+// ---- bf16 on the matrix cores -------------------------------------------------------------------
+// Both kernels below compute transposed with v_mfma_f32_16x16x32_bf16: S^T = K Q^T (A: 16 keys x 32 dims,
+// B: Q^T), O^T += V^T P^T (A: 16 value columns x 32 keys through LDS transpose reads, B: P^T).  The S^T
+// accumulators of two 16-key blocks (register i of lane l: key 4 (l / 16) + i) are a legal key order for
+// the second product, so P stays in registers.  The weights are fp32: P goes into the product as the
+// sum of two bf16 numbers (its rounding and what the rounding left), 16 bits of mantissa and more, and
+// the row sums are taken over the fp32 values.
+// Where a score cap of at most kBoundedCap holds, weights need no running maximum: e^{+-cap} and its sums
+// stay inside fp32, so nothing is rescaled and partial results of different keys simply add up.
+
+constexpr float kBoundedCap = 60.0f;
+
+// Raw product -> base-2 exponent of the weight.
+struct Weighting {
+    float in, out;      // cap: exponent = out - 2 out / (1 + 2^{in s}); none: exponent = in s
+    bool capped;
+};
+static Weighting weighting_of(float scale, float cap) {
+    constexpr float kLog2e = 1.4426950408889634f;
+    if (cap > 0.f) return Weighting{2.0f * kLog2e * scale / cap, kLog2e * cap, true};
+    return Weighting{kLog2e * scale, 0.f, false};
+}
+__device__ __forceinline__ float exponent_of(const Weighting &w, bool capped, float s) {
+    if (capped) return fmaf(-2.0f * w.out, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(w.in * s)), w.out);
+    return w.in * s;
+}
+
+// Portions: a workgroup of four wavefronts takes 4 * 16 * NQ queries of one head and walks the keys of
+// their chunks in tiles of 64; K and V tiles go through registers into LDS, one tile ahead of the products.
+// DK, DV: sizes the registers are laid out for; the model's own sizes (multiples of 8) may be smaller.
+template <int DK, int DV, int NQ, bool kBounded>
+__global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kernel(const ChunkAttnArgs a, const Weighting w,
+                                                                                  const int32_t q_tiles) {
+    constexpr int kBM = 64 * NQ, kBN = 64;
+    constexpr int kKPitch = DK * 2 + 16, kVPitch = DV * 2 + 32;      // bytes; chosen so that operand reads spread over the banks
+    constexpr int kKPieces = DK / 32, kVPieces = DV / 32;           // 16-byte pieces of a tile per thread
+    __shared__ __attribute__((aligned(16))) unsigned char smem[2 * kBN * (kKPitch + kVPitch)];
+    const lds_char_ptr lds = (lds_char_ptr)(&smem[0]);
+    // kv heads fastest, query tiles last to first: as in the prefill kernel for whole contexts, the
+    // workgroups that share keys run close together on one XCD
+    const int group = a.heads / a.kv_heads;
+    const int g_kv = blockIdx.x % a.kv_heads;
+    int rest = blockIdx.x / a.kv_heads;
+    const int head = g_kv * group + rest % group;
+    rest /= group;
+    const int row0 = (q_tiles - 1 - rest % q_tiles) * kBM;
+    const int seq = rest / q_tiles;
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int r = lane & 15, g = lane >> 4;
+    const int t0 = a.cu[seq], lq = a.cu[seq + 1] - t0;
+    if (row0 >= lq) return;
+    const int start = a.klen[seq] - lq;
+    if (start < 0) return;
+    const int last_row = min(row0 + kBM, lq) - 1;
+    const int key_end = start + last_row;                            // last key any query of the tile sees
+    const int key_begin = (start + row0) / a.chunk * a.chunk & ~(kBN - 1);
+    const int ntiles = (key_end - key_begin) / kBN + 1;
+    const bf16_t *kc = static_cast<const bf16_t *>(a.k_cache) + static_cast<int64_t>(g_kv) * a.dim;
+    const bf16_t *vc = static_cast<const bf16_t *>(a.v_cache) + static_cast<int64_t>(g_kv) * a.vdim;
+    const int64_t kstride = static_cast<int64_t>(a.kv_heads) * a.dim, vstride = static_cast<int64_t>(a.kv_heads) * a.vdim;
+    const int bmask = (1 << a.block_shift) - 1;
+
+    // queries of this wavefront
+    int pos[NQ], lo[NQ];
+    u32x4_t qf[NQ][DK / 32];
+#pragma unroll
+    for (int qa = 0; qa < NQ; ++qa) {
+        const int row = row0 + wave * 16 * NQ + 16 * qa + r;
+        pos[qa] = start + row;
+        lo[qa] = pos[qa] / a.chunk * a.chunk;
+        const bf16_t *q = static_cast<const bf16_t *>(a.q) + static_cast<int64_t>(t0 + min(row, lq - 1)) * a.q_stride +
+                          static_cast<int64_t>(head) * a.dim + 8 * g;
+#pragma unroll
+        for (int ks = 0; ks < DK / 32; ++ks) {
+            qf[qa][ks] = u32x4_t{0, 0, 0, 0};
+            if (32 * ks + 8 * g < a.dim) qf[qa][ks] = *reinterpret_cast<const u32x4_t *>(q + 32 * ks);
+        }
+    }
+    const int w_first = start + row0 + wave * 16 * NQ;               // the wavefront's queries: first and last position
+    const int w_last = min(w_first + 16 * NQ - 1, key_end);
+    const bool w_live = row0 + wave * 16 * NQ < lq;
+    const int w_lo = w_first / a.chunk * a.chunk;                    // oldest key one of them sees
+    const int w_lo_all = w_last / a.chunk * a.chunk;                 // keys from here to w_first are seen by all
+
+    u32x4_t kreg[kKPieces], vreg[kVPieces];
+    auto fetch = [&](int tile) __attribute__((always_inline)) {
+        const int key0 = key_begin + tile * kBN;
+        const int col = key0 >> a.block_shift;
+        const int blk = col < a.max_blocks ? a.block_tables[seq * a.bt_stride + col] : -1;
+        const bool ok = static_cast<uint32_t>(blk) < static_cast<uint32_t>(a.num_blocks);
+        const int64_t base = (static_cast<int64_t>(ok ? blk : 0) << a.block_shift) + (key0 & bmask);
+#pragma unroll
+        for (int i = 0; i < kKPieces; ++i) {
+            const int p = i * 256 + tid, row = p / (DK / 8), e = p % (DK / 8) * 8;
+            kreg[i] = u32x4_t{0, 0, 0, 0};
+            if (ok && key0 + row <= key_end && e < a.dim) kreg[i] = *reinterpret_cast<const u32x4_t *>(kc + (base + row) * kstride + e);
+        }
+#pragma unroll
+        for (int i = 0; i < kVPieces; ++i) {
+            const int p = i * 256 + tid, row = p / (DV / 8), e = p % (DV / 8) * 8;
+            vreg[i] = u32x4_t{0, 0, 0, 0};
+            if (ok && key0 + row <= key_end && e < a.vdim) vreg[i] = *reinterpret_cast<const u32x4_t *>(vc + (base + row) * vstride + e);
+        }
+        return ok;
+    };
+    auto put = [&](int buf) __attribute__((always_inline)) {
+        const lds_char_ptr kl = lds + buf * kBN * kKPitch, vl = lds + 2 * kBN * kKPitch + buf * kBN * kVPitch;
+#pragma unroll
+        for (int i = 0; i < kKPieces; ++i) {
+            const int p = i * 256 + tid;
+            *(lds_u32x4_ptr)(kl + p / (DK / 8) * kKPitch + p % (DK / 8) * 16) = kreg[i];
+        }
+#pragma unroll
+        for (int i = 0; i < kVPieces; ++i) {
+            const int p = i * 256 + tid;
+            *(lds_u32x4_ptr)(vl + p / (DV / 8) * kVPitch + p % (DV / 8) * 16) = vreg[i];
+        }
+    };
+
+    f32x4_t oacc[DV / 16][NQ];
+    float lsum[NQ], m[NQ];
+#pragma unroll
+    for (int qa = 0; qa < NQ; ++qa) {
+        lsum[qa] = 0.f;
+        m[qa] = -INFINITY;
+#pragma unroll
+        for (int db = 0; db < DV / 16; ++db) oacc[db][qa] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    }
+
+    auto attend = [&](auto masked_c, int key0, int buf, bool ok) __attribute__((always_inline)) {
+        constexpr bool kMasked = decltype(masked_c)::value;
+        const lds_char_ptr kl = lds + buf * kBN * kKPitch + r * kKPitch + 16 * g;
+        const lds_char_ptr vl = lds + 2 * kBN * kKPitch + buf * kBN * kVPitch + (4 * g + (r >> 2)) * kVPitch + 8 * (r & 3);
+        f32x4_t sacc[4][NQ];
+#pragma unroll
+        for (int kb = 0; kb < 4; ++kb) {
+#pragma unroll
+            for (int qa = 0; qa < NQ; ++qa) sacc[kb][qa] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int ks = 0; ks < DK / 32; ++ks) {
+                const u32x4_t kf = *(lds_u32x4_ptr)(kl + kb * 16 * kKPitch + ks * 64);
+#pragma unroll
+                for (int qa = 0; qa < NQ; ++qa) sacc[kb][qa] = mfma16(kf, qf[qa][ks], sacc[kb][qa]);
+            }
+        }
+        auto seen = [&](int qa, int kb, int i) __attribute__((always_inline)) -> bool {
+            const int key = key0 + 16 * kb + 4 * g + i;
+            return !kMasked || (ok && key >= lo[qa] && key <= pos[qa]);
+        };
+        if (!kBounded) {
+#pragma unroll
+            for (int qa = 0; qa < NQ; ++qa) {
+                float mx = -INFINITY;
+#pragma unroll
+                for (int kb = 0; kb < 4; ++kb)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) {
+                        sacc[kb][qa][i] = exponent_of(w, w.capped, sacc[kb][qa][i]);
+                        if (seen(qa, kb, i)) mx = fmaxf(mx, sacc[kb][qa][i]);
+                    }
+                mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+                mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+                const float m_new = fmaxf(m[qa], mx);
+                const float keep = m[qa] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m[qa] - m_new);
+                m[qa] = m_new;
+                lsum[qa] *= keep;
+#pragma unroll
+                for (int db = 0; db < DV / 16; ++db)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) oacc[db][qa][i] *= keep;
+            }
+        }
+#pragma unroll
+        for (int half = 0; half < 2; ++half) {
+            u32x4_t ph[NQ], pl[NQ];
+#pragma unroll
+            for (int qa = 0; qa < NQ; ++qa)
+#pragma unroll
+                for (int kb2 = 0; kb2 < 2; ++kb2) {
+                    float p[4];
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) {
+                        const float s = sacc[2 * half + kb2][qa][i];
+                        const bool vis = seen(qa, 2 * half + kb2, i);
+                        const float x = kBounded ? exponent_of(w, true, s) : s - m[qa];
+                        p[i] = vis ? __builtin_amdgcn_exp2f(x) : 0.f;
+                        lsum[qa] += p[i];
+                    }
+                    uint32_t h0, l0, h1, l1;
+                    split_pair(p[0], p[1], h0, l0);
+                    split_pair(p[2], p[3], h1, l1);
+                    ph[qa][2 * kb2] = h0; ph[qa][2 * kb2 + 1] = h1;
+                    pl[qa][2 * kb2] = l0; pl[qa][2 * kb2 + 1] = l1;
+                }
+#pragma unroll
+            for (int db = 0; db < DV / 16; ++db) {
+                const s16x4_t v0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_ptr)(vl + (32 * half) * kVPitch + 32 * db));
+                const s16x4_t v1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_ptr)(vl + (32 * half + 16) * kVPitch + 32 * db));
+                const u32x4_t vf = __builtin_bit_cast(u32x4_t, __builtin_shufflevector(v0, v1, 0, 1, 2, 3, 4, 5, 6, 7));
+#pragma unroll
+                for (int qa = 0; qa < NQ; ++qa) {
+                    oacc[db][qa] = mfma16(vf, ph[qa], oacc[db][qa]);
+                    oacc[db][qa] = mfma16(vf, pl[qa], oacc[db][qa]);
+                }
+            }
+        }
+    };
+
+    bool ok = fetch(0);
+    put(0);
+    __syncthreads();
+    for (int tile = 0; tile < ntiles; ++tile) {
+        const int buf = tile & 1;
+        bool ok_next = false;
+        if (tile + 1 < ntiles) ok_next = fetch(tile + 1);
+        const int key0 = key_begin + tile * kBN;
+        if (w_live && key0 <= w_last && key0 + kBN > w_lo) {
+            if (ok && key0 >= w_lo_all && key0 + kBN - 1 <= w_first) attend(std::false_type{}, key0, buf, ok);
+            else attend(std::true_type{}, key0, buf, ok);
+        }
+        if (tile + 1 < ntiles) put(buf ^ 1);             // (the buffer was read two tiles ago, a barrier lies between)
+        ok = ok_next;
+        __syncthreads();
+    }
+    if (!w_live) return;
+#pragma unroll
+    for (int qa = 0; qa < NQ; ++qa) {
+        float l = lsum[qa];
+        l += __shfl_xor(l, 16, 64);
+        l += __shfl_xor(l, 32, 64);
+        const float inv = l > 0.f ? 1.0f / l : 0.f;
+        const int row = row0 + wave * 16 * NQ + 16 * qa + r;
+        if (row >= lq) continue;
+        bf16_t *out = static_cast<bf16_t *>(a.out) + (static_cast<int64_t>(t0 + row) * a.heads + head) * a.vdim + 4 * g;
+#pragma unroll
+        for (int db = 0; db < DV / 16; ++db)
+            if (16 * db + 4 * g < a.vdim) {
+                const f32x4_t o = oacc[db][qa];
+                *reinterpret_cast<u32x2_t *>(out + 16 * db) = u32x2_t{pack_bf16x2(o[0] * inv, o[1] * inv), pack_bf16x2(o[2] * inv, o[3] * inv)};
+            }
+    }
+}
+
+// Single tokens: a workgroup takes one (sequence, kv head, range of keys), its wavefronts tiles of 32 keys
+// in turn; up to 16 query heads of the kv head are the columns of the products.  K goes from memory
+// straight into operand registers, V through wavefront-private LDS for the transpose.  The four wavefronts
+// meet in LDS; with more than one range per pair the results are partial (fp32 sums with their
+// weights' sum and reference) and chunk_merge_kernel adds them up.
+struct SplitArgs {
+    float *partials;         // [n, splits, heads, vdim + 2]: sums, sum of the weights, reference exponent
+    int32_t splits, keys;    // ranges per sequence, keys per range (a multiple of 128)
+    int32_t head_groups;     // groups of 16 query heads per kv head
+};
+
+template <int DK, int DV, bool kBounded>
+__global__ __launch_bounds__(256) void chunk_decode_kernel(const ChunkAttnArgs a, const Weighting w, const SplitArgs sp) {
+    constexpr int kVPitch = DV * 2 + 32;
+    constexpr int kWaveBytes = 32 * kVPitch > 16 * DV * 4 ? 32 * kVPitch : 16 * DV * 4;
+    constexpr int kVPieces = DV / 16;                    // 16-byte pieces of a 32-key V tile per lane
+    __shared__ __attribute__((aligned(16))) unsigned char smem[4 * kWaveBytes];
+    __shared__ float sh_l[4][16], sh_m[4][16];
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int r = lane & 15, g = lane >> 4;
+    const int g_kv = blockIdx.x % a.kv_heads;
+    int rest = blockIdx.x / a.kv_heads;
+    const int hg = rest % sp.head_groups;
+    rest /= sp.head_groups;
+    const int split = rest % sp.splits, seq = rest / sp.splits;
+    const int group = a.heads / a.kv_heads;
+    const int head0 = g_kv * group + hg * 16, nheads = min(16, group - hg * 16);
+    const int pos = a.klen[seq] - 1;
+    bf16_t *out = static_cast<bf16_t *>(a.out) + (static_cast<int64_t>(seq) * a.heads + head0) * a.vdim;
+    if (pos < 0) {
+        if (sp.splits == 1)
+            for (int i = tid; i < nheads * a.vdim; i += 256) out[i] = 0;
+        return;
+    }
+    const int lo = pos / a.chunk * a.chunk, first = (lo & ~31) + split * sp.keys;
+    const int last = min(pos, first + sp.keys - 1);      // last key of this range
+    if (first > last) return;
+    const int ntiles = (last - first) / 32 + 1;
+    const bf16_t *kc = static_cast<const bf16_t *>(a.k_cache) + static_cast<int64_t>(g_kv) * a.dim;
+    const bf16_t *vc = static_cast<const bf16_t *>(a.v_cache) + static_cast<int64_t>(g_kv) * a.vdim;
+    const int64_t kstride = static_cast<int64_t>(a.kv_heads) * a.dim, vstride = static_cast<int64_t>(a.kv_heads) * a.vdim;
+    const int bmask = (1 << a.block_shift) - 1;
+    const lds_char_ptr vlds = (lds_char_ptr)(&smem[0]) + wave * kWaveBytes;
+
+    auto block_of = [&](int tile) __attribute__((always_inline)) -> int {
+        const int col = (first + tile * 32) >> a.block_shift;
+        return tile < ntiles && col < a.max_blocks ? a.block_tables[seq * a.bt_stride + col] : -1;
+    };
+    u32x4_t kreg[2][DK / 32], vreg[kVPieces];
+    auto fetch = [&](int tile, int blk) __attribute__((always_inline)) {
+        const int key0 = first + tile * 32;
+        const bool ok = static_cast<uint32_t>(blk) < static_cast<uint32_t>(a.num_blocks);
+        const int64_t base = (static_cast<int64_t>(ok ? blk : 0) << a.block_shift) + (key0 & bmask);
+#pragma unroll
+        for (int kb = 0; kb < 2; ++kb) {
+            const int row = 16 * kb + r;
+            const bf16_t *k = kc + (base + row) * kstride + 8 * g;
+#pragma unroll
+            for (int ks = 0; ks < DK / 32; ++ks) {
+                kreg[kb][ks] = u32x4_t{0, 0, 0, 0};
+                if (ok && key0 + row <= last && 32 * ks + 8 * g < a.dim)
+                    kreg[kb][ks] = __builtin_nontemporal_load(reinterpret_cast<const u32x4_t *>(k + 32 * ks));
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < kVPieces; ++i) {
+            const int p = i * 64 + lane, row = p / (DV / 8), e = p % (DV / 8) * 8;
+            vreg[i] = u32x4_t{0, 0, 0, 0};
+            if (ok && key0 + row <= last && e < a.vdim)
+                vreg[i] = __builtin_nontemporal_load(reinterpret_cast<const u32x4_t *>(vc + (base + row) * vstride + e));
+        }
+    };
+    int tile = wave;
+    int blk = block_of(tile), blk_next = block_of(tile + 4);
+    if (tile < ntiles) fetch(tile, blk);
+    u32x4_t qf[DK / 32];
+    {
+        const bf16_t *q = static_cast<const bf16_t *>(a.q) + static_cast<int64_t>(seq) * a.q_stride +
+                          static_cast<int64_t>(head0 + min(r, nheads - 1)) * a.dim + 8 * g;
+#pragma unroll
+        for (int ks = 0; ks < DK / 32; ++ks) {
+            qf[ks] = u32x4_t{0, 0, 0, 0};
+            if (32 * ks + 8 * g < a.dim) qf[ks] = *reinterpret_cast<const u32x4_t *>(q + 32 * ks);
+        }
+    }
+    f32x4_t oacc[DV / 16];
+#pragma unroll
+    for (int db = 0; db < DV / 16; ++db) oacc[db] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    float lsum = 0.f, m = -INFINITY;
+    const lds_char_ptr vl = vlds + (4 * g + (r >> 2)) * kVPitch + 8 * (r & 3);
+    for (; tile < ntiles; tile += 4) {
+        const int key0 = first + tile * 32;
+        const bool ok = static_cast<uint32_t>(blk) < static_cast<uint32_t>(a.num_blocks);
+#pragma unroll
+        for (int i = 0; i < kVPieces; ++i) {
+            const int p = i * 64 + lane;
+            *(lds_u32x4_ptr)(vlds + p / (DV / 8) * kVPitch + p % (DV / 8) * 16) = vreg[i];
+        }
+        f32x4_t s[2];
+#pragma unroll
+        for (int kb = 0; kb < 2; ++kb) {
+            s[kb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int ks = 0; ks < DK / 32; ++ks) s[kb] = mfma16(kreg[kb][ks], qf[ks], s[kb]);
+        }
+        const int blk_this = blk_next;                   // of tile + 4
+        blk_next = block_of(tile + 8);
+        if (tile + 4 < ntiles) fetch(tile + 4, blk_this);
+        blk = blk_this;
+        float x[2][4], mx = -INFINITY;
+        bool vis[2][4];
+#pragma unroll
+        for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int key = key0 + 16 * kb + 4 * g + i;
+                vis[kb][i] = ok && key >= lo && key <= last;
+                x[kb][i] = exponent_of(w, kBounded || w.capped, s[kb][i]);
+                if (vis[kb][i]) mx = fmaxf(mx, x[kb][i]);
+            }
+        float ref = 0.f;
+        if (!kBounded) {
+            mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+            mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+            const float m_new = fmaxf(m, mx);
+            const float keep = m == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m - m_new);
+            m = m_new;
+            ref = m_new == -INFINITY ? 0.f : m_new;
+            lsum *= keep;
+#pragma unroll
+            for (int db = 0; db < DV / 16; ++db)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) oacc[db][i] *= keep;
+        }
+        u32x4_t ph, pl;
+#pragma unroll
+        for (int kb = 0; kb < 2; ++kb) {
+            float p[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                p[i] = vis[kb][i] ? __builtin_amdgcn_exp2f(x[kb][i] - ref) : 0.f;
+                lsum += p[i];
+            }
+            uint32_t h0, l0, h1, l1;
+            split_pair(p[0], p[1], h0, l0);
+            split_pair(p[2], p[3], h1, l1);
+            ph[2 * kb] = h0; ph[2 * kb + 1] = h1;
+            pl[2 * kb] = l0; pl[2 * kb + 1] = l1;
+        }
+        // (wavefront-private LDS: in order within the wavefront, no barrier)
+#pragma unroll
+        for (int db = 0; db < DV / 16; ++db) {
+            const s16x4_t v0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_ptr)(vl + 32 * db));
+            const s16x4_t v1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_ptr)(vl + 16 * kVPitch + 32 * db));
+            const u32x4_t vf = __builtin_bit_cast(u32x4_t, __builtin_shufflevector(v0, v1, 0, 1, 2, 3, 4, 5, 6, 7));
+            oacc[db] = mfma16(vf, ph, oacc[db]);
+            oacc[db] = mfma16(vf, pl, oacc[db]);
+        }
+    }
+    lsum += __shfl_xor(lsum, 16, 64);
+    lsum += __shfl_xor(lsum, 32, 64);
+    if (g == 0) { sh_l[wave][r] = lsum; sh_m[wave][r] = m; }
+    // the wavefront's sums over its own V tile (read for the last time above)
+    float *osh = reinterpret_cast<float *>(&smem[wave * kWaveBytes]);
+#pragma unroll
+    for (int db = 0; db < DV / 16; ++db) *reinterpret_cast<f32x4_t *>(osh + r * DV + 16 * db + 4 * g) = oacc[db];
+    __syncthreads();
+    for (int i = tid; i < nheads * a.vdim; i += 256) {
+        const int h = i / a.vdim, c = i % a.vdim;
+        float top = 0.f, l = 0.f, o = 0.f;
+        if (!kBounded) top = fmaxf(fmaxf(sh_m[0][h], sh_m[1][h]), fmaxf(sh_m[2][h], sh_m[3][h]));
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            const float f = kBounded ? 1.0f : (sh_m[v][h] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(sh_m[v][h] - top));
+            l = fmaf(sh_l[v][h], f, l);
+            o = fmaf(reinterpret_cast<const float *>(&smem[v * kWaveBytes])[h * DV + c], f, o);
+        }
+        if (sp.splits == 1) {
+            out[i] = f32_to_bf16(l > 0.f ? o / l : 0.f);
+        } else {
+            float *part = sp.partials + ((static_cast<int64_t>(seq) * sp.splits + split) * a.heads + head0 + h) * (a.vdim + 2);
+            part[c] = o;
+            if (c == 0) { part[a.vdim] = l; part[a.vdim + 1] = kBounded ? 0.f : top; }
+        }
+    }
+}
+
+// One wavefront per (row, head): adds the partial results of the ranges that hold keys.
+__global__ __launch_bounds__(256) void chunk_merge_kernel(const ChunkAttnArgs a, const SplitArgs sp) {
+    const int lane = threadIdx.x & 63;
+    const int64_t item = static_cast<int64_t>(blockIdx.x) * 4 + (threadIdx.x >> 6);
+    if (item >= static_cast<int64_t>(a.n) * a.heads) return;
+    const int seq = static_cast<int>(item / a.heads), head = static_cast<int>(item % a.heads);
+    const int pos = a.klen[seq] - 1;
+    bf16_t *out = static_cast<bf16_t *>(a.out) + item * a.vdim;
+    const int lo = pos < 0 ? 0 : pos / a.chunk * a.chunk & ~31;
+    const int count = pos < 0 ? 0 : min(sp.splits, (pos - lo) / sp.keys + 1);
+    const int pitch = a.vdim + 2;
+    const float *part = sp.partials + (static_cast<int64_t>(seq) * sp.splits * a.heads + head) * pitch;
+    const int64_t step = static_cast<int64_t>(a.heads) * pitch;
+    // lane j holds sum and reference of range j (up to 64 ranges)
+    const float my_l = lane < count ? part[lane * step + a.vdim] : 0.f;
+    const float my_m = lane < count ? part[lane * step + a.vdim + 1] : -INFINITY;
+    const float top = wave_max(my_m);
+    const float f = my_m == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(my_m - top);
+    const float l = wave_sum(my_l * f);
+    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    for (int c = lane; c < a.vdim; c += 64) {
+        float o = 0.f;
+        for (int j = 0; j < count; ++j) o = fmaf(part[j * step + c], __shfl(f, j, 64), o);
+        out[c] = f32_to_bf16(o * inv);
+    }
+}
+
+// How the keys of a decode step are split: enough ranges to fill the machine, not more than 64, none
+// shorter than 256 keys.  Depends on shapes only.
+static SplitArgs plan_splits(int64_t n, int32_t heads, int32_t kv_heads, int32_t max_blocks, int32_t block_size, int32_t chunk) {
+    SplitArgs sp{};
+    sp.head_groups = (heads / kv_heads + 15) / 16;
+    const int64_t most = std::min(static_cast<int64_t>(chunk), static_cast<int64_t>(max_blocks) * block_size) + 31;   // keys one query can see, from a multiple of 32 on
+    const int64_t pairs = std::max(static_cast<int64_t>(1), n * kv_heads * sp.head_groups);
+    int64_t keys = std::max(static_cast<int64_t>(256), most * pairs / 4096);
+    keys = std::max(keys, (most + 63) / 64);
+    keys = (keys + 127) / 128 * 128;
+    sp.keys = static_cast<int32_t>(keys);
+    sp.splits = static_cast<int32_t>(std::max(static_cast<int64_t>(1), (most + keys - 1) / keys));
+    return sp;
+}
+
+template <int DK, int DV>
+static int launch_matrix(const ChunkAttnArgs &a, const SplitArgs &sp, int32_t max_q, hipStream_t s) {
+    const bool bounded = a.cap > 0.f && a.cap <= kBoundedCap;
+    const Weighting w = weighting_of(a.scale, a.cap);
+    if (a.cu == nullptr) {
+        const int64_t wgs = static_cast<int64_t>(a.n) * sp.splits * sp.head_groups * a.kv_heads;
+        if (wgs > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
+        const dim3 grid(static_cast<uint32_t>(wgs)), block(256);
+        if (bounded) hipLaunchKernelGGL((chunk_decode_kernel<DK, DV, true>), grid, block, 0, s, a, w, sp);
+        else hipLaunchKernelGGL((chunk_decode_kernel<DK, DV, false>), grid, block, 0, s, a, w, sp);
+        const int rc = launch_status();
+        if (rc != NVA_OK || sp.splits == 1) return rc;
+        hipLaunchKernelGGL(chunk_merge_kernel, dim3(static_cast<uint32_t>((static_cast<int64_t>(a.n) * a.heads + 3) / 4)), block, 0, s, a, sp);
+        return launch_status();
+    }
+    constexpr int NQ = DK > 128 || DV > 128 ? 1 : 2;
+    const int32_t q_tiles = (max_q + 64 * NQ - 1) / (64 * NQ);
+    const int64_t wgs = static_cast<int64_t>(a.n_seqs) * q_tiles * a.heads;
+    if (wgs > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
+    if (wgs == 0) return NVA_OK;
+    const dim3 grid(static_cast<uint32_t>(wgs)), block(256);
+    if (bounded) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, true>), grid, block, 0, s, a, w, q_tiles);
+    else hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, false>), grid, block, 0, s, a, w, q_tiles);
+    return launch_status();
+}
+
+template <int DK>
+static int launch_matrix_dk(const ChunkAttnArgs &a, const SplitArgs &sp, int32_t max_q, hipStream_t s) {
+    if (a.vdim <= 64) return launch_matrix<DK, 64>(a, sp, max_q, s);
+    if (a.vdim <= 128) return launch_matrix<DK, 128>(a, sp, max_q, s);
+    return launch_matrix<DK, 256>(a, sp, max_q, s);
+}
+
+static bool matrix_ok(const ChunkAttnArgs &a) {
+    return a.dim % 8 == 0 && a.vdim % 8 == 0 && a.dim <= 256 && a.vdim <= 256 && a.q_stride % 8 == 0 && aligned16(a.q) &&
+           aligned16(a.k_cache) && aligned16(a.v_cache) && aligned16(a.out);
+}
+
 template <typename T>
 static int launch_any(const ChunkAttnArgs &a, hipStream_t s) {
     const int64_t items = static_cast<int64_t>(a.n) * a.heads;
@@ -105,10 +621,18 @@ static int launch_any(const ChunkAttnArgs &a, hipStream_t s) {
 
 }  // namespace nva
 
+extern "C" size_t nva_chunk_attn_workspace_bytes(int32_t n_tokens, int32_t num_heads, int32_t num_kv_heads, int32_t v_dim,
+                                                 int32_t max_blocks, int32_t block_size, int32_t chunk) {
+    if (n_tokens <= 0 || num_heads <= 0 || num_kv_heads <= 0 || v_dim <= 0 || max_blocks < 0 || block_size <= 0 || chunk <= 0) return 0;
+    const nva::SplitArgs sp = nva::plan_splits(n_tokens, num_heads, num_kv_heads, max_blocks, block_size, chunk);
+    if (sp.splits == 1) return 0;
+    return static_cast<size_t>(n_tokens) * sp.splits * num_heads * (v_dim + 2) * sizeof(float);
+}
+
 extern "C" int nva_chunk_attn(const void *q, int64_t q_row_stride, const void *k_cache, const void *v_cache,
                               const int32_t *block_tables, int64_t bt_row_stride, int32_t max_blocks,
                               const int32_t *cu_seqlens_q, const int32_t *seq_lens, const int32_t *token_seq, void *out,
-                              int32_t n_tokens, int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads,
+                              void *workspace, size_t workspace_bytes, int32_t n_tokens, int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads,
                               int32_t num_kv_heads, int32_t qk_dim, int32_t v_dim, int32_t block_size,
                               int32_t num_blocks, int32_t chunk, float scale, float softcap, int32_t dtype,
                               void *stream) {
@@ -132,5 +656,21 @@ extern "C" int nva_chunk_attn(const void *q, int64_t q_row_stride, const void *k
     a.block_shift = shift; a.num_blocks = num_blocks; a.max_blocks = max_blocks; a.chunk = chunk; a.scale = scale;
     a.cap = softcap;
     hipStream_t s = static_cast<hipStream_t>(stream);
+    if (dtype == NVA_DTYPE_BF16 && matrix_ok(a)) {
+        SplitArgs sp{};
+        if (decode) {
+            sp = plan_splits(n_tokens, num_heads, num_kv_heads, max_blocks, block_size, chunk);
+            sp.partials = static_cast<float *>(workspace);
+            if (sp.splits > 1) {
+                if (!workspace) return NVA_ERR_NULL_POINTER;
+                if (!aligned16(workspace)) return NVA_ERR_MISALIGNED;
+                if (workspace_bytes < nva_chunk_attn_workspace_bytes(n_tokens, num_heads, num_kv_heads, v_dim, max_blocks, block_size, chunk))
+                    return NVA_ERR_WORKSPACE_TOO_SMALL;
+            }
+        }
+        if (qk_dim <= 64) return launch_matrix_dk<64>(a, sp, max_seqlen_q, s);
+        if (qk_dim <= 128) return launch_matrix_dk<128>(a, sp, max_seqlen_q, s);
+        return launch_matrix_dk<256>(a, sp, max_seqlen_q, s);
+    }
     return dtype == NVA_DTYPE_BF16 ? launch_any<bf16_t>(a, s) : launch_any<float>(a, s);
 }

@@ -39,6 +39,24 @@ def _need_cuda(*tensors) -> None:
             raise RuntimeError("nanovllm_amd ops run on the GPU only (there is no CPU fallback)")
 
 
+_scratch: Dict[torch.device, torch.Tensor] = {}
+_retired_scratch: list = []
+
+
+def scratch(device: torch.device, nbytes: int) -> torch.Tensor:
+    """Scratch memory of the mixers' kernels, one buffer per device (their calls are ordered on one
+    stream).  It grows outside graph capture only: a captured call is preceded by an eager one of the
+    same shape.  A replaced buffer lives on, because graphs captured earlier hold its address."""
+    ws = _scratch.get(device)
+    if ws is None or ws.numel() < nbytes:
+        if torch.cuda.is_current_stream_capturing():
+            raise RuntimeError("scratch memory must be sized by an eager call before graph capture")
+        if ws is not None:
+            _retired_scratch.append(ws)
+        ws = _scratch[device] = torch.empty(max(nbytes, 1 << 20), dtype=torch.uint8, device=device)
+    return ws
+
+
 # ---- ops -----------------------------------------------------------------------------------------
 
 def embed_norm(ids: torch.Tensor, table: torch.Tensor, scale: float, norm: Tuple[torch.Tensor, torch.Tensor], eps: float):
@@ -116,10 +134,14 @@ def chunk_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     assert out.is_contiguous() and q.dtype == out.dtype == k_cache.dtype == v_cache.dtype
     table = group.block_tables
     assert table.dtype == torch.int32 and table.shape[0] == group.num_seqs and table.stride(1) == 1
-    rc = _lib.load().nva_chunk_attn(
+    chunk, lib, ws = min(chunk, 1 << 30), _lib.load(), None
+    if group.cu is None and q.dtype == torch.bfloat16:
+        nbytes = lib.nva_chunk_attn_workspace_bytes(group.count, heads, kv_heads, vdim, table.shape[1], block, chunk)
+        ws = scratch(q.device, nbytes) if nbytes else None
+    rc = lib.nva_chunk_attn(
         q.data_ptr(), q.stride(0), k_cache.data_ptr(), v_cache.data_ptr(), table.data_ptr(), table.stride(0), table.shape[1],
-        _ptr(group.cu), group.seq_lens.data_ptr(), _ptr(group.token_seq), out.data_ptr(), group.count, group.num_seqs,
-        group.max_q, heads, kv_heads, dim, vdim, block, num_blocks, min(chunk, 1 << 30), float(scale), float(softcap or 0.0),
+        _ptr(group.cu), group.seq_lens.data_ptr(), _ptr(group.token_seq), out.data_ptr(), _ptr(ws), 0 if ws is None else ws.numel(),
+        group.count, group.num_seqs, group.max_q, heads, kv_heads, dim, vdim, block, num_blocks, chunk, float(scale), float(softcap or 0.0),
         _DTYPE[q.dtype], _stream())
     _lib.check(rc, "nva_chunk_attn")
 
@@ -131,10 +153,14 @@ def retention(qkvg: torch.Tensor, state: torch.Tensor, group: RowGroup, position
     assert qkvg.stride(1) == 1 and qkvg.shape == (group.count, 2 * heads * (dim + vdim))
     assert out.shape == (group.count, heads * vdim) and out.is_contiguous() and out.dtype == qkvg.dtype
     assert state.dtype == torch.float32 and state.is_contiguous() and log2_decay.dtype == torch.float32
-    rc = _lib.load().nva_retention(
+    lib, ws = _lib.load(), None
+    if group.cu is not None:
+        nbytes = lib.nva_retention_workspace_bytes(group.num_seqs, group.max_q, heads, dim, vdim, rot_dims, _DTYPE[qkvg.dtype])
+        ws = scratch(qkvg.device, nbytes) if nbytes else None
+    rc = lib.nva_retention(
         qkvg.data_ptr(), qkvg.stride(0), state.data_ptr(), group.state_slots.data_ptr(), _ptr(group.cu),
-        group.seq_lens.data_ptr(), positions.data_ptr(), _ptr(rope), log2_decay.data_ptr(), out.data_ptr(), group.count,
-        group.num_seqs, group.max_q, heads, dim, vdim, rot_dims, 1 if rope is None else rope.shape[0], slots, float(k_scale),
+        group.seq_lens.data_ptr(), positions.data_ptr(), _ptr(rope), log2_decay.data_ptr(), out.data_ptr(), _ptr(ws),
+        0 if ws is None else ws.numel(), group.count, group.num_seqs, group.max_q, heads, dim, vdim, rot_dims, 1 if rope is None else rope.shape[0], slots, float(k_scale),
         float(eps), _DTYPE[qkvg.dtype], _stream())
     _lib.check(rc, "nva_retention")
 
