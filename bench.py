@@ -15,6 +15,7 @@ already resident in HBM.  Workloads (shapes are the five benchmark configuration
     glue      residual add + RMSNorm (--glue add-rms-norm) or SiLU(gate) * up (--glue silu-mul), 16,384 rows (--tokens N)
     decode-e2e-shape / decode-longctx-shape / copy   profiling helpers: the decode attention of configs 4 / 5
               alone (one layer); a plain copy of known size
+    kaparax   the Kaparax family beside Qwen3 at equal size: engine prefill / decode tok/s and every kernel beside its like
     read-probe    calibration: a bare streaming read at the sizes of the bandwidth-bound workloads
 The line carries `roofline` (algorithmic bytes or flops of the dominant kernel per launch,
 divided by its average duration measured with HIP events on the launch stream) and
@@ -830,9 +831,242 @@ def bench_longctx(args, dev):
     return result, (lambda: None)
 
 
-WORKLOADS = {"rope-scatter": bench_rope_scatter, "glue": bench_glue, "e2e": bench_e2e, "longctx": bench_longctx, "decode-e2e-shape": bench_decode_e2e_shape,
+def _kaparax_config(layers, width, heads, kv_heads, dim, ff, ret_heads, ret_dim, chunk, vocab):
+    """Attention and retention layers in turn, each with a feed-forward: as many layers as the model it is put beside."""
+    from nanovllm_amd.engine.kaparax import KaparaxConfig
+    ret = dict(type="retention", mixer=dict(heads=ret_heads, dim=ret_dim, vdim=ret_dim, rot=dict(base=1e6, dims=ret_dim),
+                                            decay=[1.0 - 2.0 ** (-5.0 - 0.5 * h) for h in range(ret_heads)]))
+    attn = dict(type="attention", mixer=dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, conv=4, mask=dict(size=chunk),
+                                             scale=dim ** -0.5, softcap=30.0, rot=dict(base=1e4, dims=dim)))
+    mlp = dict(kind="dense", ff=ff, limit=7.0)
+    return KaparaxConfig.from_raw(dict(architecture="Kaparax", vocab=vocab, width=width, embedding=dict(scale=width ** 0.5),
+                                       norm=dict(eps=1e-6), layers=[dict(attn if i % 2 == 0 else ret, mlp=mlp) for i in range(layers)]))
+
+
+def _kernel_row(name, us, alg, bound, like=None):
+    """One kernel beside the like kernel of the Qwen3 path: time, achieved share of the bounding peak, and how
+    many times farther from it."""
+    peak = HBM_PEAK_GBPS * 1e9 if bound == "hbm" else MFMA_BF16_PEAK_TFLOPS * 1e12
+    frac = alg / (us * 1e-6) / peak
+    row = {"kernel": name, "us": round(us, 2), "bound": bound, "algorithmic": int(alg), "frac": round(frac, 4)}
+    if like is not None:
+        lname, lus, lalg, lbound = like
+        lpeak = HBM_PEAK_GBPS * 1e9 if lbound == "hbm" else MFMA_BF16_PEAK_TFLOPS * 1e12
+        lfrac = lalg / (lus * 1e-6) / lpeak
+        row.update(like=lname, like_us=round(lus, 2), like_frac=round(lfrac, 4), times_farther=round(lfrac / frac, 2))
+    return row
+
+
+def kaparax_kernels(dev, steps=60, only=None):
+    """Every kernel of the Kaparax layers at sizes of a real layer (16 / 8 heads of 128, width 1024, feed-forward
+    3072; retention 8 heads of 128 x 128), each beside the Qwen3 path's like kernel at equal size, in one process.
+    Launches rotate through separate buffers where re-reads could come from a cache."""
+    import torch
+    import nanovllm_amd as nva
+    from nanovllm_amd.context import DecodePlan, RowGroup
+    from nanovllm_amd.engine import layers, mixers
+    from nanovllm_amd import synthetic
+    bf = torch.bfloat16
+    rnd = lambda *shape: torch.randn(*shape, device=dev).to(bf)
+    i32 = lambda x: torch.as_tensor(x, dtype=torch.int32).to(dev)
+    rows = []
+    want = lambda name: only is None or only in name
+    heads, kv, d, width, ff, rh = 16, 8, 128, 1024, 3072, 8
+    table = mixers.RopeTables(16384 + 256, dev).get(mixers.Rotary(1e4, d))
+    graph_us = lambda fns, n=200: _graph_time_ms(fns, n, 10)[0] / n * 1e3
+    event_us = lambda fns, n=steps: _steady_time_ms(fns, n, max(3, n // 10))[0] / n * 1e3
+
+    # ---- attention over portions
+    for what, lens, chunk in (("2x16384, one chunk", [16384, 16384], 16384), ("2x16384, chunks of 2048", [16384, 16384], 2048),
+                              ("16 x U[100,1024], chunks of 8192", None, 8192)):
+        if not want("attention prefill"):
+            continue
+        if lens is None:
+            g = torch.Generator().manual_seed(0)
+            lens = torch.randint(100, 1025, (16,), generator=g).tolist()
+        n, need = sum(lens), [-(-l // 256) for l in lens]
+        ids = torch.randperm(sum(need)).tolist()
+        tabs, at = [], 0
+        for k in need:
+            tabs.append(ids[at: at + k] + [-1] * (max(need) - k))
+            at += k
+        cu = [0]
+        for l in lens:
+            cu.append(cu[-1] + l)
+        kc, vc = rnd(sum(need), 256, kv, d), rnd(sum(need), 256, kv, d)
+        group = RowGroup(0, n, len(lens), i32(lens), i32([0] * n), i32(tabs), i32([0] * len(lens)), i32(cu),
+                         i32([i for i, l in enumerate(lens) for _ in range(l)]), max(lens))
+        q, out = rnd(n, heads * d), torch.empty(n, heads * d, dtype=bf, device=dev)
+        mine = event_us([lambda: mixers.chunk_attention(q, kc, vc, group, out, heads, chunk, d ** -0.5, 30.0)])
+        theirs = event_us([lambda: nva.varlen_prefill_attention(q.view(n, heads, d), kc, vc, group.cu, group.cu, max(lens), max(lens),
+                                                                d ** -0.5, block_table=group.block_tables)])
+        full = sum(l * (l + 1) // 2 for l in lens)
+        seen = sum((l // chunk) * (chunk * (chunk + 1) // 2) + (l % chunk) * (l % chunk + 1) // 2 for l in lens)
+        rows.append(_kernel_row("attention prefill, " + what, mine, 4 * d * heads * seen, "mfma",
+                                ("prefill_attn_kernel (whole context)", theirs, 4 * d * heads * full, "mfma")))
+        del kc, vc, q, out
+
+    # ---- attention of single tokens
+    for what, batch, ctx, chunk, pools in (("batch 64, ctx U[100,2048]", 64, (100, 2048), 8192, 4), ("batch 256, ctx U[300,1326]", 256, (300, 1326), 8192, 2),
+                                           ("batch 16, ctx U[4096,8192]", 16, (4096, 8192), 8192, 4), ("batch 1, ctx 8192", 1, (8192, 8192), 8192, 4)):
+        if not want("attention decode"):
+            continue
+        g = torch.Generator().manual_seed(1)
+        lens = torch.randint(ctx[0], ctx[1] + 1, (batch,), generator=g)
+        blocks = int(((lens + 255) // 256).sum())
+        tabs = synthetic.decode_tables(lens.tolist(), blocks, g).to(dev)
+        group = RowGroup(0, batch, batch, i32(lens), i32([0] * batch), tabs, i32([0] * batch))
+        q, out = rnd(batch, heads * d), torch.empty(batch, heads * d, dtype=bf, device=dev)
+        caches = [(rnd(blocks, 256, kv, d), rnd(blocks, 256, kv, d)) for _ in range(pools)]
+        mine = graph_us([lambda c=c: mixers.chunk_attention(q, c[0], c[1], group, out, heads, chunk, d ** -0.5, 30.0) for c in caches], 56)
+        alg = int(lens.sum()) * kv * d * 4 + 4 * q.numel()
+        state = {"n": 0, "plan": None}
+
+        def like(c):
+            if state["n"] % 28 == 0:
+                state["plan"] = DecodePlan(torch.cuda.is_current_stream_capturing())
+            state["n"] += 1
+            nva.paged_decode_attention(q.view(batch, heads, d), c[0], c[1], group.seq_lens, tabs, d ** -0.5, plan=state["plan"])
+        fns = [lambda c=c: like(c) for c in caches]
+        state["n"] = 0
+        theirs = _event_time_ms(fns, 84, 28) / 84 * 1e3
+        rows.append(_kernel_row("attention decode, " + what, mine, alg, "hbm", ("decode_stream_kernel + merge", theirs, alg, "hbm")))
+        del caches
+
+    # ---- retention
+    for what, lens in (("1x16384", [16384]), ("2x16384", [16384, 16384]), ("16x1024", [1024] * 16), ("29 x U[100,1024]", None)):
+        if not want("retention prefill"):
+            continue
+        if lens is None:
+            g = torch.Generator().manual_seed(0)
+            lens = torch.randint(100, 1025, (29,), generator=g).tolist()
+        n = sum(lens)
+        cu = [0]
+        for l in lens:
+            cu.append(cu[-1] + l)
+        group = RowGroup(0, n, len(lens), i32(lens), i32([0] * n), None, i32(list(range(len(lens)))), i32(cu), i32([0] * n), max(lens))
+        x, out = rnd(n, 4 * rh * d), torch.empty(n, rh * d, dtype=bf, device=dev)
+        pos = torch.cat([torch.arange(l) for l in lens]).to(dev)
+        state = torch.zeros(len(lens), rh, d, d, device=dev)
+        decay = torch.full((rh,), -0.01, device=dev)
+        mine = event_us([lambda: mixers.retention(x, state, group, pos, table, decay, out, d, d ** -0.5, 1e-6)])
+        rows.append(_kernel_row("retention prefill, " + what, mine, n * rh * d * 5 * 2 + state.numel() * 4 + n * d * 4, "hbm"))
+        rows[-1]["tokens_per_s"] = round(n / mine * 1e6)
+        rows[-1]["tflops_of_one_product_each"] = round(n * rh * (8 * d * d + 4 * 32 * d / 2) / mine / 1e6, 1)
+    for batch in (1, 64, 256):
+        if not want("retention decode"):
+            continue
+        states = [torch.zeros(batch, rh, d, d, device=dev) for _ in range(4)]
+        group = RowGroup(0, batch, batch, i32([800] * batch), i32([0] * batch), None, i32(list(range(batch))))
+        x, out = rnd(batch, 4 * rh * d), torch.empty(batch, rh * d, dtype=bf, device=dev)
+        pos = torch.full((batch,), 799, dtype=torch.int64, device=dev)
+        decay = torch.full((rh,), -0.01, device=dev)
+        mine = graph_us([lambda s=s: mixers.retention(x, s, group, pos, table, decay, out, d, d ** -0.5, 1e-6) for s in states])
+        rows.append(_kernel_row("retention decode, batch %d" % batch, mine, states[0].numel() * 8, "hbm"))
+        del states
+
+    # ---- steps around them
+    for n in (256, 16384):
+        if want("norm"):
+            y, r32, r16 = rnd(n, width), torch.randn(n, width, device=dev), rnd(n, width)
+            w = [rnd(width) for _ in range(4)]
+            mine = graph_us([lambda: mixers.post_add_norm(y, r32, (w[0], w[1]), (w[2], w[3]), 1e-6)])
+            theirs = graph_us([lambda: layers.add_rms_norm(y, r16, w[0], 1e-6)])
+            rows.append(_kernel_row("norm + add + norm, %d rows" % n, mine, n * width * (2 + 4 + 4 + 2), "hbm",
+                                    ("rms_norm_kernel (add)", theirs, n * width * 8, "hbm")))
+        if want("gate"):
+            x = rnd(n, 2 * ff)
+            rows.append(_kernel_row("clamped gate, %d rows" % n, graph_us([lambda: mixers.clamped_gate(x, 7.0, 1.702)]), n * ff * 6, "hbm",
+                                    ("silu_and_mul_kernel", graph_us([lambda: layers.silu_and_mul(x)]), n * ff * 6, "hbm")))
+        if want("convolution"):
+            single = n == 256
+            ch = (heads + 2 * kv) * d
+            x, conv, q = rnd(n, ch), rnd(4, ch), torch.empty(n, heads * d, dtype=bf, device=dev)
+            blocks = n // 256 + n if single else n // 256
+            kc, vc = (torch.empty(n // 256, 256, kv, d, dtype=bf, device=dev) for _ in range(2))
+            slots = i32(torch.randperm(n) if single else list(range(n)))
+            nseq = n if single else 16
+            st = rnd(nseq, 3, ch)
+            per = n // nseq
+            pos = (torch.full((n,), 700, dtype=torch.int64) if single else torch.arange(n) % per).to(dev)
+            group = RowGroup(0, n, nseq, i32([701] * n if single else [per] * 16), slots, None, i32(list(range(nseq))))
+            if not single:
+                group.cu, group.token_seq, group.max_q = i32(list(range(0, n + 1, per))), i32([i // per for i in range(n)]), per
+            mine = graph_us([lambda: mixers.conv_rope_store(x, conv, st, group, pos, table, q, kc, vc, heads, d)])
+            ones, rope = rnd(d), layers.build_rope_cache(d, 4096, 1e4, dev)
+            theirs = graph_us([lambda: layers.qk_norm_rope(x, pos, ones, ones, rope, heads, kv, d, 1e-6, kv_store=(kc, vc, slots))])
+            # read once, q / k / v written once; carried rows read and written (decode), cos / sin per token
+            alg = n * ch * 4 + n * d * 4 + (n * 6 * ch * 2 if single else 0)
+            alg_like = n * (ch * 4 + kv * d * 2) + n * d * 4
+            rows.append(_kernel_row("convolution + rotation + cache write, %d rows" % n, mine, alg, "hbm", ("qk_norm_rope_kernel", theirs, alg_like, "hbm")))
+    return rows
+
+
+def _engine_rates(model, dev, batch, prompt_len, new_tokens, slots):
+    """Prefill and decode tokens/s of the engine: ``batch`` prompts of ``prompt_len`` tokens, ``new_tokens`` each."""
+    import gc
+    import random
+    import torch
+    from nanovllm_amd.engine import SamplingParams
+    from nanovllm_amd.engine.llm import LLM
+    blocks = batch * (-(-(prompt_len + new_tokens + 1) // 256)) + 8
+    llm = LLM(model, max_model_len=4096, max_num_seqs=slots, num_kvcache_blocks=blocks)
+    rng = random.Random(0)
+    vocab = model.vocab_size
+
+    def run(tag, n_new):
+        prompts = [[rng.randrange(vocab) for _ in range(prompt_len)] for _ in range(batch)]
+        for p in prompts:
+            llm.add_request(p, SamplingParams(temperature=0.6, ignore_eos=True, max_tokens=n_new))
+        torch.cuda.synchronize()
+        t, kinds = time.perf_counter(), {True: [0.0, 0], False: [0.0, 0]}
+        while not llm.is_finished():
+            _, k = llm.step()
+            if not llm.scheduler.waiting and k > 0:       # prefill ends here: everything behind it is decoding
+                torch.cuda.synchronize()
+            now = time.perf_counter()
+            kinds[k > 0][0] += now - t
+            kinds[k > 0][1] += abs(k)
+            t = now
+        return kinds
+    run("warm", 8)
+    k = run("timed", new_tokens)
+    del llm
+    gc.collect()
+    torch.cuda.empty_cache()
+    return {"prefill_tok_s": round(k[True][1] / k[True][0]), "decode_tok_s": round(k[False][1] / k[False][0])}
+
+
+def bench_kaparax(args, dev):
+    """The Kaparax family beside Qwen3 at equal size: engine throughput (prompts of 1024 tokens, then 128 decoded
+    tokens each) for two layer sizes and two batches, and every kernel beside its like (--kaparax-part)."""
+    from nanovllm_amd.engine import ModelConfig, qwen3_0_6b
+    part = args.kaparax_part
+    kernels = kaparax_kernels(dev, only=args.kernel) if part in ("all", "kernels") else []
+    engines = {}
+    if part in ("all", "engine"):
+        sizes = {"28 layers, width 1024, 16/8 heads x 128, ff 3072": (
+                     _kaparax_config(28, 1024, 16, 8, 128, 3072, 8, 128, 8192, 151936), qwen3_0_6b()),
+                 "8 layers, width 4096, 32/8 heads x 128, ff 12288": (
+                     _kaparax_config(8, 4096, 32, 8, 128, 12288, 16, 128, 8192, 151936),
+                     ModelConfig(hidden_size=4096, num_hidden_layers=8, num_attention_heads=32, num_key_value_heads=8,
+                                 intermediate_size=12288, tie_word_embeddings=False))}
+        for what, (mine, like) in sizes.items():
+            for batch in (16, 128):
+                engines["%s; batch %d" % (what, batch)] = {"kaparax": _engine_rates(mine, dev, batch, 1024, 128, 128),
+                                                           "qwen3": _engine_rates(like, dev, batch, 1024, 128, 128)}
+    first = next(iter(engines.values()))["kaparax"]["decode_tok_s"] if engines else None
+    result = {"metric": "Kaparax decode tok/s (28 layers of width 1024, batch 16, prompts of 1024)", "value": first, "unit": "tok/s",
+              "ms_per_step": round(16e3 / first, 3) if first else None,
+              "config": {"workload": "random weights; attention and retention layers in turn, chunks of 8192, score cap 30", "engine": engines,
+                         "kernels": kernels},
+              "roofline": None}
+    return result, lambda: None
+
+
+WORKLOADS = {"kaparax": bench_kaparax, "rope-scatter": bench_rope_scatter, "glue": bench_glue, "e2e": bench_e2e, "longctx": bench_longctx, "decode-e2e-shape": bench_decode_e2e_shape,
              "decode-longctx-shape": bench_decode_longctx_shape, "copy": bench_copy, "read-probe": bench_read_probe, "decode": bench_decode, "scatter": bench_scatter, "prefill": bench_prefill, "sampler": bench_sampler}
-DEFAULT_STEPS = {"rope-scatter": 100, "glue": 100, "e2e": 1, "longctx": 1, "decode-e2e-shape": 1, "decode-longctx-shape": 1, "copy": 50, "read-probe": 60, "decode": 200, "scatter": 400, "prefill": 50, "sampler": 100}
+DEFAULT_STEPS = {"kaparax": 60, "rope-scatter": 100, "glue": 100, "e2e": 1, "longctx": 1, "decode-e2e-shape": 1, "decode-longctx-shape": 1, "copy": 50, "read-probe": 60, "decode": 200, "scatter": 400, "prefill": 50, "sampler": 100}
 
 
 def main():
@@ -853,6 +1087,8 @@ def main():
     ap.add_argument("--glue", choices=["add-rms-norm", "silu-mul", "last-token-norm"], default="add-rms-norm", help="glue: which elementwise kernel")
     ap.add_argument("--uniform", default=None, metavar="SxL", help="prefill: S packed sequences of L tokens each instead of config 3 (e.g. 2x16384)")
     ap.add_argument("--bucket-step", type=int, default=16, help="e2e only: spacing of the captured decode batch sizes")
+    ap.add_argument("--kaparax-part", choices=["all", "kernels", "engine"], default="all", help="kaparax: which half of the workload")
+    ap.add_argument("--kernel", default=None, help="kaparax: only kernels whose row name contains this")
     ap.add_argument("--no-extra", action="store_true", help="e2e only: skip the per-configuration rooflines and the eager pass")
     args = ap.parse_args()
     if args.gpus != 1:
