@@ -128,15 +128,20 @@ __device__ __forceinline__ float exponent_of(const Weighting &w, bool capped, fl
 }
 
 // Portions: a workgroup of four wavefronts takes 4 * 16 * NQ queries of one head and walks the keys of
-// their chunks in tiles of 64; K and V tiles go through registers into LDS, one tile ahead of the products.
-// DK, DV: sizes the registers are laid out for; the model's own sizes (multiples of 8) may be smaller.
-template <int DK, int DV, int NQ, bool kBounded>
+// their chunks in tiles of 64, double-buffered in LDS.  DK, DV: sizes the registers are laid out for.
+// kDirect (the model's sizes are exactly these): tiles travel global -> LDS without a register in between,
+// the LDS image laid out in 1 KB blocks of 16 keys x 32 dims with the 16-byte pieces permuted so that
+// operand reads spread over the banks -- the scheme of the prefill kernel for whole contexts, whose
+// description gives the permutations.  Otherwise (smaller sizes, multiples of 8) tiles go through registers
+// into padded rows, zero-filled to DK and DV.
+template <int DK, int DV, int NQ, bool kBounded, bool kDirect>
 __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kernel(const ChunkAttnArgs a, const Weighting w,
                                                                                   const int32_t q_tiles) {
     constexpr int kBM = 64 * NQ, kBN = 64;
     constexpr int kKPitch = DK * 2 + 16, kVPitch = DV * 2 + 32;      // bytes; chosen so that operand reads spread over the banks
     constexpr int kKPieces = DK / 32, kVPieces = DV / 32;           // 16-byte pieces of a tile per thread
-    __shared__ __attribute__((aligned(16))) unsigned char smem[2 * kBN * (kKPitch + kVPitch)];
+    constexpr int kKTile = kDirect ? kBN * DK * 2 : kBN * kKPitch, kVTile = kDirect ? kBN * DV * 2 : kBN * kVPitch;
+    __shared__ __attribute__((aligned(1024))) unsigned char smem[2 * (kKTile + kVTile)];
     const lds_char_ptr lds = (lds_char_ptr)(&smem[0]);
     // kv heads fastest, query tiles last to first: as in the prefill kernel for whole contexts, the
     // workgroups that share keys run close together on one XCD
@@ -185,38 +190,65 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
     const int w_lo = w_first / a.chunk * a.chunk;                    // oldest key one of them sees
     const int w_lo_all = w_last / a.chunk * a.chunk;                 // keys from here to w_first are seen by all
 
-    u32x4_t kreg[kKPieces], vreg[kVPieces];
-    auto fetch = [&](int tile) __attribute__((always_inline)) {
+    // ---- tiles into LDS.  Direct: a tile's block id is asked for one tile ahead (in a vector register, so
+    // that nothing waits for it before it is used), its loads go out while the tile before it is multiplied.
+    int lane_zero;
+    asm volatile("v_mov_b32 %0, 0" : "=v"(lane_zero));
+    auto block_of = [&](int tile) __attribute__((always_inline)) -> int {
+        const int col = (key_begin + tile * kBN) >> a.block_shift;
+        return a.block_tables[seq * a.bt_stride + min(col, a.max_blocks - 1) + lane_zero];
+    };
+    u32x4_t kreg[kDirect ? 1 : kKPieces], vreg[kDirect ? 1 : kVPieces];
+    const int lk16 = lane >> 2, lj = lane & 3;
+    const uint32_t lds_k0 = __builtin_amdgcn_readfirstlane(static_cast<uint32_t>(reinterpret_cast<uintptr_t>(lds)) + wave * (DK / 32) * 1024);
+    const uint32_t lds_v0 = __builtin_amdgcn_readfirstlane(static_cast<uint32_t>(reinterpret_cast<uintptr_t>(lds)) + 2 * kKTile + wave * (DV / 32) * 1024);
+    uint32_t koff = 0, voff = 0;
+    auto fetch = [&](int tile, int blk_v, int buf) __attribute__((always_inline)) -> bool {
         const int key0 = key_begin + tile * kBN;
-        const int col = key0 >> a.block_shift;
-        const int blk = col < a.max_blocks ? a.block_tables[seq * a.bt_stride + col] : -1;
+        const int blk = __builtin_amdgcn_readfirstlane(blk_v);
         const bool ok = static_cast<uint32_t>(blk) < static_cast<uint32_t>(a.num_blocks);
         const int64_t base = (static_cast<int64_t>(ok ? blk : 0) << a.block_shift) + (key0 & bmask);
+        if constexpr (kDirect) {
+            const int row = min(wave * 16 + lk16, key_end - key0);   // rows past the last key repeat it and are masked
+            koff = static_cast<uint32_t>(row * kstride + (lj ^ ((0 - (lk16 >> 2)) & 3)) * 8) * 2;
+            voff = static_cast<uint32_t>(row * vstride + (lj ^ (2 * ((lk16 >> 2) & 1))) * 8) * 2;
+            const char *kb = reinterpret_cast<const char *>(kc + base * kstride), *vb = reinterpret_cast<const char *>(vc + base * vstride);
 #pragma unroll
-        for (int i = 0; i < kKPieces; ++i) {
-            const int p = i * 256 + tid, row = p / (DK / 8), e = p % (DK / 8) * 8;
-            kreg[i] = u32x4_t{0, 0, 0, 0};
-            if (ok && key0 + row <= key_end && e < a.dim) kreg[i] = *reinterpret_cast<const u32x4_t *>(kc + (base + row) * kstride + e);
-        }
+            for (int x = 0; x < DK / 32; ++x) load_to_lds_16(kb + 64 * x, koff, lds_k0 + buf * kKTile + 1024 * x);
 #pragma unroll
-        for (int i = 0; i < kVPieces; ++i) {
-            const int p = i * 256 + tid, row = p / (DV / 8), e = p % (DV / 8) * 8;
-            vreg[i] = u32x4_t{0, 0, 0, 0};
-            if (ok && key0 + row <= key_end && e < a.vdim) vreg[i] = *reinterpret_cast<const u32x4_t *>(vc + (base + row) * vstride + e);
+            for (int x = 0; x < DV / 32; ++x) load_to_lds_16(vb + 64 * x, voff, lds_v0 + buf * kVTile + 1024 * x);
+        } else {
+#pragma unroll
+            for (int i = 0; i < kKPieces; ++i) {
+                const int p = i * 256 + tid, row = p / (DK / 8), e = p % (DK / 8) * 8;
+                kreg[i] = u32x4_t{0, 0, 0, 0};
+                if (ok && key0 + row <= key_end && e < a.dim) kreg[i] = *reinterpret_cast<const u32x4_t *>(kc + (base + row) * kstride + e);
+            }
+#pragma unroll
+            for (int i = 0; i < kVPieces; ++i) {
+                const int p = i * 256 + tid, row = p / (DV / 8), e = p % (DV / 8) * 8;
+                vreg[i] = u32x4_t{0, 0, 0, 0};
+                if (ok && key0 + row <= key_end && e < a.vdim) vreg[i] = *reinterpret_cast<const u32x4_t *>(vc + (base + row) * vstride + e);
+            }
         }
         return ok;
     };
     auto put = [&](int buf) __attribute__((always_inline)) {
-        const lds_char_ptr kl = lds + buf * kBN * kKPitch, vl = lds + 2 * kBN * kKPitch + buf * kBN * kVPitch;
+        if constexpr (kDirect) {
+            loads_issued(koff, voff);
+            asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        } else {
+            const lds_char_ptr kl = lds + buf * kKTile, vl = lds + 2 * kKTile + buf * kVTile;
 #pragma unroll
-        for (int i = 0; i < kKPieces; ++i) {
-            const int p = i * 256 + tid;
-            *(lds_u32x4_ptr)(kl + p / (DK / 8) * kKPitch + p % (DK / 8) * 16) = kreg[i];
-        }
+            for (int i = 0; i < kKPieces; ++i) {
+                const int p = i * 256 + tid;
+                *(lds_u32x4_ptr)(kl + p / (DK / 8) * kKPitch + p % (DK / 8) * 16) = kreg[i];
+            }
 #pragma unroll
-        for (int i = 0; i < kVPieces; ++i) {
-            const int p = i * 256 + tid;
-            *(lds_u32x4_ptr)(vl + p / (DV / 8) * kVPitch + p % (DV / 8) * 16) = vreg[i];
+            for (int i = 0; i < kVPieces; ++i) {
+                const int p = i * 256 + tid;
+                *(lds_u32x4_ptr)(vl + p / (DV / 8) * kVPitch + p % (DV / 8) * 16) = vreg[i];
+            }
         }
     };
 
@@ -230,25 +262,35 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
         for (int db = 0; db < DV / 16; ++db) oacc[db][qa] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
 
-    auto attend = [&](auto masked_c, int key0, int buf, bool ok) __attribute__((always_inline)) {
+    auto attend = [&](auto masked_c, int key0, int buf) __attribute__((always_inline)) {
         constexpr bool kMasked = decltype(masked_c)::value;
-        const lds_char_ptr kl = lds + buf * kBN * kKPitch + r * kKPitch + 16 * g;
-        const lds_char_ptr vl = lds + 2 * kBN * kKPitch + buf * kBN * kVPitch + (4 * g + (r >> 2)) * kVPitch + 8 * (r & 3);
+        const lds_char_ptr kl = lds + buf * kKTile + (kDirect ? 16 * (4 * r + (g ^ ((0 - (r >> 2)) & 3))) : r * kKPitch + 16 * g);
+        const lds_char_ptr vl = lds + 2 * kKTile + buf * kVTile + (4 * g + (r >> 2)) * (kDirect ? 64 : kVPitch) + 8 * (r & 3);
+        auto kpiece = [&](int kb, int ks) __attribute__((always_inline)) -> u32x4_t {
+            return *(lds_u32x4_ptr)(kl + (kDirect ? (kb * (DK / 32) + ks) * 1024 : kb * 16 * kKPitch + ks * 64));
+        };
+        auto vpiece = [&](int kb, int db) __attribute__((always_inline)) -> s16x4_t {
+            return __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_ptr)(
+                vl + (kDirect ? (kb * (DV / 32) + (db >> 1)) * 1024 + 32 * ((g ^ db) & 1) : kb * 16 * kVPitch + 32 * db)));
+        };
         f32x4_t sacc[4][NQ];
-#pragma unroll
-        for (int kb = 0; kb < 4; ++kb) {
+        auto scores = [&](int kb) __attribute__((always_inline)) {
 #pragma unroll
             for (int qa = 0; qa < NQ; ++qa) sacc[kb][qa] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int ks = 0; ks < DK / 32; ++ks) {
-                const u32x4_t kf = *(lds_u32x4_ptr)(kl + kb * 16 * kKPitch + ks * 64);
+                const u32x4_t kf = kpiece(kb, ks);
 #pragma unroll
                 for (int qa = 0; qa < NQ; ++qa) sacc[kb][qa] = mfma16(kf, qf[qa][ks], sacc[kb][qa]);
             }
+        };
+        if (!kBounded) {
+#pragma unroll
+            for (int kb = 0; kb < 4; ++kb) scores(kb);
         }
         auto seen = [&](int qa, int kb, int i) __attribute__((always_inline)) -> bool {
             const int key = key0 + 16 * kb + 4 * g + i;
-            return !kMasked || (ok && key >= lo[qa] && key <= pos[qa]);
+            return !kMasked || (key >= lo[qa] && key <= pos[qa]);
         };
         if (!kBounded) {
 #pragma unroll
@@ -275,6 +317,10 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
         }
 #pragma unroll
         for (int half = 0; half < 2; ++half) {
+            if (kBounded) {                              // half a tile at a time: fewer registers
+                scores(2 * half);
+                scores(2 * half + 1);
+            }
             u32x4_t ph[NQ], pl[NQ];
 #pragma unroll
             for (int qa = 0; qa < NQ; ++qa)
@@ -297,8 +343,7 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
                 }
 #pragma unroll
             for (int db = 0; db < DV / 16; ++db) {
-                const s16x4_t v0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_ptr)(vl + (32 * half) * kVPitch + 32 * db));
-                const s16x4_t v1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_ptr)(vl + (32 * half + 16) * kVPitch + 32 * db));
+                const s16x4_t v0 = vpiece(2 * half, db), v1 = vpiece(2 * half + 1, db);
                 const u32x4_t vf = __builtin_bit_cast(u32x4_t, __builtin_shufflevector(v0, v1, 0, 1, 2, 3, 4, 5, 6, 7));
 #pragma unroll
                 for (int qa = 0; qa < NQ; ++qa) {
@@ -309,19 +354,23 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
         }
     };
 
-    bool ok = fetch(0);
+    int blk_next = block_of(1);
+    bool ok = fetch(0, block_of(0), 0);
     put(0);
     __syncthreads();
     for (int tile = 0; tile < ntiles; ++tile) {
         const int buf = tile & 1;
         bool ok_next = false;
-        if (tile + 1 < ntiles) ok_next = fetch(tile + 1);
-        const int key0 = key_begin + tile * kBN;
-        if (w_live && key0 <= w_last && key0 + kBN > w_lo) {
-            if (ok && key0 >= w_lo_all && key0 + kBN - 1 <= w_first) attend(std::false_type{}, key0, buf, ok);
-            else attend(std::true_type{}, key0, buf, ok);
+        if (tile + 1 < ntiles) {
+            ok_next = fetch(tile + 1, blk_next, buf ^ 1);            // (that buffer was read one tile ago, a barrier lies between)
+            blk_next = block_of(tile + 2);
         }
-        if (tile + 1 < ntiles) put(buf ^ 1);             // (the buffer was read two tiles ago, a barrier lies between)
+        const int key0 = key_begin + tile * kBN;
+        if (ok && w_live && key0 <= w_last && key0 + kBN > w_lo) {
+            if (key0 >= w_lo_all && key0 + kBN - 1 <= w_first) attend(std::false_type{}, key0, buf);
+            else attend(std::true_type{}, key0, buf);
+        }
+        if (tile + 1 < ntiles) put(buf ^ 1);
         ok = ok_next;
         __syncthreads();
     }
@@ -595,8 +644,13 @@ static int launch_matrix(const ChunkAttnArgs &a, const SplitArgs &sp, int32_t ma
     if (wgs > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
     if (wgs == 0) return NVA_OK;
     const dim3 grid(static_cast<uint32_t>(wgs)), block(256);
-    if (bounded) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, true>), grid, block, 0, s, a, w, q_tiles);
-    else hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, false>), grid, block, 0, s, a, w, q_tiles);
+    if (a.dim == DK && a.vdim == DV) {
+        if (bounded) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, true, true>), grid, block, 0, s, a, w, q_tiles);
+        else hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, false, true>), grid, block, 0, s, a, w, q_tiles);
+    } else {
+        if (bounded) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, true, false>), grid, block, 0, s, a, w, q_tiles);
+        else hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, false, false>), grid, block, 0, s, a, w, q_tiles);
+    }
     return launch_status();
 }
 

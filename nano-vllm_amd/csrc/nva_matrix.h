@@ -37,4 +37,23 @@ __device__ __forceinline__ void split8(const float (&v)[8], u32x4_t &hi, u32x4_t
     }
 }
 
+// global -> LDS without a register in between: lane l's 16 bytes at base + voff land at LDS byte
+// address lds_addr + 16 l.  Written as inline assembly on purpose: the compiler would make every
+// LDS read that follows its own builtin wait for the load (it cannot tell the two LDS buffers
+// apart), which would serialise the prefetch of the next tile with the arithmetic of this one.
+// The caller waits with s_waitcnt vmcnt(0) before the barrier that publishes the tile.
+// (s_nop 0: the load needs one wait state after the write of m0, which the compiler cannot provide
+// for an instruction it does not see.  Its scalar operands are always results of scalar
+// arithmetic; one written by a vector instruction -- v_readfirstlane -- would need five.)
+__device__ __forceinline__ void load_to_lds_16(const void *base, uint32_t &voff, uint32_t lds_addr) {
+    // Not volatile, and the offset register is declared as written although it keeps its value: the
+    // statement is then an ordinary instruction that the scheduler may place anywhere between the
+    // computation of its operands and the next use of the offset (a volatile statement is a fence
+    // for every LDS read and cuts the block into separately scheduled pieces).  The loads of one
+    // tensor form a chain through the offset; loads_issued() ends the chains before the wait.
+    asm("s_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, %1"
+        : "+v"(voff) : "s"(base), "s"(lds_addr) : "m0");
+}
+__device__ __forceinline__ void loads_issued(uint32_t koff, uint32_t voff) { asm volatile("" :: "v"(koff), "v"(voff)); }
+
 }  // namespace nva

@@ -41,22 +41,13 @@
 //
 // The causal mask is aligned to the end of the keys: query i sees keys j <= i + (Lk - Lq).
 // Work: 4 * 128 flop per (query, visible key, head).
-#include "nva_common.h"
+#include "nva_matrix.h"
 
 #include <math.h>
 
 #include <type_traits>
 
 namespace nva {
-
-typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
-typedef float f32x4_t __attribute__((ext_vector_type(4)));
-typedef uint32_t u32x4_t __attribute__((ext_vector_type(4)));   // plain vectors: stay in registers
-typedef short s16x4_t __attribute__((ext_vector_type(4)));
-typedef short s16x8_t __attribute__((ext_vector_type(8)));
-typedef __attribute__((address_space(3))) char *lds_char_ptr;
-typedef __attribute__((address_space(3))) u32x4_t *lds_u32x4_ptr;
-typedef __attribute__((address_space(3))) s16x4_t *lds_s16x4_ptr;
 
 constexpr int kPfThreads = 256;
 constexpr int kPfBM = 128;            // queries per workgroup
@@ -76,27 +67,6 @@ struct PrefillArgs {
     int32_t block_shift;     // log2 of the tokens per KV block
     float scale_log2e;
 };
-
-__device__ __forceinline__ bf16x8_t as_bf16x8(const u32x4_t &u) { return __builtin_bit_cast(bf16x8_t, u); }
-
-// global -> LDS without a register in between: lane l's 16 bytes at base + voff land at LDS byte
-// address lds_addr + 16 l.  Written as inline assembly on purpose: the compiler would make every
-// LDS read that follows its own builtin wait for the load (it cannot tell the two LDS buffers
-// apart), which would serialise the prefetch of the next tile with the arithmetic of this one.
-// The caller waits with s_waitcnt vmcnt(0) before the barrier that publishes the tile.
-// (s_nop 0: the load needs one wait state after the write of m0, which the compiler cannot provide
-// for an instruction it does not see.  Its scalar operands are always results of scalar
-// arithmetic; one written by a vector instruction -- v_readfirstlane -- would need five.)
-__device__ __forceinline__ void load_to_lds_16(const void *base, uint32_t &voff, uint32_t lds_addr) {
-    // Not volatile, and the offset register is declared as written although it keeps its value: the
-    // statement is then an ordinary instruction that the scheduler may place anywhere between the
-    // computation of its operands and the next use of the offset (a volatile statement is a fence
-    // for every LDS read and cuts the block into separately scheduled pieces).  The loads of one
-    // tensor form a chain through the offset; loads_issued() ends the chains before the wait.
-    asm("s_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, %1"
-        : "+v"(voff) : "s"(base), "s"(lds_addr) : "m0");
-}
-__device__ __forceinline__ void loads_issued(uint32_t koff, uint32_t voff) { asm volatile("" :: "v"(koff), "v"(voff)); }
 
 template <bool kPaged>
 __global__ __launch_bounds__(kPfThreads, 2) void prefill_attn_kernel(const PrefillArgs a) {
