@@ -949,7 +949,7 @@ def kaparax_kernels(dev, steps=60, only=None):
         pos = torch.cat([torch.arange(l) for l in lens]).to(dev)
         state = torch.zeros(len(lens), rh, d, d, device=dev)
         decay = torch.full((rh,), -0.01, device=dev)
-        mine = event_us([lambda: mixers.retention(x, state, group, pos, table, decay, out, d, d ** -0.5, 1e-6)])
+        mine = event_us([lambda: mixers.retention(x, state, group, table, decay, out, d, d ** -0.5, 1e-6)])
         rows.append(_kernel_row("retention prefill, " + what, mine, n * rh * d * 5 * 2 + state.numel() * 4 + n * d * 4, "hbm"))
         rows[-1]["tokens_per_s"] = round(n / mine * 1e6)
         rows[-1]["tflops_of_one_product_each"] = round(n * rh * (8 * d * d + 4 * 32 * d / 2) / mine / 1e6, 1)
@@ -961,7 +961,7 @@ def kaparax_kernels(dev, steps=60, only=None):
         x, out = rnd(batch, 4 * rh * d), torch.empty(batch, rh * d, dtype=bf, device=dev)
         pos = torch.full((batch,), 799, dtype=torch.int64, device=dev)
         decay = torch.full((rh,), -0.01, device=dev)
-        mine = graph_us([lambda s=s: mixers.retention(x, s, group, pos, table, decay, out, d, d ** -0.5, 1e-6) for s in states])
+        mine = graph_us([lambda s=s: mixers.retention(x, s, group, table, decay, out, d, d ** -0.5, 1e-6) for s in states])
         rows.append(_kernel_row("retention decode, batch %d" % batch, mine, states[0].numel() * 8, "hbm"))
         del states
 
@@ -992,7 +992,7 @@ def kaparax_kernels(dev, steps=60, only=None):
             group = RowGroup(0, n, nseq, i32([701] * n if single else [per] * 16), slots, None, i32(list(range(nseq))))
             if not single:
                 group.cu, group.token_seq, group.max_q = i32(list(range(0, n + 1, per))), i32([i // per for i in range(n)]), per
-            mine = graph_us([lambda: mixers.conv_rope_store(x, conv, st, group, pos, table, q, kc, vc, heads, d)])
+            mine = graph_us([lambda: mixers.conv_rope_store(x, conv, st, group, table, q, kc, vc, heads, d)])
             ones, rope = rnd(d), layers.build_rope_cache(d, 4096, 1e4, dev)
             theirs = graph_us([lambda: layers.qk_norm_rope(x, pos, ones, ones, rope, heads, kv, d, 1e-6, kv_store=(kc, vc, slots))])
             # read once, q / k / v written once; carried rows read and written (decode), cos / sin per token

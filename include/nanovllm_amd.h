@@ -334,7 +334,7 @@ int nva_clamped_gate(const void *x, int64_t x_row_stride, void *out, int32_t row
  * rope_cache: fp32 [max_position, rot_dims], cos in the first half of a row, sin in the second. */
 int nva_conv_rope_store(const void *qkv, int64_t qkv_row_stride, const void *conv_weight, void *conv_state,
                         const int32_t *state_slots_of_seq, const int32_t *cu_seqlens_q, const int32_t *seq_lens,
-                        const int32_t *token_seq, const int64_t *positions, const float *rope_cache,
+                        const int32_t *token_seq, const float *rope_cache,
                         void *q_out, void *k_cache, void *v_cache, const int32_t *slot_mapping,
                         int64_t num_slots, int32_t n_tokens, int32_t n_seqs, int32_t num_heads,
                         int32_t num_kv_heads, int32_t qk_dim, int32_t v_dim, int32_t rot_dims, int32_t taps,
@@ -370,7 +370,7 @@ int nva_chunk_attn(const void *q, int64_t q_row_stride, const void *k_cache, con
 size_t nva_retention_workspace_bytes(int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads, int32_t qk_dim,
                                      int32_t v_dim, int32_t rot_dims, int32_t dtype);
 int nva_retention(const void *qkvg, int64_t row_stride, float *state, const int32_t *state_slots_of_seq,
-                  const int32_t *cu_seqlens_q, const int32_t *seq_lens, const int64_t *positions,
+                  const int32_t *cu_seqlens_q, const int32_t *seq_lens,
                   const float *rope_cache, const float *log2_decay, void *out, void *workspace,
                   size_t workspace_bytes, int32_t n_tokens, int32_t n_seqs,
                   int32_t max_seqlen_q, int32_t num_heads, int32_t qk_dim, int32_t v_dim, int32_t rot_dims,

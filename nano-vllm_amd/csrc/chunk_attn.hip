@@ -405,7 +405,7 @@ struct SplitArgs {
 };
 
 template <int DK, int DV, bool kBounded>
-__global__ __launch_bounds__(256) void chunk_decode_kernel(const ChunkAttnArgs a, const Weighting w, const SplitArgs sp) {
+__global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 3) void chunk_decode_kernel(const ChunkAttnArgs a, const Weighting w, const SplitArgs sp) {
     constexpr int kVPitch = DV * 2 + 32;
     constexpr int kWaveBytes = 32 * kVPitch > 16 * DV * 4 ? 32 * kVPitch : 16 * DV * 4;
     constexpr int kVPieces = DV / 16;                    // 16-byte pieces of a 32-key V tile per lane
@@ -414,11 +414,14 @@ __global__ __launch_bounds__(256) void chunk_decode_kernel(const ChunkAttnArgs a
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int r = lane & 15, g = lane >> 4;
-    const int g_kv = blockIdx.x % a.kv_heads;
-    int rest = blockIdx.x / a.kv_heads;
-    const int hg = rest % sp.head_groups;
-    rest /= sp.head_groups;
-    const int split = rest % sp.splits, seq = rest / sp.splits;
+    // Workgroups are handed out in order, round-robin over XCDs and their CUs: sequences are the fastest index, so
+    // that ranges past the end of short sequences do not fall on the same CUs again and again (with the
+    // ranges of a sequence next to one another half the machine idled at four ranges)
+    const int seq = blockIdx.x % a.n;
+    int rest = blockIdx.x / a.n;
+    const int split = rest % sp.splits;
+    rest /= sp.splits;
+    const int g_kv = rest % a.kv_heads, hg = rest / a.kv_heads;
     const int group = a.heads / a.kv_heads;
     const int head0 = g_kv * group + hg * 16, nheads = min(16, group - hg * 16);
     const int pos = a.klen[seq] - 1;
@@ -608,15 +611,13 @@ __global__ __launch_bounds__(256) void chunk_merge_kernel(const ChunkAttnArgs a,
     }
 }
 
-// How the keys of a decode step are split: enough ranges to fill the machine, not more than 64, none
-// shorter than 256 keys.  Depends on shapes only.
-static SplitArgs plan_splits(int64_t n, int32_t heads, int32_t kv_heads, int32_t max_blocks, int32_t block_size, int32_t chunk) {
+// How the keys of a decode step are split: ranges of 512 keys, longer ones where that would be more than 64.
+// Depends on shapes only.
+static SplitArgs plan_splits(int32_t heads, int32_t kv_heads, int32_t max_blocks, int32_t block_size, int32_t chunk) {
     SplitArgs sp{};
     sp.head_groups = (heads / kv_heads + 15) / 16;
     const int64_t most = std::min(static_cast<int64_t>(chunk), static_cast<int64_t>(max_blocks) * block_size) + 31;   // keys one query can see, from a multiple of 32 on
-    const int64_t pairs = std::max(static_cast<int64_t>(1), n * kv_heads * sp.head_groups);
-    int64_t keys = std::max(static_cast<int64_t>(256), most * pairs / 4096);
-    keys = std::max(keys, (most + 63) / 64);
+    int64_t keys = std::max(static_cast<int64_t>(512), (most + 63) / 64);
     keys = (keys + 127) / 128 * 128;
     sp.keys = static_cast<int32_t>(keys);
     sp.splits = static_cast<int32_t>(std::max(static_cast<int64_t>(1), (most + keys - 1) / keys));
@@ -678,7 +679,7 @@ static int launch_any(const ChunkAttnArgs &a, hipStream_t s) {
 extern "C" size_t nva_chunk_attn_workspace_bytes(int32_t n_tokens, int32_t num_heads, int32_t num_kv_heads, int32_t v_dim,
                                                  int32_t max_blocks, int32_t block_size, int32_t chunk) {
     if (n_tokens <= 0 || num_heads <= 0 || num_kv_heads <= 0 || v_dim <= 0 || max_blocks < 0 || block_size <= 0 || chunk <= 0) return 0;
-    const nva::SplitArgs sp = nva::plan_splits(n_tokens, num_heads, num_kv_heads, max_blocks, block_size, chunk);
+    const nva::SplitArgs sp = nva::plan_splits(num_heads, num_kv_heads, max_blocks, block_size, chunk);
     if (sp.splits == 1) return 0;
     return static_cast<size_t>(n_tokens) * sp.splits * num_heads * (v_dim + 2) * sizeof(float);
 }
@@ -713,7 +714,7 @@ extern "C" int nva_chunk_attn(const void *q, int64_t q_row_stride, const void *k
     if (dtype == NVA_DTYPE_BF16 && matrix_ok(a)) {
         SplitArgs sp{};
         if (decode) {
-            sp = plan_splits(n_tokens, num_heads, num_kv_heads, max_blocks, block_size, chunk);
+            sp = plan_splits(num_heads, num_kv_heads, max_blocks, block_size, chunk);
             sp.partials = static_cast<float *>(workspace);
             if (sp.splits > 1) {
                 if (!workspace) return NVA_ERR_NULL_POINTER;

@@ -217,7 +217,6 @@ struct ConvRopeArgs {
     const int32_t *cu;              // portions: [n_seqs + 1] row bounds
     const int32_t *klen;            // tokens of every sequence once its rows are in (decode: 0 = padded row)
     const int32_t *token_seq;       // portions: sequence of every row
-    const int64_t *positions;       // [n]
     const float *rope;              // [max_position, rot_dims]: cos | sin
     void *q_out;                    // [n, H * dim]
     void *k_cache, *v_cache;        // flat [num_slots, G * dim], [num_slots, G * vdim]
@@ -227,12 +226,11 @@ struct ConvRopeArgs {
 };
 
 // A thread owns one group of V channels (two groups, i and i + half, where the rotation pairs them) and
-// walks kTokens consecutive rows with the taps - 1 rows before it in registers.  kTaps >= taps: missing
-// old taps have weight zero and are not read.  kDecode: every row is a sequence of its own, and the
-// thread also shifts its channels of the carried rows.
-template <typename T, int kTaps, int V, bool kDecode>
+// walks kTokens consecutive rows with the taps - 1 rows before it in registers and the next row on its way.
+// kTaps >= taps: missing old taps have weight zero and are not read.  kDecode: every row is a sequence of
+// its own, and the thread also shifts its channels of the carried rows.
+template <typename T, int kTaps, int V, int kTokens, bool kDecode>
 __global__ __launch_bounds__(256) void conv_rope_store_kernel(ConvRopeArgs a) {
-    constexpr int kTokens = kDecode ? 1 : 4;
     constexpr int kHist = kTaps - 1;
     const int pairs = a.half / V, rest = (a.dim - 2 * a.half) / V, per_head = pairs + rest;
     const int qk_units = (a.heads + a.kv_heads) * per_head;
@@ -261,6 +259,35 @@ __global__ __launch_bounds__(256) void conv_rope_store_kernel(ConvRopeArgs a) {
     const int64_t c1 = pair ? c0 + a.half : c0;
     const T *qkv = static_cast<const T *>(a.qkv);
     T *state = static_cast<T *>(a.state);
+    const int t_end = static_cast<int>(min(static_cast<int64_t>(a.n), t0 + kTokens));
+
+    // the sequence of the first row: its rows [first, row_end), its tokens before them
+    int seq, first, row_end, start, slot_s;
+    auto enter = [&](int s) __attribute__((always_inline)) {
+        seq = s;
+        if (kDecode) {
+            first = seq;
+            row_end = seq + 1;
+            start = a.klen[seq] - 1;
+        } else {
+            first = a.cu[seq];
+            row_end = a.cu[seq + 1];
+            start = a.klen[seq] - (row_end - first);
+        }
+        slot_s = a.taps > 1 ? a.slots_of_seq[seq] : -1;
+    };
+    enter(kDecode ? static_cast<int>(t0) : min(max(a.token_seq[t0], 0), a.n_seqs - 1));
+    if (kDecode && start < 0) {                           // padded row of a batch bucket
+        float zero[V];
+#pragma unroll
+        for (int i = 0; i < V; ++i) zero[i] = 0.f;
+        if (!is_v && head < a.heads) {
+            T *q = static_cast<T *>(a.q_out) + t0 * a.heads * a.dim + static_cast<int64_t>(head) * a.dim + off;
+            store_f32<T, V>(q, zero);
+            if (pair) store_f32<T, V>(q + a.half, zero);
+        }
+        return;
+    }
 
     float w0[kTaps][V], w1[kTaps][V];
 #pragma unroll
@@ -276,42 +303,30 @@ __global__ __launch_bounds__(256) void conv_rope_store_kernel(ConvRopeArgs a) {
     }
 
     float h0[kHist > 0 ? kHist : 1][V], h1[kHist > 0 ? kHist : 1][V];   // [b]: the row b + 1 back
-    int prev_seq = -1;
+    float x0[V], x1[V], n0[V], n1[V];
+    load_f32<T, V>(qkv + t0 * a.stride + c0, n0);
+    load_f32<T, V>(qkv + t0 * a.stride + c1, n1);
+    bool fresh = true;                                    // the history has to be read for this row's sequence
+#pragma unroll 4
+    for (int t = static_cast<int>(t0); t < t_end; ++t) {
 #pragma unroll
-    for (int step = 0; step < kTokens; ++step) {
-        const int64_t t = t0 + step;
-        if (t >= a.n) return;
-        int seq, first, start;
-        if (kDecode) {
-            seq = static_cast<int>(t);
-            first = seq;
-            start = a.klen[seq] - 1;
-        } else {
-            seq = min(max(a.token_seq[t], 0), a.n_seqs - 1);
-            first = a.cu[seq];
-            start = a.klen[seq] - (a.cu[seq + 1] - first);
+        for (int i = 0; i < V; ++i) { x0[i] = n0[i]; x1[i] = n1[i]; }
+        if (t + 1 < t_end) {
+            load_f32<T, V>(qkv + static_cast<int64_t>(t + 1) * a.stride + c0, n0);
+            load_f32<T, V>(qkv + static_cast<int64_t>(t + 1) * a.stride + c1, n1);
         }
-        const int slot_s = a.taps > 1 ? a.slots_of_seq[seq] : -1;
-        const bool have_state = start > 0 && static_cast<uint32_t>(slot_s) < static_cast<uint32_t>(a.state_slots);
-        if (kDecode && start < 0) {                       // padded row of a batch bucket
-            float zero[V];
-#pragma unroll
-            for (int i = 0; i < V; ++i) zero[i] = 0.f;
-            if (!is_v && head < a.heads) {
-                T *q = static_cast<T *>(a.q_out) + t * a.heads * a.dim + static_cast<int64_t>(head) * a.dim + off;
-                store_f32<T, V>(q, zero);
-                if (pair) store_f32<T, V>(q + a.half, zero);
-            }
-            return;
+        if (!kDecode && t >= row_end) {
+            int s = seq;
+            while (s + 1 < a.n_seqs && t >= a.cu[s + 1]) ++s;
+            enter(s);
+            fresh = true;
         }
-        float x0[V], x1[V];
-        load_f32<T, V>(qkv + t * a.stride + c0, x0);
-        load_f32<T, V>(qkv + t * a.stride + c1, x1);
-        if (seq != prev_seq) {
+        if (fresh) {
+            const bool have_state = start > 0 && static_cast<uint32_t>(slot_s) < static_cast<uint32_t>(a.state_slots);
 #pragma unroll
             for (int b = 0; b < kHist; ++b) {
-                const int64_t src = t - (b + 1);          // row b + 1 back, if it belongs to this portion
-                const int row_s = a.taps - 1 - (first - static_cast<int>(src));   // else this row of the carried ones
+                const int src = t - (b + 1);              // row b + 1 back, if it belongs to this portion
+                const int row_s = a.taps - 1 - (first - src);   // else this row of the carried ones
                 if (b + 1 < a.taps && src >= first) {
                     load_f32<T, V>(qkv + src * a.stride + c0, h0[b]);
                     load_f32<T, V>(qkv + src * a.stride + c1, h1[b]);
@@ -324,7 +339,7 @@ __global__ __launch_bounds__(256) void conv_rope_store_kernel(ConvRopeArgs a) {
                     for (int i = 0; i < V; ++i) h0[b][i] = h1[b][i] = 0.f;
                 }
             }
-            prev_seq = seq;
+            fresh = false;
         }
         float y0[V], y1[V];
 #pragma unroll
@@ -338,8 +353,8 @@ __global__ __launch_bounds__(256) void conv_rope_store_kernel(ConvRopeArgs a) {
             }
         }
         if (pair) {
-            const int64_t pos = min(max(a.positions[t], static_cast<int64_t>(0)), static_cast<int64_t>(a.max_position) - 1);
-            const float *cs = a.rope + pos * (2 * a.half) + ri;
+            const int pos = min(max(start + (t - first), 0), a.max_position - 1);
+            const float *cs = a.rope + static_cast<int64_t>(pos) * (2 * a.half) + ri;
             float c[V], s[V];
             load_f32<float, V>(cs, c);
             load_f32<float, V>(cs + a.half, s);
@@ -351,7 +366,7 @@ __global__ __launch_bounds__(256) void conv_rope_store_kernel(ConvRopeArgs a) {
             }
         }
         if (!is_v && head < a.heads) {
-            T *q = static_cast<T *>(a.q_out) + t * a.heads * a.dim + static_cast<int64_t>(head) * a.dim + off;
+            T *q = static_cast<T *>(a.q_out) + static_cast<int64_t>(t) * a.heads * a.dim + static_cast<int64_t>(head) * a.dim + off;
             store_f32<T, V>(q, y0);
             if (pair) store_f32<T, V>(q + a.half, y1);
         } else {
@@ -418,23 +433,25 @@ __global__ __launch_bounds__(256) void conv_state_update_kernel(ConvRopeArgs a, 
     }
 }
 
-template <typename T, int V, bool kDecode>
+template <typename T, int V, int kTokens, bool kDecode>
 static void launch_conv_rope(const ConvRopeArgs &a, hipStream_t s) {
     const int64_t units = static_cast<int64_t>(a.heads + a.kv_heads) * (a.dim - a.half) / V + static_cast<int64_t>(a.kv_heads) * a.vdim / V;
-    const int64_t groups = kDecode ? a.n : (a.n + 3) / 4;
+    const int64_t groups = (a.n + kTokens - 1) / kTokens;
     const dim3 grid(static_cast<uint32_t>((units * groups + 255) / 256)), block(256);
-    if (a.taps <= 1) hipLaunchKernelGGL((conv_rope_store_kernel<T, 1, V, kDecode>), grid, block, 0, s, a);
-    else if (a.taps <= 2) hipLaunchKernelGGL((conv_rope_store_kernel<T, 2, V, kDecode>), grid, block, 0, s, a);
-    else if (a.taps <= 4) hipLaunchKernelGGL((conv_rope_store_kernel<T, 4, V, kDecode>), grid, block, 0, s, a);
-    else hipLaunchKernelGGL((conv_rope_store_kernel<T, 8, V, kDecode>), grid, block, 0, s, a);
+    if (a.taps <= 1) hipLaunchKernelGGL((conv_rope_store_kernel<T, 1, V, kTokens, kDecode>), grid, block, 0, s, a);
+    else if (a.taps <= 2) hipLaunchKernelGGL((conv_rope_store_kernel<T, 2, V, kTokens, kDecode>), grid, block, 0, s, a);
+    else if (a.taps <= 4) hipLaunchKernelGGL((conv_rope_store_kernel<T, 4, V, kTokens, kDecode>), grid, block, 0, s, a);
+    else hipLaunchKernelGGL((conv_rope_store_kernel<T, 8, V, kTokens, kDecode>), grid, block, 0, s, a);
 }
 
 template <typename T>
 static int run_conv_rope(const ConvRopeArgs &a, bool decode, bool vector, hipStream_t s) {
     if (vector) {
-        if (decode) launch_conv_rope<T, 8, true>(a, s); else launch_conv_rope<T, 8, false>(a, s);
+        if (decode) launch_conv_rope<T, 8, 1, true>(a, s);
+        else if (a.n < 4096) launch_conv_rope<T, 8, 4, false>(a, s);
+        else launch_conv_rope<T, 8, 16, false>(a, s);     // enough rows to fill the machine: fewer rows are read twice
     } else {
-        if (decode) launch_conv_rope<T, 1, true>(a, s); else launch_conv_rope<T, 1, false>(a, s);
+        if (decode) launch_conv_rope<T, 1, 1, true>(a, s); else launch_conv_rope<T, 1, 4, false>(a, s);
     }
     int rc = launch_status();
     if (rc != NVA_OK || decode || a.taps <= 1) return rc;
@@ -513,7 +530,7 @@ extern "C" int nva_clamped_gate(const void *x, int64_t x_row_stride, void *out, 
 
 extern "C" int nva_conv_rope_store(const void *qkv, int64_t qkv_row_stride, const void *conv_weight, void *conv_state,
                                    const int32_t *state_slots_of_seq, const int32_t *cu_seqlens_q, const int32_t *seq_lens,
-                                   const int32_t *token_seq, const int64_t *positions, const float *rope_cache,
+                                   const int32_t *token_seq, const float *rope_cache,
                                    void *q_out, void *k_cache, void *v_cache, const int32_t *slot_mapping,
                                    int64_t num_slots, int32_t n_tokens, int32_t n_seqs, int32_t num_heads,
                                    int32_t num_kv_heads, int32_t qk_dim, int32_t v_dim, int32_t rot_dims, int32_t taps,
@@ -525,7 +542,7 @@ extern "C" int nva_conv_rope_store(const void *qkv, int64_t qkv_row_stride, cons
     if (rot_dims % 2 != 0 || taps > 8 || !known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     if (n_tokens == 0) return NVA_OK;
     const bool decode = cu_seqlens_q == nullptr;
-    if (!qkv || !conv_weight || !seq_lens || !positions || !q_out || !k_cache || !v_cache || !slot_mapping)
+    if (!qkv || !conv_weight || !seq_lens || !q_out || !k_cache || !v_cache || !slot_mapping)
         return NVA_ERR_NULL_POINTER;
     if (taps > 1 && (!conv_state || !state_slots_of_seq)) return NVA_ERR_NULL_POINTER;
     if (rot_dims > 0 && !rope_cache) return NVA_ERR_NULL_POINTER;
@@ -537,7 +554,7 @@ extern "C" int nva_conv_rope_store(const void *qkv, int64_t qkv_row_stride, cons
     if (channels * n_tokens / 256 > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
     ConvRopeArgs a{};
     a.qkv = qkv; a.stride = qkv_row_stride; a.weight = conv_weight; a.state = conv_state; a.slots_of_seq = state_slots_of_seq;
-    a.cu = cu_seqlens_q; a.klen = seq_lens; a.token_seq = token_seq; a.positions = positions; a.rope = rope_cache;
+    a.cu = cu_seqlens_q; a.klen = seq_lens; a.token_seq = token_seq; a.rope = rope_cache;
     a.q_out = q_out; a.k_cache = k_cache; a.v_cache = v_cache; a.slot_mapping = slot_mapping; a.num_slots = num_slots;
     a.n = n_tokens; a.n_seqs = n_seqs; a.heads = num_heads; a.kv_heads = num_kv_heads; a.dim = qk_dim; a.vdim = v_dim;
     a.half = rot_dims / 2; a.taps = taps; a.max_position = max_position; a.state_slots = num_state_slots;

@@ -20,7 +20,6 @@ struct RetentionArgs {
     const int32_t *slots;            // [n_seqs]
     const int32_t *cu;               // portions: [n_seqs + 1]; decode: null, row i is sequence i
     const int32_t *klen;             // tokens of every sequence, this step's included (decode: 0 = padded row)
-    const int64_t *positions;        // [n]
     const float *rope;               // [max_position, 2 half]: cos | sin
     const float *log2_decay;         // [H]
     void *out;                       // [n, H vdim] dense
@@ -62,7 +61,7 @@ __global__ __launch_bounds__(256) void retention_scan_any_kernel(RetentionArgs a
         const T *row = static_cast<const T *>(a.x) + static_cast<int64_t>(first + t) * a.stride;
         const T *q = row + static_cast<int64_t>(head) * a.dim, *k = q + qk;
         const T *v = row + 2 * qk + static_cast<int64_t>(head) * a.vdim, *gate = v + static_cast<int64_t>(a.heads) * a.vdim;
-        const int64_t pos = min(max(a.positions[first + t], static_cast<int64_t>(0)), static_cast<int64_t>(a.max_position) - 1);
+        const int64_t pos = min(start + t, a.max_position - 1);
         for (int i = tid; i < a.dim; i += 256) {
             float qv = Elem<T>::to_f32(q[i]), kv = Elem<T>::to_f32(k[i]);
             if (i < 2 * a.half) {
@@ -159,7 +158,7 @@ __global__ __launch_bounds__(256) void retention_step_kernel(RetentionArgs a) {
     const T *row = static_cast<const T *>(a.x) + static_cast<int64_t>(seq) * a.stride;
     const T *q = row + static_cast<int64_t>(head) * a.dim, *k = q + qk;
     const T *v = row + 2 * qk + static_cast<int64_t>(head) * a.vdim, *gate = v + static_cast<int64_t>(a.heads) * a.vdim;
-    const int64_t pos = min(max(a.positions[seq], static_cast<int64_t>(0)), static_cast<int64_t>(a.max_position) - 1);
+    const int64_t pos = min(start, a.max_position - 1);
     for (int i = tid; i < a.dim; i += 256) {
         float qv = Elem<T>::to_f32(q[i]), kv = Elem<T>::to_f32(k[i]);
         if (i < 2 * a.half) {
@@ -600,7 +599,7 @@ extern "C" size_t nva_retention_workspace_bytes(int32_t n_seqs, int32_t max_seql
 }
 
 extern "C" int nva_retention(const void *qkvg, int64_t row_stride, float *state, const int32_t *state_slots_of_seq,
-                             const int32_t *cu_seqlens_q, const int32_t *seq_lens, const int64_t *positions,
+                             const int32_t *cu_seqlens_q, const int32_t *seq_lens,
                              const float *rope_cache, const float *log2_decay, void *out, void *workspace,
                              size_t workspace_bytes, int32_t n_tokens, int32_t n_seqs,
                              int32_t max_seqlen_q, int32_t num_heads, int32_t qk_dim, int32_t v_dim, int32_t rot_dims,
@@ -612,14 +611,14 @@ extern "C" int nva_retention(const void *qkvg, int64_t row_stride, float *state,
         return NVA_ERR_BAD_SHAPE;
     if (rot_dims % 2 != 0 || qk_dim > kScanMaxDim || v_dim > kScanMaxDim || !known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     if (n_tokens == 0 || n_seqs == 0) return NVA_OK;
-    if (!qkvg || !state || !state_slots_of_seq || !seq_lens || !positions || !log2_decay || !out) return NVA_ERR_NULL_POINTER;
+    if (!qkvg || !state || !state_slots_of_seq || !seq_lens || !log2_decay || !out) return NVA_ERR_NULL_POINTER;
     if (rot_dims > 0 && !rope_cache) return NVA_ERR_NULL_POINTER;
     if (cu_seqlens_q == nullptr && n_seqs != n_tokens) return NVA_ERR_BAD_SHAPE;
     if (row_stride < 2 * static_cast<int64_t>(num_heads) * (qk_dim + v_dim)) return NVA_ERR_BAD_STRIDE;
     if (static_cast<int64_t>(n_seqs) * num_heads > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
     RetentionArgs a{};
     a.x = qkvg; a.stride = row_stride; a.state = state; a.slots = state_slots_of_seq; a.cu = cu_seqlens_q; a.klen = seq_lens;
-    a.positions = positions; a.rope = rope_cache; a.log2_decay = log2_decay; a.out = out; a.n = n_tokens; a.n_seqs = n_seqs;
+    a.rope = rope_cache; a.log2_decay = log2_decay; a.out = out; a.n = n_tokens; a.n_seqs = n_seqs;
     a.heads = num_heads; a.dim = qk_dim; a.vdim = v_dim; a.half = rot_dims / 2; a.num_slots = num_state_slots;
     a.max_position = max_position; a.k_scale = k_scale; a.eps = eps;
     hipStream_t s = static_cast<hipStream_t>(stream);

@@ -54,13 +54,13 @@ SIGNATURES = {
     "nva_embed_norm": (C.c_int, [_vp, _vp, _f32, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _f32, _i32, _vp]),
     "nva_post_add_norm": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _f32, _i32, _vp]),
     "nva_clamped_gate": (C.c_int, [_vp, _i64, _vp, _i32, _i32, _f32, _f32, _i32, _vp]),
-    "nva_conv_rope_store": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp,
+    "nva_conv_rope_store": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp,
                                       _i64, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _vp]),
     "nva_chunk_attn_workspace_bytes": (_sz, [_i32, _i32, _i32, _i32, _i32, _i32, _i32]),
     "nva_chunk_attn": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _i64, _i32, _vp, _vp, _vp, _vp, _vp, _sz, _i32, _i32, _i32, _i32,
                                  _i32, _i32, _i32, _i32, _i32, _i32, _f32, _f32, _i32, _vp]),
     "nva_retention_workspace_bytes": (_sz, [_i32, _i32, _i32, _i32, _i32, _i32, _i32]),
-    "nva_retention": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _sz, _i32, _i32, _i32, _i32, _i32,
+    "nva_retention": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _sz, _i32, _i32, _i32, _i32, _i32,
                                 _i32, _i32, _i32, _i32, _f32, _f32, _i32, _vp]),
     "nva_probe_stream_read": (C.c_int, [_vp, _i64, _vp, _vp]),
 }

@@ -197,7 +197,7 @@ class Kaparax(nn.Module):
     def forward_layers(self, input_ids, positions, hidden, residual, first: int, last: int):
         """Layers ``[first, last)``: ``hidden`` is the normed input of the next sublayer, ``residual`` the
         fp32 stream, updated in place.  After the last layer ``hidden`` is the final norm -- of the rows in
-        the Context's ``logit_rows`` only, when they are given."""
+        the Context's ``logit_rows`` only, when they are given.  (Positions follow from the row groups.)"""
         eps, layers = self.cfg.norm_eps, self.layers
         if first == 0:
             residual, hidden = mixers.embed_norm(input_ids, self.embed, self.cfg.embed_scale, layers[0].weights.norm1.pair, eps)
@@ -206,7 +206,7 @@ class Kaparax(nn.Module):
             nxt, rows = self.final.pair, get_context().logit_rows
             if i + 1 < len(layers):
                 nxt, rows = layers[i + 1].weights.norm1.pair, None
-            y = layer.mixer(hidden, positions)
+            y = layer.mixer(hidden)
             post = w.norm1b.pair
             if layer.mlp is not None:
                 hidden = mixers.post_add_norm(y, residual, post, w.norm2.pair, eps)

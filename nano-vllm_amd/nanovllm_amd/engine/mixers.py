@@ -105,7 +105,7 @@ def clamped_gate(x: torch.Tensor, limit: float, alpha: float) -> torch.Tensor:
 
 
 def conv_rope_store(qkv: torch.Tensor, conv_weight: torch.Tensor, conv_state: Optional[torch.Tensor], group: RowGroup,
-                    positions: torch.Tensor, rope: Optional[torch.Tensor], q_out: torch.Tensor, k_cache: torch.Tensor,
+                    rope: Optional[torch.Tensor], q_out: torch.Tensor, k_cache: torch.Tensor,
                     v_cache: torch.Tensor, heads: int, rot_dims: int) -> None:
     """Short convolution of q, k and v, rotation of q and k, cache write; see ``nva_conv_rope_store``."""
     taps = conv_weight.shape[0]
@@ -114,12 +114,12 @@ def conv_rope_store(qkv: torch.Tensor, conv_weight: torch.Tensor, conv_state: Op
     assert qkv.stride(1) == 1 and qkv.shape[1] == (heads + kv_heads) * dim + kv_heads * vdim == conv_weight.shape[1]
     assert q_out.shape == (qkv.shape[0], heads * dim) and q_out.is_contiguous() and qkv.dtype == q_out.dtype == k_cache.dtype
     assert k_cache.is_contiguous() and v_cache.is_contiguous() and conv_weight.is_contiguous()
-    assert group.slot_mapping.numel() == qkv.shape[0] == positions.numel() == group.count
+    assert group.slot_mapping.numel() == qkv.shape[0] == group.count
     slots = k_cache.shape[0] * k_cache.shape[1]
     state_slots = 0 if conv_state is None else conv_state.shape[0]
     rc = _lib.load().nva_conv_rope_store(
         qkv.data_ptr(), qkv.stride(0), conv_weight.data_ptr(), _ptr(conv_state), _ptr(group.state_slots), _ptr(group.cu),
-        group.seq_lens.data_ptr(), _ptr(group.token_seq), positions.data_ptr(), _ptr(rope), q_out.data_ptr(),
+        group.seq_lens.data_ptr(), _ptr(group.token_seq), _ptr(rope), q_out.data_ptr(),
         k_cache.data_ptr(), v_cache.data_ptr(), group.slot_mapping.data_ptr(), slots, group.count, group.num_seqs, heads,
         kv_heads, dim, vdim, rot_dims, taps, 1 if rope is None else rope.shape[0], state_slots, _DTYPE[qkv.dtype], _stream())
     _lib.check(rc, "nva_conv_rope_store")
@@ -146,7 +146,7 @@ def chunk_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     _lib.check(rc, "nva_chunk_attn")
 
 
-def retention(qkvg: torch.Tensor, state: torch.Tensor, group: RowGroup, positions: torch.Tensor, rope: Optional[torch.Tensor],
+def retention(qkvg: torch.Tensor, state: torch.Tensor, group: RowGroup, rope: Optional[torch.Tensor],
               log2_decay: torch.Tensor, out: torch.Tensor, rot_dims: int, k_scale: float, eps: float) -> None:
     """Retention with its rotation, head norm and output gate; see ``nva_retention``."""
     slots, heads, dim, vdim = state.shape
@@ -159,7 +159,7 @@ def retention(qkvg: torch.Tensor, state: torch.Tensor, group: RowGroup, position
         ws = scratch(qkvg.device, nbytes) if nbytes else None
     rc = lib.nva_retention(
         qkvg.data_ptr(), qkvg.stride(0), state.data_ptr(), group.state_slots.data_ptr(), _ptr(group.cu),
-        group.seq_lens.data_ptr(), positions.data_ptr(), _ptr(rope), log2_decay.data_ptr(), out.data_ptr(), _ptr(ws),
+        group.seq_lens.data_ptr(), _ptr(rope), log2_decay.data_ptr(), out.data_ptr(), _ptr(ws),
         0 if ws is None else ws.numel(), group.count, group.num_seqs, group.max_q, heads, dim, vdim, rot_dims, 1 if rope is None else rope.shape[0], slots, float(k_scale),
         float(eps), _DTYPE[qkvg.dtype], _stream())
     _lib.check(rc, "nva_retention")
@@ -293,14 +293,14 @@ class ChunkAttention:
     def unbind(self) -> None:
         self.k_cache = self.v_cache = self.conv_state = None
 
-    def __call__(self, h: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
+    def __call__(self, h: torch.Tensor) -> torch.Tensor:
         s, w = self.spec, self.weights
         qkv = F.linear(h, w.qkv)
         q = torch.empty((h.shape[0], s.heads * s.dim), dtype=h.dtype, device=h.device)
         o = torch.empty((h.shape[0], s.heads * s.vdim), dtype=h.dtype, device=h.device)
         for group in get_context().groups:
             rows = slice(group.first, group.first + group.count)
-            conv_rope_store(qkv[rows], w.conv, self.conv_state, group, positions[rows], self.rope, q[rows], self.k_cache,
+            conv_rope_store(qkv[rows], w.conv, self.conv_state, group, self.rope, q[rows], self.k_cache,
                             self.v_cache, s.heads, s.rot.dims)
             chunk_attention(q[rows], self.k_cache, self.v_cache, group, o[rows], s.heads, s.chunk, s.scale, s.softcap)
         return F.linear(o, w.o)
@@ -329,13 +329,13 @@ class Retention:
     def unbind(self) -> None:
         self.state = None
 
-    def __call__(self, h: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
+    def __call__(self, h: torch.Tensor) -> torch.Tensor:
         s, w = self.spec, self.weights
         qkvg = F.linear(h, w.qkvg)
         o = torch.empty((h.shape[0], s.heads * s.vdim), dtype=h.dtype, device=h.device)
         for group in get_context().groups:
             rows = slice(group.first, group.first + group.count)
-            retention(qkvg[rows], self.state, group, positions[rows], self.rope, self.log2_decay, o[rows], s.rot.dims,
+            retention(qkvg[rows], self.state, group, self.rope, self.log2_decay, o[rows], s.rot.dims,
                       s.dim ** -0.5, self.eps)
         return F.linear(o, w.o)
 

@@ -155,7 +155,7 @@ def test_convolution_rotation_and_cache_write(dev, dtype, shape):
         vc = torch.full((batch.num_blocks, BLOCK, kv, vdim), 7.0, dtype=dtype, device=dev)
         x = batch.rows(full).to(dev)
         q = torch.empty((x.shape[0], heads * dim), dtype=dtype, device=dev)
-        mixers.conv_rope_store(x, weight.to(dev), state, batch.group, batch.positions, table, q, kc, vc, heads, rot)
+        mixers.conv_rope_store(x, weight.to(dev), state, batch.group, table, q, kc, vc, heads, rot)
         ref = [plain.short_conv(f.double(), weight.t().double()) for f in full]
         n = x.shape[0] - batch.pad
         split = [r.split([heads * dim, kv * dim, kv * vdim], dim=1) for r in ref]
@@ -271,7 +271,7 @@ def test_retention_with_norm_and_gate(dev, dtype, shape, decays):
         before, state = state.clone(), state.to(dev)
         rows = batch.rows(full).to(dev)
         out = torch.full((rows.shape[0], heads * vdim), 9.0, dtype=dtype, device=dev)
-        mixers.retention(rows, state, batch.group, batch.positions, table, log2, out, rot, dim ** -0.5, 1e-5)
+        mixers.retention(rows, state, batch.group, table, log2, out, rot, dim ** -0.5, 1e-5)
         what = f"{shape} {decays} single {batch.single} spans {batch.spans}"
         # (without any memory o is (q . k) v, and dividing by its size magnifies rounding where q . k is near 0)
         _close(out, batch.rows(want), _tol(dtype, 8e-3, 2e-5 if min(decay) > 0 else 1e-4), what)
