@@ -876,6 +876,12 @@ def kaparax_kernels(dev, steps=60, only=None):
     graph_us = lambda fns, n=200: _graph_time_ms(fns, n, 10)[0] / n * 1e3
     event_us = lambda fns, n=steps: _steady_time_ms(fns, n, max(3, n // 10))[0] / n * 1e3
 
+    def like_prefill(lens, q=None):
+        q = rnd(sum(lens), heads * d) if q is None else q
+        k, v = rnd(sum(lens), kv, d), rnd(sum(lens), kv, d)
+        cu = torch.tensor([0] + lens).cumsum(0).to(torch.int32).to(dev)
+        return lambda: nva.varlen_prefill_attention(q.view(-1, heads, d), k, v, cu, cu, max(lens), max(lens), d ** -0.5)
+
     # ---- attention over portions
     for what, lens, chunk in (("2x16384, one chunk", [16384, 16384], 16384), ("2x16384, chunks of 2048", [16384, 16384], 2048),
                               ("16 x U[100,1024], chunks of 8192", None, 8192)):
@@ -898,12 +904,12 @@ def kaparax_kernels(dev, steps=60, only=None):
                          i32([i for i, l in enumerate(lens) for _ in range(l)]), max(lens))
         q, out = rnd(n, heads * d), torch.empty(n, heads * d, dtype=bf, device=dev)
         mine = event_us([lambda: mixers.chunk_attention(q, kc, vc, group, out, heads, chunk, d ** -0.5, 30.0)])
-        theirs = event_us([lambda: nva.varlen_prefill_attention(q.view(n, heads, d), kc, vc, group.cu, group.cu, max(lens), max(lens),
-                                                                d ** -0.5, block_table=group.block_tables)])
-        full = sum(l * (l + 1) // 2 for l in lens)
+        # the like kernel on the same visible pairs: every chunk a sequence of its own
+        parts = [min(chunk, l - k) for l in lens for k in range(0, l, chunk)]
+        theirs = event_us([like_prefill(parts, q)])
         seen = sum((l // chunk) * (chunk * (chunk + 1) // 2) + (l % chunk) * (l % chunk + 1) // 2 for l in lens)
         rows.append(_kernel_row("attention prefill, " + what, mine, 4 * d * heads * seen, "mfma",
-                                ("prefill_attn_kernel (whole context)", theirs, 4 * d * heads * full, "mfma")))
+                                ("prefill_attn_kernel", theirs, 4 * d * heads * seen, "mfma")))
         del kc, vc, q, out
 
     # ---- attention of single tokens
@@ -946,11 +952,12 @@ def kaparax_kernels(dev, steps=60, only=None):
             cu.append(cu[-1] + l)
         group = RowGroup(0, n, len(lens), i32(lens), i32([0] * n), None, i32(list(range(len(lens)))), i32(cu), i32([0] * n), max(lens))
         x, out = rnd(n, 4 * rh * d), torch.empty(n, rh * d, dtype=bf, device=dev)
-        pos = torch.cat([torch.arange(l) for l in lens]).to(dev)
         state = torch.zeros(len(lens), rh, d, d, device=dev)
         decay = torch.full((rh,), -0.01, device=dev)
         mine = event_us([lambda: mixers.retention(x, state, group, table, decay, out, d, d ** -0.5, 1e-6)])
-        rows.append(_kernel_row("retention prefill, " + what, mine, n * rh * d * 5 * 2 + state.numel() * 4 + n * d * 4, "hbm"))
+        theirs = event_us([like_prefill(lens)])
+        rows.append(_kernel_row("retention prefill, " + what, mine, n * rh * d * 5 * 2 + state.numel() * 4 + n * d * 4, "hbm",
+                                ("prefill_attn_kernel", theirs, 4 * d * heads * sum(l * (l + 1) // 2 for l in lens), "mfma")))
         rows[-1]["tokens_per_s"] = round(n / mine * 1e6)
         rows[-1]["tflops_of_one_product_each"] = round(n * rh * (8 * d * d + 4 * 32 * d / 2) / mine / 1e6, 1)
     for batch in (1, 64, 256):
@@ -959,10 +966,13 @@ def kaparax_kernels(dev, steps=60, only=None):
         states = [torch.zeros(batch, rh, d, d, device=dev) for _ in range(4)]
         group = RowGroup(0, batch, batch, i32([800] * batch), i32([0] * batch), None, i32(list(range(batch))))
         x, out = rnd(batch, 4 * rh * d), torch.empty(batch, rh * d, dtype=bf, device=dev)
-        pos = torch.full((batch,), 799, dtype=torch.int64, device=dev)
         decay = torch.full((rh,), -0.01, device=dev)
         mine = graph_us([lambda s=s: mixers.retention(x, s, group, table, decay, out, d, d ** -0.5, 1e-6) for s in states])
-        rows.append(_kernel_row("retention decode, batch %d" % batch, mine, states[0].numel() * 8, "hbm"))
+        # as many bytes of keys and values through the decode attention: 2 * d * 4 bytes of state are d / kv tokens of K and V
+        ctx = torch.full((batch,), states[0][0].numel() * 8 // (kv * d * 4), dtype=torch.int32)
+        roof = decode_shape_roofline(dev, [(rnd(batch, 256, kv, d), rnd(batch, 256, kv, d)) for _ in range(4)], batch, ctx, heads, "", layers=28)
+        rows.append(_kernel_row("retention decode, batch %d" % batch, mine, states[0].numel() * 8, "hbm",
+                                ("decode_stream_kernel + merge", roof["us_per_launch"], roof["algorithmic_bytes_per_launch"], "hbm")))
         del states
 
     # ---- steps around them
@@ -982,7 +992,6 @@ def kaparax_kernels(dev, steps=60, only=None):
             single = n == 256
             ch = (heads + 2 * kv) * d
             x, conv, q = rnd(n, ch), rnd(4, ch), torch.empty(n, heads * d, dtype=bf, device=dev)
-            blocks = n // 256 + n if single else n // 256
             kc, vc = (torch.empty(n // 256, 256, kv, d, dtype=bf, device=dev) for _ in range(2))
             slots = i32(torch.randperm(n) if single else list(range(n)))
             nseq = n if single else 16

@@ -294,6 +294,7 @@ __global__ __launch_bounds__(256, DK * NV > 256 ? 1 : 2) void retention_chunk_ke
     for (int qb = 0; qb < 2; ++qb) gq[qb] = __builtin_amdgcn_exp2f(l2 * (16 * qb + r + 1));
 #pragma unroll
     for (int e = 0; e < 8; ++e) vfac[e] = __builtin_amdgcn_exp2f(l2 * (kC - 1 - chunk_token(g, e >> 2, e & 3)));
+    const float inv_vdim = 1.0f / static_cast<float>(a.vdim);
     float g_chunk = __builtin_amdgcn_exp2f(l2 * kC);
 
     const int64_t qk = static_cast<int64_t>(a.heads) * a.dim;
@@ -301,63 +302,102 @@ __global__ __launch_bounds__(256, DK * NV > 256 ? 1 : 2) void retention_chunk_ke
     const bf16_t *xv = static_cast<const bf16_t *>(a.x) + 2 * qk + static_cast<int64_t>(head) * a.vdim;
     const bf16_t *xg = xv + static_cast<int64_t>(a.heads) * a.vdim;
     const int pairs = a.half / 8, units = DK / 8 - pairs;            // per row: pairs of pieces that rotate, then single pieces
+    struct Unit { int e0, e1; bool pair; };
+    auto unit_of = [&](int w) __attribute__((always_inline)) -> Unit {
+        const bool pair = w < pairs;
+        const int e0 = pair ? 8 * w : 2 * a.half + 8 * (w - pairs);
+        return Unit{e0, pair ? e0 + a.half : e0, pair};
+    };
+    // a thread's first unit of q and k and its pieces of v (32 rows of 64 NV columns) are loaded one chunk ahead
+    u32x4_t rq0, rq1, rk0, rk1, rv[NV];
+    const int my_row = tid / units;
+    const Unit my_unit = unit_of(tid % units);
+    auto fetch = [&](int row, const Unit &w, int t0) __attribute__((always_inline)) {
+        rq0 = rq1 = rk0 = rk1 = u32x4_t{0, 0, 0, 0};
+        if (row < kC && t0 + row < t_end && w.e0 < a.dim) {
+            const bf16_t *x = xq + static_cast<int64_t>(first + t0 + row) * a.stride;
+            if (!kSums) {
+                rq0 = *reinterpret_cast<const u32x4_t *>(x + w.e0);
+                rq1 = *reinterpret_cast<const u32x4_t *>(x + w.e1);
+            }
+            rk0 = *reinterpret_cast<const u32x4_t *>(x + qk + w.e0);
+            rk1 = *reinterpret_cast<const u32x4_t *>(x + qk + w.e1);
+        }
+    };
+    float rcos[8], rsin[8];
+    auto fetch_turn = [&](int row, const Unit &w, int t0) __attribute__((always_inline)) {
+        if (w.pair) {
+            const float *cs = a.rope + static_cast<int64_t>(min(start + t0 + row, a.max_position - 1)) * (2 * a.half) + w.e0;
+            load_f32<float, 8>(cs, rcos);
+            load_f32<float, 8>(cs + a.half, rsin);
+        }
+    };
+    auto fetch_v = [&](int t0) __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int p = i * 256 + tid, row = p / (kVW / 8), e = p % (kVW / 8) * 8;
+            rv[i] = u32x4_t{0, 0, 0, 0};
+            if (t0 + row < t_end && e < a.vdim) rv[i] = *reinterpret_cast<const u32x4_t *>(xv + static_cast<int64_t>(first + t0 + row) * a.stride + e);
+        }
+    };
+    fetch(my_row, my_unit, t_begin);
+    fetch_turn(my_row, my_unit, t_begin);
+    fetch_v(t_begin);
 
     for (int t0 = t_begin; t0 < t_end; t0 += kC) {
         const int L = min(kC, t_end - t0);
-        // ---- q and k: load, rotate, split; v: load ------------------------------------------------
-        for (int u = tid; u < kC * units; u += 256) {
-            const int row = u / units, w = u % units;
-            const bool pair = w < pairs;
-            const int e0 = pair ? 8 * w : 2 * a.half + 8 * (w - pairs), e1 = pair ? e0 + a.half : e0;
-            const bool in = row < L && e0 < a.dim;
-            const bf16_t *x = xq + static_cast<int64_t>(first + t0 + min(row, L - 1)) * a.stride;
-            u32x4_t rq0 = {0, 0, 0, 0}, rq1 = rq0, rk0 = rq0, rk1 = rq0;
-            float c[8], s[8];
-            if (in) {
-                if (!kSums) {
-                    rq0 = *reinterpret_cast<const u32x4_t *>(x + e0);
-                    rq1 = *reinterpret_cast<const u32x4_t *>(x + e1);
-                }
-                rk0 = *reinterpret_cast<const u32x4_t *>(x + qk + e0);
-                rk1 = *reinterpret_cast<const u32x4_t *>(x + qk + e1);
-            }
+        // ---- q and k: rotate, split; v; all into LDS ------------------------------------------------
+        auto place = [&](const u32x4_t &p0, const u32x4_t &p1, bool pair, const float (&c)[8], const float (&s)[8], float scale,
+                         lds_char_ptr dst0, lds_char_ptr dst1) __attribute__((always_inline)) {
+            float x0[8], x1[8], y[8];
+            u32x4_t hi, lo;
+            unpack8(make_uint4(p0[0], p0[1], p0[2], p0[3]), x0);
             if (pair) {
-                const int64_t pos = min(start + t0 + row, a.max_position - 1);
-                load_f32<float, 8>(a.rope + pos * (2 * a.half) + e0, c);
-                load_f32<float, 8>(a.rope + pos * (2 * a.half) + a.half + e0, s);
-            }
-            auto place = [&](u32x4_t &p0, u32x4_t &p1, float scale, int at) __attribute__((always_inline)) {
-                float x0[8], x1[8];
-                unpack8(make_uint4(p0[0], p0[1], p0[2], p0[3]), x0);
                 unpack8(make_uint4(p1[0], p1[1], p1[2], p1[3]), x1);
-                float y0[8], y1[8];
 #pragma unroll
-                for (int i = 0; i < 8; ++i) {
-                    y0[i] = scale * (pair ? x0[i] * c[i] - x1[i] * s[i] : x0[i]);
-                    y1[i] = scale * (pair ? x1[i] * c[i] + x0[i] * s[i] : 0.f);
-                }
-                u32x4_t hi, lo;
-                split8(y0, hi, lo);
-                const lds_char_ptr dst = lds + at + row * kPitch;
-                *(lds_u32x4_ptr)(dst + 2 * e0) = hi;
-                *(lds_u32x4_ptr)(dst + kC * kPitch + 2 * e0) = lo;
-                if (pair) {
-                    split8(y1, hi, lo);
-                    *(lds_u32x4_ptr)(dst + 2 * e1) = hi;
-                    *(lds_u32x4_ptr)(dst + kC * kPitch + 2 * e1) = lo;
-                }
-            };
-            if (!kSums) place(rq0, rq1, 1.0f, kQ);
-            place(rk0, rk1, a.k_scale, kK);
+                for (int i = 0; i < 8; ++i) y[i] = x1[i] * c[i] + x0[i] * s[i];
+                split8(y, hi, lo);
+                *(lds_u32x4_ptr)dst1 = hi;
+                *(lds_u32x4_ptr)(dst1 + kC * kPitch) = lo;
+#pragma unroll
+                for (int i = 0; i < 8; ++i) y[i] = x0[i] * c[i] - x1[i] * s[i];
+            } else {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) y[i] = x0[i] * scale;
+            }
+            split8(y, hi, lo);
+            *(lds_u32x4_ptr)dst0 = hi;
+            *(lds_u32x4_ptr)(dst0 + kC * kPitch) = lo;
+        };
+        auto place_unit = [&](int row, const Unit &w) __attribute__((always_inline)) {
+            float c[8], s[8];
+#pragma unroll
+            for (int i = 0; i < 8; ++i) { c[i] = rcos[i]; s[i] = rsin[i]; }
+            const lds_char_ptr d0 = lds + row * kPitch + 2 * w.e0, d1 = lds + row * kPitch + 2 * w.e1;
+            if (!kSums) place(rq0, rq1, w.pair, c, s, 1.0f, d0 + kQ, d1 + kQ);
+            if (w.pair)
+#pragma unroll
+                for (int i = 0; i < 8; ++i) { c[i] *= a.k_scale; s[i] *= a.k_scale; }
+            place(rk0, rk1, w.pair, c, s, a.k_scale, d0 + kK, d1 + kK);
+        };
+        if (tid < kC * units) place_unit(my_row, my_unit);
+        for (int u = tid + 256; u < kC * units; u += 256) {          // (sizes with more than one unit per thread)
+            const int row = u / units;
+            const Unit w = unit_of(u % units);
+            fetch(row, w, t0);
+            fetch_turn(row, w, t0);
+            place_unit(row, w);
         }
 #pragma unroll
-        for (int i = 0; i < NV; ++i) {                   // 32 rows of 64 NV columns: NV pieces per thread
-            const int p = i * 256 + tid, row = p / (kVW / 8), e = p % (kVW / 8) * 8;
-            u32x4_t v = {0, 0, 0, 0};
-            if (row < L && e < a.vdim) v = *reinterpret_cast<const u32x4_t *>(xv + static_cast<int64_t>(first + t0 + row) * a.stride + e);
-            *(lds_u32x4_ptr)(lds + kV + row * kVPitch + 2 * e) = v;
+        for (int i = 0; i < NV; ++i) {
+            const int p = i * 256 + tid;
+            *(lds_u32x4_ptr)(lds + kV + p / (kVW / 8) * kVPitch + p % (kVW / 8) * 16) = rv[i];
         }
         __syncthreads();
+        if (t0 + kC < t_end) {
+            fetch(my_row, my_unit, t0 + kC);
+            fetch_v(t0 + kC);
+        }
         if (L < kC) {                                    // the last chunk of the segment
 #pragma unroll
             for (int e = 0; e < 8; ++e) {
@@ -457,6 +497,19 @@ __global__ __launch_bounds__(256, DK * NV > 256 ? 1 : 2) void retention_chunk_ke
             for (int e = 0; e < 8; ++e) f[e] *= vfac[e];
             split8(f, vh[vb], vl[vb]);
         }
+        // what the end of this chunk and the start of the next one wait for: gates, angles
+        u32x2_t gate[kSums ? 1 : 2][NV];
+        if (!kSums) {
+#pragma unroll
+            for (int qb = 0; qb < 2; ++qb)
+#pragma unroll
+                for (int vb = 0; vb < NV; ++vb) {
+                    const int v = v0 + 16 * vb + 4 * g;
+                    if (16 * qb + r < L && v < a.vdim)
+                        gate[qb][vb] = *reinterpret_cast<const u32x2_t *>(xg + static_cast<int64_t>(first + t0 + 16 * qb + r) * a.stride + v);
+                }
+        }
+        if (t0 + kC < t_end) fetch_turn(my_row, my_unit, t0 + kC);
 #pragma unroll
         for (int db = 0; db < kDB; ++db) {
             const u32x4_t kh = token_frag(kK, kPitch, 16 * db), kl = token_frag(kK + kC * kPitch, kPitch, 16 * db);
@@ -489,7 +542,7 @@ __global__ __launch_bounds__(256, DK * NV > 256 ? 1 : 2) void retention_chunk_ke
             for (int qb = 0; qb < 2; ++qb) {
                 const int row = 16 * qb + r;
                 const float ss = (sh_ss[0][row] + sh_ss[1][row]) + (sh_ss[2][row] + sh_ss[3][row]);
-                const float inv = rsqrtf(ss / static_cast<float>(a.vdim) + a.eps);
+                const float inv = rsqrtf(fmaf(ss, inv_vdim, a.eps));
                 if (row >= L) continue;
                 const int64_t t = first + t0 + row;
                 bf16_t *out = static_cast<bf16_t *>(a.out) + (t * a.heads + head) * a.vdim;
@@ -497,7 +550,7 @@ __global__ __launch_bounds__(256, DK * NV > 256 ? 1 : 2) void retention_chunk_ke
                 for (int vb = 0; vb < NV; ++vb) {
                     const int v = v0 + 16 * vb + 4 * g;
                     if (v < a.vdim) {
-                        const u32x2_t z = *reinterpret_cast<const u32x2_t *>(xg + t * a.stride + v);
+                        const u32x2_t z = gate[qb][vb];
                         const float zf[4] = {bf16lo_to_f32(z[0]), bf16hi_to_f32(z[0]), bf16lo_to_f32(z[1]), bf16hi_to_f32(z[1])};
                         float y[4];
 #pragma unroll
@@ -533,11 +586,19 @@ __global__ __launch_bounds__(256) void retention_segment_scan_kernel(const Reten
     float run = carried ? a.state[(static_cast<int64_t>(slot) * a.heads + head) * size + e] : 0.f;
     const float decay = exp2f(a.log2_decay[head] * static_cast<float>(sg.length));
     const int segments = min(sg.segments, (count - 1) / sg.length + 1);
-    for (int seg = 0; seg < segments; ++seg) {
-        float *p = sg.sums + ((static_cast<int64_t>(seq) * sg.segments + seg) * a.heads + head) * size + e;
-        const float own = seg + 1 < segments ? *p : 0.f;
-        *p = run;
-        run = fmaf(decay, run, own);
+    float *p = sg.sums + (static_cast<int64_t>(seq) * sg.segments * a.heads + head) * size + e;
+    const int64_t step = static_cast<int64_t>(a.heads) * size;
+    constexpr int kAhead = 8;                             // loads in flight together
+    for (int s0 = 0; s0 < segments; s0 += kAhead) {
+        float own[kAhead];
+#pragma unroll
+        for (int i = 0; i < kAhead; ++i) own[i] = s0 + i + 1 < segments ? p[(s0 + i) * step] : 0.f;
+#pragma unroll
+        for (int i = 0; i < kAhead; ++i)
+            if (s0 + i < segments) {
+                p[(s0 + i) * step] = run;
+                run = fmaf(decay, run, own[i]);
+            }
     }
 }
 
@@ -546,7 +607,7 @@ __global__ __launch_bounds__(256) void retention_segment_scan_kernel(const Reten
 static SegmentArgs plan_segments(int32_t n_seqs, int32_t heads, int32_t max_q) {
     SegmentArgs sg{};
     const int64_t walks = std::max<int64_t>(1, static_cast<int64_t>(n_seqs) * heads);
-    const int64_t want = std::min<int64_t>((768 + walks - 1) / walks, std::max(1, max_q / 256));
+    const int64_t want = std::min<int64_t>(std::max<int64_t>(1, 512 / walks), std::max(1, max_q / 256));
     const int64_t length = (max_q + want - 1) / want;
     sg.length = static_cast<int32_t>(std::max<int64_t>(kRetChunk, (length + kRetChunk - 1) / kRetChunk * kRetChunk));
     sg.segments = std::max(1, (max_q + sg.length - 1) / sg.length);
