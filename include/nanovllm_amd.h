@@ -328,7 +328,7 @@ int nva_clamped_gate(const void *x, int64_t x_row_stride, void *out, int32_t row
  * the first rot_dims elements of each q and k head (pairs i, i + rot_dims / 2), q to q_out, k and v to
  * their cache slots.
  * qkv: [n_tokens, channels], channels = (num_heads + num_kv_heads) * qk_dim + num_kv_heads * v_dim.
- * conv_weight: [taps, channels], tap taps - 1 meets the row itself; 1 <= taps <= 8.
+ * conv_weight: [taps, channels], tap taps - 1 meets the row itself; 1 <= taps <= 16.
  * conv_state: [num_state_slots, taps - 1, channels], the last projected rows of every sequence, oldest
  * first; read for rows before a portion, updated by the call.
  * rope_cache: fp32 [max_position, rot_dims], cos in the first half of a row, sin in the second. */

@@ -441,7 +441,8 @@ static void launch_conv_rope(const ConvRopeArgs &a, hipStream_t s) {
     if (a.taps <= 1) hipLaunchKernelGGL((conv_rope_store_kernel<T, 1, V, kTokens, kDecode>), grid, block, 0, s, a);
     else if (a.taps <= 2) hipLaunchKernelGGL((conv_rope_store_kernel<T, 2, V, kTokens, kDecode>), grid, block, 0, s, a);
     else if (a.taps <= 4) hipLaunchKernelGGL((conv_rope_store_kernel<T, 4, V, kTokens, kDecode>), grid, block, 0, s, a);
-    else hipLaunchKernelGGL((conv_rope_store_kernel<T, 8, V, kTokens, kDecode>), grid, block, 0, s, a);
+    else if (V == 8 || a.taps <= 8) hipLaunchKernelGGL((conv_rope_store_kernel<T, 8, V, kTokens, kDecode>), grid, block, 0, s, a);
+    else hipLaunchKernelGGL((conv_rope_store_kernel<T, V == 8 ? 8 : 16, V, kTokens, kDecode>), grid, block, 0, s, a);
 }
 
 template <typename T>
@@ -539,7 +540,7 @@ extern "C" int nva_conv_rope_store(const void *qkv, int64_t qkv_row_stride, cons
     if (n_tokens < 0 || n_seqs < 0 || num_heads <= 0 || num_kv_heads <= 0 || qk_dim <= 0 || v_dim <= 0 || rot_dims < 0 ||
         rot_dims > qk_dim || num_slots < 0 || num_state_slots < 0 || max_position <= 0 || taps <= 0)
         return NVA_ERR_BAD_SHAPE;
-    if (rot_dims % 2 != 0 || taps > 8 || !known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
+    if (rot_dims % 2 != 0 || taps > 16 || !known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     if (n_tokens == 0) return NVA_OK;
     const bool decode = cu_seqlens_q == nullptr;
     if (!qkv || !conv_weight || !seq_lens || !q_out || !k_cache || !v_cache || !slot_mapping)
@@ -558,7 +559,7 @@ extern "C" int nva_conv_rope_store(const void *qkv, int64_t qkv_row_stride, cons
     a.q_out = q_out; a.k_cache = k_cache; a.v_cache = v_cache; a.slot_mapping = slot_mapping; a.num_slots = num_slots;
     a.n = n_tokens; a.n_seqs = n_seqs; a.heads = num_heads; a.kv_heads = num_kv_heads; a.dim = qk_dim; a.vdim = v_dim;
     a.half = rot_dims / 2; a.taps = taps; a.max_position = max_position; a.state_slots = num_state_slots;
-    const bool vector = qk_dim % 8 == 0 && v_dim % 8 == 0 && a.half % 8 == 0 && qkv_row_stride % 8 == 0 && aligned16(qkv) &&
+    const bool vector = taps <= 8 && qk_dim % 8 == 0 && v_dim % 8 == 0 && a.half % 8 == 0 && qkv_row_stride % 8 == 0 && aligned16(qkv) &&
                         aligned16(conv_weight) && aligned16(conv_state) && aligned16(rope_cache) && aligned16(q_out) &&
                         aligned16(k_cache) && aligned16(v_cache);
     hipStream_t s = static_cast<hipStream_t>(stream);

@@ -6,7 +6,7 @@ may have no feed-forward, and a layer may run another layer's weights with a cac
 from __future__ import annotations
 
 from dataclasses import dataclass
-from typing import Dict, List, Optional, Tuple, Union
+from typing import List, Optional, Tuple, Union
 
 import torch
 import torch.nn.functional as F
@@ -30,7 +30,7 @@ def _rotary(raw: dict) -> Rotary:
 def _attention_spec(raw: dict) -> AttentionSpec:
     spec = AttentionSpec(heads=int(raw["heads"]), kv_heads=int(raw["kv_heads"]), dim=int(raw["dim"]), vdim=int(raw["vdim"]),
                          taps=int(raw["conv"]), chunk=int(raw["mask"]["size"]), scale=float(raw["scale"]),
-                         softcap=float(raw["softcap"]), rot=_rotary(raw["rot"]))
+                         softcap=float(raw.get("softcap") or 0.0), rot=_rotary(raw["rot"]))
     if spec.heads % spec.kv_heads or spec.taps < 1 or spec.chunk < 1 or spec.rot.dims > spec.dim:
         raise ValueError(f"inconsistent attention sizes: {spec}")
     return spec
@@ -77,22 +77,22 @@ class KaparaxConfig:
 
     @classmethod
     def from_raw(cls, raw: dict) -> "KaparaxConfig":
+        entries = raw["layers"]
         layers: List[LayerSpec] = []
-        for i, entry in enumerate(raw["layers"]):
+        for i, entry in enumerate(entries):
             kind = entry["type"]
             if kind not in _MIXER_PARSERS:
                 raise ValueError(f"layer {i}: unknown mixer {kind!r}")
-            source = entry.get("weights_of")
-            if source is None:
-                source = i
-            elif not 0 <= source < i:
-                raise ValueError(f"layer {i}: weights_of {source} is not an earlier layer")
-            else:
-                source = layers[source].weights_of
-            spec = LayerSpec(_MIXER_PARSERS[kind](entry["mixer"]), _mlp_spec(entry["mlp"]), source)
-            if source != i and (spec.mixer, spec.mlp) != (layers[source].mixer, layers[source].mlp):
-                raise ValueError(f"layer {i} differs from layer {source}, whose weights it shares")
-            layers.append(spec)
+            source, seen = i, set()
+            while entries[source].get("weights_of") is not None:      # (a shared layer may itself name another)
+                seen.add(source)
+                source = entries[source]["weights_of"]
+                if not 0 <= source < len(entries) or source in seen:
+                    raise ValueError(f"layer {i}: weights_of leads to no layer with tensors of its own")
+            layers.append(LayerSpec(_MIXER_PARSERS[kind](entry["mixer"]), _mlp_spec(entry.get("mlp")), source))
+        for i, spec in enumerate(layers):
+            if (spec.mixer, spec.mlp) != (layers[spec.weights_of].mixer, layers[spec.weights_of].mlp):
+                raise ValueError(f"layer {i} differs from layer {spec.weights_of}, whose weights it shares")
         if not layers:
             raise ValueError("a model needs at least one layer")
         return cls(int(raw["vocab"]), int(raw["width"]), float(raw["embedding"]["scale"]), float(raw["norm"]["eps"]), tuple(layers))

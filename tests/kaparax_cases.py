@@ -36,7 +36,7 @@ def model(width, vocab, layers, scale=3.5, eps=1e-5):
 
 def configs():
     """name -> configuration.  Together: one and several kv heads and a group of 1, equal and unequal
-    key and value sizes, whole, part and no rotation, 1 to 6 taps, chunks shorter and longer than a
+    key and value sizes, whole, part and no rotation, 1 to 11 taps, chunks shorter and longer than a
     page, any pattern of feed-forwards, shared weights of both mixers, a score cap beyond what an
     unreferenced exponential could hold, sizes off every vector width."""
     a1 = attention(6, 2, 48, 40, 3, 37, 32)
@@ -48,13 +48,14 @@ def configs():
     a4 = attention(5, 1, 64, 96, 6, 500, 0)
     r4 = retention(4, 64, 160, 64, decay=[0.2, 0.9, 0.99, 0.9999])
     a5 = attention(4, 4, 96, 64, 1, 129, 64, cap=5.0)
+    a6 = attention(4, 2, 32, 24, 11, 90, 20)
     r5 = retention(2, 192, 64, 96)
     return {
         "mixed": model(104, 320, [(r1, mlp(72)), (a1, None), (a1, mlp(56)), (r1, None), (a1, None, 1), (r1, mlp(72), 0), (a1, mlp(56), 2)]),
         "wide": model(256, 512, [(a2, mlp(384)), (r2, None), (a2, mlp(384), 0), (r2, None, 1)], eps=1e-6),
         "odd": model(50, 301, [(a3, mlp(27)), (r3, mlp(31)), (a3, None), (r3, None)], scale=0.7),
         "deep_state": model(128, 256, [(r4, None), (a4, mlp(96)), (r4, mlp(64)), (a4, None)]),
-        "no_conv": model(192, 256, [(a5, mlp(128, limit=0.4)), (r5, mlp(128)), (a5, None)]),
+        "taps": model(192, 256, [(a5, mlp(128, limit=0.4)), (r5, mlp(128)), (a5, None), (a6, mlp(64))]),
     }
 
 

@@ -216,3 +216,70 @@ def test_probe_validation():
     assert f(A, 1000, A, None) == _lib.ERR_MISALIGNED               # not a multiple of 16
     assert f(A, -16, A, None) == _lib.ERR_BAD_SHAPE
     assert f(A, 0, A, None) == _lib.OK                               # nothing to read
+
+
+def _with(ok, f, **kw):
+    """Calls ``f`` with the values of ``ok`` (in order), some of them replaced."""
+    assert not set(kw) - set(ok), set(kw) - set(ok)
+    return f(*dict(ok, **kw).values())
+
+
+def test_norms_and_gate_of_layered_models_validation():
+    lib = _lib.load()
+    ok = dict(ids=A, table=A, scale=1.0, w=A, b=A, res=A, out=A, rows=4, width=64, vocab=10, eps=1e-5, dtype=0, stream=None)
+    for kw, rc in ((dict(ids=None), _lib.ERR_NULL_POINTER), (dict(res=None), _lib.ERR_NULL_POINTER), (dict(width=0), _lib.ERR_BAD_SHAPE),
+                   (dict(vocab=0), _lib.ERR_BAD_SHAPE), (dict(dtype=2), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, ids=None), _lib.OK)):
+        assert _with(ok, lib.nva_embed_norm, **kw) == rc, kw
+    ok = dict(y=A, ys=64, res=A, pw=A, pb=A, nw=A, nb=A, out=A, rows_of=None, rows=4, src=4, width=64, eps=1e-5, dtype=1, stream=None)
+    for kw, rc in ((dict(y=None), _lib.ERR_NULL_POINTER), (dict(nb=None), _lib.ERR_NULL_POINTER), (dict(ys=63), _lib.ERR_BAD_STRIDE),
+                   (dict(rows=3), _lib.ERR_BAD_SHAPE), (dict(rows_of=A, src=0), _lib.ERR_BAD_SHAPE), (dict(rows=0, src=0), _lib.OK),
+                   (dict(dtype=-1), _lib.ERR_UNSUPPORTED_GEOMETRY)):
+        assert _with(ok, lib.nva_post_add_norm, **kw) == rc, kw
+    ok = dict(x=A, xs=128, out=A, rows=4, inter=64, limit=1.0, alpha=1.7, dtype=0, stream=None)
+    for kw, rc in ((dict(x=None), _lib.ERR_NULL_POINTER), (dict(xs=127), _lib.ERR_BAD_STRIDE), (dict(inter=0), _lib.ERR_BAD_SHAPE),
+                   (dict(rows=-1), _lib.ERR_BAD_SHAPE), (dict(rows=0, x=None), _lib.OK)):
+        assert _with(ok, lib.nva_clamped_gate, **kw) == rc, kw
+
+
+def test_conv_rope_store_validation():
+    f = _lib.load().nva_conv_rope_store
+    ok = dict(qkv=A, stride=192, w=A, state=A, slots=A, cu=A, lens=A, tseq=A, rope=A, q=A, kc=A, vc=A, sm=A, num_slots=512, n=9, seqs=2,
+              heads=4, kv=1, dim=32, vdim=32, rot=32, taps=4, max_pos=64, state_slots=4, dtype=0, stream=None)
+    for kw, rc in ((dict(qkv=None), _lib.ERR_NULL_POINTER), (dict(state=None), _lib.ERR_NULL_POINTER), (dict(slots=None), _lib.ERR_NULL_POINTER),
+                   (dict(tseq=None), _lib.ERR_NULL_POINTER), (dict(rope=None), _lib.ERR_NULL_POINTER), (dict(vc=None), _lib.ERR_NULL_POINTER),
+                   (dict(stride=191), _lib.ERR_BAD_STRIDE), (dict(rot=34), _lib.ERR_BAD_SHAPE), (dict(rot=31), _lib.ERR_UNSUPPORTED_GEOMETRY),
+                   (dict(taps=17), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(taps=0), _lib.ERR_BAD_SHAPE), (dict(cu=None), _lib.ERR_BAD_SHAPE),
+                   (dict(dtype=7), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(n=0, qkv=None), _lib.OK)):
+        assert _with(ok, f, **kw) == rc, kw
+
+
+def test_chunk_attention_validation_and_workspace():
+    lib = _lib.load()
+    ws = lib.nva_chunk_attn_workspace_bytes
+    assert ws(8, 16, 8, 128, 2, 256, 400) == 0                       # one range of keys holds them all
+    assert ws(8, 16, 8, 128, 16, 256, 1 << 20) == 8 * 9 * 16 * 130 * 4   # 4096 keys and up to 31 before a multiple of 32, ranges of 512
+    assert ws(0, 16, 8, 128, 16, 256, 100) == 0
+    ok = dict(q=A, qs=2048, kc=A, vc=A, bt=A, bts=16, mb=16, cu=None, lens=A, tseq=None, out=A, ws=A, wsb=1 << 30, n=8, seqs=8, mq=1,
+              heads=16, kv=8, dim=128, vdim=128, bs=256, nb=64, chunk=8192, scale=0.1, cap=30.0, dtype=0, stream=None)
+    for kw, rc in ((dict(q=None), _lib.ERR_NULL_POINTER), (dict(ws=None), _lib.ERR_NULL_POINTER), (dict(ws=A + 8), _lib.ERR_MISALIGNED),
+                   (dict(wsb=100), _lib.ERR_WORKSPACE_TOO_SMALL), (dict(heads=12), _lib.ERR_BAD_SHAPE), (dict(chunk=0), _lib.ERR_BAD_SHAPE),
+                   (dict(bs=64), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(dim=520), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(qs=2047), _lib.ERR_BAD_STRIDE),
+                   (dict(bts=15), _lib.ERR_BAD_STRIDE), (dict(cu=A), _lib.ERR_NULL_POINTER), (dict(seqs=7), _lib.ERR_BAD_SHAPE),
+                   (dict(dtype=3), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(n=0, q=None), _lib.OK)):
+        assert _with(ok, lib.nva_chunk_attn, **kw) == rc, kw
+
+
+def test_retention_validation_and_workspace():
+    lib = _lib.load()
+    ws = lib.nva_retention_workspace_bytes
+    assert ws(1, 200, 8, 128, 128, 128, 0) == 0 and ws(600, 4096, 8, 128, 128, 128, 0) == 0       # short, or enough sequences
+    assert ws(1, 4096, 8, 128, 128, 128, 0) == 16 * 8 * 128 * 128 * 4                             # segments of 256 tokens
+    assert ws(1, 4096, 8, 128, 128, 128, 1) == 0 and ws(1, 4096, 8, 100, 128, 0, 0) == 0          # sizes that walk token by token
+    ok = dict(x=A, xs=4096, state=A, slots=A, cu=A, lens=A, rope=A, decay=A, out=A, ws=A, wsb=1 << 30, n=4096, seqs=1, mq=4096, heads=8,
+              dim=128, vdim=128, rot=128, max_pos=64, state_slots=4, ks=0.1, eps=1e-6, dtype=0, stream=None)
+    for kw, rc in ((dict(x=None), _lib.ERR_NULL_POINTER), (dict(state=None), _lib.ERR_NULL_POINTER), (dict(rope=None), _lib.ERR_NULL_POINTER),
+                   (dict(decay=None), _lib.ERR_NULL_POINTER), (dict(ws=None), _lib.ERR_NULL_POINTER), (dict(ws=A + 4), _lib.ERR_MISALIGNED),
+                   (dict(wsb=1000), _lib.ERR_WORKSPACE_TOO_SMALL), (dict(xs=4095), _lib.ERR_BAD_STRIDE), (dict(rot=130), _lib.ERR_BAD_SHAPE),
+                   (dict(rot=127), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(dim=1024, xs=1 << 20), _lib.ERR_UNSUPPORTED_GEOMETRY),
+                   (dict(cu=None), _lib.ERR_BAD_SHAPE), (dict(n=0, x=None), _lib.OK)):
+        assert _with(ok, lib.nva_retention, **kw) == rc, kw

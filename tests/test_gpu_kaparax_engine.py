@@ -168,6 +168,25 @@ def test_long_decoding_over_many_chunks(dev, folder):
     _check(torch.cat(rows), want, "bfloat16", "long decoding")
 
 
+@pytest.mark.parametrize("name", ["mixed", "wide"])
+def test_decode_graphs_replay_like_eager_steps(dev, folder, name):
+    """Four requests decoded side by side, by replayed graphs and by eager launches, portions of other
+    work and eager runs of other models' memory between the replays: bit for bit the same logits."""
+    path, cfg, _ = folder(name)
+    graph, eager = TraceReplayer(path, "bfloat16", 2048), TraceReplayer(path, "bfloat16", 2048, enforce_eager=True)
+    assert graph.runner.graph_bs == [1, 2, 4] and not eager.runner.graph_bs
+    prompts = {k: cases.tokens(n, cfg["vocab"], 90 + n) for k, n in (("a", 250), ("b", 31), ("c", 256), ("d", 77))}
+    start = [dict(id=k, tokens=ids, want=[]) for k, ids in prompts.items()]
+    graph.step(start, []), eager.step(start, [])
+    for i in range(12):
+        step = [dict(id=k, tokens=[(7 * i + j) % cfg["vocab"]], want=[0]) for j, k in enumerate(prompts)]
+        got, want = graph.step(step, []), eager.step(step, [])
+        assert torch.equal(got, want), i
+        if i % 4 == 3:                                           # two requests move on in portions, unasked
+            more = [dict(id=k, tokens=cases.tokens(5, cfg["vocab"], i), want=[]) for k in "ac"]
+            graph.step(more, []), eager.step(more, [])
+
+
 def _greedy_follows_plain(name, cfg, weights, prompt, out, slack):
     """Every generated token is the plain model's best, or ties with it within ``slack``."""
     logits = plain.forward(cfg, weights, prompt + out)[len(prompt) - 1: -1]
@@ -222,3 +241,16 @@ def test_trace_command(dev, folder, tmp_path, dtype):
     got = np.fromfile(tmp_path / "1.f32", dtype="<f4").reshape(3, cfg["vocab"])
     _check(torch.from_numpy(got), want[[0, 129, 63]], dtype, "step 1")
     _check(torch.from_numpy(np.fromfile(tmp_path / "2.f32", dtype="<f4").reshape(1, -1)), want[[1]], dtype, "step 2")
+
+
+def test_generate_command(dev, folder):
+    path, cfg, weights = folder("mixed")
+    prompts = [cases.tokens(70, cfg["vocab"], 3), [1]]
+    p = subprocess.run([os.path.join(ROOT, "bin", "generate"), "--model", path, "--max-tokens", "5", "--max-model-len", "512", "--max-num-seqs", "4",
+                        "--dtype", "float32"], input="".join(json.dumps(x) + "\n" for x in prompts), capture_output=True, text=True, timeout=100)
+    assert p.returncode == 0, p.stderr[-2000:]
+    lines = [json.loads(l) for l in p.stdout.splitlines()]
+    assert [l["prompt"] for l in lines] == prompts
+    for l in lines:
+        assert len(l["token_ids"]) == 5
+        _greedy_follows_plain("mixed", cfg, weights, l["prompt"], l["token_ids"], 1e-3)

@@ -130,7 +130,7 @@ def test_clamped_gate(dev, dtype, ff):
 
 ATTN = [  # heads, kv heads, key size, value size, rotated, taps
     (6, 2, 48, 40, 32, 3), (4, 1, 64, 32, 64, 4), (8, 2, 128, 128, 128, 4), (3, 3, 20, 12, 12, 2), (5, 1, 64, 96, 0, 6),
-    (4, 4, 96, 64, 64, 1), (2, 1, 256, 192, 128, 8)]
+    (4, 4, 96, 64, 64, 1), (2, 1, 256, 192, 128, 8), (4, 2, 32, 24, 20, 11)]
 
 
 @pytest.mark.parametrize("dtype", [BF16, F32])

@@ -76,11 +76,15 @@ def test_config_is_read_and_checked(tmp_path):
     assert registry.load_config(str(tmp_path)) == cfg and registry.model_class(cfg) is Kaparax
     (tmp_path / "config.json").write_text(json.dumps({"hidden_size": 64, "num_attention_heads": 4}))
     assert isinstance(registry.load_config(str(tmp_path)), ModelConfig)
+    chain = json.loads(json.dumps(raw))
+    chain["layers"][1]["weights_of"], chain["layers"][1]["mlp"] = 4, None     # towards a later layer, which has tensors then
+    del chain["layers"][4]["weights_of"]
+    assert [l.weights_of for l in KaparaxConfig.from_raw(chain).layers][1] == 4
     bad = json.loads(json.dumps(raw))
     bad["layers"][4]["mixer"]["dim"] = 64
     with pytest.raises(ValueError, match="shares"):
         KaparaxConfig.from_raw(bad)
-    for path, value in ((("layers", 0, "type"), "other"), (("layers", 0, "mlp", "kind"), "routed"), (("layers", 4, "weights_of"), 4)):
+    for path, value in ((("layers", 0, "type"), "other"), (("layers", 0, "mlp", "kind"), "routed"), (("layers", 4, "weights_of"), 4), (("layers", 4, "weights_of"), 70)):
         bad = json.loads(json.dumps(raw))
         at = bad
         for p in path[:-1]:
