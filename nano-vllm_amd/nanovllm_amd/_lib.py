@@ -1,7 +1,9 @@
 """ctypes binding of the C ABI declared in include/nanovllm_amd.h.
 
-The shared library is built in-tree (``libnanovllm_amd.so`` next to this file) by
-``csrc/Makefile``.  There is no fallback: if the library is missing every op raises.
+Two shared libraries are built in-tree, next to this file, by ``csrc/Makefile``:
+``libnanovllm_amd.so`` (the attention hot path) and ``libnanovllm_mixers.so`` (mixers of layered
+models).  Each is opened when one of its symbols is first used, so a model needs only its own.  There
+is no fallback: an op whose library is missing raises.
 """
 from __future__ import annotations
 
@@ -10,6 +12,7 @@ import os
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libnanovllm_amd.so")
+MIXERS_LIB_PATH = os.path.join(_HERE, "libnanovllm_mixers.so")
 
 # status codes of enum nva_status
 OK = 0
@@ -65,32 +68,68 @@ SIGNATURES = {
     "nva_probe_stream_read": (C.c_int, [_vp, _i64, _vp, _vp]),
 }
 
-_lib = None
+# symbols of libnanovllm_mixers.so; the common ones are in both libraries, every other one in libnanovllm_amd.so
+MIXER_SYMBOLS = {"nva_embed_norm", "nva_post_add_norm", "nva_clamped_gate", "nva_conv_rope_store", "nva_chunk_attn",
+                 "nva_chunk_attn_workspace_bytes", "nva_retention", "nva_retention_workspace_bytes"}
+COMMON_SYMBOLS = {"nva_version", "nva_status_string", "nva_device_count", "nva_stage_decode_inputs"}
 
 
 class HipLibraryMissing(RuntimeError):
     pass
 
 
+class _Symbols:
+    """The entry points as attributes, bound (with their signatures) on first use."""
+
+    def __init__(self):
+        self._opened = {}
+
+    def __getattr__(self, name: str):
+        if name not in SIGNATURES:
+            raise AttributeError(name)
+        paths = [MIXERS_LIB_PATH] if name in MIXER_SYMBOLS else [LIB_PATH]
+        if name in COMMON_SYMBOLS:
+            paths.append(MIXERS_LIB_PATH)
+        path = next((p for p in paths if os.path.exists(p)), None)
+        if path is None:
+            raise _missing(paths[0])
+        if path not in self._opened:
+            self._opened[path] = C.CDLL(path)
+        fn = getattr(self._opened[path], name)
+        fn.restype, fn.argtypes = SIGNATURES[name]
+        setattr(self, name, fn)
+        return fn
+
+
+_lib = None
+_symbols = _Symbols()
+
+
+def _missing(path: str) -> HipLibraryMissing:
+    return HipLibraryMissing(f"{path} not found: build it with `make -C nano-vllm_amd/csrc` "
+                             "(or __graft_entry__.build()); there is no CPU fallback")
+
+
 def load():
-    """Load the library once; raise loudly when it has not been built."""
+    """The entry points of the attention hot path (and, where it is built, of the mixers); raises loudly
+    when the library has not been built."""
     global _lib
     if _lib is None:
         if not os.path.exists(LIB_PATH):
-            raise HipLibraryMissing(
-                f"{LIB_PATH} not found: build it with `make -C nano-vllm_amd/csrc` "
-                "(or __graft_entry__.build()); there is no CPU fallback")
-        lib = C.CDLL(LIB_PATH)
-        for name, (res, args) in SIGNATURES.items():
-            fn = getattr(lib, name)
-            fn.restype = res
-            fn.argtypes = args
-        _lib = lib
+            raise _missing(LIB_PATH)
+        _lib = _symbols
     return _lib
 
 
+def load_mixers():
+    """The entry points of the mixers' library and the common ones; needs that library only."""
+    if not os.path.exists(MIXERS_LIB_PATH):
+        raise _missing(MIXERS_LIB_PATH)
+    return _symbols
+
+
 def status_string(code: int) -> str:
-    return load().nva_status_string(int(code)).decode()
+    return _symbols.nva_status_string(int(code)).decode()
 
 
 def check(code: int, what: str) -> None:

@@ -67,7 +67,7 @@ def embed_norm(ids: torch.Tensor, table: torch.Tensor, scale: float, norm: Tuple
     n = ids.numel()
     residual = torch.empty((n, width), dtype=torch.float32, device=table.device)
     out = torch.empty((n, width), dtype=table.dtype, device=table.device)
-    rc = _lib.load().nva_embed_norm(ids.data_ptr(), table.data_ptr(), float(scale), norm[0].data_ptr(), norm[1].data_ptr(),
+    rc = _lib.load_mixers().nva_embed_norm(ids.data_ptr(), table.data_ptr(), float(scale), norm[0].data_ptr(), norm[1].data_ptr(),
                                     residual.data_ptr(), out.data_ptr(), n, width, vocab, float(eps), _DTYPE[table.dtype],
                                     _stream())
     _lib.check(rc, "nva_embed_norm")
@@ -85,7 +85,7 @@ def post_add_norm(y: torch.Tensor, residual: torch.Tensor, post: Tuple[torch.Ten
     if rows is not None:
         assert rows.dtype == torch.int32 and rows.is_contiguous()
     out = torch.empty((count, width), dtype=y.dtype, device=y.device)
-    rc = _lib.load().nva_post_add_norm(y.data_ptr(), y.stride(0), residual.data_ptr(), post[0].data_ptr(), post[1].data_ptr(),
+    rc = _lib.load_mixers().nva_post_add_norm(y.data_ptr(), y.stride(0), residual.data_ptr(), post[0].data_ptr(), post[1].data_ptr(),
                                        nxt[0].data_ptr(), nxt[1].data_ptr(), out.data_ptr(), _ptr(rows), count, n, width,
                                        float(eps), _DTYPE[y.dtype], _stream())
     _lib.check(rc, "nva_post_add_norm")
@@ -98,7 +98,7 @@ def clamped_gate(x: torch.Tensor, limit: float, alpha: float) -> torch.Tensor:
     _need_cuda(x)
     inter = x.shape[1] // 2
     out = torch.empty((x.shape[0], inter), dtype=x.dtype, device=x.device)
-    rc = _lib.load().nva_clamped_gate(x.data_ptr(), x.stride(0), out.data_ptr(), x.shape[0], inter, float(limit),
+    rc = _lib.load_mixers().nva_clamped_gate(x.data_ptr(), x.stride(0), out.data_ptr(), x.shape[0], inter, float(limit),
                                       float(alpha), _DTYPE[x.dtype], _stream())
     _lib.check(rc, "nva_clamped_gate")
     return out
@@ -117,7 +117,7 @@ def conv_rope_store(qkv: torch.Tensor, conv_weight: torch.Tensor, conv_state: Op
     assert group.slot_mapping.numel() == qkv.shape[0] == group.count
     slots = k_cache.shape[0] * k_cache.shape[1]
     state_slots = 0 if conv_state is None else conv_state.shape[0]
-    rc = _lib.load().nva_conv_rope_store(
+    rc = _lib.load_mixers().nva_conv_rope_store(
         qkv.data_ptr(), qkv.stride(0), conv_weight.data_ptr(), _ptr(conv_state), _ptr(group.state_slots), _ptr(group.cu),
         group.seq_lens.data_ptr(), _ptr(group.token_seq), _ptr(rope), q_out.data_ptr(),
         k_cache.data_ptr(), v_cache.data_ptr(), group.slot_mapping.data_ptr(), slots, group.count, group.num_seqs, heads,
@@ -134,7 +134,7 @@ def chunk_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     assert out.is_contiguous() and q.dtype == out.dtype == k_cache.dtype == v_cache.dtype
     table = group.block_tables
     assert table.dtype == torch.int32 and table.shape[0] == group.num_seqs and table.stride(1) == 1
-    chunk, lib, ws = min(chunk, 1 << 30), _lib.load(), None
+    chunk, lib, ws = min(chunk, 1 << 30), _lib.load_mixers(), None
     if group.cu is None and q.dtype == torch.bfloat16:
         nbytes = lib.nva_chunk_attn_workspace_bytes(group.count, heads, kv_heads, vdim, table.shape[1], block, chunk)
         ws = scratch(q.device, nbytes) if nbytes else None
@@ -153,7 +153,7 @@ def retention(qkvg: torch.Tensor, state: torch.Tensor, group: RowGroup, rope: Op
     assert qkvg.stride(1) == 1 and qkvg.shape == (group.count, 2 * heads * (dim + vdim))
     assert out.shape == (group.count, heads * vdim) and out.is_contiguous() and out.dtype == qkvg.dtype
     assert state.dtype == torch.float32 and state.is_contiguous() and log2_decay.dtype == torch.float32
-    lib, ws = _lib.load(), None
+    lib, ws = _lib.load_mixers(), None
     if group.cu is not None:
         nbytes = lib.nva_retention_workspace_bytes(group.num_seqs, group.max_q, heads, dim, vdim, rot_dims, _DTYPE[qkvg.dtype])
         ws = scratch(qkvg.device, nbytes) if nbytes else None

@@ -249,6 +249,10 @@ class ModelRunner:
         assert cfg.num_kvcache_blocks > 0, "no memory left for the KV cache"
         self.model.bind_cache(cfg.num_kvcache_blocks, bs, slots)
 
+    def _kernels(self):
+        """The library this model's steps run on."""
+        return _lib.load_mixers() if self.portions else _lib.load()
+
     # ---- host -> device inputs -----------------------------------------------------------------
     def _to_device(self, array: np.ndarray, dtype: torch.dtype) -> torch.Tensor:
         t = torch.from_numpy(np.ascontiguousarray(array)).to(dtype)
@@ -289,7 +293,7 @@ class ModelRunner:
             host[at: at + raw.size] = raw
             views.append(self._pf_dev[at: at + raw.size].view(dtype).view(array.shape))
             at += (raw.size + 255) // 256 * 256
-        rc = _lib.load().nva_stage_decode_inputs(self._pf_dev.data_ptr(), self._pf_host[self._pf_turn].data_ptr(), at,
+        rc = self._kernels().nva_stage_decode_inputs(self._pf_dev.data_ptr(), self._pf_host[self._pf_turn].data_ptr(), at,
                                                  0, 0, 0, None, 0, torch.cuda.current_stream().cuda_stream)
         _lib.check(rc, "nva_stage_decode_inputs")
         return views
@@ -435,7 +439,7 @@ class ModelRunner:
         if not n_pending:
             st["token_src"][:bs] = -1
         ids_off, idx_off = self._stage_offsets["input_ids"], self._stage_offsets["token_src"]
-        rc = _lib.load().nva_stage_decode_inputs(
+        rc = self._kernels().nva_stage_decode_inputs(
             self._stage_dev.data_ptr(), self._stage_host[self._stage_turn].data_ptr(), self._stage_dev.numel(),
             ids_off, idx_off, bs, prev.tokens_dev.data_ptr() if n_pending else None,
             prev.tokens_dev.numel() if n_pending else 0, torch.cuda.current_stream().cuda_stream)

@@ -39,7 +39,7 @@ def configs():
     key and value sizes, whole, part and no rotation, 1 to 11 taps, chunks shorter and longer than a
     page, any pattern of feed-forwards, shared weights of both mixers, a score cap beyond what an
     unreferenced exponential could hold, sizes off every vector width."""
-    a1 = attention(6, 2, 48, 40, 3, 37, 32)
+    a1 = attention(6, 2, 48, 40, 3, 37, 32, cap=2.5)
     r1 = retention(3, 32, 48, 16)
     a2 = attention(8, 2, 128, 128, 4, 300, 128, scale=0.15)
     r2 = retention(2, 128, 128, 128)

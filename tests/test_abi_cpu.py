@@ -191,6 +191,13 @@ def test_missing_library_fails_loudly(monkeypatch):
     monkeypatch.setattr(_lib, "LIB_PATH", "/nonexistent/libnanovllm_amd.so")
     with pytest.raises(_lib.HipLibraryMissing, match="no CPU fallback"):
         _lib.load()
+    fresh = _lib._Symbols()                                            # the mixers' library alone serves its own and the common symbols
+    assert fresh.nva_version() >= 1 and fresh.nva_retention_workspace_bytes(0, 0, 1, 8, 8, 0, 0) == 0
+    with pytest.raises(_lib.HipLibraryMissing, match="no CPU fallback"):
+        fresh.nva_rms_norm
+    monkeypatch.setattr(_lib, "MIXERS_LIB_PATH", "/nonexistent/libnanovllm_mixers.so")
+    with pytest.raises(_lib.HipLibraryMissing, match="no CPU fallback"):
+        _lib.load_mixers()
 
 
 def test_sample_static_validation():

@@ -224,3 +224,41 @@ def test_trace_command_refuses_what_no_model_does(tmp_path):
     from nanovllm_amd.engine import trace
     (tmp_path / "config.json").write_text(json.dumps({"hidden_size": 64, "num_attention_heads": 4}))
     assert trace.main(["--model", str(tmp_path), "--dtype", "float32", "--out", str(tmp_path), "--max-tokens", "64"]) == 3
+
+
+# ---- the engine tests' models show a planted mistake ---------------------------------------------------
+
+def _reset_state_at(at):
+    true = plain.retention
+    return lambda q, k, v, decay: torch.cat([true(q[:at], k[:at], v[:at], decay), true(q[at:], k[at:], v[at:], decay)])
+
+
+def _forget_rows_before(at):
+    true = plain.short_conv
+    return lambda u, w: torch.cat([true(u[:at], w), true(u[at:], w)])
+
+
+_true = {n: getattr(plain, n) for n in ("chunk_visible", "rotate", "short_conv", "capped", "gated_mlp", "layer_norm", "unit_rms")}
+MISTAKES = {
+    "a chunk one key longer": dict(chunk_visible=lambda t, size: _true["chunk_visible"](t, size + 1)),
+    "keys of the page before unseen": dict(chunk_visible=lambda t, size: _true["chunk_visible"](t, size) & _true["chunk_visible"](t, 256)),
+    "a state lost at token 256": dict(retention=_reset_state_at(256)),
+    "carried rows lost at token 256": dict(short_conv=_forget_rows_before(256)),
+    "rotation of neighbours": dict(rotate=lambda x, base, dims: _true["rotate"](x.flip(-1), base, dims).flip(-1) if dims else x),
+    "taps in the wrong order": dict(short_conv=lambda u, w: _true["short_conv"](u, w.flip(1))),
+    "no score cap": dict(capped=lambda s, cap: s),
+    "no limit in the feed-forward": dict(gated_mlp=lambda h, g, u, d, limit: _true["gated_mlp"](h, g, u, d, 1e9)),
+    "a norm without its shift": dict(layer_norm=lambda x, w, b, eps: _true["layer_norm"](x, w, 0 * b, eps)),
+}
+
+
+@pytest.mark.parametrize("mistake", sorted(MISTAKES))
+def test_planted_mistakes_show_in_the_logits(monkeypatch, mistake):
+    cfg = cases.configs()["mixed"]
+    weights = cases.random_weights(cfg, 1)
+    ids = cases.tokens(300, cfg["vocab"], 5)
+    want = plain.forward(cfg, weights, ids)
+    for name, wrong in MISTAKES[mistake].items():
+        monkeypatch.setattr(plain, name, wrong)
+    err = cases.row_error(plain.forward(cfg, weights, ids), want)
+    assert float(err.max()) > 0.12, (mistake, float(err.max()), float(err.mean()))     # beyond the bf16 limit, far beyond the fp32 one
