@@ -574,30 +574,36 @@ __global__ __launch_bounds__(256, DK * NV > 256 ? 1 : 2) void retention_chunk_ke
             }
 }
 
-// Replaces every segment's own sums by the state the segment starts from; one thread per state element.
+// Replaces every segment's own sums by the state the segment starts from; one thread per four state elements
+// (the value size is a multiple of 8).
 __global__ __launch_bounds__(256) void retention_segment_scan_kernel(const RetentionArgs a, const SegmentArgs sg) {
     const int head = blockIdx.x % a.heads, seq = blockIdx.x / a.heads;
     const int64_t size = static_cast<int64_t>(a.dim) * a.vdim;
-    const int64_t e = static_cast<int64_t>(blockIdx.y) * 256 + threadIdx.x;
+    const int64_t e = (static_cast<int64_t>(blockIdx.y) * 256 + threadIdx.x) * 4;
     const int count = a.cu[seq + 1] - a.cu[seq], start = a.klen[seq] - count;
     if (e >= size || count <= 0 || start < 0) return;
     const int slot = a.slots[seq];
     const bool carried = start > 0 && static_cast<uint32_t>(slot) < static_cast<uint32_t>(a.num_slots);
-    float run = carried ? a.state[(static_cast<int64_t>(slot) * a.heads + head) * size + e] : 0.f;
+    f32x4_t run = {0.f, 0.f, 0.f, 0.f};
+    if (carried) run = *reinterpret_cast<const f32x4_t *>(a.state + (static_cast<int64_t>(slot) * a.heads + head) * size + e);
     const float decay = exp2f(a.log2_decay[head] * static_cast<float>(sg.length));
     const int segments = min(sg.segments, (count - 1) / sg.length + 1);
     float *p = sg.sums + (static_cast<int64_t>(seq) * sg.segments * a.heads + head) * size + e;
     const int64_t step = static_cast<int64_t>(a.heads) * size;
-    constexpr int kAhead = 8;                             // loads in flight together
+    constexpr int kAhead = 16;                            // loads in flight together
     for (int s0 = 0; s0 < segments; s0 += kAhead) {
-        float own[kAhead];
+        f32x4_t own[kAhead];
 #pragma unroll
-        for (int i = 0; i < kAhead; ++i) own[i] = s0 + i + 1 < segments ? p[(s0 + i) * step] : 0.f;
+        for (int i = 0; i < kAhead; ++i) {
+            own[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+            if (s0 + i + 1 < segments) own[i] = *reinterpret_cast<const f32x4_t *>(p + (s0 + i) * step);
+        }
 #pragma unroll
         for (int i = 0; i < kAhead; ++i)
             if (s0 + i < segments) {
-                p[(s0 + i) * step] = run;
-                run = fmaf(decay, run, own[i]);
+                *reinterpret_cast<f32x4_t *>(p + (s0 + i) * step) = run;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) run[j] = fmaf(decay, run[j], own[i][j]);
             }
     }
 }
@@ -621,7 +627,7 @@ static int launch_chunks(const RetentionArgs &a, const SegmentArgs &sg, hipStrea
         hipLaunchKernelGGL((retention_chunk_kernel<DK, NV, true>), grid, block, 0, s, a, sg);
         int rc = launch_status();
         if (rc != NVA_OK) return rc;
-        hipLaunchKernelGGL(retention_segment_scan_kernel, dim3(a.n_seqs * a.heads, (a.dim * a.vdim + 255) / 256), block, 0, s, a, sg);
+        hipLaunchKernelGGL(retention_segment_scan_kernel, dim3(a.n_seqs * a.heads, (a.dim * a.vdim + 1023) / 1024), block, 0, s, a, sg);
         rc = launch_status();
         if (rc != NVA_OK) return rc;
     }
@@ -690,7 +696,7 @@ extern "C" int nva_retention(const void *qkvg, int64_t row_stride, float *state,
         return launch_status();
     }
     if (cu_seqlens_q != nullptr && dtype == NVA_DTYPE_BF16 && chunks_ok(qk_dim, v_dim, a.half) && row_stride % 8 == 0 &&
-        aligned16(qkvg) && aligned16(out) && aligned16(rope_cache)) {
+        aligned16(state) && aligned16(qkvg) && aligned16(out) && aligned16(rope_cache)) {
         SegmentArgs sg = plan_segments(n_seqs, num_heads, max_seqlen_q);
         sg.sums = static_cast<float *>(workspace);
         if (sg.segments > 1) {
