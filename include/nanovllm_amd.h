@@ -378,6 +378,112 @@ int nva_retention(const void *qkvg, int64_t row_stride, float *state, const int3
                   void *stream);
 
 /*
+ * ---- layered models whose mixer and feed-forward branch off one point of the stream ---------
+ * Same conventions for rows, dtypes, slots and padded rows as the mixers above.
+ */
+
+/* residual[r] = table[ids[r]] * scale (fp32); out1[r] = residual[r] / rms * (weight_offset + weight1), out2 the
+ * same with weight2 (weight2 may be NULL: one norm).  rms = sqrt(mean(x^2) + eps).  clear (may be NULL):
+ * clear_count int32 counters set to zero, for a router that runs behind this. */
+int nva_embed_rms_norms(const int64_t *ids, const void *table, float scale, const void *weight1, const void *weight2,
+                        float weight_offset, float *residual, void *out1, void *out2, int32_t *clear,
+                        int32_t clear_count, int32_t rows, int32_t width, int32_t vocab, float eps, int32_t dtype,
+                        void *stream);
+
+/* residual[r] += mult * (gain1 * y1[r] + gain2 * sum_k term_weight[r, k] * y2[r * terms + k]), in place, fp32; then
+ * the norms as above.  y1 or y2, either gain ([width]) and term_weight (fp32) may be NULL (absent; one; one).
+ * rows_of (int32 [rows], may be NULL): out[r] is computed from row rows_of[r] (clamped to [0, src_rows)) and
+ * residual is not written; without it rows == src_rows. */
+int nva_branches_rms_norms(const void *y1, int64_t y1_row_stride, const void *gain1, const void *y2,
+                           const float *term_weight, int32_t terms, const void *gain2, float mult, float *residual,
+                           const void *weight1, const void *weight2, float weight_offset, void *out1, void *out2,
+                           const int32_t *rows_of, int32_t *clear, int32_t clear_count, int32_t rows,
+                           int32_t src_rows, int32_t width, float eps, int32_t dtype, void *stream);
+
+/* out[r, g] = W_g x[r, g] for every row and group: x + r * x_row_stride + g * x_group_stride, weight [groups, n_out, k_in],
+ * out + r * out_row_stride + g * out_group_stride (elements).  out_dtype fp32 keeps the fp32 sums of bf16 products. */
+int nva_grouped_linear(const void *x, int64_t x_row_stride, int64_t x_group_stride, const void *weight, void *out,
+                       int64_t out_row_stride, int64_t out_group_stride, int32_t rows, int32_t groups, int32_t n_out,
+                       int32_t k_in, int32_t dtype, int32_t out_dtype, void *stream);
+
+/* Router of a mixture of experts: logits = weight x (fp32), softmax over all experts, the `top` best (ties: the lower
+ * index) in descending order, their scores divided by their sum (+ 1e-20) and multiplied by scale.
+ * choice int32, choice_weight fp32: [rows, top].  lists int32 [experts, list_stride], counts int32 [experts]: the
+ * assignments row * top + k of every expert, in no particular order; counts must be zero on entry;
+ * list_stride >= rows.  experts <= 1024, top <= 128. */
+int nva_router(const void *x, int64_t x_row_stride, const void *weight, int32_t *choice, float *choice_weight,
+               int32_t *lists, int32_t *counts, int64_t list_stride, int32_t rows, int32_t width, int32_t experts,
+               int32_t top, float scale, int32_t dtype, void *stream);
+
+/* out[p] = W_e x[p / terms] (x_per_row) or W_e x[p], for every assignment p of lists to its expert e.
+ * weight: [experts, n_out, k_in], or gated: [experts, 2 n_out, k_in] (gate | up) and out = silu(gate) * up.
+ * out: [rows * terms, n_out] dense. */
+int nva_routed_linear(const void *x, int64_t x_row_stride, const void *weight, void *out, const int32_t *lists,
+                      const int32_t *counts, int64_t list_stride, int32_t rows, int32_t terms, int32_t experts,
+                      int32_t n_out, int32_t k_in, int32_t x_per_row, int32_t gated, int32_t dtype, void *stream);
+
+/* Latent attention, what a row leaves behind and its query latent.
+ * x: [n_tokens, q_rank | kv_rank | rot_dim] (row stride in elements).
+ * q_out [n_tokens, q_rank] = first part / rms * q_norm_weight; cache row slot_mapping[i] of [num_slots, kv_rank + rot_dim] =
+ * (second part / rms * kv_norm_weight | third part, neighbours (2i, 2i + 1) rotated by the row's position).
+ * cache NULL: the queries only (x then has q_rank columns).  rope_cache: fp32 [max_position, rot_dim], cos in the
+ * first half of a row, sin in the second. */
+int nva_latent_prepare(const void *x, int64_t x_row_stride, const void *q_norm_weight, const void *kv_norm_weight,
+                       const float *rope_cache, void *q_out, void *cache, const int32_t *slot_mapping, int64_t num_slots,
+                       const int32_t *cu_seqlens_q, const int32_t *seq_lens, const int32_t *token_seq, int32_t n_tokens,
+                       int32_t n_seqs, int32_t q_rank, int32_t kv_rank, int32_t rot_dim, int32_t max_position, float eps,
+                       int32_t dtype, void *stream);
+
+/* Absorbed form: the query at position p meets the cached rows (p - window, p] of its sequence,
+ *   score = (q_latent . c + rotate(q_rot) . k_rot) * scale,  out = sigmoid(gate) * sum softmax(score) c.
+ * q_latent [n_tokens, num_heads, kv_rank] dense; q_rot [n_tokens, num_heads, rot_dim], not yet rotated; gate
+ * [n_tokens, num_heads] logits; cache [num_blocks, block_size, kv_rank + rot_dim]; out [n_tokens, num_heads, kv_rank] dense.
+ * A key behind a table entry outside [0, num_blocks) is not seen.  kv_rank + rot_dim <= 1024.
+ * workspace: partial results, nva_latent_attn_workspace_bytes() bytes, 16-byte aligned (NULL where that is 0). */
+size_t nva_latent_attn_workspace_bytes(int32_t n_tokens, int32_t num_heads, int32_t kv_rank, int32_t rot_dim,
+                                       int32_t max_blocks, int32_t block_size, int32_t window, int32_t dtype);
+int nva_latent_attn(const void *q_latent, const void *q_rot, int64_t qr_row_stride, int64_t qr_head_stride, const void *gate,
+                    int64_t gate_row_stride, const float *rope_cache, const void *cache, const int32_t *block_tables,
+                    int64_t bt_row_stride, int32_t max_blocks, const int32_t *cu_seqlens_q, const int32_t *seq_lens,
+                    const int32_t *token_seq, void *out, void *workspace, size_t workspace_bytes, int32_t n_tokens,
+                    int32_t n_seqs, int32_t num_heads, int32_t kv_rank, int32_t rot_dim, int32_t block_size,
+                    int32_t num_blocks, int32_t window, int32_t max_position, float scale, int32_t dtype, void *stream);
+
+/* Expanded form, for portions.  nva_latent_gather copies the cache rows of the last key_cu[s + 1] - key_cu[s] tokens of
+ * every sequence s to out [n_keys, row_width]; the caller multiplies the latents out to kv [n_keys, num_heads * dim |
+ * num_heads * v_dim]; nva_latent_prefill attends:
+ *   score = (q[:dim] . k + rotate(q[dim:]) . k_rot) * scale,  out = sigmoid(gate) * sum softmax(score) v
+ * over the positions (p - window, p] that were gathered.  q [n_tokens, num_heads, dim + rot_dim], bf16 only, sizes
+ * multiples of 8 (nva_latent_prefill_supported). */
+int nva_latent_gather(const void *cache, const int32_t *block_tables, int64_t bt_row_stride, int32_t max_blocks,
+                      const int32_t *key_cu, const int32_t *seq_lens, void *out, int32_t n_keys, int32_t n_seqs,
+                      int32_t row_width, int32_t block_size, int32_t num_blocks, int32_t dtype, void *stream);
+int nva_latent_prefill_supported(int32_t dim, int32_t rot_dim, int32_t v_dim, int32_t dtype);
+int nva_latent_prefill(const void *q, int64_t q_row_stride, const void *kv, int64_t kv_row_stride, const void *k_rot,
+                       int64_t kr_row_stride, const void *gate, int64_t gate_row_stride, const float *rope_cache,
+                       const int32_t *cu_seqlens_q, const int32_t *seq_lens, const int32_t *key_cu, void *out,
+                       int32_t n_tokens, int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads, int32_t dim, int32_t rot_dim,
+                       int32_t v_dim, int32_t window, int32_t max_position, float scale, int32_t dtype, void *stream);
+
+/* Matrix memory with exponential gates, head norm and output gate.  With i = cap tanh((z_i + b_i) / cap) and
+ * f = log sigmoid(cap tanh((z_f + b_f) / cap)):  m_t = max(f + m_{t-1}, i),  S_t = e^{f + m_{t-1} - m_t} S_{t-1} +
+ * e^{i - m_t} k v^T,  n_t likewise with k,  o = S_t^T q / (max(|n_t . q|, e^{-m_t}) + 1e-6), q scaled by q_scale;
+ * out = o / rms(o) * norm_weight * sigmoid(gate).
+ * qkvg: [n_tokens, 2 * num_heads * (qk_dim + v_dim)] (q | k | v | gate, row stride in elements); gate_logits fp32
+ * [n_tokens, 2 * num_heads] dense (input gates | forget gates), gate_bias fp32 [2 * num_heads], norm_weight
+ * [num_heads * v_dim]; state / mass / top: fp32 [num_state_slots, num_heads, (qk_dim, v_dim | qk_dim | -)], carried across
+ * calls; out: [n_tokens, num_heads * v_dim] dense.  workspace: states between the segments of long portions,
+ * nva_mlstm_workspace_bytes() bytes, 16-byte aligned (NULL where that is 0, and for single tokens). */
+size_t nva_mlstm_workspace_bytes(int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads, int32_t qk_dim, int32_t v_dim,
+                                 int32_t dtype);
+int nva_mlstm(const void *qkvg, int64_t row_stride, const float *gate_logits, const float *gate_bias,
+              const void *norm_weight, float *state, float *mass, float *top, const int32_t *state_slots_of_seq,
+              const int32_t *cu_seqlens_q, const int32_t *seq_lens, void *out, void *workspace,
+              size_t workspace_bytes, int32_t n_tokens, int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads,
+              int32_t qk_dim, int32_t v_dim, int32_t num_state_slots, float q_scale, float gate_cap, float eps,
+              int32_t dtype, void *stream);
+
+/*
  * Calibration, no counterpart in the reference: streams nbytes from src with the access discipline of
  * the decode kernel (2048 wavefront workers, contiguous slices, 16-byte non-temporal loads) and keeps
  * nothing.  Its duration is what any kernel that reads that many bytes needs at least on this GPU;

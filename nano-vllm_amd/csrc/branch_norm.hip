@@ -1,0 +1,217 @@
+// The residual step of layers whose mixer and feed-forward branch off the same point of the stream:
+//   embed_norms     residual = embed[id] * scale, then the norms below
+//   branches_norms  residual += mult * (gain1 * y1 + gain2 * sum_k weight_k y2_k)   (y2: the outputs of a
+//                   row's experts, or one dense branch), then
+//                   out1 = residual / rms * (offset + w1)     out2 = residual / rms * (offset + w2)
+// in one pass over the row.  Tensors are bf16 or fp32, the stream and all sums fp32.
+#include "nva_elem.h"
+
+#include <math.h>
+
+namespace nva {
+
+struct BranchArgs {
+    const int64_t *ids;              // embed: token ids [rows]
+    const void *x;                   // embed: table [vocab, width]; otherwise y1 [*, width] (may be null)
+    int64_t x_stride;
+    const void *gain1;               // [width] or null (1)
+    const void *y2;                  // [* x terms, width]: rows r * terms + k belong to row r (null: none)
+    const float *term_weight;        // [* x terms] or null (1)
+    const void *gain2;               // [width] or null (1)
+    float *residual;                 // fp32 [*, width] dense
+    const void *w1, *w2;             // [width]; w2 null: one norm only
+    void *out1, *out2;               // [rows, width] dense
+    const int32_t *rows_of;          // optional: output row r is computed from row rows_of[r], residual left alone
+    int32_t *clear;                  // optional: counters set to zero
+    int32_t clear_count, terms;
+    int32_t rows, src_rows, width, vocab;
+    float scale, mult, offset, eps;
+};
+
+__device__ __forceinline__ void clear_counters(const BranchArgs &a) {
+    if (a.clear != nullptr && blockIdx.x == 0)
+        for (int i = threadIdx.x; i < a.clear_count; i += 256) a.clear[i] = 0;
+}
+
+__device__ __forceinline__ int64_t branch_source_row(const BranchArgs &a, int row, bool embed) {
+    if (embed || a.rows_of == nullptr) return row;
+    return min(max(a.rows_of[row], 0), a.src_rows - 1);      // device data the host could not check
+}
+
+// V consecutive elements of the new residual
+template <typename T, int V, bool kEmbed>
+__device__ __forceinline__ void new_residual(const BranchArgs &a, const T *xp, int64_t src, int e, float (&r)[V]) {
+    float v[V];
+    if (kEmbed) {
+        load_f32<T, V>(xp + e, v);
+#pragma unroll
+        for (int i = 0; i < V; ++i) r[i] = v[i] * a.scale;
+        return;
+    }
+    float sum[V];
+#pragma unroll
+    for (int i = 0; i < V; ++i) sum[i] = 0.f;
+    load_f32<float, V>(a.residual + src * a.width + e, r);
+    if (a.x != nullptr) {
+        load_f32<T, V>(xp + e, v);
+        if (a.gain1 != nullptr) load_f32<T, V>(static_cast<const T *>(a.gain1) + e, sum);
+#pragma unroll
+        for (int i = 0; i < V; ++i) sum[i] = a.gain1 != nullptr ? sum[i] * v[i] : v[i];
+    }
+    if (a.y2 != nullptr) {
+        float part[V];
+#pragma unroll
+        for (int i = 0; i < V; ++i) part[i] = 0.f;
+        const T *yp = static_cast<const T *>(a.y2) + src * a.terms * a.width + e;
+#pragma unroll 4
+        for (int k = 0; k < a.terms; ++k) {
+            const float w = a.term_weight != nullptr ? a.term_weight[src * a.terms + k] : 1.0f;
+            load_f32<T, V>(yp + static_cast<int64_t>(k) * a.width, v);
+#pragma unroll
+            for (int i = 0; i < V; ++i) part[i] = fmaf(w, v[i], part[i]);
+        }
+        float gain[V];
+        if (a.gain2 != nullptr) load_f32<T, V>(static_cast<const T *>(a.gain2) + e, gain);
+#pragma unroll
+        for (int i = 0; i < V; ++i) sum[i] = a.gain2 != nullptr ? fmaf(gain[i], part[i], sum[i]) : sum[i] + part[i];
+    }
+#pragma unroll
+    for (int i = 0; i < V; ++i) r[i] = fmaf(a.mult, sum[i], r[i]);
+}
+
+// One wavefront per row, the row in registers; NC pieces of 512 elements (width % 8 == 0, width <= 4096).
+template <typename T, int NC, bool kEmbed>
+__global__ __launch_bounds__(256) void branch_norm_kernel(BranchArgs a) {
+    clear_counters(a);
+    const int lane = threadIdx.x & 63;
+    const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (row >= a.rows) return;
+    const int64_t src = branch_source_row(a, row, kEmbed);
+    int64_t xrow = src;
+    if (kEmbed) xrow = min(max(a.ids[row], static_cast<int64_t>(0)), static_cast<int64_t>(a.vocab) - 1);
+    const T *xp = static_cast<const T *>(a.x) + xrow * a.x_stride;
+    float r[NC][8];
+    float sq = 0.f;
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+        const int e = c * 512 + lane * 8;
+        if (e < a.width) {
+            new_residual<T, 8, kEmbed>(a, xp, src, e, r[c]);
+            if (kEmbed || a.rows_of == nullptr) store_f32<float, 8>(a.residual + src * a.width + e, r[c]);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) sq = fmaf(r[c][i], r[c][i], sq);
+        }
+    }
+    const float rstd = rsqrtf(wave_sum(sq) / static_cast<float>(a.width) + a.eps);
+    const int64_t at = static_cast<int64_t>(row) * a.width;
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+        const int e = c * 512 + lane * 8;
+        if (e < a.width) {
+            float w[8], y[8];
+            load_f32<T, 8>(static_cast<const T *>(a.w1) + e, w);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) y[i] = r[c][i] * rstd * (a.offset + w[i]);
+            store_f32<T, 8>(static_cast<T *>(a.out1) + at + e, y);
+            if (a.w2 != nullptr) {
+                load_f32<T, 8>(static_cast<const T *>(a.w2) + e, w);
+#pragma unroll
+                for (int i = 0; i < 8; ++i) y[i] = r[c][i] * rstd * (a.offset + w[i]);
+                store_f32<T, 8>(static_cast<T *>(a.out2) + at + e, y);
+            }
+        }
+    }
+}
+
+// Any width: one workgroup per row; a thread re-reads the residual elements it wrote itself (or, where
+// they are not written, computes them again).
+template <typename T, bool kEmbed>
+__global__ __launch_bounds__(256) void branch_norm_any_kernel(BranchArgs a) {
+    __shared__ float sh[4];
+    clear_counters(a);
+    const int row = blockIdx.x;
+    const int64_t src = branch_source_row(a, row, kEmbed);
+    int64_t xrow = src;
+    if (kEmbed) xrow = min(max(a.ids[row], static_cast<int64_t>(0)), static_cast<int64_t>(a.vocab) - 1);
+    const T *xp = static_cast<const T *>(a.x) + xrow * a.x_stride;
+    const bool keep = kEmbed || a.rows_of == nullptr;
+    float sq = 0.f;
+    for (int e = threadIdx.x; e < a.width; e += 256) {
+        float r[1];
+        new_residual<T, 1, kEmbed>(a, xp, src, e, r);
+        if (keep) a.residual[src * a.width + e] = r[0];
+        sq = fmaf(r[0], r[0], sq);
+    }
+    sq = wave_sum(sq);
+    if ((threadIdx.x & 63) == 0) sh[threadIdx.x >> 6] = sq;
+    __syncthreads();
+    const float rstd = rsqrtf(((sh[0] + sh[1]) + (sh[2] + sh[3])) / static_cast<float>(a.width) + a.eps);
+    const int64_t at = static_cast<int64_t>(row) * a.width;
+    for (int e = threadIdx.x; e < a.width; e += 256) {
+        float r[1];
+        if (keep) r[0] = a.residual[src * a.width + e];
+        else new_residual<T, 1, kEmbed>(a, xp, src, e, r);
+        static_cast<T *>(a.out1)[at + e] = Elem<T>::from_f32(r[0] * rstd * (a.offset + Elem<T>::to_f32(static_cast<const T *>(a.w1)[e])));
+        if (a.w2 != nullptr)
+            static_cast<T *>(a.out2)[at + e] = Elem<T>::from_f32(r[0] * rstd * (a.offset + Elem<T>::to_f32(static_cast<const T *>(a.w2)[e])));
+    }
+}
+
+template <typename T, bool kEmbed>
+static int launch_branch_norm(const BranchArgs &a, hipStream_t s) {
+    const bool vector = a.width % 8 == 0 && a.width <= 4096 && a.x_stride % 8 == 0 && aligned16(a.x) && aligned16(a.residual) &&
+                        aligned16(a.gain1) && aligned16(a.y2) && aligned16(a.gain2) && aligned16(a.w1) && aligned16(a.w2) &&
+                        aligned16(a.out1) && aligned16(a.out2);
+    if (!vector) {
+        hipLaunchKernelGGL((branch_norm_any_kernel<T, kEmbed>), dim3(a.rows), dim3(256), 0, s, a);
+        return launch_status();
+    }
+    const dim3 grid((a.rows + 3) / 4), block(256);
+    switch ((a.width + 511) / 512) {
+        case 1: hipLaunchKernelGGL((branch_norm_kernel<T, 1, kEmbed>), grid, block, 0, s, a); break;
+        case 2: hipLaunchKernelGGL((branch_norm_kernel<T, 2, kEmbed>), grid, block, 0, s, a); break;
+        case 3: case 4: hipLaunchKernelGGL((branch_norm_kernel<T, 4, kEmbed>), grid, block, 0, s, a); break;
+        default: hipLaunchKernelGGL((branch_norm_kernel<T, 8, kEmbed>), grid, block, 0, s, a); break;
+    }
+    return launch_status();
+}
+
+}  // namespace nva
+
+extern "C" int nva_embed_rms_norms(const int64_t *ids, const void *table, float scale, const void *weight1, const void *weight2,
+                                   float weight_offset, float *residual, void *out1, void *out2, int32_t *clear,
+                                   int32_t clear_count, int32_t rows, int32_t width, int32_t vocab, float eps, int32_t dtype,
+                                   void *stream) {
+    using namespace nva;
+    if (rows < 0 || width <= 0 || vocab <= 0 || clear_count < 0) return NVA_ERR_BAD_SHAPE;
+    if (!known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
+    if (rows == 0) return NVA_OK;
+    if (!ids || !table || !weight1 || !residual || !out1 || (weight2 && !out2)) return NVA_ERR_NULL_POINTER;
+    BranchArgs a{};
+    a.ids = ids; a.x = table; a.x_stride = width; a.residual = residual; a.w1 = weight1; a.w2 = weight2; a.out1 = out1; a.out2 = out2;
+    a.clear = clear; a.clear_count = clear ? clear_count : 0; a.rows = rows; a.src_rows = rows; a.width = width; a.vocab = vocab;
+    a.scale = scale; a.offset = weight_offset; a.eps = eps;
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    return dtype == NVA_DTYPE_BF16 ? launch_branch_norm<bf16_t, true>(a, s) : launch_branch_norm<float, true>(a, s);
+}
+
+extern "C" int nva_branches_rms_norms(const void *y1, int64_t y1_row_stride, const void *gain1, const void *y2,
+                                      const float *term_weight, int32_t terms, const void *gain2, float mult, float *residual,
+                                      const void *weight1, const void *weight2, float weight_offset, void *out1, void *out2,
+                                      const int32_t *rows_of, int32_t *clear, int32_t clear_count, int32_t rows,
+                                      int32_t src_rows, int32_t width, float eps, int32_t dtype, void *stream) {
+    using namespace nva;
+    if (rows < 0 || src_rows < 0 || width <= 0 || terms < 0 || clear_count < 0) return NVA_ERR_BAD_SHAPE;
+    if (!known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
+    if (rows == 0) return NVA_OK;
+    if (src_rows == 0 || (!rows_of && rows != src_rows) || (y2 && terms == 0)) return NVA_ERR_BAD_SHAPE;
+    if (!residual || !weight1 || !out1 || (weight2 && !out2)) return NVA_ERR_NULL_POINTER;
+    if (y1 && y1_row_stride < width) return NVA_ERR_BAD_STRIDE;
+    BranchArgs a{};
+    a.x = y1; a.x_stride = y1 ? y1_row_stride : 0; a.gain1 = gain1; a.y2 = y2; a.term_weight = term_weight; a.terms = terms; a.gain2 = gain2;
+    a.mult = mult; a.residual = residual; a.w1 = weight1; a.w2 = weight2; a.offset = weight_offset; a.out1 = out1; a.out2 = out2;
+    a.rows_of = rows_of; a.clear = clear; a.clear_count = clear ? clear_count : 0; a.rows = rows; a.src_rows = src_rows;
+    a.width = width; a.eps = eps;
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    return dtype == NVA_DTYPE_BF16 ? launch_branch_norm<bf16_t, false>(a, s) : launch_branch_norm<float, false>(a, s);
+}

@@ -1,0 +1,390 @@
+// Matrix products whose weights come in groups, and the router that assigns rows to them.
+//   dense groups   out[r, g] = W_g x[r, g] for every row r and group g (per-head products; one group: a plain
+//                  product with few outputs, in fp32 where asked for)
+//   routed groups  out[p] = W_e x[p / terms] for every assignment p = row * terms + k of a row to an expert e;
+//                  lists[e] holds the assignments of expert e in any order, counts[e] their number
+//   gated          W has 2 n_out rows (gate | up): out = silu(gate) * up
+//   router         logits in fp32, softmax over all experts, the best `terms`, their normalised weights, lists
+// bf16 tensors go through the matrix cores, fp32 ones and odd sizes through plain fp32 kernels.
+#include "nva_elem.h"
+#include "nva_matrix.h"
+
+#include <math.h>
+
+#include <algorithm>
+
+namespace nva {
+
+struct LinearArgs {
+    const void *x;
+    int64_t x_stride, x_group;       // elements between rows, between groups (dense)
+    const void *w;                   // [groups][n_out or 2 n_out][k]
+    void *out;
+    int64_t o_stride, o_group;
+    const int32_t *lists, *counts;   // routed: [groups, list_stride], [groups]
+    int64_t list_stride;
+    int32_t rows, groups, n_out, k;  // rows: dense rows, or assignments in all
+    int32_t x_div;                   // routed: x row = assignment / x_div
+};
+
+// number of rows of a group, and where its i-th row comes from and goes to
+__device__ __forceinline__ int group_rows(const LinearArgs &a, int g) {
+    return a.lists == nullptr ? a.rows : min(max(a.counts[g], 0), static_cast<int32_t>(a.list_stride));
+}
+__device__ __forceinline__ int group_row(const LinearArgs &a, int g, int i) {
+    return a.lists == nullptr ? i : min(max(a.lists[g * a.list_stride + i], 0), a.rows - 1);
+}
+__device__ __forceinline__ int64_t x_offset(const LinearArgs &a, int g, int row) {
+    return a.lists == nullptr ? row * a.x_stride + g * a.x_group : row / a.x_div * a.x_stride;
+}
+__device__ __forceinline__ int64_t out_offset(const LinearArgs &a, int g, int row) {
+    return row * a.o_stride + (a.lists == nullptr ? g * a.o_group : 0);
+}
+
+template <typename T> __device__ __forceinline__ float silu_of(float z) { return z * sigmoid_of<T>(z); }
+
+// ---- any sizes, bf16 or fp32: tiles of 16 rows x 64 outputs in plain fp32 arithmetic ----------------
+template <typename T, typename O, bool kGated>
+__global__ __launch_bounds__(256) void linear_any_kernel(LinearArgs a) {
+    constexpr int kParts = kGated ? 2 : 1, kK = 32;
+    __shared__ float sx[16][kK + 1], sw[kParts][64][kK + 1];
+    const int g = blockIdx.y, n0 = blockIdx.x * 64, tid = threadIdx.x;
+    const int r = tid >> 4, c = tid & 15;
+    const int count = group_rows(a, g);
+    const T *w = static_cast<const T *>(a.w) + static_cast<int64_t>(g) * kParts * a.n_out * a.k;
+    for (int m0 = blockIdx.z * 16; m0 < count; m0 += gridDim.z * 16) {
+        float acc[kParts][4];
+#pragma unroll
+        for (int p = 0; p < kParts; ++p)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) acc[p][j] = 0.f;
+        const int row = group_row(a, g, min(m0 + r, count - 1));
+        const T *x = static_cast<const T *>(a.x) + x_offset(a, g, row);
+        for (int k0 = 0; k0 < a.k; k0 += kK) {
+            for (int i = c; i < kK; i += 16) sx[r][i] = k0 + i < a.k ? Elem<T>::to_f32(x[k0 + i]) : 0.f;
+            for (int i = tid; i < kParts * 64 * kK; i += 256) {
+                const int kk = i % kK, n = i / kK % 64, p = i / kK / 64;
+                sw[p][n][kk] = k0 + kk < a.k && n0 + n < a.n_out ? Elem<T>::to_f32(w[(static_cast<int64_t>(p) * a.n_out + n0 + n) * a.k + k0 + kk]) : 0.f;
+            }
+            __syncthreads();
+#pragma unroll 8
+            for (int kk = 0; kk < kK; ++kk)
+#pragma unroll
+                for (int p = 0; p < kParts; ++p)
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) acc[p][j] = fmaf(sx[r][kk], sw[p][c + 16 * j][kk], acc[p][j]);
+            __syncthreads();
+        }
+        if (m0 + r < count) {
+            O *out = static_cast<O *>(a.out) + out_offset(a, g, row);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int n = n0 + c + 16 * j;
+                if (n < a.n_out) out[n] = Elem<O>::from_f32(kGated ? silu_of<T>(acc[0][j]) * acc[kParts - 1][j] : acc[0][j]);
+            }
+        }
+    }
+}
+
+// ---- bf16, few rows per group: the weights are streamed once per 16 MT rows ------------------------
+// A workgroup takes 16 outputs of a group (16 gates and the 16 ups that belong to them), its four
+// wavefronts a quarter of the inner dimension each, weights and rows straight from memory into operands
+// (weights first operand: an accumulator holds four consecutive outputs of one row).  The quarters meet in LDS.
+template <int MT, bool kGated, typename O>
+__global__ __launch_bounds__(256) void linear_skinny_kernel(LinearArgs a) {
+    constexpr int kParts = kGated ? 2 : 1, kAhead = MT == 1 ? 8 : 4;
+    __shared__ __attribute__((aligned(16))) float part[4][MT * 16][kParts * 16 + 4];
+    const int g = blockIdx.y, n0 = blockIdx.x * 16;
+    const int tid = threadIdx.x, lane = tid & 63, r = lane & 15, q = lane >> 4;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int count = group_rows(a, g);
+    const int steps = (a.k + 31) / 32, per_wave = (steps + 3) / 4;
+    const int s_begin = wave * per_wave, s_end = min(steps, s_begin + per_wave);
+    const bf16_t *w = static_cast<const bf16_t *>(a.w) + static_cast<int64_t>(g) * kParts * a.n_out * a.k +
+                      static_cast<int64_t>(min(n0 + r, a.n_out - 1)) * a.k;
+    const int64_t up = static_cast<int64_t>(a.n_out) * a.k;
+    for (int m0 = blockIdx.z * 16 * MT; m0 < count; m0 += gridDim.z * 16 * MT) {
+        const bf16_t *x[MT];
+#pragma unroll
+        for (int m = 0; m < MT; ++m)
+            x[m] = static_cast<const bf16_t *>(a.x) + x_offset(a, g, group_row(a, g, min(m0 + 16 * m + r, count - 1)));
+        f32x4_t acc[MT][kParts];
+#pragma unroll
+        for (int m = 0; m < MT; ++m)
+#pragma unroll
+            for (int p = 0; p < kParts; ++p) acc[m][p] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        for (int s0 = s_begin; s0 < s_end; s0 += kAhead) {
+            u32x4_t wf[kAhead][kParts], xf[kAhead][MT];
+#pragma unroll
+            for (int j = 0; j < kAhead; ++j) {
+                const int e = (s0 + j) * 32 + 8 * q;
+                const bool in = s0 + j < s_end && e < a.k;
+#pragma unroll
+                for (int p = 0; p < kParts; ++p) {
+                    wf[j][p] = u32x4_t{0, 0, 0, 0};
+                    if (in) wf[j][p] = *reinterpret_cast<const u32x4_t *>(w + p * up + e);
+                }
+#pragma unroll
+                for (int m = 0; m < MT; ++m) {
+                    xf[j][m] = u32x4_t{0, 0, 0, 0};
+                    if (in) xf[j][m] = *reinterpret_cast<const u32x4_t *>(x[m] + e);
+                }
+            }
+#pragma unroll
+            for (int j = 0; j < kAhead; ++j)
+#pragma unroll
+                for (int m = 0; m < MT; ++m)
+#pragma unroll
+                    for (int p = 0; p < kParts; ++p) acc[m][p] = mfma16(wf[j][p], xf[j][m], acc[m][p]);
+        }
+#pragma unroll
+        for (int m = 0; m < MT; ++m)
+#pragma unroll
+            for (int p = 0; p < kParts; ++p) *reinterpret_cast<f32x4_t *>(&part[wave][16 * m + r][16 * p + 4 * q]) = acc[m][p];
+        __syncthreads();
+        for (int i = tid; i < MT * 16 * 16; i += 256) {
+            const int m = i >> 4, n = i & 15;
+            if (m0 + m >= count || n0 + n >= a.n_out) continue;
+            float v[kParts];
+#pragma unroll
+            for (int p = 0; p < kParts; ++p) {
+                const int c = 16 * p + n;
+                v[p] = (part[0][m][c] + part[1][m][c]) + (part[2][m][c] + part[3][m][c]);
+            }
+            static_cast<O *>(a.out)[out_offset(a, g, group_row(a, g, m0 + m)) + n0 + n] =
+                Elem<O>::from_f32(kGated ? silu_of<bf16_t>(v[0]) * v[kParts - 1] : v[0]);
+        }
+        __syncthreads();
+    }
+}
+
+template <typename T, typename O, bool kGated>
+static int launch_any_linear(const LinearArgs &a, int32_t most_rows, hipStream_t s) {
+    const dim3 grid((a.n_out + 63) / 64, a.groups, std::min(std::max(1, (most_rows + 15) / 16), a.lists ? 64 : 65535));
+    hipLaunchKernelGGL((linear_any_kernel<T, O, kGated>), grid, dim3(256), 0, s, a);
+    return launch_status();
+}
+
+// rows_hint: rows a group is expected to have
+template <bool kGated, typename O>
+static int launch_skinny(const LinearArgs &a, int32_t rows_hint, int32_t most_rows, hipStream_t s) {
+    const int mt = rows_hint <= 16 ? 1 : rows_hint <= 32 ? 2 : 4;
+    const int passes = std::max(1, (most_rows + 16 * mt - 1) / (16 * mt));
+    const dim3 grid((a.n_out + 15) / 16, a.groups, a.lists ? 1 : std::min(passes, 65535)), block(256);
+    if (mt == 1) hipLaunchKernelGGL((linear_skinny_kernel<1, kGated, O>), grid, block, 0, s, a);
+    else if (mt == 2) hipLaunchKernelGGL((linear_skinny_kernel<2, kGated, O>), grid, block, 0, s, a);
+    else hipLaunchKernelGGL((linear_skinny_kernel<4, kGated, O>), grid, block, 0, s, a);
+    return launch_status();
+}
+
+static bool linear_matrix_ok(const LinearArgs &a) {
+    return a.k % 8 == 0 && a.x_stride % 8 == 0 && a.x_group % 8 == 0 && aligned16(a.x) && aligned16(a.w);
+}
+
+// ---- router ------------------------------------------------------------------------------------------
+
+struct RouterArgs {
+    const void *x;                   // [rows, width]
+    int64_t x_stride;
+    const void *w;                   // [experts, width]
+    int32_t *choice;                 // [rows, top]
+    float *weight;                   // [rows, top]
+    int32_t *lists, *counts;         // [experts, list_stride], [experts] (zero on entry)
+    int64_t list_stride;
+    int32_t rows, width, experts, top;
+    float scale;
+};
+
+// 16 TG rows per workgroup of eight wavefronts; KS = 8 / TG wavefronts share a group's inner dimension.
+constexpr float kWeightGuard = 1e-20f;
+
+template <typename T, int TG, bool kMatrix>
+__global__ __launch_bounds__(512) void router_kernel(RouterArgs a) {
+    constexpr int KS = 8 / TG, kRows = 16 * TG;
+    extern __shared__ __attribute__((aligned(16))) unsigned char router_smem[];
+    float *logits = reinterpret_cast<float *>(router_smem);                    // [kRows][experts]
+    float *partial = logits + kRows * a.experts;                               // [KS][kRows][64 + 4] (matrix form)
+    int *have = reinterpret_cast<int *>(partial + (kMatrix ? KS * kRows * 68 : 0)); // [experts]: this workgroup's assignments
+    int *base = have + a.experts;                                              // [experts]
+    int *mine = base + a.experts;                                              // [kRows * top]: expert, place among this workgroup's
+    const int tid = threadIdx.x, lane = tid & 63, r = lane & 15, q = lane >> 4;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int row0 = blockIdx.x * kRows;
+    const int rows = min(kRows, a.rows - row0);
+    for (int e = tid; e < a.experts; e += 512) have[e] = 0;
+    if constexpr (kMatrix) {
+        const int tg = wave / KS, part = wave % KS;
+        const int steps = (a.width + 31) / 32, per = (steps + KS - 1) / KS;
+        const int s_begin = part * per, s_end = min(steps, s_begin + per);
+        const bf16_t *x = static_cast<const bf16_t *>(a.x) + static_cast<int64_t>(row0 + min(16 * tg + r, rows - 1)) * a.x_stride;
+        for (int e0 = 0; e0 < a.experts; e0 += 64) {
+            const int blocks = min(4, (a.experts - e0 + 15) / 16);
+            f32x4_t acc[4];
+            const bf16_t *w[4];
+#pragma unroll
+            for (int b = 0; b < 4; ++b) {
+                acc[b] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+                w[b] = static_cast<const bf16_t *>(a.w) + static_cast<int64_t>(min(e0 + 16 * b + r, a.experts - 1)) * a.width;
+            }
+#pragma unroll 4
+            for (int s = s_begin; s < s_end; ++s) {
+                const int e = s * 32 + 8 * q;
+                const bool in = e < a.width;
+                u32x4_t xf = {0, 0, 0, 0};
+                if (in) xf = *reinterpret_cast<const u32x4_t *>(x + e);
+#pragma unroll
+                for (int b = 0; b < 4; ++b) {
+                    if (b >= blocks) continue;
+                    u32x4_t wf = {0, 0, 0, 0};
+                    if (in) wf = *reinterpret_cast<const u32x4_t *>(w[b] + e);
+                    acc[b] = mfma16(wf, xf, acc[b]);
+                }
+            }
+#pragma unroll
+            for (int b = 0; b < 4; ++b) *reinterpret_cast<f32x4_t *>(partial + (part * kRows + 16 * tg + r) * 68 + 16 * b + 4 * q) = acc[b];
+            __syncthreads();
+            for (int i = tid; i < kRows * 64; i += 512) {
+                const int row = i >> 6, e = i & 63;
+                if (e0 + e >= a.experts) continue;
+                float z = 0.f;
+#pragma unroll
+                for (int p = 0; p < KS; ++p) z += partial[(p * kRows + row) * 68 + e];
+                logits[row * a.experts + e0 + e] = z;
+            }
+            __syncthreads();
+        }
+    } else {
+        for (int i = tid; i < rows * a.experts; i += 512) {
+            const int row = i / a.experts, e = i % a.experts;
+            const T *x = static_cast<const T *>(a.x) + static_cast<int64_t>(row0 + row) * a.x_stride;
+            const T *w = static_cast<const T *>(a.w) + static_cast<int64_t>(e) * a.width;
+            float z = 0.f;
+            for (int k = 0; k < a.width; ++k) z = fmaf(Elem<T>::to_f32(x[k]), Elem<T>::to_f32(w[k]), z);
+            logits[i] = z;
+        }
+        __syncthreads();
+    }
+    // one wavefront per row: softmax over the experts, then the best one `top` times (ties: the lower index)
+    for (int row = wave; row < rows; row += 8) {
+        float *z = logits + row * a.experts;
+        float mx = -INFINITY;
+        for (int e = lane; e < a.experts; e += 64) mx = fmaxf(mx, z[e]);
+        mx = wave_max(mx);
+        float sum = 0.f;
+        for (int e = lane; e < a.experts; e += 64) sum += exp_of<T>(z[e] - mx);
+        const float inv = 1.0f / wave_sum(sum);
+        const int64_t at = static_cast<int64_t>(row0 + row) * a.top;
+        float chosen = 0.f;
+        for (int k = 0; k < a.top; ++k) {
+            float best = -INFINITY;
+            int who = 0x7fffffff;
+            for (int e = lane; e < a.experts; e += 64)
+                if (z[e] > best) { best = z[e]; who = e; }
+#pragma unroll
+            for (int d = 1; d < 64; d <<= 1) {
+                const float ob = __shfl_xor(best, d, 64);
+                const int ow = __shfl_xor(who, d, 64);
+                if (ob > best || (ob == best && ow < who)) { best = ob; who = ow; }
+            }
+            if (who >= a.experts) who = 0;                   // (only where logits are not numbers)
+            const float s = exp_of<T>(best - mx) * inv;
+            chosen += s;
+            if (lane == 0) {
+                a.choice[at + k] = who;
+                a.weight[at + k] = s;                        // scaled below, by the same lane
+                mine[2 * (row * a.top + k)] = who;
+                mine[2 * (row * a.top + k) + 1] = atomicAdd(&have[who], 1);
+                z[who] = -INFINITY;
+            }
+            __builtin_amdgcn_wave_barrier();
+            __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+        }
+        const float f = a.scale / (chosen + kWeightGuard);
+        if (lane == 0)
+            for (int k = 0; k < a.top; ++k) a.weight[at + k] *= f;
+    }
+    __syncthreads();
+    for (int e = tid; e < a.experts; e += 512) base[e] = have[e] > 0 ? atomicAdd(&a.counts[e], have[e]) : 0;
+    __syncthreads();
+    for (int i = tid; i < rows * a.top; i += 512) {
+        const int e = mine[2 * i], place = base[e] + mine[2 * i + 1];
+        if (place < a.list_stride) a.lists[e * a.list_stride + place] = row0 * a.top + i;
+    }
+}
+
+static size_t router_lds(int32_t experts, int32_t top, int tg, bool matrix) {
+    const size_t rows = 16 * static_cast<size_t>(tg);
+    return 4 * (rows * experts + (matrix ? 8 / tg * rows * 68 : 0) + 2 * static_cast<size_t>(experts) + 2 * rows * top);
+}
+
+template <typename T, int TG, bool kMatrix>
+static int launch_router_tg(const RouterArgs &a, hipStream_t s) {
+    const size_t lds = router_lds(a.experts, a.top, TG, kMatrix);
+    if (lds > 64 * 1024 &&
+        hipFuncSetAttribute(reinterpret_cast<const void *>(&router_kernel<T, TG, kMatrix>), hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds)) != hipSuccess)
+        return NVA_ERR_LAUNCH_FAILED;
+    hipLaunchKernelGGL((router_kernel<T, TG, kMatrix>), dim3((a.rows + 16 * TG - 1) / (16 * TG)), dim3(512), lds, s, a);
+    return launch_status();
+}
+
+}  // namespace nva
+
+extern "C" int nva_grouped_linear(const void *x, int64_t x_row_stride, int64_t x_group_stride, const void *weight, void *out,
+                                  int64_t out_row_stride, int64_t out_group_stride, int32_t rows, int32_t groups, int32_t n_out,
+                                  int32_t k_in, int32_t dtype, int32_t out_dtype, void *stream) {
+    using namespace nva;
+    if (rows < 0 || groups < 0 || n_out <= 0 || k_in <= 0) return NVA_ERR_BAD_SHAPE;
+    if (!known_dtype(dtype) || !known_dtype(out_dtype) || (dtype == NVA_DTYPE_F32 && out_dtype != NVA_DTYPE_F32)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
+    if (rows == 0 || groups == 0) return NVA_OK;
+    if (!x || !weight || !out) return NVA_ERR_NULL_POINTER;
+    if (groups > 65535) return NVA_ERR_BAD_SHAPE;
+    if (x_row_stride < k_in || out_row_stride < n_out || (groups > 1 && (x_group_stride < 0 || out_group_stride < n_out))) return NVA_ERR_BAD_STRIDE;
+    LinearArgs a{};
+    a.x = x; a.x_stride = x_row_stride; a.x_group = groups > 1 ? x_group_stride : 0; a.w = weight; a.out = out; a.o_stride = out_row_stride;
+    a.o_group = groups > 1 ? out_group_stride : 0; a.rows = rows; a.groups = groups; a.n_out = n_out; a.k = k_in; a.x_div = 1;
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    if (dtype == NVA_DTYPE_F32) return launch_any_linear<float, float, false>(a, rows, s);
+    if (!linear_matrix_ok(a))
+        return out_dtype == NVA_DTYPE_F32 ? launch_any_linear<bf16_t, float, false>(a, rows, s) : launch_any_linear<bf16_t, bf16_t, false>(a, rows, s);
+    return out_dtype == NVA_DTYPE_F32 ? launch_skinny<false, float>(a, rows, rows, s) : launch_skinny<false, bf16_t>(a, rows, rows, s);
+}
+
+extern "C" int nva_routed_linear(const void *x, int64_t x_row_stride, const void *weight, void *out, const int32_t *lists,
+                                 const int32_t *counts, int64_t list_stride, int32_t rows, int32_t terms, int32_t experts,
+                                 int32_t n_out, int32_t k_in, int32_t x_per_row, int32_t gated, int32_t dtype, void *stream) {
+    using namespace nva;
+    if (rows < 0 || terms <= 0 || experts <= 0 || n_out <= 0 || k_in <= 0 || list_stride < rows || terms > experts) return NVA_ERR_BAD_SHAPE;
+    if (!known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
+    if (rows == 0) return NVA_OK;
+    if (!x || !weight || !out || !lists || !counts) return NVA_ERR_NULL_POINTER;
+    if (experts > 65535 || static_cast<int64_t>(rows) * terms > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
+    if (x_row_stride < k_in) return NVA_ERR_BAD_STRIDE;
+    LinearArgs a{};
+    a.x = x; a.x_stride = x_row_stride; a.w = weight; a.out = out; a.o_stride = n_out; a.lists = lists; a.counts = counts;
+    a.list_stride = list_stride; a.rows = rows * terms; a.groups = experts; a.n_out = n_out; a.k = k_in; a.x_div = x_per_row ? terms : 1;
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    const int32_t hint = static_cast<int32_t>((static_cast<int64_t>(rows) * terms * 3 / 2 + experts - 1) / experts);
+    if (dtype == NVA_DTYPE_F32) return gated ? launch_any_linear<float, float, true>(a, rows, s) : launch_any_linear<float, float, false>(a, rows, s);
+    if (!linear_matrix_ok(a)) return gated ? launch_any_linear<bf16_t, bf16_t, true>(a, rows, s) : launch_any_linear<bf16_t, bf16_t, false>(a, rows, s);
+    return gated ? launch_skinny<true, bf16_t>(a, hint, rows, s) : launch_skinny<false, bf16_t>(a, hint, rows, s);
+}
+
+extern "C" int nva_router(const void *x, int64_t x_row_stride, const void *weight, int32_t *choice, float *choice_weight,
+                          int32_t *lists, int32_t *counts, int64_t list_stride, int32_t rows, int32_t width, int32_t experts,
+                          int32_t top, float scale, int32_t dtype, void *stream) {
+    using namespace nva;
+    if (rows < 0 || width <= 0 || experts <= 0 || top <= 0 || top > experts || list_stride < rows) return NVA_ERR_BAD_SHAPE;
+    if (!known_dtype(dtype) || experts > 1024 || top > 128) return NVA_ERR_UNSUPPORTED_GEOMETRY;
+    if (rows == 0) return NVA_OK;
+    if (!x || !weight || !choice || !choice_weight || !lists || !counts) return NVA_ERR_NULL_POINTER;
+    if (x_row_stride < width) return NVA_ERR_BAD_STRIDE;
+    if (static_cast<int64_t>(rows) * top > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
+    RouterArgs a{};
+    a.x = x; a.x_stride = x_row_stride; a.w = weight; a.choice = choice; a.weight = choice_weight; a.lists = lists; a.counts = counts;
+    a.list_stride = list_stride; a.rows = rows; a.width = width; a.experts = experts; a.top = top; a.scale = scale;
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    const bool many = rows >= 4096 && experts <= 128 && top <= 32;       // more rows per workgroup: fewer additions to the counters
+    if (dtype == NVA_DTYPE_F32) return launch_router_tg<float, 1, false>(a, s);
+    if (width % 8 != 0 || x_row_stride % 8 != 0 || !aligned16(x) || !aligned16(weight)) return launch_router_tg<bf16_t, 1, false>(a, s);
+    return many ? launch_router_tg<bf16_t, 4, true>(a, s) : launch_router_tg<bf16_t, 1, true>(a, s);
+}

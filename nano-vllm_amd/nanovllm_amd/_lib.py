@@ -1,8 +1,8 @@
 """ctypes binding of the C ABI declared in include/nanovllm_amd.h.
 
-Two shared libraries are built in-tree, next to this file, by ``csrc/Makefile``:
-``libnanovllm_amd.so`` (the attention hot path) and ``libnanovllm_mixers.so`` (mixers of layered
-models).  Each is opened when one of its symbols is first used, so a model needs only its own.  There
+Shared libraries are built in-tree, next to this file, by ``csrc/Makefile``: ``libnanovllm_amd.so``
+(the attention hot path), ``libnanovllm_mixers.so`` (chunked attention and retention of layered models)
+and ``libnanovllm_latent.so`` (latent attention, matrix memory, routed experts).  Each is opened when one of its symbols is first used, so a model needs only its own.  There
 is no fallback: an op whose library is missing raises.
 """
 from __future__ import annotations
@@ -13,6 +13,7 @@ import os
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libnanovllm_amd.so")
 MIXERS_LIB_PATH = os.path.join(_HERE, "libnanovllm_mixers.so")
+LATENT_LIB_PATH = os.path.join(_HERE, "libnanovllm_latent.so")
 
 # status codes of enum nva_status
 OK = 0
@@ -65,12 +66,33 @@ SIGNATURES = {
     "nva_retention_workspace_bytes": (_sz, [_i32, _i32, _i32, _i32, _i32, _i32, _i32]),
     "nva_retention": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _sz, _i32, _i32, _i32, _i32, _i32,
                                 _i32, _i32, _i32, _i32, _f32, _f32, _i32, _vp]),
+    "nva_embed_rms_norms": (C.c_int, [_vp, _vp, _f32, _vp, _vp, _f32, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _i32, _f32, _i32, _vp]),
+    "nva_branches_rms_norms": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _i32, _vp, _f32, _vp, _vp, _vp, _f32, _vp, _vp, _vp, _vp, _i32,
+                                         _i32, _i32, _i32, _f32, _i32, _vp]),
+    "nva_grouped_linear": (C.c_int, [_vp, _i64, _i64, _vp, _vp, _i64, _i64, _i32, _i32, _i32, _i32, _i32, _i32, _vp]),
+    "nva_router": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _f32, _i32, _vp]),
+    "nva_routed_linear": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _vp]),
+    "nva_latent_prepare": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _vp, _vp, _vp, _i32, _i32, _i32, _i32, _i32,
+                                     _i32, _f32, _i32, _vp]),
+    "nva_latent_attn_workspace_bytes": (_sz, [_i32] * 8),
+    "nva_latent_attn": (C.c_int, [_vp, _vp, _i64, _i64, _vp, _i64, _vp, _vp, _vp, _i64, _i32, _vp, _vp, _vp, _vp, _vp, _sz,
+                                  _i32, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _f32, _i32, _vp]),
+    "nva_latent_gather": (C.c_int, [_vp, _vp, _i64, _i32, _vp, _vp, _vp, _i32, _i32, _i32, _i32, _i32, _i32, _vp]),
+    "nva_latent_prefill_supported": (C.c_int, [_i32, _i32, _i32, _i32]),
+    "nva_latent_prefill": (C.c_int, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _i32,
+                                     _i32, _i32, _i32, _i32, _i32, _f32, _i32, _vp]),
+    "nva_mlstm_workspace_bytes": (_sz, [_i32] * 6),
+    "nva_mlstm": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _sz, _i32, _i32, _i32, _i32, _i32,
+                            _i32, _i32, _f32, _f32, _f32, _i32, _vp]),
     "nva_probe_stream_read": (C.c_int, [_vp, _i64, _vp, _vp]),
 }
 
-# symbols of libnanovllm_mixers.so; the common ones are in both libraries, every other one in libnanovllm_amd.so
+# symbols of the libraries of layered models; the common ones are in every library, all others in libnanovllm_amd.so
 MIXER_SYMBOLS = {"nva_embed_norm", "nva_post_add_norm", "nva_clamped_gate", "nva_conv_rope_store", "nva_chunk_attn",
                  "nva_chunk_attn_workspace_bytes", "nva_retention", "nva_retention_workspace_bytes"}
+LATENT_SYMBOLS = {"nva_embed_rms_norms", "nva_branches_rms_norms", "nva_grouped_linear", "nva_router", "nva_routed_linear",
+                  "nva_latent_prepare", "nva_latent_attn", "nva_latent_attn_workspace_bytes", "nva_latent_gather",
+                  "nva_latent_prefill", "nva_latent_prefill_supported", "nva_mlstm", "nva_mlstm_workspace_bytes"}
 COMMON_SYMBOLS = {"nva_version", "nva_status_string", "nva_device_count", "nva_stage_decode_inputs"}
 
 
@@ -87,9 +109,9 @@ class _Symbols:
     def __getattr__(self, name: str):
         if name not in SIGNATURES:
             raise AttributeError(name)
-        paths = [MIXERS_LIB_PATH] if name in MIXER_SYMBOLS else [LIB_PATH]
+        paths = [MIXERS_LIB_PATH] if name in MIXER_SYMBOLS else [LATENT_LIB_PATH] if name in LATENT_SYMBOLS else [LIB_PATH]
         if name in COMMON_SYMBOLS:
-            paths.append(MIXERS_LIB_PATH)
+            paths += [MIXERS_LIB_PATH, LATENT_LIB_PATH]
         path = next((p for p in paths if os.path.exists(p)), None)
         if path is None:
             raise _missing(paths[0])
@@ -126,6 +148,21 @@ def load_mixers():
     if not os.path.exists(MIXERS_LIB_PATH):
         raise _missing(MIXERS_LIB_PATH)
     return _symbols
+
+
+def load_latent():
+    """The entry points of the library of latent attention, matrix memory and experts, and the common ones."""
+    if not os.path.exists(LATENT_LIB_PATH):
+        raise _missing(LATENT_LIB_PATH)
+    return _symbols
+
+
+# kernel sets by name: the make target that builds one, its library and its loader
+LIBRARIES = {"path": (LIB_PATH, load), "mixers": (MIXERS_LIB_PATH, load_mixers), "latent": (LATENT_LIB_PATH, load_latent)}
+
+
+def load_set(name: str):
+    return LIBRARIES[name][1]()
 
 
 def status_string(code: int) -> str:

@@ -49,6 +49,8 @@ class RowGroup:
     cu: Optional[torch.Tensor] = None            # [num_seqs + 1] row bounds, relative to ``first``
     token_seq: Optional[torch.Tensor] = None     # [count] sequence of every row
     max_q: int = 1                               # longest portion
+    spans: Optional[list] = None                 # portions: (start, count) of every sequence, on the host
+    shared: dict = field(default_factory=dict)   # what layers derive from the group once for all of them
 
 
 @dataclass

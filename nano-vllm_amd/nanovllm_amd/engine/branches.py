@@ -1,0 +1,62 @@
+"""The residual step of layers whose mixer and feed-forward read the same point of the stream: both branches'
+results are added at once and the next layer's two norms are taken in the same pass over the row."""
+from __future__ import annotations
+
+from typing import Optional, Tuple
+
+import torch
+
+from .. import _lib
+from .mixers import _DTYPE, _need_cuda, _ptr, _stream
+
+
+def _outputs(rows: int, table: torch.Tensor, second: Optional[torch.Tensor]):
+    width = table.shape[-1]
+    out1 = torch.empty((rows, width), dtype=table.dtype, device=table.device)
+    return out1, None if second is None else torch.empty_like(out1)
+
+
+def embed_rms_norms(ids: torch.Tensor, table: torch.Tensor, scale: float, weights: Tuple[torch.Tensor, Optional[torch.Tensor]],
+                    eps: float, weight_offset: float = 0.0, clear: Optional[torch.Tensor] = None):
+    """``residual = table[ids] * scale`` (fp32) and its RMS norms with one or two weights (stored as the
+    deviation from ``weight_offset``); ``clear``: int32 counters to zero.  Returns (residual, out1, out2)."""
+    vocab, width = table.shape
+    assert ids.dtype == torch.int64 and ids.is_contiguous() and table.is_contiguous()
+    _need_cuda(ids, table)
+    n = ids.numel()
+    residual = torch.empty((n, width), dtype=torch.float32, device=table.device)
+    out1, out2 = _outputs(n, table, weights[1])
+    rc = _lib.load_latent().nva_embed_rms_norms(
+        ids.data_ptr(), table.data_ptr(), float(scale), weights[0].data_ptr(), _ptr(weights[1]), float(weight_offset),
+        residual.data_ptr(), out1.data_ptr(), _ptr(out2), _ptr(clear), 0 if clear is None else clear.numel(), n, width, vocab,
+        float(eps), _DTYPE[table.dtype], _stream())
+    _lib.check(rc, "nva_embed_rms_norms")
+    return residual, out1, out2
+
+
+def branches_rms_norms(residual: torch.Tensor, mult: float, y1: Optional[torch.Tensor], gain1: Optional[torch.Tensor],
+                       y2: Optional[torch.Tensor], term_weight: Optional[torch.Tensor], gain2: Optional[torch.Tensor],
+                       weights: Tuple[torch.Tensor, Optional[torch.Tensor]], eps: float, weight_offset: float = 0.0,
+                       rows: Optional[torch.Tensor] = None, clear: Optional[torch.Tensor] = None):
+    """``residual += mult * (gain1 * y1 + gain2 * sum_k term_weight[:, k] * y2[:, k])`` in place (``y2 [n * terms,
+    width]``), then the norms.  With ``rows`` (int32) only those rows are computed and the residual stays as it is."""
+    n, width = residual.shape
+    assert residual.dtype == torch.float32 and residual.is_contiguous()
+    _need_cuda(residual, weights[0])
+    terms = 0
+    if y1 is not None:
+        assert y1.shape == residual.shape and y1.stride(1) == 1 and y1.dtype == weights[0].dtype
+    if y2 is not None:
+        terms = y2.shape[0] // max(n, 1)
+        assert y2.shape == (n * terms, width) and y2.is_contiguous() and y2.dtype == weights[0].dtype
+        assert term_weight is None or (term_weight.shape == (n, terms) and term_weight.dtype == torch.float32 and term_weight.is_contiguous())
+    count = n if rows is None else rows.numel()
+    if rows is not None:
+        assert rows.dtype == torch.int32 and rows.is_contiguous()
+    out1, out2 = _outputs(count, weights[0], weights[1])
+    rc = _lib.load_latent().nva_branches_rms_norms(
+        _ptr(y1), 0 if y1 is None else y1.stride(0), _ptr(gain1), _ptr(y2), _ptr(term_weight), terms, _ptr(gain2), float(mult),
+        residual.data_ptr(), weights[0].data_ptr(), _ptr(weights[1]), float(weight_offset), out1.data_ptr(), _ptr(out2), _ptr(rows),
+        _ptr(clear), 0 if clear is None else clear.numel(), count, n, width, float(eps), _DTYPE[weights[0].dtype], _stream())
+    _lib.check(rc, "nva_branches_rms_norms")
+    return out1, out2

@@ -14,7 +14,7 @@ from torch import nn
 
 from ..context import get_context
 from . import mixers
-from .loader import TensorFolder
+from .layered import LayeredModel
 from .mixers import AttentionSpec, MlpSpec, RetentionSpec, RopeTables, Rotary
 
 MixerSpec = Union[AttentionSpec, RetentionSpec]
@@ -145,59 +145,24 @@ class _Layer:
         self.mlp = mixers.ClampedGateMLP(spec.mlp, weights.mlp) if spec.mlp is not None else None
 
 
-class Kaparax(nn.Module):
+class Kaparax(LayeredModel):
 
     def __init__(self, cfg: KaparaxConfig, max_position: int, device, seed: int = 0):
-        super().__init__()
-        # 32-bit accumulation in the library's matrix products, and full fp32 ones
-        torch.backends.cuda.matmul.allow_bf16_reduced_precision_reduction = False
-        torch.backends.cuda.matmul.allow_tf32 = False
-        self.cfg = cfg
-        self.embed = nn.Parameter(torch.empty(cfg.vocab_size, cfg.hidden_size))
-        self.head = nn.Parameter(torch.empty(cfg.vocab_size, cfg.hidden_size))
+        super().__init__(cfg)
         self.final = _Norm(cfg.hidden_size)
         self.layer_weights = nn.ModuleDict({str(i): LayerWeights(s, cfg.hidden_size)
                                             for i, s in enumerate(cfg.layers) if s.weights_of == i})
         ropes = RopeTables(max_position, device)
         self.layers = [_Layer(s, self.layer_weights[str(s.weights_of)], ropes, cfg.norm_eps) for s in cfg.layers]
-        gen = torch.Generator(device=device).manual_seed(seed)
-        with torch.no_grad():
-            for p in self.parameters():
-                if p.dim() == 2:
-                    p.normal_(0.0, 0.02 if p.shape[0] > 8 else 0.5, generator=gen)
+        self.random_weights(device, seed)
 
-    @torch.no_grad()
-    def load_weights(self, folder: str) -> None:
-        tensors = TensorFolder(folder)
-        take, width = tensors.take, self.cfg.hidden_size
-        self.embed.copy_(take("embed", self.embed.shape))
-        self.head.copy_(take("head", self.head.shape))
+    def load_tensors(self, take) -> None:
+        width = self.cfg.hidden_size
         self.final.load(width, take, "final.norm")
         for i, weights in self.layer_weights.items():
             weights.load(self.cfg.layers[int(i)], width, take, f"l{i}.")
-        if tensors.unused():
-            raise ValueError(f"tensors without a place in the model: {', '.join(tensors.unused()[:5])}")
 
-    # ---- cache and state ---------------------------------------------------------------------------
-    def kv_bytes_per_token(self) -> int:
-        return self.embed.element_size() * sum(l.mixer.kv_elements_per_token() for l in self.layers)
-
-    def state_bytes_per_slot(self) -> int:
-        return sum(l.mixer.state_bytes_per_slot(self.embed.element_size()) for l in self.layers)
-
-    def bind_cache(self, num_blocks: int, block: int, slots: int) -> None:
-        for l in self.layers:
-            l.mixer.bind(num_blocks, block, slots, self.embed.dtype, self.embed.device)
-
-    def unbind_cache(self) -> None:
-        for l in self.layers:
-            l.mixer.unbind()
-
-    # ---- forward -------------------------------------------------------------------------------------
     def forward_layers(self, input_ids, positions, hidden, residual, first: int, last: int):
-        """Layers ``[first, last)``: ``hidden`` is the normed input of the next sublayer, ``residual`` the
-        fp32 stream, updated in place.  After the last layer ``hidden`` is the final norm -- of the rows in
-        the Context's ``logit_rows`` only, when they are given.  (Positions follow from the row groups.)"""
         eps, layers = self.cfg.norm_eps, self.layers
         if first == 0:
             residual, hidden = mixers.embed_norm(input_ids, self.embed, self.cfg.embed_scale, layers[0].weights.norm1.pair, eps)
@@ -213,12 +178,6 @@ class Kaparax(nn.Module):
                 y, post = layer.mlp(hidden), w.norm2b.pair
             hidden = mixers.post_add_norm(y, residual, post, nxt, eps, rows)
         return hidden, residual
-
-    def finish(self, hidden, residual) -> torch.Tensor:
-        return hidden
-
-    def forward(self, input_ids, positions) -> torch.Tensor:
-        return self.forward_layers(input_ids, positions, None, None, 0, len(self.layers))[0]
 
     def compute_logits(self, hidden: torch.Tensor) -> torch.Tensor:
         return F.linear(hidden, self.head)

@@ -169,7 +169,8 @@ def retention(qkvg: torch.Tensor, state: torch.Tensor, group: RowGroup, rope: Op
 
 @dataclass(frozen=True)
 class Rotary:
-    """Rotation of the first ``dims`` elements of a head, pairs (i, i + dims / 2), by position * base^(-2i/dims)."""
+    """Rotation of the first ``dims`` elements of a head by position * base^(-2i/dims); which elements make pair i
+    (i and i + dims / 2, or neighbours) is the mixer's affair."""
     base: float
     dims: int
 

@@ -251,7 +251,7 @@ class ModelRunner:
 
     def _kernels(self):
         """The library this model's steps run on."""
-        return _lib.load_mixers() if self.portions else _lib.load()
+        return _lib.load_set(registry.kernels_for(self.cfg))
 
     # ---- host -> device inputs -----------------------------------------------------------------
     def _to_device(self, array: np.ndarray, dtype: torch.dtype) -> torch.Tensor:
@@ -333,7 +333,8 @@ class ModelRunner:
                 continue
             single, n = name == "singles", h[name]["token_seq"].size
             groups.append(RowGroup(first, n, len(h[name]["seq_lens"]), lens, slots[first: first + n], tables, state,
-                                   None if single else cu, None if single else token_seq, h[name]["max_q"]))
+                                   None if single else cu, None if single else token_seq, h[name]["max_q"],
+                                   [(s.start, s.count) for s in spans if (s.count == 1) == single]))
             first += n
         set_row_groups(groups, torch.empty(0, dtype=torch.int32, device=self.device) if rows is None else rows)
         return ids, pos

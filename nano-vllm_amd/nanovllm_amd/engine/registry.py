@@ -21,6 +21,7 @@ _DEFAULT = "Qwen3ForCausalLM"
 class Family:
     config: str                  # "module:class", relative to this package
     model: str
+    kernels: str = "path"        # the kernel set its steps run on (``_lib.LIBRARIES``)
 
     @staticmethod
     def _resolve(where: str):
@@ -39,12 +40,13 @@ class Family:
 _families: Dict[str, Family] = {}
 
 
-def register(architecture: str, config: str, model: str) -> None:
-    _families[architecture] = Family(config, model)
+def register(architecture: str, config: str, model: str, kernels: str = "path") -> None:
+    _families[architecture] = Family(config, model, kernels)
 
 
 register("Qwen3ForCausalLM", ".config:ModelConfig", ".model:Qwen3ForCausalLM")
-register("Kaparax", ".kaparax:KaparaxConfig", ".kaparax:Kaparax")
+register("Kaparax", ".kaparax:KaparaxConfig", ".kaparax:Kaparax", "mixers")
+register("Pidutar", ".pidutar:PidutarConfig", ".pidutar:Pidutar", "latent")
 
 
 def family_of_raw(raw: dict) -> Family:
@@ -54,18 +56,35 @@ def family_of_raw(raw: dict) -> Family:
     return _families[name]
 
 
-def load_config(model_dir: str):
+def _read(model_dir: str) -> dict:
     with open(os.path.join(model_dir, "config.json")) as f:
-        raw = json.load(f)
+        return json.load(f)
+
+
+def load_config(model_dir: str):
+    raw = _read(model_dir)
     return family_of_raw(raw).config_class.from_raw(raw)
+
+
+def kernels_of(model_dir: str) -> str:
+    """The kernel set a model folder needs, without importing the family."""
+    return family_of_raw(_read(model_dir)).kernels
 
 
 def is_config(obj) -> bool:
     return any(isinstance(obj, f.config_class) for f in _families.values())
 
 
-def model_class(cfg):
+def _family_of(cfg) -> Family:
     for f in _families.values():
         if isinstance(cfg, f.config_class):
-            return f.model_class
+            return f
     raise ValueError(f"no model class for {type(cfg).__name__}")
+
+
+def model_class(cfg):
+    return _family_of(cfg).model_class
+
+
+def kernels_for(cfg) -> str:
+    return _family_of(cfg).kernels

@@ -63,7 +63,7 @@ class TraceReplayer:
         return out
 
 
-def main(argv=None) -> int:
+def main(argv=None, before_loading=None) -> int:
     ap = argparse.ArgumentParser(prog="trace_run", description="Feeds token ids through a model step by step and writes logits. "
                                  "Reads one JSON object a line: {\"step\", \"entries\": [{\"id\", \"tokens\", \"want\"}], \"end\": [ids]}.")
     ap.add_argument("--model", required=True, help="folder with config.json and *.safetensors")
@@ -74,6 +74,8 @@ def main(argv=None) -> int:
     if args.dtype not in registry.load_config(args.model).dtypes:
         print(f"this model does not run in {args.dtype}", file=sys.stderr)
         return 3
+    if before_loading is not None:
+        before_loading(args.model)
     replayer = TraceReplayer(args.model, args.dtype, args.max_tokens)
     for line in sys.stdin:
         if not line.strip():
