@@ -290,3 +290,81 @@ def test_retention_validation_and_workspace():
                    (dict(rot=127), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(dim=1024, xs=1 << 20), _lib.ERR_UNSUPPORTED_GEOMETRY),
                    (dict(cu=None), _lib.ERR_BAD_SHAPE), (dict(n=0, x=None), _lib.OK)):
         assert _with(ok, lib.nva_retention, **kw) == rc, kw
+
+
+def test_branches_and_experts_validation():
+    lib = _lib.load()
+    ok = dict(ids=A, table=A, scale=1.0, w1=A, w2=A, off=1.0, res=A, o1=A, o2=A, clear=None, nclear=0, rows=4, width=64, vocab=10, eps=1e-5, dtype=0, stream=None)
+    for kw, rc in ((dict(ids=None), _lib.ERR_NULL_POINTER), (dict(o2=None), _lib.ERR_NULL_POINTER), (dict(width=0), _lib.ERR_BAD_SHAPE),
+                   (dict(nclear=-1), _lib.ERR_BAD_SHAPE), (dict(dtype=2), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, ids=None), _lib.OK)):
+        assert _with(ok, lib.nva_embed_rms_norms, **kw) == rc, kw
+    ok = dict(y1=A, ys=64, g1=A, y2=A, tw=A, terms=2, g2=A, mult=1.0, res=A, w1=A, w2=A, off=1.0, o1=A, o2=A, rows_of=None, clear=None, nclear=0,
+              rows=4, src=4, width=64, eps=1e-5, dtype=1, stream=None)
+    for kw, rc in ((dict(res=None), _lib.ERR_NULL_POINTER), (dict(w1=None), _lib.ERR_NULL_POINTER), (dict(o2=None), _lib.ERR_NULL_POINTER),
+                   (dict(ys=63), _lib.ERR_BAD_STRIDE), (dict(terms=0), _lib.ERR_BAD_SHAPE), (dict(rows=3), _lib.ERR_BAD_SHAPE),
+                   (dict(rows_of=A, src=0), _lib.ERR_BAD_SHAPE), (dict(rows=0, src=0), _lib.OK), (dict(dtype=-1), _lib.ERR_UNSUPPORTED_GEOMETRY)):
+        assert _with(ok, lib.nva_branches_rms_norms, **kw) == rc, kw
+    ok = dict(x=A, xs=256, xg=64, w=A, out=A, os=256, og=64, rows=4, groups=4, n_out=64, k=64, dtype=0, odt=0, stream=None)
+    for kw, rc in ((dict(x=None), _lib.ERR_NULL_POINTER), (dict(w=None), _lib.ERR_NULL_POINTER), (dict(xs=63), _lib.ERR_BAD_STRIDE),
+                   (dict(og=63), _lib.ERR_BAD_STRIDE), (dict(k=0), _lib.ERR_BAD_SHAPE), (dict(groups=70000), _lib.ERR_BAD_SHAPE),
+                   (dict(dtype=1, odt=0), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, x=None), _lib.OK), (dict(groups=0, x=None), _lib.OK)):
+        assert _with(ok, lib.nva_grouped_linear, **kw) == rc, kw
+    ok = dict(x=A, xs=64, w=A, choice=A, cw=A, lists=A, counts=A, ls=16, rows=16, width=64, experts=8, top=2, scale=1.0, dtype=0, stream=None)
+    for kw, rc in ((dict(counts=None), _lib.ERR_NULL_POINTER), (dict(cw=None), _lib.ERR_NULL_POINTER), (dict(top=9), _lib.ERR_BAD_SHAPE),
+                   (dict(ls=15), _lib.ERR_BAD_SHAPE), (dict(xs=63), _lib.ERR_BAD_STRIDE), (dict(experts=1025), _lib.ERR_UNSUPPORTED_GEOMETRY),
+                   (dict(experts=512, top=129), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, x=None), _lib.OK)):
+        assert _with(ok, lib.nva_router, **kw) == rc, kw
+    ok = dict(x=A, xs=64, w=A, out=A, lists=A, counts=A, ls=16, rows=16, terms=2, experts=8, n_out=32, k=64, per_row=1, gated=1, dtype=0, stream=None)
+    for kw, rc in ((dict(lists=None), _lib.ERR_NULL_POINTER), (dict(out=None), _lib.ERR_NULL_POINTER), (dict(terms=9), _lib.ERR_BAD_SHAPE),
+                   (dict(ls=15), _lib.ERR_BAD_SHAPE), (dict(xs=63), _lib.ERR_BAD_STRIDE), (dict(dtype=5), _lib.ERR_UNSUPPORTED_GEOMETRY),
+                   (dict(rows=0, x=None), _lib.OK)):
+        assert _with(ok, lib.nva_routed_linear, **kw) == rc, kw
+
+
+def test_latent_attention_validation_and_workspace():
+    lib = _lib.load()
+    ok = dict(x=A, xs=400, wq=A, wkv=A, rope=A, q=A, cache=A, sm=A, slots=512, cu=A, lens=A, tseq=A, n=9, seqs=2, q_rank=96, rank=128, rot=32, max_pos=64,
+              eps=1e-5, dtype=0, stream=None)
+    for kw, rc in ((dict(x=None), _lib.ERR_NULL_POINTER), (dict(wkv=None), _lib.ERR_NULL_POINTER), (dict(rope=None), _lib.ERR_NULL_POINTER),
+                   (dict(tseq=None), _lib.ERR_NULL_POINTER), (dict(cu=None), _lib.ERR_BAD_SHAPE), (dict(xs=255), _lib.ERR_BAD_STRIDE),
+                   (dict(rot=31), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rank=0), _lib.ERR_BAD_SHAPE), (dict(n=0, x=None), _lib.OK)):
+        assert _with(ok, lib.nva_latent_prepare, **kw) == rc, kw
+    ws = lib.nva_latent_attn_workspace_bytes
+    assert ws(2000, 16, 512, 64, 16, 256, 4096, 0) == 0               # enough rows for the machine: one range of keys each
+    assert ws(1, 16, 512, 64, 16, 256, 1 << 20, 0) == 33 * 16 * 516 * 4   # 4096 keys and up to 31 before a multiple of 32, ranges of 128
+    assert ws(1, 16, 512, 64, 16, 256, 90, 0) == 0 and ws(1, 16, 512, 64, 16, 256, 4096, 1) == 0 and ws(1, 16, 516, 64, 16, 256, 4096, 0) == 0
+    ok = dict(ql=A, qr=A, qrs=3072, qrh=192, gate=A, gs=16, rope=A, cache=A, bt=A, bts=16, mb=16, cu=None, lens=A, tseq=None, out=A, ws=A, wsb=1 << 30,
+              n=8, seqs=8, heads=16, rank=512, rot=64, bs=256, nb=64, window=4096, max_pos=4096, scale=0.1, dtype=0, stream=None)
+    for kw, rc in ((dict(ql=None), _lib.ERR_NULL_POINTER), (dict(qr=None), _lib.ERR_NULL_POINTER), (dict(ws=None), _lib.ERR_NULL_POINTER),
+                   (dict(ws=A + 8), _lib.ERR_MISALIGNED), (dict(wsb=100), _lib.ERR_WORKSPACE_TOO_SMALL), (dict(window=0), _lib.ERR_BAD_SHAPE),
+                   (dict(bs=64), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rank=1000), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(gs=15), _lib.ERR_BAD_STRIDE),
+                   (dict(qrs=2000), _lib.ERR_BAD_STRIDE), (dict(bts=15), _lib.ERR_BAD_STRIDE), (dict(cu=A), _lib.ERR_NULL_POINTER),
+                   (dict(seqs=7), _lib.ERR_BAD_SHAPE), (dict(n=0, ql=None), _lib.OK)):
+        assert _with(ok, lib.nva_latent_attn, **kw) == rc, kw
+    ok = dict(cache=A, bt=A, bts=16, mb=16, kcu=A, lens=A, out=A, keys=90, seqs=2, width=576, bs=256, nb=64, dtype=0, stream=None)
+    for kw, rc in ((dict(kcu=None), _lib.ERR_NULL_POINTER), (dict(bts=15), _lib.ERR_BAD_STRIDE), (dict(nb=0), _lib.ERR_BAD_SHAPE),
+                   (dict(bs=100), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(keys=0, cache=None), _lib.OK)):
+        assert _with(ok, lib.nva_latent_gather, **kw) == rc, kw
+    fits = lib.nva_latent_prefill_supported
+    assert fits(128, 64, 128, 0) == 1 and fits(128, 64, 128, 1) == 0 and fits(100, 64, 128, 0) == 0 and fits(264, 64, 128, 0) == 0 and fits(8, 136, 8, 0) == 0
+    ok = dict(q=A, qs=3072, kv=A, kvs=4096, kr=A, krs=576, gate=A, gs=16, rope=A, cu=A, lens=A, kcu=A, out=A, n=9, seqs=2, mq=7, heads=16, dim=128, rot=64,
+              vdim=128, window=100, max_pos=4096, scale=0.1, dtype=0, stream=None)
+    for kw, rc in ((dict(q=None), _lib.ERR_NULL_POINTER), (dict(kr=None), _lib.ERR_NULL_POINTER), (dict(kcu=None), _lib.ERR_NULL_POINTER),
+                   (dict(kvs=4088), _lib.ERR_BAD_STRIDE), (dict(qs=3076), _lib.ERR_BAD_STRIDE), (dict(kv=A + 2), _lib.ERR_MISALIGNED),
+                   (dict(dtype=1), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(window=0), _lib.ERR_BAD_SHAPE), (dict(n=0, q=None), _lib.OK)):
+        assert _with(ok, lib.nva_latent_prefill, **kw) == rc, kw
+
+
+def test_matrix_memory_validation_and_workspace():
+    lib = _lib.load()
+    ws = lib.nva_mlstm_workspace_bytes
+    assert ws(1, 200, 8, 128, 128, 0) == 0 and ws(600, 4096, 8, 128, 128, 0) == 0                 # short, or enough sequences
+    assert ws(1, 4096, 8, 128, 128, 0) == 16 * 8 * (128 * 129 + 4) * 4                            # segments of 256 tokens
+    assert ws(1, 4096, 8, 128, 128, 1) == 0 and ws(1, 4096, 8, 100, 128, 0) == 0                  # sizes that walk token by token
+    ok = dict(x=A, xs=4096, z=A, bias=A, nw=A, state=A, mass=A, top=A, slots=A, cu=A, lens=A, out=A, ws=A, wsb=1 << 30, n=4096, seqs=1, mq=4096, heads=8,
+              dim=128, vdim=128, state_slots=4, qs=0.1, cap=5.0, eps=1e-6, dtype=0, stream=None)
+    for kw, rc in ((dict(x=None), _lib.ERR_NULL_POINTER), (dict(z=None), _lib.ERR_NULL_POINTER), (dict(mass=None), _lib.ERR_NULL_POINTER),
+                   (dict(ws=None), _lib.ERR_NULL_POINTER), (dict(ws=A + 4), _lib.ERR_MISALIGNED), (dict(wsb=1000), _lib.ERR_WORKSPACE_TOO_SMALL),
+                   (dict(xs=4095), _lib.ERR_BAD_STRIDE), (dict(cap=0.0), _lib.ERR_BAD_SHAPE), (dict(dim=1024, xs=1 << 20), _lib.ERR_UNSUPPORTED_GEOMETRY),
+                   (dict(cu=None), _lib.ERR_BAD_SHAPE), (dict(n=0, x=None), _lib.OK)):
+        assert _with(ok, lib.nva_mlstm, **kw) == rc, kw
