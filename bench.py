@@ -15,6 +15,7 @@ already resident in HBM.  Workloads (shapes are the five benchmark configuration
     glue      residual add + RMSNorm (--glue add-rms-norm) or SiLU(gate) * up (--glue silu-mul), 16,384 rows (--tokens N)
     decode-e2e-shape / decode-longctx-shape / copy   profiling helpers: the decode attention of configs 4 / 5
               alone (one layer); a plain copy of known size
+    pidutar   the Pidutar family beside Kaparax at equal size: engine prefill / decode tok/s and every kernel beside its like
     kaparax   the Kaparax family beside Qwen3 at equal size: engine prefill / decode tok/s and every kernel beside its like
     read-probe    calibration: a bare streaming read at the sizes of the bandwidth-bound workloads
 The line carries `roofline` (algorithmic bytes or flops of the dominant kernel per launch,
@@ -1011,6 +1012,241 @@ def kaparax_kernels(dev, steps=60, only=None):
     return rows
 
 
+def _pidutar_config(layers, width, heads, q_rank, kv_rank, mem_heads, mem_dim, experts, top, ff, window, vocab):
+    """Latent attention (128 + 64 key elements, 128 value elements a head) and matrix memory in turn, each beside routed
+    experts; every second attention layer reads the cache of the one before it."""
+    from nanovllm_amd.engine.pidutar import PidutarConfig
+    mlp = dict(kind="moe", expert=dict(ff=ff), router=dict(experts=experts, top=top, scale=1.0))
+    out = []
+    for i in range(layers):
+        if i % 2:
+            out.append(dict(type="mlstm", mixer=dict(heads=mem_heads, dim=mem_dim, vdim=mem_dim, gate_cap=15.0), mlp=mlp))
+            continue
+        m = dict(heads=heads, dim=128, rot_dim=64, vdim=128, q_rank=q_rank, kv_rank=kv_rank, mask=dict(size=window), scale=192 ** -0.5,
+                 rot=dict(base=1e4, dims=64))
+        if i % 4 == 2:
+            m["kv_from"] = i - 2
+        out.append(dict(type="latent_attention", mixer=m, mlp=mlp))
+    return PidutarConfig.from_raw(dict(architecture="Pidutar", vocab=vocab, width=width, embedding=dict(scale=1.0), residual_mult=0.5,
+                                       logit_scale=1.0, norm=dict(eps=1e-6), layers=out))
+
+
+def _portions(dev, lens, seed=0):
+    """Whole prompts of the given lengths in randomly scattered pages, as one group of portions."""
+    import torch
+    from nanovllm_amd.context import RowGroup
+    i32 = lambda x: torch.as_tensor(x, dtype=torch.int32).to(dev)
+    need = [-(-l // 256) for l in lens]
+    ids = torch.randperm(sum(need), generator=torch.Generator().manual_seed(seed)).tolist()
+    tabs, slots, at = [], [], 0
+    for k, l in zip(need, lens):
+        mine = ids[at: at + k]
+        tabs.append(mine + [-1] * (max(need) - k))
+        slots += [mine[p // 256] * 256 + p % 256 for p in range(l)]
+        at += k
+    cu = torch.tensor([0] + lens).cumsum(0)
+    return RowGroup(0, sum(lens), len(lens), i32(lens), i32(slots), i32(tabs), i32(list(range(len(lens)))), i32(cu),
+                    torch.repeat_interleave(torch.arange(len(lens)), torch.tensor(lens)).to(torch.int32).to(dev), max(lens),
+                    [(0, l) for l in lens]), sum(need)
+
+
+def pidutar_kernels(dev, steps=60, only=None):
+    """Every kernel of the Pidutar layers at sizes of a real layer (width 1024, 16 heads of 128 + 64 / 128 over latents of 512,
+    memory of 8 heads of 128 x 128, 32 experts of 768 of which a row uses 4), each beside the like kernel of the closest
+    model at equal size -- Kaparax's attention, retention, norms and gate, the dense products of its feed-forward -- in one process."""
+    import torch
+    import torch.nn.functional as F
+    from nanovllm_amd import synthetic
+    from nanovllm_amd.context import RowGroup
+    from nanovllm_amd.engine import branches, experts, latent, mixers
+    from nanovllm_amd.engine.mlstm import mlstm
+    bf = torch.bfloat16
+    rnd = lambda *shape: torch.randn(*shape, device=dev).to(bf)
+    i32 = lambda x: torch.as_tensor(x, dtype=torch.int32).to(dev)
+    rows = []
+    want = lambda name: only is None or only in name
+    heads, dim, rot, vdim, rank, q_rank, width = 16, 128, 64, 128, 512, 512, 1024
+    n_exp, top, ff, mh = 32, 4, 768, 8
+    ropes = mixers.RopeTables(16384 + 256, dev)
+    rope, rope128 = ropes.get(mixers.Rotary(1e4, rot)), ropes.get(mixers.Rotary(1e4, 128))
+    graph_us = lambda fns, n=200: _graph_time_ms(fns, n, 10)[0] / n * 1e3
+    event_us = lambda fns, n=steps: _steady_time_ms(fns, n, max(3, n // 10))[0] / n * 1e3
+    scale = (dim + rot) ** -0.5
+
+    def lengths(count, lo, hi, seed=0):
+        return torch.randint(lo, hi + 1, (count,), generator=torch.Generator().manual_seed(seed)).tolist()
+
+    # ---- attention over portions: gather, keys and values multiplied out (library product), attention
+    for what, lens, window in (("2x16384, window 16384", [16384, 16384], 16384), ("2x16384, window 2048", [16384, 16384], 2048),
+                               ("16 x U[100,1024], window 8192", lengths(16, 100, 1024), 8192)):
+        if not want("attention prefill"):
+            continue
+        group, blocks = _portions(dev, lens)
+        n = sum(lens)
+        q, kv, keys, gate = rnd(n, heads * (dim + rot)), rnd(n, heads * (dim + vdim)), rnd(n, rank + rot), rnd(n, heads)
+        out = torch.empty(n, heads * vdim, dtype=bf, device=dev)
+        mine = event_us([lambda: latent.latent_prefill(q, kv, keys[:, rank:], gate, rope, group, group.cu, out, dim, vdim, window, scale)])
+        seen = sum(sum(min(p + 1, window) for p in range(l)) for l in lens)
+        # the like kernel: as many heads of 128, one key and value head each, the same visible pairs in whole chunks
+        parts = window if max(lens) > window else max(lens)
+        q1, kc, vc = rnd(n, heads * 128), rnd(blocks, 256, heads, 128), rnd(blocks, 256, heads, 128)
+        theirs = event_us([lambda: mixers.chunk_attention(q1, kc, vc, group, out, heads, parts, 128 ** -0.5, 30.0)])
+        chunked = sum((l // parts) * (parts * (parts + 1) // 2) + (l % parts) * (l % parts + 1) // 2 for l in lens)
+        rows.append(_kernel_row("latent attention prefill, " + what, mine, 2 * heads * seen * (dim + rot + vdim), "mfma",
+                                ("chunk_prefill_kernel", theirs, 4 * 128 * heads * chunked, "mfma")))
+        cache = rnd(blocks, 256, rank + rot)
+        # (gather: read and written once; like: a plain copy of the rows)
+        mine = graph_us([lambda: latent.latent_gather(cache, group, group.cu, n)], 50)
+        dst = torch.empty_like(keys)
+        rows.append(_kernel_row("latent gather, " + what, mine, 4 * n * (rank + rot), "hbm", ("copy by torch", graph_us([lambda: dst.copy_(keys)], 50), 4 * n * (rank + rot), "hbm")))
+        del q, kv, keys, out, kc, vc, cache, dst
+
+    # ---- attention of single tokens: latents met as they lie
+    for what, batch, ctx, window, pools in (("batch 64, ctx U[100,2048]", 64, (100, 2048), 8192, 4), ("batch 256, ctx U[300,1326]", 256, (300, 1326), 8192, 3),
+                                            ("batch 16, ctx U[4096,8192]", 16, (4096, 8192), 8192, 4), ("batch 64, ctx 8192, window 1024", 64, (8192, 8192), 1024, 2),
+                                            ("batch 1, ctx 8192", 1, (8192, 8192), 8192, 8)):
+        if not want("attention decode"):
+            continue
+        g = torch.Generator().manual_seed(1)
+        lens = torch.randint(ctx[0], ctx[1] + 1, (batch,), generator=g)
+        blocks = int(((lens + 255) // 256).sum())
+        tabs = synthetic.decode_tables(lens.tolist(), blocks, g).to(dev)
+        group = RowGroup(0, batch, batch, i32(lens), i32([0] * batch), tabs, i32([0] * batch))
+        met, qr, gate, out = rnd(batch, heads, rank), rnd(batch, heads, rot), rnd(batch, heads), torch.empty(batch, heads, rank, dtype=bf, device=dev)
+        caches = [rnd(blocks, 256, rank + rot) for _ in range(pools)]
+        mine = graph_us([lambda c=c: latent.latent_attention(met, qr, gate, rope, c, group, out, window, scale) for c in caches], 56)
+        keys = int(torch.clamp(lens, max=window).sum())
+        alg = keys * (rank + rot) * 2 + 4 * met.numel()
+        del caches
+        # the like kernel: as many bytes of keys and values (2 heads of 128 and a window of whole chunks; 8 query heads each)
+        kv = 2
+        caches = [(rnd(blocks, 256, kv, 128), rnd(blocks, 256, kv, 128)) for _ in range(pools)]
+        q1, o1 = rnd(batch, heads * 128), torch.empty(batch, heads * 128, dtype=bf, device=dev)
+        theirs = graph_us([lambda c=c: mixers.chunk_attention(q1, c[0], c[1], group, o1, heads, window, 128 ** -0.5, 30.0) for c in caches], 56)
+        like_keys = int(((lens - 1) % window + 1).sum())
+        rows.append(_kernel_row("latent attention decode, " + what, mine, alg, "hbm", ("chunk_decode_kernel + merge", theirs, like_keys * kv * 512 + 4 * q1.numel(), "hbm")))
+        del caches
+
+    # ---- per-head products around the absorbed form
+    for batch in (16, 256):
+        if not want("per-head"):
+            continue
+        q, met = rnd(batch, heads, dim + rot), torch.empty(batch, heads, rank, dtype=bf, device=dev)
+        ws = [(rnd(heads, rank, dim), rnd(heads, vdim, rank)) for _ in range(24)]
+        o = torch.empty(batch, heads, vdim, dtype=bf, device=dev)
+        x, wl = rnd(batch, rank), [rnd(heads * dim, rank) for _ in range(24)]
+        like = graph_us([lambda w=w: F.linear(x, w) for w in wl])
+        lalg = 2 * (heads * dim * rank + batch * (rank + heads * dim))
+        mine = graph_us([lambda w=w: experts.grouped_linear(q[..., :dim], w[0], met) for w in ws])
+        rows.append(_kernel_row("per-head product to the latent, %d rows" % batch, mine, 2 * (heads * dim * rank + batch * heads * (dim + rank)), "hbm", ("library product", like, lalg, "hbm")))
+        mine = graph_us([lambda w=w: experts.grouped_linear(met, w[1], o) for w in ws])
+        rows.append(_kernel_row("per-head product from the latent, %d rows" % batch, mine, 2 * (heads * vdim * rank + batch * heads * (vdim + rank)), "hbm", ("library product", like, lalg, "hbm")))
+
+    # ---- matrix memory
+    for what, lens in (("1x16384", [16384]), ("2x16384", [16384, 16384]), ("16x1024", [1024] * 16), ("29 x U[100,1024]", lengths(29, 100, 1024))):
+        if not want("memory prefill"):
+            continue
+        group, _ = _portions(dev, lens)
+        n = sum(lens)
+        x, z, out, w = rnd(n, 4 * mh * 128), torch.randn(n, 2 * mh, device=dev), torch.empty(n, mh * 128, dtype=bf, device=dev), rnd(mh * 128)
+        state, mass, mtop = torch.zeros(len(lens), mh, 128, 128, device=dev), torch.zeros(len(lens), mh, 128, device=dev), torch.zeros(len(lens), mh, device=dev)
+        bias = torch.cat([torch.zeros(mh), torch.full((mh,), 4.0)]).to(dev)
+        mine = event_us([lambda: mlstm(x, z, bias, w, state, mass, mtop, group, out, 128 ** -0.5, 15.0, 1e-6)])
+        alg = n * mh * 128 * 5 * 2 + state.numel() * 4
+        theirs = event_us([lambda: mixers.retention(x, state, group, rope128, bias[:mh] - 0.01, out, 128, 128 ** -0.5, 1e-6)])
+        rows.append(_kernel_row("memory prefill, " + what, mine, alg + n * mh * 8, "hbm", ("retention_chunk_kernel", theirs, alg + n * 128 * 4, "hbm")))
+    for batch in (1, 64, 256):
+        if not want("memory decode"):
+            continue
+        states = [torch.zeros(batch, mh, 128, 128, device=dev) for _ in range(4)]
+        mass, mtop = torch.zeros(batch, mh, 128, device=dev), torch.zeros(batch, mh, device=dev)
+        group = RowGroup(0, batch, batch, i32([800] * batch), i32([0] * batch), None, i32(list(range(batch))))
+        x, z, out, w = rnd(batch, 4 * mh * 128), torch.randn(batch, 2 * mh, device=dev), torch.empty(batch, mh * 128, dtype=bf, device=dev), rnd(mh * 128)
+        bias = torch.cat([torch.zeros(mh), torch.full((mh,), 4.0)]).to(dev)
+        mine = graph_us([lambda s=s: mlstm(x, z, bias, w, s, mass, mtop, group, out, 128 ** -0.5, 15.0, 1e-6) for s in states])
+        theirs = graph_us([lambda s=s: mixers.retention(x, s, group, rope128, bias[:mh] - 0.01, out, 128, 128 ** -0.5, 1e-6) for s in states])
+        rows.append(_kernel_row("memory decode, batch %d" % batch, mine, states[0].numel() * 8, "hbm", ("retention_step_kernel", theirs, states[0].numel() * 8, "hbm")))
+        del states
+    for n in (16, 256, 16384):
+        if want("gate products"):
+            h = rnd(n, width)
+            ws, wl = [rnd(2 * mh, width) for _ in range(8)], [rnd(2 * mh, width) for _ in range(8)]
+            alg = 2 * n * width + 4 * mh * width + 8 * mh * n
+            rows.append(_kernel_row("gate products in fp32, %d rows" % n, graph_us([lambda w=w: experts.linear_f32(h, w) for w in ws]), alg, "hbm",
+                                    ("library product", graph_us([lambda w=w: F.linear(h, w) for w in wl]), alg, "hbm")))
+
+    # ---- experts
+    for n in (1, 16, 128, 512, 2048, 16384):
+        if not want("experts"):
+            continue
+        h = rnd(n, width)
+        spec = experts.ExpertsSpec(n_exp, top, ff, 1.0)
+        copies = 6 if n <= 512 else 1
+        runs = []
+        for _ in range(copies):
+            with torch.device(dev):
+                w = experts.ExpertWeights(spec, width).to(bf).requires_grad_(False)
+            for p in w.parameters():
+                p.normal_(0.0, 0.03)
+            counters = torch.zeros(n_exp, dtype=torch.int32, device=dev)
+            a = experts.route(h, w.router, top, 1.0, counters)
+            runs.append((w, a, experts.routed_linear(h, w.gate_up, a, True), torch.zeros(n_exp, dtype=torch.int32, device=dev)))
+        hit = sum(int((r[1].counts > 0).sum()) for r in runs) / copies
+        dense = [(rnd(2 * top * ff, width), rnd(width, top * ff)) for _ in range(copies)]
+        mid, act = rnd(n, 2 * top * ff), rnd(n, top * ff)
+        time = graph_us if n <= 512 else event_us
+        n_calls = (200,) if n <= 512 else (steps,)
+        up = time([lambda r=r: experts.routed_linear(h, r[0].gate_up, r[1], True) for r in runs], *n_calls)
+        down = time([lambda r=r: experts.routed_linear(r[2], r[0].down, r[1], False) for r in runs], *n_calls)
+        lup = time([lambda d=d: mixers.clamped_gate(F.linear(h, d[0]), 7.0, 1.702) for d in dense], *n_calls)
+        ldown = time([lambda d=d: F.linear(act, d[1]) for d in dense], *n_calls)
+        if n >= 512:
+            rows.append(_kernel_row("experts gate | up, %d rows" % n, up, 4 * n * top * ff * width, "mfma", ("library product + clamped_gate_kernel", lup, 4 * n * top * ff * width, "mfma")))
+            rows.append(_kernel_row("experts down, %d rows" % n, down, 2 * n * top * ff * width, "mfma", ("library product", ldown, 2 * n * top * ff * width, "mfma")))
+        else:
+            wu, io = hit * 2 * ff * width * 2, 2 * n * (width + top * ff)
+            rows.append(_kernel_row("experts gate | up, %d rows" % n, up, wu + io, "hbm", ("library product + clamped_gate_kernel", lup, 2 * top * ff * width * 2 + io, "hbm")))
+            wd, io = hit * ff * width * 2, 2 * n * (top * ff + top * width)
+            rows.append(_kernel_row("experts down, %d rows" % n, down, wd + io, "hbm", ("library product", ldown, top * ff * width * 2 + 2 * n * (top * ff + width), "hbm")))
+
+        def routed(r):
+            r[3].zero_()
+            experts.route(h, r[0].router, top, 1.0, r[3])
+        both = time([lambda r=r: routed(r) for r in runs], *n_calls)
+        clear = time([lambda r=r: r[3].zero_() for r in runs], *n_calls)
+        plain = [rnd(n_exp, width) for _ in range(copies)]
+        lrouter = time([lambda w=w: F.linear(h, w) for w in plain], *n_calls)
+        alg = 2 * n * width + 2 * n_exp * width + n * top * 12
+        rows.append(_kernel_row("experts router, %d rows" % n, both - clear, alg, "hbm", ("library product (logits only)", lrouter, alg, "hbm")))
+        del runs, dense
+
+    # ---- steps around them
+    for n in (16, 256, 16384):
+        if want("branches"):
+            y1, y2, r32 = rnd(n, width), rnd(n * top, width), torch.randn(n, width, device=dev)
+            tw, w = torch.rand(n, top, device=dev), [rnd(width) for _ in range(4)]
+            cnt = torch.zeros(n_exp, dtype=torch.int32, device=dev)
+            mine = graph_us([lambda: branches.branches_rms_norms(r32, 0.5, y1, w[0], y2, tw, w[1], (w[2], w[3]), 1e-6, 1.0, clear=cnt)])
+            theirs = graph_us([lambda: mixers.post_add_norm(y1, r32, (w[0], w[1]), (w[2], w[3]), 1e-6)])
+            rows.append(_kernel_row("branches + norms, %d rows" % n, mine, n * width * (2 + 2 * top + 8 + 4), "hbm", ("norm_rows_kernel", theirs, n * width * 12, "hbm")))
+        if want("prepare"):
+            x, qo = rnd(n, q_rank + rank + rot + heads), torch.empty(n, q_rank, dtype=bf, device=dev)
+            wq, wkv = rnd(q_rank), rnd(rank)
+            cache = torch.empty(max(1, n // 256), 256, rank + rot, dtype=bf, device=dev)
+            if n >= 16384:
+                group, _ = _portions(dev, [1024] * 16)
+            else:
+                group = RowGroup(0, n, n, i32([701] * n), i32(torch.randperm(n)), None, i32(list(range(n))))
+            mine = graph_us([lambda: latent.latent_prepare(x, wq, wkv, rope, qo, cache, group, rot, 1e-6)])
+            ch = (heads + 2 * 8) * 128
+            xc, conv, q1 = rnd(n, ch), rnd(1, ch), torch.empty(n, heads * 128, dtype=bf, device=dev)
+            kc, vc = (torch.empty(max(1, n // 256), 256, 8, 128, dtype=bf, device=dev) for _ in range(2))
+            theirs = graph_us([lambda: mixers.conv_rope_store(xc, conv, None, group, rope128, q1, kc, vc, heads, 128)])
+            rows.append(_kernel_row("prepare: latents, rotation, cache write, %d rows" % n, mine, n * (q_rank + rank + rot) * 4 + n * rot * 4, "hbm",
+                                    ("conv_rope_store_kernel, one tap", theirs, n * ch * 4 + n * 512, "hbm")))
+    return rows
+
+
 def _engine_rates(model, dev, batch, prompt_len, new_tokens, slots):
     """Prefill and decode tokens/s of the engine: ``batch`` prompts of ``prompt_len`` tokens, ``new_tokens`` each."""
     import gc
@@ -1048,9 +1284,9 @@ def _engine_rates(model, dev, batch, prompt_len, new_tokens, slots):
 
 def bench_kaparax(args, dev):
     """The Kaparax family beside Qwen3 at equal size: engine throughput (prompts of 1024 tokens, then 128 decoded
-    tokens each) for two layer sizes and two batches, and every kernel beside its like (--kaparax-part)."""
+    tokens each) for two layer sizes and two batches, and every kernel beside its like (--part)."""
     from nanovllm_amd.engine import ModelConfig, qwen3_0_6b
-    part = args.kaparax_part
+    part = args.part
     kernels = kaparax_kernels(dev, only=args.kernel) if part in ("all", "kernels") else []
     engines = {}
     if part in ("all", "engine"):
@@ -1073,9 +1309,33 @@ def bench_kaparax(args, dev):
     return result, lambda: None
 
 
-WORKLOADS = {"kaparax": bench_kaparax, "rope-scatter": bench_rope_scatter, "glue": bench_glue, "e2e": bench_e2e, "longctx": bench_longctx, "decode-e2e-shape": bench_decode_e2e_shape,
+def bench_pidutar(args, dev):
+    """The Pidutar family beside Kaparax at equal size: engine throughput (prompts of 1024 tokens, then 128 decoded
+    tokens each) for two layer sizes and two batches, and every kernel beside its like (--part)."""
+    part = args.part
+    kernels = pidutar_kernels(dev, only=args.kernel) if part in ("all", "kernels") else []
+    engines = {}
+    if part in ("all", "engine"):
+        sizes = {"28 layers, width 1024, 16 heads, 4 of 32 experts of 768": (
+                     _pidutar_config(28, 1024, 16, 512, 512, 8, 128, 32, 4, 768, 8192, 151936), _kaparax_config(28, 1024, 16, 8, 128, 3072, 8, 128, 8192, 151936)),
+                 "8 layers, width 4096, 32 heads, 4 of 32 experts of 3072": (
+                     _pidutar_config(8, 4096, 32, 1536, 512, 16, 128, 32, 4, 3072, 8192, 151936), _kaparax_config(8, 4096, 32, 8, 128, 12288, 16, 128, 8192, 151936))}
+        for what, (mine, like) in sizes.items():
+            for batch in (16, 128):
+                engines["%s; batch %d" % (what, batch)] = {"pidutar": _engine_rates(mine, dev, batch, 1024, 128, 128),
+                                                           "kaparax": _engine_rates(like, dev, batch, 1024, 128, 128)}
+    first = next(iter(engines.values()))["pidutar"]["decode_tok_s"] if engines else None
+    result = {"metric": "Pidutar decode tok/s (28 layers of width 1024, batch 16, prompts of 1024)", "value": first, "unit": "tok/s",
+              "ms_per_step": round(16e3 / first, 3) if first else None,
+              "config": {"workload": "random weights; latent attention and matrix memory in turn, window 8192, every layer beside routed experts",
+                         "engine": engines, "kernels": kernels},
+              "roofline": None}
+    return result, lambda: None
+
+
+WORKLOADS = {"pidutar": bench_pidutar, "kaparax": bench_kaparax, "rope-scatter": bench_rope_scatter, "glue": bench_glue, "e2e": bench_e2e, "longctx": bench_longctx, "decode-e2e-shape": bench_decode_e2e_shape,
              "decode-longctx-shape": bench_decode_longctx_shape, "copy": bench_copy, "read-probe": bench_read_probe, "decode": bench_decode, "scatter": bench_scatter, "prefill": bench_prefill, "sampler": bench_sampler}
-DEFAULT_STEPS = {"kaparax": 60, "rope-scatter": 100, "glue": 100, "e2e": 1, "longctx": 1, "decode-e2e-shape": 1, "decode-longctx-shape": 1, "copy": 50, "read-probe": 60, "decode": 200, "scatter": 400, "prefill": 50, "sampler": 100}
+DEFAULT_STEPS = {"pidutar": 60, "kaparax": 60, "rope-scatter": 100, "glue": 100, "e2e": 1, "longctx": 1, "decode-e2e-shape": 1, "decode-longctx-shape": 1, "copy": 50, "read-probe": 60, "decode": 200, "scatter": 400, "prefill": 50, "sampler": 100}
 
 
 def main():
@@ -1096,8 +1356,8 @@ def main():
     ap.add_argument("--glue", choices=["add-rms-norm", "silu-mul", "last-token-norm"], default="add-rms-norm", help="glue: which elementwise kernel")
     ap.add_argument("--uniform", default=None, metavar="SxL", help="prefill: S packed sequences of L tokens each instead of config 3 (e.g. 2x16384)")
     ap.add_argument("--bucket-step", type=int, default=16, help="e2e only: spacing of the captured decode batch sizes")
-    ap.add_argument("--kaparax-part", choices=["all", "kernels", "engine"], default="all", help="kaparax: which half of the workload")
-    ap.add_argument("--kernel", default=None, help="kaparax: only kernels whose row name contains this")
+    ap.add_argument("--part", "--kaparax-part", choices=["all", "kernels", "engine"], default="all", help="kaparax / pidutar: which half of the workload")
+    ap.add_argument("--kernel", default=None, help="kaparax / pidutar: only kernels whose row name contains this")
     ap.add_argument("--no-extra", action="store_true", help="e2e only: skip the per-configuration rooflines and the eager pass")
     args = ap.parse_args()
     if args.gpus != 1:

@@ -158,6 +158,169 @@ __global__ __launch_bounds__(256) void linear_skinny_kernel(LinearArgs a) {
     }
 }
 
+// ---- bf16, many rows per expert: tiles of BM rows x 128 weight rows ---------------------------------
+// Routed only.  A workgroup of four wavefronts (2 x 2) takes BM assignments of one expert and 128 rows of its weights
+// (gated: 64 gates and the 64 ups that belong to them, side by side in every wavefront).  Both operands travel
+// global -> LDS without a register in between, in steps of 32 inner elements through three buffers: while one
+// step is multiplied the next one has landed or is about to and the one after it is on its way, and the wait
+// before the barrier leaves those loads in flight.  The LDS image is made of 1 KB blocks of 16 rows x 32 elements with the
+// 16-byte pieces of a row permuted so that operand reads spread over the banks.
+// Tiles are numbered expert by expert, weight tiles fastest, and dealt out so that each XCD walks one
+// stretch of that order: neighbours share rows or weights in its L2.
+constexpr int kTileN = 128;
+
+template <int BM, bool kGated>
+__global__ __launch_bounds__(256, 2) void linear_tile_kernel(const LinearArgs a, const int32_t n_tiles) {
+    constexpr int kTB = BM / 32;                         // blocks of 16 rows per wavefront
+    constexpr int kBlocksX = BM / 16, kBlocksW = kTileN / 16, kStage = (kBlocksX + kBlocksW) * 1024;
+    constexpr int kLX = kBlocksX / 4, kLW = kBlocksW / 4;                       // blocks a wavefront loads per step
+    __shared__ __attribute__((aligned(1024))) unsigned char smem[3 * kStage];
+    const int tid = threadIdx.x, lane = tid & 63, r = lane & 15, g = lane >> 4;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int wm = wave & 1, wn = wave >> 1;
+    // ---- which tile: row tiles of every expert, 64 experts at a time
+    int total = 0;
+    for (int e0 = 0; e0 < a.groups; e0 += 64) {
+        const int e = e0 + lane;
+        int t = e < a.groups ? (group_rows(a, e) + BM - 1) / BM : 0;
+#pragma unroll
+        for (int d = 1; d < 64; d <<= 1) t += __shfl_xor(t, d, 64);
+        total += t;
+    }
+    total = __builtin_amdgcn_readfirstlane(total) * n_tiles;
+    const int stretch = (total + 7) / 8;
+    const int in_stretch = blockIdx.x / 8;
+    const int tile = blockIdx.x % 8 * stretch + in_stretch;
+    if (in_stretch >= stretch || tile >= total) return;
+    const int n_tile = tile % n_tiles;
+    int m_tile = tile / n_tiles, expert = 0;
+    for (int e0 = 0; e0 < a.groups; e0 += 64) {
+        const int e = e0 + lane;
+        const int own = e < a.groups ? (group_rows(a, e) + BM - 1) / BM : 0;
+        int upto = own;
+#pragma unroll
+        for (int d = 1; d < 64; d <<= 1) {
+            const int o = __shfl_up(upto, d, 64);
+            if (lane >= d) upto += o;
+        }
+        const unsigned long long here = __ballot(m_tile < upto);
+        if (here != 0) {
+            const int first = __ffsll(here) - 1;
+            expert = e0 + first;
+            m_tile -= __shfl(upto, first, 64) - __shfl(own, first, 64);
+            break;
+        }
+        m_tile -= __shfl(upto, 63, 64);
+    }
+    expert = __builtin_amdgcn_readfirstlane(expert);
+    m_tile = __builtin_amdgcn_readfirstlane(m_tile);
+    const int count = group_rows(a, expert), m0 = m_tile * BM;
+
+    // ---- what this wavefront loads: byte offsets of its lanes' pieces in the first step
+    const int l16 = lane >> 2, piece = ((lane & 3) ^ ((0 - (l16 >> 2)) & 3)) * 8;
+    uint32_t xoff[kLX], woff[kLW];
+#pragma unroll
+    for (int i = 0; i < kLX; ++i)
+        xoff[i] = static_cast<uint32_t>(x_offset(a, expert, group_row(a, expert, min(m0 + 16 * (wave * kLX + i) + l16, count - 1))) + piece) * 2;
+#pragma unroll
+    for (int i = 0; i < kLW; ++i) {
+        const int row = 16 * (wave * kLW + i) + l16;     // of the tile; gated: 32 gates, their 32 ups, twice
+        int n;
+        if (kGated) n = min(n_tile * 64 + row / 64 * 32 + row % 32, a.n_out - 1) + (row % 64 < 32 ? 0 : a.n_out);
+        else n = min(n_tile * kTileN + row, a.n_out - 1);
+        woff[i] = static_cast<uint32_t>(n * static_cast<int64_t>(a.k) + piece) * 2;
+    }
+    const char *xb = static_cast<const char *>(a.x);
+    const char *wb = static_cast<const char *>(a.w) + static_cast<int64_t>(expert) * (kGated ? 2 : 1) * a.n_out * a.k * 2;
+    const lds_char_ptr lds = (lds_char_ptr)(&smem[0]);
+    const uint32_t lds0 = __builtin_amdgcn_readfirstlane(static_cast<uint32_t>(reinterpret_cast<uintptr_t>(lds)));
+    auto fetch = [&](int step, int buf) __attribute__((always_inline)) {
+        const char *x = xb + 64 * static_cast<int64_t>(step), *w = wb + 64 * static_cast<int64_t>(step);
+        const uint32_t at = lds0 + buf * kStage;
+#pragma unroll
+        for (int i = 0; i < kLX; ++i) load_to_lds_16(x, xoff[i], at + (wave * kLX + i) * 1024);
+#pragma unroll
+        for (int i = 0; i < kLW; ++i) load_to_lds_16(w, woff[i], at + (kBlocksX + wave * kLW + i) * 1024);
+    };
+    // the loads above are ordinary instructions to the compiler: these two keep them on their side of a barrier
+    auto after_barrier = [&]() __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < kLX; ++i) asm volatile("" : "+v"(xoff[i]));
+#pragma unroll
+        for (int i = 0; i < kLW; ++i) asm volatile("" : "+v"(woff[i]));
+    };
+
+    f32x4_t acc[4][kTB];
+#pragma unroll
+    for (int n = 0; n < 4; ++n)
+#pragma unroll
+        for (int m = 0; m < kTB; ++m) acc[n][m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    const int steps = a.k / 32;
+    const lds_char_ptr frag = lds + 16 * (4 * r + (g ^ ((0 - (r >> 2)) & 3)));
+    fetch(0, 0);
+    after_barrier();
+    if (steps > 1) {
+        fetch(1, 1);
+        after_barrier();
+        asm volatile("s_waitcnt vmcnt(%0)" :: "i"(kLX + kLW) : "memory");
+    } else {
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    }
+    __syncthreads();
+    int buf = 0;
+    for (int step = 0; step < steps; ++step) {
+        after_barrier();
+        if (step + 2 < steps) fetch(step + 2, buf == 0 ? 2 : buf - 1);          // (the buffer of the step before this one)
+        const lds_char_ptr xl = frag + buf * kStage + wm * kTB * 1024, wl = frag + buf * kStage + (kBlocksX + wn * 4) * 1024;
+        u32x4_t wf[4];
+#pragma unroll
+        for (int n = 0; n < 4; ++n) wf[n] = *(lds_u32x4_ptr)(wl + n * 1024);
+#pragma unroll
+        for (int m = 0; m < kTB; ++m) {
+            const u32x4_t xf = *(lds_u32x4_ptr)(xl + m * 1024);
+#pragma unroll
+            for (int n = 0; n < 4; ++n) acc[n][m] = mfma16(wf[n], xf, acc[n][m]);
+        }
+        after_barrier();
+        if (step + 2 < steps) asm volatile("s_waitcnt vmcnt(%0)" :: "i"(kLX + kLW) : "memory");
+        else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();
+        buf = buf == 2 ? 0 : buf + 1;
+    }
+    // ---- four consecutive outputs of a row per accumulator
+#pragma unroll
+    for (int m = 0; m < kTB; ++m) {
+        const int i = m0 + 16 * (wm * kTB + m) + r;
+        if (i >= count) continue;
+        bf16_t *out = static_cast<bf16_t *>(a.out) + out_offset(a, expert, group_row(a, expert, i));
+#pragma unroll
+        for (int n = 0; n < (kGated ? 2 : 4); ++n) {
+            const int c = kGated ? n_tile * 64 + 32 * wn + 16 * n + 4 * g : n_tile * kTileN + 64 * wn + 16 * n + 4 * g;
+            if (c >= a.n_out) continue;
+            float y[4];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) y[j] = kGated ? silu_of<bf16_t>(acc[n][m][j]) * acc[kGated ? n + 2 : n][m][j] : acc[n][m][j];
+            *reinterpret_cast<u32x2_t *>(out + c) = u32x2_t{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
+        }
+    }
+}
+
+// Sizes the tiled form is built for: whole steps, whole 8-byte stores, 32-bit offsets.
+static bool tiles_ok(const LinearArgs &a, bool gated, int32_t x_rows) {
+    return a.k % 32 == 0 && a.n_out % 4 == 0 && aligned16(a.out) && static_cast<int64_t>(x_rows) * a.x_stride < (1LL << 30) &&
+           static_cast<int64_t>(a.n_out) * (gated ? 2 : 1) * a.k < (1LL << 30);
+}
+
+template <int BM, bool kGated>
+static int launch_tiles(const LinearArgs &a, hipStream_t s) {
+    const int32_t n_tiles = (a.n_out + (kGated ? 64 : kTileN) - 1) / (kGated ? 64 : kTileN);
+    const int64_t most = (static_cast<int64_t>(a.rows) / BM + a.groups) * n_tiles;      // row tiles there can be, whatever the counts are
+    const int64_t grid = (most + 7) / 8 * 8 + 8;
+    if (grid > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
+    hipLaunchKernelGGL((linear_tile_kernel<BM, kGated>), dim3(static_cast<uint32_t>(grid)), dim3(256), 0, s, a, n_tiles);
+    return launch_status();
+}
+
 template <typename T, typename O, bool kGated>
 static int launch_any_linear(const LinearArgs &a, int32_t most_rows, hipStream_t s) {
     const dim3 grid((a.n_out + 63) / 64, a.groups, std::min(std::max(1, (most_rows + 15) / 16), a.lists ? 64 : 65535));
@@ -234,9 +397,8 @@ __global__ __launch_bounds__(512) void router_kernel(RouterArgs a) {
                 if (in) xf = *reinterpret_cast<const u32x4_t *>(x + e);
 #pragma unroll
                 for (int b = 0; b < 4; ++b) {
-                    if (b >= blocks) continue;
                     u32x4_t wf = {0, 0, 0, 0};
-                    if (in) wf = *reinterpret_cast<const u32x4_t *>(w[b] + e);
+                    if (in && b < blocks) wf = *reinterpret_cast<const u32x4_t *>(w[b] + e);
                     acc[b] = mfma16(wf, xf, acc[b]);
                 }
             }
@@ -366,6 +528,11 @@ extern "C" int nva_routed_linear(const void *x, int64_t x_row_stride, const void
     const int32_t hint = static_cast<int32_t>((static_cast<int64_t>(rows) * terms * 3 / 2 + experts - 1) / experts);
     if (dtype == NVA_DTYPE_F32) return gated ? launch_any_linear<float, float, true>(a, rows, s) : launch_any_linear<float, float, false>(a, rows, s);
     if (!linear_matrix_ok(a)) return gated ? launch_any_linear<bf16_t, bf16_t, true>(a, rows, s) : launch_any_linear<bf16_t, bf16_t, false>(a, rows, s);
+    const int32_t average = static_cast<int32_t>(static_cast<int64_t>(rows) * terms / experts);
+    if (average >= 48 && tiles_ok(a, gated, x_per_row ? rows : rows * terms)) {
+        if (average >= 192) return gated ? launch_tiles<256, true>(a, s) : launch_tiles<256, false>(a, s);
+        return gated ? launch_tiles<128, true>(a, s) : launch_tiles<128, false>(a, s);
+    }
     return gated ? launch_skinny<true, bf16_t>(a, hint, rows, s) : launch_skinny<false, bf16_t>(a, hint, rows, s);
 }
 

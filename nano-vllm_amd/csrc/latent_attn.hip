@@ -206,32 +206,38 @@ __global__ __launch_bounds__(256) void latent_attn_any_kernel(LatentAttnArgs a) 
 }
 
 // bf16 on the matrix cores (v_mfma_f32_16x16x32_bf16, transposed: S^T = K Q^T, O^T += C^T P^T).  A workgroup takes
-// one (row, range of keys, 16 NH heads) and walks the range in tiles of 32 keys, the next tile on its way in
-// registers.  A tile lies in LDS once: its rows are the keys and, read through the transpose, the values.
-// Every wavefront forms all scores of the tile (so that nothing is exchanged) and its quarter of the
-// latent columns.  The score accumulators of two 16-key blocks (register i of lane l: key 4 (l / 16) + i) are
-// a legal key order for the second product, so P stays in registers; its fp32 weights enter as the sum of two
-// bf16 numbers.  With more than one range per row the results are partial (fp32 sums, sum of the weights,
-// reference exponent) and latent_merge_kernel adds them up.
+// one (row, range of keys, 16 NH heads) and walks the range in tiles of 64 keys.  Wavefront w loads 16 of them from memory
+// straight into operand registers, forms their scores, and puts the latents into LDS, where every wavefront reads
+// its quarter of the latent columns through the transpose.  The score accumulators (register i of lane l: key 4 (l / 16) + i)
+// are a legal key order for the second product, so the weights go to the other wavefronts lane by lane; fp32, they
+// enter it as the sum of two bf16 numbers.  The next tile's loads go out as soon as the registers are free.  The
+// reference of the weights is shared by the wavefronts and moves only when a score passes it by more than 2^8.  With
+// more than one range per row the results are partial (fp32 sums, sum of the weights, reference exponent)
+// and latent_merge_kernel adds them up.  kExact: the model's sizes are those the registers are laid out for.
 struct LatentSplit {
     float *partials;         // [n, splits, heads, R + 4]: sums, sum of the weights, reference exponent
-    int32_t splits, keys;    // ranges per row, keys per range (a multiple of 32)
+    int32_t splits, keys;    // ranges per row, keys per range (a multiple of 64)
     int32_t head_groups;     // groups of 16 NH heads
 };
+constexpr int kRowTile = 64;
 
-template <int RK, int DR, int NH>
+template <int RK, int DR, int NH, bool kExact>
 __global__ __launch_bounds__(256, 2) void latent_rows_kernel(const LatentAttnArgs a, const LatentSplit sp) {
-    constexpr int kKS = RK / 32, kAll = (RK + DR) / 32, kPitch = (RK + DR) * 2 + 16, kPieces = (RK + DR) * 32 / 8 / 256;
+    constexpr int kKS = RK / 32, kAll = (RK + DR) / 32, kPitch = RK * 2 + 32;
     constexpr int kDB = RK / 64;                         // value blocks of 16 columns per wavefront
-    static_assert((RK + DR) * 32 / 8 % 256 == 0, "whole pieces per thread");
-    __shared__ __attribute__((aligned(16))) unsigned char smem[32 * kPitch];
+    __shared__ __attribute__((aligned(16))) unsigned char smem[kRowTile * kPitch];
+    __shared__ u32x4_t sh_p[NH][4][64];
+    __shared__ float sh_m[NH][4][16], sh_l[NH][4][16];
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int r = lane & 15, g = lane >> 4;
-    // rows are the fastest index: ranges past the end of short sequences spread over the CUs
-    const int64_t t = blockIdx.x % a.rows.n;
-    const int rest = blockIdx.x / a.rows.n;
-    const int split = rest % sp.splits, head0 = rest / sp.splits * 16 * NH;
+    // (row, range) pairs are dealt out over the XCDs, a pair's head groups to the same one; rows are the fastest
+    // index, so that ranges past the end of short sequences spread over the CUs
+    const int hg = blockIdx.x / 8 % sp.head_groups;
+    const int64_t item = static_cast<int64_t>(blockIdx.x) / (8 * sp.head_groups) * 8 + blockIdx.x % 8;
+    if (item >= static_cast<int64_t>(a.rows.n) * sp.splits) return;
+    const int64_t t = item % a.rows.n;
+    const int split = static_cast<int>(item / a.rows.n), head0 = hg * 16 * NH;
     const int nheads = min(16 * NH, a.heads - head0);
     int seq, pos;
     place_of(a.rows, t, seq, pos);
@@ -241,30 +247,31 @@ __global__ __launch_bounds__(256, 2) void latent_rows_kernel(const LatentAttnArg
             for (int i = tid; i < nheads * a.rank; i += 256) out[i] = 0;
         return;
     }
-    const int lo = max(0, pos - a.window + 1), first = (lo & ~31) + split * sp.keys;
+    const int lo = max(0, pos - a.window + 1), first = (lo & ~(kRowTile - 1)) + split * sp.keys;
     const int last = min(pos, first + sp.keys - 1);      // last key of this range
     if (first > last) return;
-    const int ntiles = (last - first) / 32 + 1, width = a.rank + a.rot;
+    const int ntiles = (last - first) / kRowTile + 1, width = a.rank + a.rot;
     const int bmask = (1 << a.block_shift) - 1;
     const lds_char_ptr lds = (lds_char_ptr)(&smem[0]);
     const bf16_t *cache = static_cast<const bf16_t *>(a.cache);
 
     auto block_of = [&](int tile) __attribute__((always_inline)) -> int {
-        const int col = (first + tile * 32) >> a.block_shift;
+        const int col = (first + tile * kRowTile) >> a.block_shift;
         return tile < ntiles && col < a.max_blocks ? a.block_tables[seq * a.bt_stride + col] : -1;
     };
-    u32x4_t reg[kPieces];
+    u32x4_t kf[kAll];
     auto fetch = [&](int tile, int blk) __attribute__((always_inline)) {
-        const int key0 = first + tile * 32;
+        const int key0 = first + tile * kRowTile;
         const bool ok = static_cast<uint32_t>(blk) < static_cast<uint32_t>(a.num_blocks);
-        const bf16_t *base = cache + ((static_cast<int64_t>(ok ? blk : 0) << a.block_shift) + (key0 & bmask)) * width;
+        if (!ok) return;
+        const int row = min(16 * wave + r, last - key0);             // rows past the last key repeat it and are masked
+        const bf16_t *base = cache + ((static_cast<int64_t>(blk) << a.block_shift) + (key0 & bmask) + row) * width + 8 * g;
 #pragma unroll
-        for (int i = 0; i < kPieces; ++i) {
-            const int p = i * 256 + tid, row = p / ((RK + DR) / 8), c = p % ((RK + DR) / 8) * 8;
-            const int e = c < RK ? c : c - RK;           // latent columns up to RK, then the rotated part
-            reg[i] = u32x4_t{0, 0, 0, 0};
-            if (ok && key0 + row <= last && e < (c < RK ? a.rank : a.rot))
-                reg[i] = __builtin_nontemporal_load(reinterpret_cast<const u32x4_t *>(base + static_cast<int64_t>(row) * width + (c < RK ? e : a.rank + e)));
+        for (int ks = 0; ks < kAll; ++ks) {
+            const int e = ks < kKS ? 32 * ks : 32 * (ks - kKS);
+            const bool in = kExact || e + 8 * g < (ks < kKS ? a.rank : a.rot);
+            if (!kExact) kf[ks] = u32x4_t{0, 0, 0, 0};
+            if (in) kf[ks] = *reinterpret_cast<const u32x4_t *>(base + (ks < kKS ? e : a.rank + e));
         }
     };
     int blk = block_of(0), blk_next = block_of(1);
@@ -282,10 +289,10 @@ __global__ __launch_bounds__(256, 2) void latent_rows_kernel(const LatentAttnArg
                 qf[h][ks] = u32x4_t{0, 0, 0, 0};
                 if (ks < kKS) {
                     const int e = 32 * ks + 8 * g;
-                    if (e < a.rank) qf[h][ks] = *reinterpret_cast<const u32x4_t *>(ql + e);
+                    if (kExact || e < a.rank) qf[h][ks] = *reinterpret_cast<const u32x4_t *>(ql + e);
                 } else {
                     const int e = 32 * (ks - kKS) + 8 * g;
-                    if (e < a.rot) {
+                    if (kExact || e < a.rot) {
                         float v[8];
                         load_f32<bf16_t, 8>(qr + e, v);
                         turn_pairs<8>(v, cs, a.rot / 2, e);
@@ -306,51 +313,49 @@ __global__ __launch_bounds__(256, 2) void latent_rows_kernel(const LatentAttnArg
         for (int db = 0; db < kDB; ++db) oacc[h][db] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
     const float to_exp2 = a.scale * 1.4426950408889634f;
-    const lds_char_ptr kl = lds + r * kPitch + 16 * g;
+    const lds_char_ptr vw = lds + (16 * wave + r) * kPitch + 16 * g;
     const lds_char_ptr vl = lds + (4 * g + (r >> 2)) * kPitch + 8 * (r & 3) + wave * (RK / 4) * 2;
     for (int tile = 0; tile < ntiles; ++tile) {
-        const int key0 = first + tile * 32;
+        const int key0 = first + tile * kRowTile;
         const bool ok = static_cast<uint32_t>(blk) < static_cast<uint32_t>(a.num_blocks);
-        if (tile > 0) __syncthreads();                   // the tile before has been read
-#pragma unroll
-        for (int i = 0; i < kPieces; ++i) {
-            const int p = i * 256 + tid;
-            *(lds_u32x4_ptr)(lds + p / ((RK + DR) / 8) * kPitch + p % ((RK + DR) / 8) * 16) = reg[i];
+        const int blk_this = blk_next;
+        if (!ok) {                                       // (the whole workgroup skips it)
+            blk = blk_this;
+            blk_next = block_of(tile + 2);
+            if (tile + 1 < ntiles) fetch(tile + 1, blk);
+            continue;
         }
-        __syncthreads();
-        blk = blk_next;
-        if (tile + 1 < ntiles) fetch(tile + 1, blk);
-        blk_next = block_of(tile + 2);
-        if (!ok) continue;
-        f32x4_t s[NH][2];
+        f32x4_t s[NH][2];                                // two chains, added below
+        float x[NH][4];
 #pragma unroll
-        for (int kb = 0; kb < 2; ++kb) {
+        for (int h = 0; h < NH; ++h) s[h][0] = s[h][1] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int h = 0; h < NH; ++h) s[h][kb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        for (int ks = 0; ks < kAll; ++ks)
 #pragma unroll
-            for (int ks = 0; ks < kAll; ++ks) {
-                const u32x4_t kf = *(lds_u32x4_ptr)(kl + kb * 16 * kPitch + ks * 64);
-#pragma unroll
-                for (int h = 0; h < NH; ++h) s[h][kb] = mfma16(kf, qf[h][ks], s[h][kb]);
-            }
-        }
-        u32x4_t ph[NH], pl[NH];
+            for (int h = 0; h < NH; ++h) s[h][ks & 1] = mfma16(kf[ks], qf[h][ks], s[h][ks & 1]);
+        const int key = key0 + 16 * wave + 4 * g;
 #pragma unroll
         for (int h = 0; h < NH; ++h) {
             float mx = -INFINITY;
-            bool vis[2][4];
 #pragma unroll
-            for (int kb = 0; kb < 2; ++kb)
-#pragma unroll
-                for (int i = 0; i < 4; ++i) {
-                    const int key = key0 + 16 * kb + 4 * g + i;
-                    vis[kb][i] = key >= lo && key <= last;
-                    s[h][kb][i] *= to_exp2;
-                    if (vis[kb][i]) mx = fmaxf(mx, s[h][kb][i]);
-                }
+            for (int i = 0; i < 4; ++i) {
+                x[h][i] = key + i >= lo && key + i <= last ? (s[h][0][i] + s[h][1][i]) * to_exp2 : -INFINITY;
+                mx = fmaxf(mx, x[h][i]);
+            }
             mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
             mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-            if (__any(mx > m[h])) {
+            if (g == 0) sh_m[h][wave][r] = mx;
+        }
+        __syncthreads();                                 // maxima are there; the tile before has been read
+#pragma unroll
+        for (int ks = 0; ks < kKS; ++ks) *(lds_u32x4_ptr)(vw + 64 * ks) = kf[ks];
+        blk = blk_this;
+        blk_next = block_of(tile + 2);
+        if (tile + 1 < ntiles) fetch(tile + 1, blk);
+#pragma unroll
+        for (int h = 0; h < NH; ++h) {
+            const float mx = fmaxf(fmaxf(sh_m[h][0][r], sh_m[h][1][r]), fmaxf(sh_m[h][2][r], sh_m[h][3][r]));
+            if (__any(mx > m[h] + 8.0f)) {               // (the same in every wavefront)
                 const float m_new = fmaxf(m[h], mx);
                 const float keep = m[h] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m[h] - m_new);
                 m[h] = m_new;
@@ -361,46 +366,60 @@ __global__ __launch_bounds__(256, 2) void latent_rows_kernel(const LatentAttnArg
                     for (int i = 0; i < 4; ++i) oacc[h][db][i] *= keep;
             }
             const float ref = m[h] == -INFINITY ? 0.f : m[h];
+            float p[4];
 #pragma unroll
-            for (int kb = 0; kb < 2; ++kb) {
-                float p[4];
-#pragma unroll
-                for (int i = 0; i < 4; ++i) {
-                    p[i] = vis[kb][i] ? __builtin_amdgcn_exp2f(s[h][kb][i] - ref) : 0.f;
-                    lsum[h] += p[i];
-                }
-                uint32_t h0, l0, h1, l1;
-                split_pair(p[0], p[1], h0, l0);
-                split_pair(p[2], p[3], h1, l1);
-                ph[h][2 * kb] = h0; ph[h][2 * kb + 1] = h1;
-                pl[h][2 * kb] = l0; pl[h][2 * kb + 1] = l1;
+            for (int i = 0; i < 4; ++i) {
+                p[i] = __builtin_amdgcn_exp2f(x[h][i] - ref);
+                lsum[h] += p[i];
             }
+            uint32_t h0, l0, h1, l1;
+            split_pair(p[0], p[1], h0, l0);
+            split_pair(p[2], p[3], h1, l1);
+            sh_p[h][wave][lane] = u32x4_t{h0, h1, l0, l1};
         }
+        __syncthreads();
 #pragma unroll
-        for (int db = 0; db < kDB; ++db) {
-            const s16x4_t v0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_ptr)(vl + 32 * db));
-            const s16x4_t v1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_ptr)(vl + 16 * kPitch + 32 * db));
-            const u32x4_t vf = __builtin_bit_cast(u32x4_t, __builtin_shufflevector(v0, v1, 0, 1, 2, 3, 4, 5, 6, 7));
+        for (int st = 0; st < 2; ++st) {
+            u32x4_t ph[NH], pl[NH];
 #pragma unroll
             for (int h = 0; h < NH; ++h) {
-                oacc[h][db] = mfma16(vf, ph[h], oacc[h][db]);
-                oacc[h][db] = mfma16(vf, pl[h], oacc[h][db]);
+                const u32x4_t p0 = sh_p[h][2 * st][lane], p1 = sh_p[h][2 * st + 1][lane];
+                ph[h] = u32x4_t{p0[0], p0[1], p1[0], p1[1]};
+                pl[h] = u32x4_t{p0[2], p0[3], p1[2], p1[3]};
+            }
+#pragma unroll
+            for (int db = 0; db < kDB; ++db) {
+                const s16x4_t v0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_ptr)(vl + 32 * st * kPitch + 32 * db));
+                const s16x4_t v1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_ptr)(vl + (32 * st + 16) * kPitch + 32 * db));
+                const u32x4_t vf = __builtin_bit_cast(u32x4_t, __builtin_shufflevector(v0, v1, 0, 1, 2, 3, 4, 5, 6, 7));
+#pragma unroll
+                for (int h = 0; h < NH; ++h) {
+                    oacc[h][db] = mfma16(vf, ph[h], oacc[h][db]);
+                    oacc[h][db] = mfma16(vf, pl[h], oacc[h][db]);
+                }
             }
         }
     }
+    // sums of the weights: a wavefront's keys are spread over its lane groups, the tile's over the wavefronts
 #pragma unroll
     for (int h = 0; h < NH; ++h) {
         lsum[h] += __shfl_xor(lsum[h], 16, 64);
         lsum[h] += __shfl_xor(lsum[h], 32, 64);
+        if (g == 0) sh_l[h][wave][r] = lsum[h];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int h = 0; h < NH; ++h) {
         const int hh = 16 * h + r;
         if (hh >= nheads) continue;
+        const float l = (sh_l[h][0][r] + sh_l[h][1][r]) + (sh_l[h][2][r] + sh_l[h][3][r]);
         if (sp.splits == 1) {
             const float z = bf16_to_f32(static_cast<const bf16_t *>(a.gate)[t * a.gate_stride + head0 + hh]);
-            const float f = lsum[h] > 0.f ? sigmoid_of<bf16_t>(z) / lsum[h] : 0.f;
+            const float f = l > 0.f ? sigmoid_of<bf16_t>(z) / l : 0.f;
 #pragma unroll
             for (int db = 0; db < kDB; ++db) {
                 const int c = wave * (RK / 4) + 16 * db + 4 * g;
-                if (c < a.rank)
+                if (kExact || c < a.rank)
                     *reinterpret_cast<u32x2_t *>(out + hh * a.rank + c) = u32x2_t{pack_bf16x2(oacc[h][db][0] * f, oacc[h][db][1] * f), pack_bf16x2(oacc[h][db][2] * f, oacc[h][db][3] * f)};
             }
         } else {
@@ -408,24 +427,26 @@ __global__ __launch_bounds__(256, 2) void latent_rows_kernel(const LatentAttnArg
 #pragma unroll
             for (int db = 0; db < kDB; ++db) {
                 const int c = wave * (RK / 4) + 16 * db + 4 * g;
-                if (c < a.rank) *reinterpret_cast<f32x4_t *>(part + c) = oacc[h][db];
+                if (kExact || c < a.rank) *reinterpret_cast<f32x4_t *>(part + c) = oacc[h][db];
             }
-            if (wave == 0 && g == 0) { part[a.rank] = lsum[h]; part[a.rank + 1] = m[h]; }
+            if (wave == 0 && g == 0) { part[a.rank] = l; part[a.rank + 1] = m[h]; }
         }
     }
 }
 
-// One wavefront per (row, head): adds the partial results of the ranges that hold keys (at most 64).
-__global__ __launch_bounds__(256) void latent_merge_kernel(const LatentAttnArgs a, const LatentSplit sp) {
+// Adds the partial results of the ranges that hold keys (at most 64): one wavefront per 256 columns of a (row,
+// head), several ranges' loads in flight together.
+__global__ __launch_bounds__(256) void latent_merge_kernel(const LatentAttnArgs a, const LatentSplit sp, const int32_t pieces) {
     const int lane = threadIdx.x & 63;
-    const int64_t item = static_cast<int64_t>(blockIdx.x) * 4 + (threadIdx.x >> 6);
+    const int64_t job = static_cast<int64_t>(blockIdx.x) * 4 + (threadIdx.x >> 6);
+    const int64_t item = job / pieces;
     if (item >= static_cast<int64_t>(a.rows.n) * a.heads) return;
+    const int c = static_cast<int>(job % pieces) * 256 + 4 * lane;
     const int64_t t = item / a.heads;
     const int head = static_cast<int>(item % a.heads);
     int seq, pos;
     place_of(a.rows, t, seq, pos);
-    bf16_t *out = static_cast<bf16_t *>(a.out) + item * a.rank;
-    const int first = max(0, pos - a.window + 1) & ~31;
+    const int first = max(0, pos - a.window + 1) & ~(kRowTile - 1);
     const int count = pos < 0 ? 0 : min(sp.splits, (pos - first) / sp.keys + 1);
     const int pitch = a.rank + 4;
     const float *part = sp.partials + (t * sp.splits * a.heads + head) * pitch;
@@ -433,47 +454,58 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const LatentAttnArgs 
     // lane j holds sum and reference of range j
     const float my_l = lane < count ? part[lane * step + a.rank] : 0.f;
     const float my_m = lane < count ? part[lane * step + a.rank + 1] : -INFINITY;
+    const float z = bf16_to_f32(static_cast<const bf16_t *>(a.gate)[t * a.gate_stride + head]);
+    constexpr int kAhead = 8;
+    f32x4_t p[kAhead], o = {0.f, 0.f, 0.f, 0.f};
+    const bool in = c < a.rank;                          // (the rank is a multiple of 8)
+    auto fetch = [&](int j0) __attribute__((always_inline)) {
+#pragma unroll
+        for (int j = 0; j < kAhead; ++j)
+            if (in && j0 + j < count) p[j] = *reinterpret_cast<const f32x4_t *>(part + (j0 + j) * step + c);
+    };
+    fetch(0);
     const float top = wave_max(my_m);
     const float f = my_m == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(my_m - top);
     const float l = wave_sum(my_l * f);
-    const float z = bf16_to_f32(static_cast<const bf16_t *>(a.gate)[t * a.gate_stride + head]);
     const float inv = l > 0.f ? sigmoid_of<bf16_t>(z) / l : 0.f;
-    for (int c = 4 * lane; c < a.rank; c += 256) {       // (the rank is a multiple of 8)
-        f32x4_t o = {0.f, 0.f, 0.f, 0.f};
-        for (int j = 0; j < count; ++j) {
-            const f32x4_t p = *reinterpret_cast<const f32x4_t *>(part + j * step + c);
-            const float w = __shfl(f, j, 64);
+    for (int j0 = 0; j0 < count; j0 += kAhead) {
 #pragma unroll
-            for (int i = 0; i < 4; ++i) o[i] = fmaf(p[i], w, o[i]);
+        for (int j = 0; j < kAhead; ++j) {
+            const float w = __shfl(f, min(j0 + j, 63), 64);
+            if (j0 + j < count)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) o[i] = fmaf(p[j][i], w, o[i]);
         }
-        *reinterpret_cast<u32x2_t *>(out + c) = u32x2_t{pack_bf16x2(o[0] * inv, o[1] * inv), pack_bf16x2(o[2] * inv, o[3] * inv)};
+        if (j0 + kAhead < count) fetch(j0 + kAhead);
     }
+    if (in)
+        *reinterpret_cast<u32x2_t *>(static_cast<bf16_t *>(a.out) + item * a.rank + c) = u32x2_t{pack_bf16x2(o[0] * inv, o[1] * inv), pack_bf16x2(o[2] * inv, o[3] * inv)};
 }
 
 // How the keys of a row are split.  Depends on shapes only.
-static LatentSplit plan_latent(int32_t rows, int32_t heads, int32_t max_blocks, int32_t block_size, int32_t window) {
+static LatentSplit plan_latent(int32_t rows, int32_t heads, int32_t rank, int32_t max_blocks, int32_t block_size, int32_t window) {
     LatentSplit sp{};
-    const int nh = heads > 16 ? 2 : 1;
+    const int nh = heads > 16 && rank <= 256 ? 2 : 1;    // (two groups' registers do not fit beside a longer latent)
     sp.head_groups = (heads + 16 * nh - 1) / (16 * nh);
-    const int64_t most = std::min(static_cast<int64_t>(window), static_cast<int64_t>(max_blocks) * block_size) + 31;   // keys one row can see, from a multiple of 32 on
+    const int64_t most = std::min(static_cast<int64_t>(window), static_cast<int64_t>(max_blocks) * block_size) + kRowTile - 1;   // keys one row can see, from a tile's start on
     const int64_t want = std::max<int64_t>(1, 1024 / std::max<int64_t>(1, static_cast<int64_t>(rows) * sp.head_groups));
-    int64_t keys = std::max({static_cast<int64_t>(128), (most + want - 1) / want, (most + 63) / 64});
-    keys = (keys + 31) / 32 * 32;
+    int64_t keys = std::max({static_cast<int64_t>(256), (most + want - 1) / want, (most + 63) / 64});
+    keys = (keys + kRowTile - 1) / kRowTile * kRowTile;
     sp.keys = static_cast<int32_t>(keys);
     sp.splits = static_cast<int32_t>(std::max(static_cast<int64_t>(1), (most + keys - 1) / keys));
     return sp;
 }
 
-template <int RK, int DR>
+template <int RK, int DR, int NH, bool kExact>
 static int launch_latent_rows(const LatentAttnArgs &a, const LatentSplit &sp, hipStream_t s) {
-    const int64_t wgs = static_cast<int64_t>(a.rows.n) * sp.splits * sp.head_groups;
-    if (wgs > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
-    const dim3 grid(static_cast<uint32_t>(wgs)), block(256);
-    if (a.heads > 16) hipLaunchKernelGGL((latent_rows_kernel<RK, DR, 2>), grid, block, 0, s, a, sp);
-    else hipLaunchKernelGGL((latent_rows_kernel<RK, DR, 1>), grid, block, 0, s, a, sp);
+    const int64_t items = (static_cast<int64_t>(a.rows.n) * sp.splits + 7) / 8 * 8;
+    if (items * sp.head_groups > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
+    const dim3 block(256);
+    hipLaunchKernelGGL((latent_rows_kernel<RK, DR, NH, kExact>), dim3(static_cast<uint32_t>(items * sp.head_groups)), block, 0, s, a, sp);
     const int rc = launch_status();
     if (rc != NVA_OK || sp.splits == 1) return rc;
-    hipLaunchKernelGGL(latent_merge_kernel, dim3(static_cast<uint32_t>((static_cast<int64_t>(a.rows.n) * a.heads + 3) / 4)), block, 0, s, a, sp);
+    const int32_t pieces = (a.rank + 255) / 256;
+    hipLaunchKernelGGL(latent_merge_kernel, dim3(static_cast<uint32_t>((static_cast<int64_t>(a.rows.n) * a.heads * pieces + 3) / 4)), block, 0, s, a, sp, pieces);
     return launch_status();
 }
 
@@ -834,7 +866,7 @@ extern "C" size_t nva_latent_attn_workspace_bytes(int32_t n_tokens, int32_t num_
                                                   int32_t max_blocks, int32_t block_size, int32_t window, int32_t dtype) {
     if (n_tokens <= 0 || num_heads <= 0 || kv_rank <= 0 || rot_dim < 0 || max_blocks < 0 || block_size <= 0 || window <= 0) return 0;
     if (!nva::latent_rows_ok(kv_rank, rot_dim, dtype)) return 0;
-    const nva::LatentSplit sp = nva::plan_latent(n_tokens, num_heads, max_blocks, block_size, window);
+    const nva::LatentSplit sp = nva::plan_latent(n_tokens, num_heads, kv_rank, max_blocks, block_size, window);
     if (sp.splits == 1) return 0;
     return static_cast<size_t>(n_tokens) * sp.splits * num_heads * (kv_rank + 4) * sizeof(float);
 }
@@ -865,7 +897,7 @@ extern "C" int nva_latent_attn(const void *q_latent, const void *q_rot, int64_t 
     hipStream_t s = static_cast<hipStream_t>(stream);
     if (latent_rows_ok(kv_rank, rot_dim, dtype) && qr_row_stride % 8 == 0 && qr_head_stride % 8 == 0 && aligned16(q_latent) && aligned16(q_rot) &&
         aligned16(cache) && aligned16(out)) {
-        LatentSplit sp = plan_latent(n_tokens, num_heads, max_blocks, block_size, window);
+        LatentSplit sp = plan_latent(n_tokens, num_heads, kv_rank, max_blocks, block_size, window);
         sp.partials = static_cast<float *>(workspace);
         if (sp.splits > 1) {
             if (!workspace) return NVA_ERR_NULL_POINTER;
@@ -873,9 +905,11 @@ extern "C" int nva_latent_attn(const void *q_latent, const void *q_rot, int64_t 
             if (workspace_bytes < nva_latent_attn_workspace_bytes(n_tokens, num_heads, kv_rank, rot_dim, max_blocks, block_size, window, dtype))
                 return NVA_ERR_WORKSPACE_TOO_SMALL;
         }
-        if (kv_rank <= 128) return launch_latent_rows<128, 64>(a, sp, s);
-        if (kv_rank <= 256) return launch_latent_rows<256, 64>(a, sp, s);
-        return launch_latent_rows<512, 64>(a, sp, s);
+        const bool wide = num_heads > 16;
+        if (kv_rank == 512 && rot_dim == 64) return launch_latent_rows<512, 64, 1, true>(a, sp, s);
+        if (kv_rank <= 128) return wide ? launch_latent_rows<128, 64, 2, false>(a, sp, s) : launch_latent_rows<128, 64, 1, false>(a, sp, s);
+        if (kv_rank <= 256) return wide ? launch_latent_rows<256, 64, 2, false>(a, sp, s) : launch_latent_rows<256, 64, 1, false>(a, sp, s);
+        return launch_latent_rows<512, 64, 1, false>(a, sp, s);
     }
     const dim3 grid(static_cast<uint32_t>((static_cast<int64_t>(n_tokens) * num_heads + 3) / 4));
     if (dtype == NVA_DTYPE_BF16) hipLaunchKernelGGL((latent_attn_any_kernel<bf16_t>), grid, dim3(256), 0, s, a);
