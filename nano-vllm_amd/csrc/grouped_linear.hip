@@ -12,6 +12,7 @@
 #include <math.h>
 
 #include <algorithm>
+#include <type_traits>
 
 namespace nva {
 
@@ -87,42 +88,43 @@ __global__ __launch_bounds__(256) void linear_any_kernel(LinearArgs a) {
 }
 
 // ---- bf16, few rows per group: the weights are streamed once per 16 MT rows ------------------------
-// A workgroup takes 16 outputs of a group (16 gates and the 16 ups that belong to them), its four
+// A workgroup takes 16 NB outputs of a group (NB blocks of 16 gates and the 16 ups that belong to them), its four
 // wavefronts a quarter of the inner dimension each, weights and rows straight from memory into operands
 // (weights first operand: an accumulator holds four consecutive outputs of one row).  The quarters meet in LDS.
-template <int MT, bool kGated, typename O>
+template <int MT, int NB, bool kGated, typename O>
 __global__ __launch_bounds__(256) void linear_skinny_kernel(LinearArgs a) {
-    constexpr int kParts = kGated ? 2 : 1, kAhead = MT == 1 ? 8 : 4;
-    __shared__ __attribute__((aligned(16))) float part[4][MT * 16][kParts * 16 + 4];
-    const int g = blockIdx.y, n0 = blockIdx.x * 16;
+    constexpr int kParts = kGated ? 2 : 1, kBlocks = kParts * NB, kAhead = MT * NB == 1 ? 8 : 4;
+    __shared__ __attribute__((aligned(16))) float part[4][MT * 16][kBlocks * 16 + 4];
+    const int g = blockIdx.y, n0 = blockIdx.x * 16 * NB;
     const int tid = threadIdx.x, lane = tid & 63, r = lane & 15, q = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int count = group_rows(a, g);
     const int steps = (a.k + 31) / 32, per_wave = (steps + 3) / 4;
     const int s_begin = wave * per_wave, s_end = min(steps, s_begin + per_wave);
-    const bf16_t *w = static_cast<const bf16_t *>(a.w) + static_cast<int64_t>(g) * kParts * a.n_out * a.k +
-                      static_cast<int64_t>(min(n0 + r, a.n_out - 1)) * a.k;
-    const int64_t up = static_cast<int64_t>(a.n_out) * a.k;
+    const bf16_t *w[kBlocks];
+#pragma unroll
+    for (int b = 0; b < kBlocks; ++b)
+        w[b] = static_cast<const bf16_t *>(a.w) + (static_cast<int64_t>(g) * kParts * a.n_out + (b / NB) * a.n_out + min(n0 + 16 * (b % NB) + r, a.n_out - 1)) * a.k;
     for (int m0 = blockIdx.z * 16 * MT; m0 < count; m0 += gridDim.z * 16 * MT) {
         const bf16_t *x[MT];
 #pragma unroll
         for (int m = 0; m < MT; ++m)
             x[m] = static_cast<const bf16_t *>(a.x) + x_offset(a, g, group_row(a, g, min(m0 + 16 * m + r, count - 1)));
-        f32x4_t acc[MT][kParts];
+        f32x4_t acc[MT][kBlocks];
 #pragma unroll
         for (int m = 0; m < MT; ++m)
 #pragma unroll
-            for (int p = 0; p < kParts; ++p) acc[m][p] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+            for (int b = 0; b < kBlocks; ++b) acc[m][b] = f32x4_t{0.f, 0.f, 0.f, 0.f};
         for (int s0 = s_begin; s0 < s_end; s0 += kAhead) {
-            u32x4_t wf[kAhead][kParts], xf[kAhead][MT];
+            u32x4_t wf[kAhead][kBlocks], xf[kAhead][MT];
 #pragma unroll
             for (int j = 0; j < kAhead; ++j) {
                 const int e = (s0 + j) * 32 + 8 * q;
                 const bool in = s0 + j < s_end && e < a.k;
 #pragma unroll
-                for (int p = 0; p < kParts; ++p) {
-                    wf[j][p] = u32x4_t{0, 0, 0, 0};
-                    if (in) wf[j][p] = *reinterpret_cast<const u32x4_t *>(w + p * up + e);
+                for (int b = 0; b < kBlocks; ++b) {
+                    wf[j][b] = u32x4_t{0, 0, 0, 0};
+                    if (in) wf[j][b] = *reinterpret_cast<const u32x4_t *>(w[b] + e);
                 }
 #pragma unroll
                 for (int m = 0; m < MT; ++m) {
@@ -135,20 +137,20 @@ __global__ __launch_bounds__(256) void linear_skinny_kernel(LinearArgs a) {
 #pragma unroll
                 for (int m = 0; m < MT; ++m)
 #pragma unroll
-                    for (int p = 0; p < kParts; ++p) acc[m][p] = mfma16(wf[j][p], xf[j][m], acc[m][p]);
+                    for (int b = 0; b < kBlocks; ++b) acc[m][b] = mfma16(wf[j][b], xf[j][m], acc[m][b]);
         }
 #pragma unroll
         for (int m = 0; m < MT; ++m)
 #pragma unroll
-            for (int p = 0; p < kParts; ++p) *reinterpret_cast<f32x4_t *>(&part[wave][16 * m + r][16 * p + 4 * q]) = acc[m][p];
+            for (int b = 0; b < kBlocks; ++b) *reinterpret_cast<f32x4_t *>(&part[wave][16 * m + r][16 * b + 4 * q]) = acc[m][b];
         __syncthreads();
-        for (int i = tid; i < MT * 16 * 16; i += 256) {
-            const int m = i >> 4, n = i & 15;
+        for (int i = tid; i < MT * 16 * 16 * NB; i += 256) {
+            const int m = i / (16 * NB), n = i % (16 * NB);
             if (m0 + m >= count || n0 + n >= a.n_out) continue;
             float v[kParts];
 #pragma unroll
             for (int p = 0; p < kParts; ++p) {
-                const int c = 16 * p + n;
+                const int c = 16 * NB * p + n;
                 v[p] = (part[0][m][c] + part[1][m][c]) + (part[2][m][c] + part[3][m][c]);
             }
             static_cast<O *>(a.out)[out_offset(a, g, group_row(a, g, m0 + m)) + n0 + n] =
@@ -175,18 +177,22 @@ __global__ __launch_bounds__(256, 2) void linear_tile_kernel(const LinearArgs a,
     constexpr int kBlocksX = BM / 16, kBlocksW = kTileN / 16, kStage = (kBlocksX + kBlocksW) * 1024;
     constexpr int kLX = kBlocksX / 4, kLW = kBlocksW / 4;                       // blocks a wavefront loads per step
     __shared__ __attribute__((aligned(1024))) unsigned char smem[3 * kStage];
+    __shared__ int sh_row[BM];
     const int tid = threadIdx.x, lane = tid & 63, r = lane & 15, g = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int wm = wave & 1, wn = wave >> 1;
     // ---- which tile: row tiles of every expert, 64 experts at a time
-    int total = 0;
-    for (int e0 = 0; e0 < a.groups; e0 += 64) {
-        const int e = e0 + lane;
-        int t = e < a.groups ? (group_rows(a, e) + BM - 1) / BM : 0;
+    auto tiles_of = [&](int e) __attribute__((always_inline)) -> int { return e < a.groups ? (group_rows(a, e) + BM - 1) / BM : 0; };
+    auto up_to = [&](int t) __attribute__((always_inline)) -> int {
 #pragma unroll
-        for (int d = 1; d < 64; d <<= 1) t += __shfl_xor(t, d, 64);
-        total += t;
-    }
+        for (int d = 1; d < 64; d <<= 1) {
+            const int o = __shfl_up(t, d, 64);
+            if (lane >= d) t += o;
+        }
+        return t;
+    };
+    int own = tiles_of(lane), upto = up_to(own), total = __shfl(upto, 63, 64);
+    for (int e0 = 64; e0 < a.groups; e0 += 64) total += __shfl(up_to(tiles_of(e0 + lane)), 63, 64);
     total = __builtin_amdgcn_readfirstlane(total) * n_tiles;
     const int stretch = (total + 7) / 8;
     const int in_stretch = blockIdx.x / 8;
@@ -194,15 +200,7 @@ __global__ __launch_bounds__(256, 2) void linear_tile_kernel(const LinearArgs a,
     if (in_stretch >= stretch || tile >= total) return;
     const int n_tile = tile % n_tiles;
     int m_tile = tile / n_tiles, expert = 0;
-    for (int e0 = 0; e0 < a.groups; e0 += 64) {
-        const int e = e0 + lane;
-        const int own = e < a.groups ? (group_rows(a, e) + BM - 1) / BM : 0;
-        int upto = own;
-#pragma unroll
-        for (int d = 1; d < 64; d <<= 1) {
-            const int o = __shfl_up(upto, d, 64);
-            if (lane >= d) upto += o;
-        }
+    for (int e0 = 0;;) {
         const unsigned long long here = __ballot(m_tile < upto);
         if (here != 0) {
             const int first = __ffsll(here) - 1;
@@ -211,10 +209,15 @@ __global__ __launch_bounds__(256, 2) void linear_tile_kernel(const LinearArgs a,
             break;
         }
         m_tile -= __shfl(upto, 63, 64);
+        e0 += 64;                                        // (m_tile < total: one of the experts has it)
+        if (e0 >= a.groups) return;
+        own = tiles_of(e0 + lane);
+        upto = up_to(own);
     }
     expert = __builtin_amdgcn_readfirstlane(expert);
     m_tile = __builtin_amdgcn_readfirstlane(m_tile);
     const int count = group_rows(a, expert), m0 = m_tile * BM;
+    if (tid < BM) sh_row[tid] = group_row(a, expert, min(m0 + tid, count - 1));       // (published by the barriers below)
 
     // ---- what this wavefront loads: byte offsets of its lanes' pieces in the first step
     const int l16 = lane >> 2, piece = ((lane & 3) ^ ((0 - (l16 >> 2)) & 3)) * 8;
@@ -287,33 +290,37 @@ __global__ __launch_bounds__(256, 2) void linear_tile_kernel(const LinearArgs a,
         __syncthreads();
         buf = buf == 2 ? 0 : buf + 1;
     }
-    // ---- four consecutive outputs of a row per accumulator
+    // ---- through LDS into whole pieces of rows (an accumulator holds four consecutive outputs of one row)
+    constexpr int kCols = kGated ? 64 : kTileN, kOutPitch = kCols * 2 + 16, kPer = kCols / 8;
+    static_assert(BM * kOutPitch <= 3 * kStage, "the tile fits the operands' buffers");
 #pragma unroll
-    for (int m = 0; m < kTB; ++m) {
-        const int i = m0 + 16 * (wm * kTB + m) + r;
-        if (i >= count) continue;
-        bf16_t *out = static_cast<bf16_t *>(a.out) + out_offset(a, expert, group_row(a, expert, i));
+    for (int m = 0; m < kTB; ++m)
 #pragma unroll
         for (int n = 0; n < (kGated ? 2 : 4); ++n) {
-            const int c = kGated ? n_tile * 64 + 32 * wn + 16 * n + 4 * g : n_tile * kTileN + 64 * wn + 16 * n + 4 * g;
-            if (c >= a.n_out) continue;
             float y[4];
 #pragma unroll
             for (int j = 0; j < 4; ++j) y[j] = kGated ? silu_of<bf16_t>(acc[n][m][j]) * acc[kGated ? n + 2 : n][m][j] : acc[n][m][j];
-            *reinterpret_cast<u32x2_t *>(out + c) = u32x2_t{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
+            *(__attribute__((address_space(3))) u32x2_t *)(lds + (16 * (wm * kTB + m) + r) * kOutPitch + 2 * ((kGated ? 32 : 64) * wn + 16 * n + 4 * g)) =
+                u32x2_t{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
         }
-    }
+    __syncthreads();
+    const int c = tid % kPer * 8, n0 = n_tile * kCols + c, end = min(BM, count - m0);
+    if (n0 < a.n_out)
+#pragma unroll 4
+        for (int i = tid / kPer; i < end; i += 256 / kPer)               // (16-byte pieces)
+            *reinterpret_cast<u32x4_t *>(static_cast<bf16_t *>(a.out) + static_cast<int64_t>(sh_row[i]) * a.o_stride + n0) = *(lds_u32x4_ptr)(lds + i * kOutPitch + 2 * c);
 }
 
-// Sizes the tiled form is built for: whole steps, whole 8-byte stores, 32-bit offsets.
+// Sizes the tiled form is built for: whole steps, whole 16-byte stores, 32-bit offsets.
 static bool tiles_ok(const LinearArgs &a, bool gated, int32_t x_rows) {
-    return a.k % 32 == 0 && a.n_out % 4 == 0 && aligned16(a.out) && static_cast<int64_t>(x_rows) * a.x_stride < (1LL << 30) &&
+    return a.k % 32 == 0 && a.n_out % 8 == 0 && aligned16(a.out) && static_cast<int64_t>(x_rows) * a.x_stride < (1LL << 30) &&
            static_cast<int64_t>(a.n_out) * (gated ? 2 : 1) * a.k < (1LL << 30);
 }
 
 template <int BM, bool kGated>
 static int launch_tiles(const LinearArgs &a, hipStream_t s) {
-    const int32_t n_tiles = (a.n_out + (kGated ? 64 : kTileN) - 1) / (kGated ? 64 : kTileN);
+    constexpr int kCols = kGated ? kTileN / 2 : kTileN;
+    const int32_t n_tiles = (a.n_out + kCols - 1) / kCols;
     const int64_t most = (static_cast<int64_t>(a.rows) / BM + a.groups) * n_tiles;      // row tiles there can be, whatever the counts are
     const int64_t grid = (most + 7) / 8 * 8 + 8;
     if (grid > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
@@ -329,15 +336,21 @@ static int launch_any_linear(const LinearArgs &a, int32_t most_rows, hipStream_t
 }
 
 // rows_hint: rows a group is expected to have
-template <bool kGated, typename O>
-static int launch_skinny(const LinearArgs &a, int32_t rows_hint, int32_t most_rows, hipStream_t s) {
+template <int NB, bool kGated, typename O>
+static int launch_skinny_nb(const LinearArgs &a, int32_t rows_hint, int32_t most_rows, hipStream_t s) {
     const int mt = rows_hint <= 16 ? 1 : rows_hint <= 32 ? 2 : 4;
     const int passes = std::max(1, (most_rows + 16 * mt - 1) / (16 * mt));
-    const dim3 grid((a.n_out + 15) / 16, a.groups, a.lists ? 1 : std::min(passes, 65535)), block(256);
-    if (mt == 1) hipLaunchKernelGGL((linear_skinny_kernel<1, kGated, O>), grid, block, 0, s, a);
-    else if (mt == 2) hipLaunchKernelGGL((linear_skinny_kernel<2, kGated, O>), grid, block, 0, s, a);
-    else hipLaunchKernelGGL((linear_skinny_kernel<4, kGated, O>), grid, block, 0, s, a);
+    const dim3 grid((a.n_out + 16 * NB - 1) / (16 * NB), a.groups, a.lists ? 1 : std::min(passes, 65535)), block(256);
+    if (mt == 1) hipLaunchKernelGGL((linear_skinny_kernel<1, NB, kGated, O>), grid, block, 0, s, a);
+    else if (mt == 2) hipLaunchKernelGGL((linear_skinny_kernel<2, NB, kGated, O>), grid, block, 0, s, a);
+    else hipLaunchKernelGGL((linear_skinny_kernel<4, NB, kGated, O>), grid, block, 0, s, a);
     return launch_status();
+}
+template <bool kGated, typename O>
+static int launch_skinny(const LinearArgs &a, int32_t rows_hint, int32_t most_rows, int32_t busy_groups, hipStream_t s) {
+    // two blocks of outputs per workgroup where that leaves enough workgroups for the machine
+    if (static_cast<int64_t>(busy_groups) * ((a.n_out + 31) / 32) >= 512) return launch_skinny_nb<2, kGated, O>(a, rows_hint, most_rows, s);
+    return launch_skinny_nb<1, kGated, O>(a, rows_hint, most_rows, s);
 }
 
 static bool linear_matrix_ok(const LinearArgs &a) {
@@ -429,41 +442,63 @@ __global__ __launch_bounds__(512) void router_kernel(RouterArgs a) {
     // one wavefront per row: softmax over the experts, then the best one `top` times (ties: the lower index)
     for (int row = wave; row < rows; row += 8) {
         float *z = logits + row * a.experts;
-        float mx = -INFINITY;
-        for (int e = lane; e < a.experts; e += 64) mx = fmaxf(mx, z[e]);
+        float mine_z = -INFINITY, mx = -INFINITY;            // (up to 64 experts: one per lane)
+        const bool narrow = a.experts <= 64;
+        if (narrow) {
+            if (lane < a.experts) mine_z = z[lane];
+            mx = mine_z;
+        } else {
+            for (int e = lane; e < a.experts; e += 64) mx = fmaxf(mx, z[e]);
+        }
         mx = wave_max(mx);
         float sum = 0.f;
-        for (int e = lane; e < a.experts; e += 64) sum += exp_of<T>(z[e] - mx);
+        if (narrow) sum = exp_of<T>(mine_z - mx);
+        else for (int e = lane; e < a.experts; e += 64) sum += exp_of<T>(z[e] - mx);
         const float inv = 1.0f / wave_sum(sum);
-        const int64_t at = static_cast<int64_t>(row0 + row) * a.top;
-        float chosen = 0.f;
+        float chosen = 0.f, my_s = 0.f;                    // lane k keeps choice k (of every 64)
+        int my_who = 0;
         for (int k = 0; k < a.top; ++k) {
-            float best = -INFINITY;
-            int who = 0x7fffffff;
-            for (int e = lane; e < a.experts; e += 64)
-                if (z[e] > best) { best = z[e]; who = e; }
-#pragma unroll
-            for (int d = 1; d < 64; d <<= 1) {
-                const float ob = __shfl_xor(best, d, 64);
-                const int ow = __shfl_xor(who, d, 64);
-                if (ob > best || (ob == best && ow < who)) { best = ob; who = ow; }
+            float best = mine_z;
+            int who = lane;
+            if (!narrow) {
+                best = -INFINITY;
+                for (int e = lane; e < a.experts; e += 64)
+                    if (z[e] > best) { best = z[e]; who = e; }
             }
-            if (who >= a.experts) who = 0;                   // (only where logits are not numbers)
-            const float s = exp_of<T>(best - mx) * inv;
+            const float best_now = wave_max(best);
+            const unsigned long long at = __ballot(best == best_now);
+            int win;
+            if (narrow) win = at != 0 ? __ffsll(at) - 1 : 0;
+            else win = 1023 - static_cast<int>(wave_max(best == best_now ? static_cast<float>(1023 - who) : 0.f));
+            if (win >= a.experts) win = 0;                   // (only where logits are not numbers)
+            const float s = exp_of<T>(best_now - mx) * inv;
             chosen += s;
-            if (lane == 0) {
-                a.choice[at + k] = who;
-                a.weight[at + k] = s;                        // scaled below, by the same lane
-                mine[2 * (row * a.top + k)] = who;
-                mine[2 * (row * a.top + k) + 1] = atomicAdd(&have[who], 1);
-                z[who] = -INFINITY;
+            if (lane == k % 64) {
+                my_s = s;
+                my_who = win;
             }
-            __builtin_amdgcn_wave_barrier();
-            __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+            if (narrow) { if (lane == win) mine_z = -INFINITY; }
+            else {
+                if (lane == 0) z[win] = -INFINITY;
+                __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+            }
+            if (k % 64 == 63 || k == a.top - 1) {            // hand over up to 64 choices at once
+                const int kk = k / 64 * 64 + lane;
+                if (kk <= k) {
+                    mine[2 * (row * a.top + kk)] = my_who;
+                    mine[2 * (row * a.top + kk) + 1] = __float_as_int(my_s);
+                }
+            }
         }
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
         const float f = a.scale / (chosen + kWeightGuard);
-        if (lane == 0)
-            for (int k = 0; k < a.top; ++k) a.weight[at + k] *= f;
+        const int64_t at = static_cast<int64_t>(row0 + row) * a.top;
+        for (int k = lane; k < a.top; k += 64) {
+            const int who = mine[2 * (row * a.top + k)];
+            a.choice[at + k] = who;
+            a.weight[at + k] = __int_as_float(mine[2 * (row * a.top + k) + 1]) * f;
+            mine[2 * (row * a.top + k) + 1] = atomicAdd(&have[who], 1);
+        }
     }
     __syncthreads();
     for (int e = tid; e < a.experts; e += 512) base[e] = have[e] > 0 ? atomicAdd(&a.counts[e], have[e]) : 0;
@@ -508,7 +543,7 @@ extern "C" int nva_grouped_linear(const void *x, int64_t x_row_stride, int64_t x
     if (dtype == NVA_DTYPE_F32) return launch_any_linear<float, float, false>(a, rows, s);
     if (!linear_matrix_ok(a))
         return out_dtype == NVA_DTYPE_F32 ? launch_any_linear<bf16_t, float, false>(a, rows, s) : launch_any_linear<bf16_t, bf16_t, false>(a, rows, s);
-    return out_dtype == NVA_DTYPE_F32 ? launch_skinny<false, float>(a, rows, rows, s) : launch_skinny<false, bf16_t>(a, rows, rows, s);
+    return out_dtype == NVA_DTYPE_F32 ? launch_skinny<false, float>(a, rows, rows, groups, s) : launch_skinny<false, bf16_t>(a, rows, rows, groups, s);
 }
 
 extern "C" int nva_routed_linear(const void *x, int64_t x_row_stride, const void *weight, void *out, const int32_t *lists,
@@ -530,10 +565,11 @@ extern "C" int nva_routed_linear(const void *x, int64_t x_row_stride, const void
     if (!linear_matrix_ok(a)) return gated ? launch_any_linear<bf16_t, bf16_t, true>(a, rows, s) : launch_any_linear<bf16_t, bf16_t, false>(a, rows, s);
     const int32_t average = static_cast<int32_t>(static_cast<int64_t>(rows) * terms / experts);
     if (average >= 48 && tiles_ok(a, gated, x_per_row ? rows : rows * terms)) {
-        if (average >= 192) return gated ? launch_tiles<256, true>(a, s) : launch_tiles<256, false>(a, s);
+        if (average >= 512) return gated ? launch_tiles<256, true>(a, s) : launch_tiles<256, false>(a, s);
         return gated ? launch_tiles<128, true>(a, s) : launch_tiles<128, false>(a, s);
     }
-    return gated ? launch_skinny<true, bf16_t>(a, hint, rows, s) : launch_skinny<false, bf16_t>(a, hint, rows, s);
+    const int32_t busy = static_cast<int32_t>(std::min(static_cast<int64_t>(experts), static_cast<int64_t>(rows) * terms));
+    return gated ? launch_skinny<true, bf16_t>(a, hint, rows, busy, s) : launch_skinny<false, bf16_t>(a, hint, rows, busy, s);
 }
 
 extern "C" int nva_router(const void *x, int64_t x_row_stride, const void *weight, int32_t *choice, float *choice_weight,

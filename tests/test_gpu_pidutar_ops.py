@@ -112,7 +112,7 @@ def test_router_prefers_the_lower_index_of_equals(dev):
 
 @pytest.mark.parametrize("dtype", [BF16, F32])
 @pytest.mark.parametrize("shape", [(6, 2, 64, 40), (3, 3, 50, 27), (16, 4, 256, 128), (1, 1, 16, 24), (40, 6, 192, 48), (4, 2, 520, 200), (8, 2, 1024, 768), (5, 2, 256, 96), (70, 35, 64, 36)])
-@pytest.mark.parametrize("n", [1, 7, 60, 700, 1500])
+@pytest.mark.parametrize("n", [1, 7, 60, 700, 1500, 4100])
 def test_experts(dev, dtype, shape, n):
     """Both products and the weighted sum, with rows spread evenly and with (nearly) all of them at one expert."""
     n_experts, top, width, ff = shape
