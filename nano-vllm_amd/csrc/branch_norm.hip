@@ -63,9 +63,22 @@ __device__ __forceinline__ void new_residual(const BranchArgs &a, const T *xp, i
 #pragma unroll
         for (int i = 0; i < V; ++i) part[i] = 0.f;
         const T *yp = static_cast<const T *>(a.y2) + src * a.terms * a.width + e;
-#pragma unroll 4
-        for (int k = 0; k < a.terms; ++k) {
-            const float w = a.term_weight != nullptr ? a.term_weight[src * a.terms + k] : 1.0f;
+        const float *tw = a.term_weight != nullptr ? a.term_weight + src * a.terms : nullptr;
+        int k = 0;
+        for (; k + 4 <= a.terms; k += 4) {
+            float y[4][V], w[4];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                load_f32<T, V>(yp + static_cast<int64_t>(k + j) * a.width, y[j]);
+                w[j] = tw != nullptr ? tw[k + j] : 1.0f;
+            }
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+#pragma unroll
+                for (int i = 0; i < V; ++i) part[i] = fmaf(w[j], y[j][i], part[i]);
+        }
+        for (; k < a.terms; ++k) {
+            const float w = tw != nullptr ? tw[k] : 1.0f;
             load_f32<T, V>(yp + static_cast<int64_t>(k) * a.width, v);
 #pragma unroll
             for (int i = 0; i < V; ++i) part[i] = fmaf(w, v[i], part[i]);
@@ -79,12 +92,15 @@ __device__ __forceinline__ void new_residual(const BranchArgs &a, const T *xp, i
     for (int i = 0; i < V; ++i) r[i] = fmaf(a.mult, sum[i], r[i]);
 }
 
-// One wavefront per row, the row in registers; NC pieces of 512 elements (width % 8 == 0, width <= 4096).
-template <typename T, int NC, bool kEmbed>
+// The row in registers, 8 elements per access (width % 8 == 0, width <= 4096): WPR = 1, one wavefront per row, NC pieces of
+// 512 elements; WPR = 4 (few rows), a workgroup per row, NC pieces of 2048.
+template <typename T, int NC, int WPR, bool kEmbed>
 __global__ __launch_bounds__(256) void branch_norm_kernel(BranchArgs a) {
+    __shared__ float sh[4];
     clear_counters(a);
-    const int lane = threadIdx.x & 63;
-    const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
+    constexpr int kStep = 512 * WPR;
+    const int at0 = (threadIdx.x & (64 * WPR - 1)) * 8;
+    const int row = WPR == 1 ? blockIdx.x * 4 + (threadIdx.x >> 6) : blockIdx.x;
     if (row >= a.rows) return;
     const int64_t src = branch_source_row(a, row, kEmbed);
     int64_t xrow = src;
@@ -94,7 +110,7 @@ __global__ __launch_bounds__(256) void branch_norm_kernel(BranchArgs a) {
     float sq = 0.f;
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
-        const int e = c * 512 + lane * 8;
+        const int e = c * kStep + at0;
         if (e < a.width) {
             new_residual<T, 8, kEmbed>(a, xp, src, e, r[c]);
             if (kEmbed || a.rows_of == nullptr) store_f32<float, 8>(a.residual + src * a.width + e, r[c]);
@@ -102,11 +118,17 @@ __global__ __launch_bounds__(256) void branch_norm_kernel(BranchArgs a) {
             for (int i = 0; i < 8; ++i) sq = fmaf(r[c][i], r[c][i], sq);
         }
     }
-    const float rstd = rsqrtf(wave_sum(sq) / static_cast<float>(a.width) + a.eps);
+    sq = wave_sum(sq);
+    if (WPR > 1) {
+        if ((threadIdx.x & 63) == 0) sh[threadIdx.x >> 6] = sq;
+        __syncthreads();
+        sq = (sh[0] + sh[1]) + (sh[2] + sh[3]);
+    }
+    const float rstd = rsqrtf(sq / static_cast<float>(a.width) + a.eps);
     const int64_t at = static_cast<int64_t>(row) * a.width;
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
-        const int e = c * 512 + lane * 8;
+        const int e = c * kStep + at0;
         if (e < a.width) {
             float w[8], y[8];
             load_f32<T, 8>(static_cast<const T *>(a.w1) + e, w);
@@ -166,12 +188,18 @@ static int launch_branch_norm(const BranchArgs &a, hipStream_t s) {
         hipLaunchKernelGGL((branch_norm_any_kernel<T, kEmbed>), dim3(a.rows), dim3(256), 0, s, a);
         return launch_status();
     }
-    const dim3 grid((a.rows + 3) / 4), block(256);
+    const dim3 block(256);
+    if (a.rows <= 1024) {
+        if (a.width <= 2048) hipLaunchKernelGGL((branch_norm_kernel<T, 1, 4, kEmbed>), dim3(a.rows), block, 0, s, a);
+        else hipLaunchKernelGGL((branch_norm_kernel<T, 2, 4, kEmbed>), dim3(a.rows), block, 0, s, a);
+        return launch_status();
+    }
+    const dim3 grid((a.rows + 3) / 4);
     switch ((a.width + 511) / 512) {
-        case 1: hipLaunchKernelGGL((branch_norm_kernel<T, 1, kEmbed>), grid, block, 0, s, a); break;
-        case 2: hipLaunchKernelGGL((branch_norm_kernel<T, 2, kEmbed>), grid, block, 0, s, a); break;
-        case 3: case 4: hipLaunchKernelGGL((branch_norm_kernel<T, 4, kEmbed>), grid, block, 0, s, a); break;
-        default: hipLaunchKernelGGL((branch_norm_kernel<T, 8, kEmbed>), grid, block, 0, s, a); break;
+        case 1: hipLaunchKernelGGL((branch_norm_kernel<T, 1, 1, kEmbed>), grid, block, 0, s, a); break;
+        case 2: hipLaunchKernelGGL((branch_norm_kernel<T, 2, 1, kEmbed>), grid, block, 0, s, a); break;
+        case 3: case 4: hipLaunchKernelGGL((branch_norm_kernel<T, 4, 1, kEmbed>), grid, block, 0, s, a); break;
+        default: hipLaunchKernelGGL((branch_norm_kernel<T, 8, 1, kEmbed>), grid, block, 0, s, a); break;
     }
     return launch_status();
 }

@@ -371,12 +371,12 @@ struct RouterArgs {
     float scale;
 };
 
-// 16 TG rows per workgroup of eight wavefronts; KS = 8 / TG wavefronts share a group's inner dimension.
+// 16 TG rows per workgroup of NW wavefronts; KS = NW / TG wavefronts share a group's inner dimension.
 constexpr float kWeightGuard = 1e-20f;
 
-template <typename T, int TG, bool kMatrix>
-__global__ __launch_bounds__(512) void router_kernel(RouterArgs a) {
-    constexpr int KS = 8 / TG, kRows = 16 * TG;
+template <typename T, int TG, int NW, bool kMatrix>
+__global__ __launch_bounds__(64 * NW) void router_kernel(RouterArgs a) {
+    constexpr int KS = NW / TG, kRows = 16 * TG, kThreads = 64 * NW;
     extern __shared__ __attribute__((aligned(16))) unsigned char router_smem[];
     float *logits = reinterpret_cast<float *>(router_smem);                    // [kRows][experts]
     float *partial = logits + kRows * a.experts;                               // [KS][kRows][64 + 4] (matrix form)
@@ -387,7 +387,7 @@ __global__ __launch_bounds__(512) void router_kernel(RouterArgs a) {
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int row0 = blockIdx.x * kRows;
     const int rows = min(kRows, a.rows - row0);
-    for (int e = tid; e < a.experts; e += 512) have[e] = 0;
+    for (int e = tid; e < a.experts; e += kThreads) have[e] = 0;
     if constexpr (kMatrix) {
         const int tg = wave / KS, part = wave % KS;
         const int steps = (a.width + 31) / 32, per = (steps + KS - 1) / KS;
@@ -402,7 +402,6 @@ __global__ __launch_bounds__(512) void router_kernel(RouterArgs a) {
                 acc[b] = f32x4_t{0.f, 0.f, 0.f, 0.f};
                 w[b] = static_cast<const bf16_t *>(a.w) + static_cast<int64_t>(min(e0 + 16 * b + r, a.experts - 1)) * a.width;
             }
-#pragma unroll 4
             for (int s = s_begin; s < s_end; ++s) {
                 const int e = s * 32 + 8 * q;
                 const bool in = e < a.width;
@@ -418,7 +417,7 @@ __global__ __launch_bounds__(512) void router_kernel(RouterArgs a) {
 #pragma unroll
             for (int b = 0; b < 4; ++b) *reinterpret_cast<f32x4_t *>(partial + (part * kRows + 16 * tg + r) * 68 + 16 * b + 4 * q) = acc[b];
             __syncthreads();
-            for (int i = tid; i < kRows * 64; i += 512) {
+            for (int i = tid; i < kRows * 64; i += kThreads) {
                 const int row = i >> 6, e = i & 63;
                 if (e0 + e >= a.experts) continue;
                 float z = 0.f;
@@ -429,7 +428,7 @@ __global__ __launch_bounds__(512) void router_kernel(RouterArgs a) {
             __syncthreads();
         }
     } else {
-        for (int i = tid; i < rows * a.experts; i += 512) {
+        for (int i = tid; i < rows * a.experts; i += kThreads) {
             const int row = i / a.experts, e = i % a.experts;
             const T *x = static_cast<const T *>(a.x) + static_cast<int64_t>(row0 + row) * a.x_stride;
             const T *w = static_cast<const T *>(a.w) + static_cast<int64_t>(e) * a.width;
@@ -440,7 +439,7 @@ __global__ __launch_bounds__(512) void router_kernel(RouterArgs a) {
         __syncthreads();
     }
     // one wavefront per row: softmax over the experts, then the best one `top` times (ties: the lower index)
-    for (int row = wave; row < rows; row += 8) {
+    for (int row = wave; row < rows; row += NW) {
         float *z = logits + row * a.experts;
         float mine_z = -INFINITY, mx = -INFINITY;            // (up to 64 experts: one per lane)
         const bool narrow = a.experts <= 64;
@@ -501,26 +500,31 @@ __global__ __launch_bounds__(512) void router_kernel(RouterArgs a) {
         }
     }
     __syncthreads();
-    for (int e = tid; e < a.experts; e += 512) base[e] = have[e] > 0 ? atomicAdd(&a.counts[e], have[e]) : 0;
+    const bool alone = gridDim.x == 1;                       // nobody else adds to the counters
+    for (int e = tid; e < a.experts; e += kThreads) {
+        base[e] = 0;
+        if (alone) a.counts[e] = have[e];
+        else if (have[e] > 0) base[e] = atomicAdd(&a.counts[e], have[e]);
+    }
     __syncthreads();
-    for (int i = tid; i < rows * a.top; i += 512) {
+    for (int i = tid; i < rows * a.top; i += kThreads) {
         const int e = mine[2 * i], place = base[e] + mine[2 * i + 1];
         if (place < a.list_stride) a.lists[e * a.list_stride + place] = row0 * a.top + i;
     }
 }
 
-static size_t router_lds(int32_t experts, int32_t top, int tg, bool matrix) {
+static size_t router_lds(int32_t experts, int32_t top, int tg, int nw, bool matrix) {
     const size_t rows = 16 * static_cast<size_t>(tg);
-    return 4 * (rows * experts + (matrix ? 8 / tg * rows * 68 : 0) + 2 * static_cast<size_t>(experts) + 2 * rows * top);
+    return 4 * (rows * experts + (matrix ? nw / tg * rows * 68 : 0) + 2 * static_cast<size_t>(experts) + 2 * rows * top);
 }
 
-template <typename T, int TG, bool kMatrix>
+template <typename T, int TG, int NW, bool kMatrix>
 static int launch_router_tg(const RouterArgs &a, hipStream_t s) {
-    const size_t lds = router_lds(a.experts, a.top, TG, kMatrix);
+    const size_t lds = router_lds(a.experts, a.top, TG, NW, kMatrix);
     if (lds > 64 * 1024 &&
-        hipFuncSetAttribute(reinterpret_cast<const void *>(&router_kernel<T, TG, kMatrix>), hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds)) != hipSuccess)
+        hipFuncSetAttribute(reinterpret_cast<const void *>(&router_kernel<T, TG, NW, kMatrix>), hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds)) != hipSuccess)
         return NVA_ERR_LAUNCH_FAILED;
-    hipLaunchKernelGGL((router_kernel<T, TG, kMatrix>), dim3((a.rows + 16 * TG - 1) / (16 * TG)), dim3(512), lds, s, a);
+    hipLaunchKernelGGL((router_kernel<T, TG, NW, kMatrix>), dim3((a.rows + 16 * TG - 1) / (16 * TG)), dim3(64 * NW), lds, s, a);
     return launch_status();
 }
 
@@ -587,7 +591,8 @@ extern "C" int nva_router(const void *x, int64_t x_row_stride, const void *weigh
     a.list_stride = list_stride; a.rows = rows; a.width = width; a.experts = experts; a.top = top; a.scale = scale;
     hipStream_t s = static_cast<hipStream_t>(stream);
     const bool many = rows >= 4096 && experts <= 128 && top <= 32;       // more rows per workgroup: fewer additions to the counters
-    if (dtype == NVA_DTYPE_F32) return launch_router_tg<float, 1, false>(a, s);
-    if (width % 8 != 0 || x_row_stride % 8 != 0 || !aligned16(x) || !aligned16(weight)) return launch_router_tg<bf16_t, 1, false>(a, s);
-    return many ? launch_router_tg<bf16_t, 4, true>(a, s) : launch_router_tg<bf16_t, 1, true>(a, s);
+    if (dtype == NVA_DTYPE_F32) return launch_router_tg<float, 1, 8, false>(a, s);
+    if (width % 8 != 0 || x_row_stride % 8 != 0 || !aligned16(x) || !aligned16(weight)) return launch_router_tg<bf16_t, 1, 8, false>(a, s);
+    if (many) return launch_router_tg<bf16_t, 4, 8, true>(a, s);
+    return rows <= 1024 && experts <= 256 ? launch_router_tg<bf16_t, 1, 16, true>(a, s) : launch_router_tg<bf16_t, 1, 8, true>(a, s);
 }

@@ -489,7 +489,8 @@ static LatentSplit plan_latent(int32_t rows, int32_t heads, int32_t rank, int32_
     sp.head_groups = (heads + 16 * nh - 1) / (16 * nh);
     const int64_t most = std::min(static_cast<int64_t>(window), static_cast<int64_t>(max_blocks) * block_size) + kRowTile - 1;   // keys one row can see, from a tile's start on
     const int64_t want = std::max<int64_t>(1, 1024 / std::max<int64_t>(1, static_cast<int64_t>(rows) * sp.head_groups));
-    int64_t keys = std::max({static_cast<int64_t>(256), (most + want - 1) / want, (most + 63) / 64});
+    const int64_t least = static_cast<int64_t>(rows) * sp.head_groups <= 32 ? 128 : 256;
+    int64_t keys = std::max({least, (most + want - 1) / want, (most + 63) / 64});
     keys = (keys + kRowTile - 1) / kRowTile * kRowTile;
     sp.keys = static_cast<int32_t>(keys);
     sp.splits = static_cast<int32_t>(std::max(static_cast<int64_t>(1), (most + keys - 1) / keys));

@@ -8,6 +8,7 @@ from dataclasses import dataclass
 from typing import Tuple
 
 import torch
+import torch.nn.functional as F
 from torch import nn
 
 from .. import _lib
@@ -29,6 +30,17 @@ def grouped_linear(x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor) -> 
 def linear_f32(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
     """``x @ weight.T`` with few outputs, kept in fp32."""
     out = torch.empty((x.shape[0], weight.shape[0]), dtype=torch.float32, device=x.device)
+    grouped_linear(x[:, None], weight[None], out[:, None])
+    return out
+
+
+def project(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """``x @ weight.T``: the library's product, or for few rows the kernel that streams the weights once, where it is faster."""
+    n, k = x.shape
+    few = n <= 16 and weight.numel() <= 1 << 24 or n <= 64 and k <= 1024
+    if not few or x.dtype != torch.bfloat16:
+        return F.linear(x, weight)
+    out = torch.empty((n, weight.shape[0]), dtype=x.dtype, device=x.device)
     grouped_linear(x[:, None], weight[None], out[:, None])
     return out
 

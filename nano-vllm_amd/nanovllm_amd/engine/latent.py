@@ -17,7 +17,7 @@ from torch import nn
 
 from .. import _lib
 from ..context import RowGroup, get_context
-from .experts import grouped_linear
+from .experts import grouped_linear, project
 from .mixers import _DTYPE, Rotary, RopeTables, _ptr, _stream, scratch
 
 EXPAND_FROM = 32                 # rows a gathered key has to serve on average before multiplying it out pays
@@ -185,14 +185,14 @@ class LatentAttention:
     def __call__(self, h: torch.Tensor) -> torch.Tensor:
         s, w, n = self.spec, self.weights, h.shape[0]
         cache = self.cache if self.source is None else self.source.cache
-        down = F.linear(h, w.down)
+        down = project(h, w.down)
         gate = down[:, s.down_rows - s.heads: s.down_rows]
         empty = lambda *shape: torch.empty(shape, dtype=h.dtype, device=h.device)
         q_latent, o = empty(n, s.q_rank), empty(n, s.heads * s.vdim)
         groups = [(g, slice(g.first, g.first + g.count)) for g in get_context().groups]
         for group, rows in groups:
             latent_prepare(down[rows], w.q_norm, w.kv_norm, self.rope, q_latent[rows], self.cache, group, s.rot_dim, self.eps)
-        q = F.linear(q_latent, w.uq)
+        q = project(q_latent, w.uq)
         expands = h.dtype == torch.bfloat16 and _lib.load_latent().nva_latent_prefill_supported(s.dim, s.rot_dim, s.vdim, _DTYPE[h.dtype])
         for group, rows in groups:
             keys = visible_keys(group, s.window, h.device) if expands else None
@@ -207,4 +207,4 @@ class LatentAttention:
             mixed = empty(group.count, s.heads, s.kv_rank)
             latent_attention(met, heads[..., s.dim:], gate[rows], self.rope, cache, group, mixed, s.window, s.scale)
             grouped_linear(mixed, w.uv, o[rows].view(-1, s.heads, s.vdim))
-        return F.linear(o, w.o)
+        return project(o, w.o)

@@ -4,12 +4,11 @@ from __future__ import annotations
 from dataclasses import dataclass
 
 import torch
-import torch.nn.functional as F
 from torch import nn
 
 from .. import _lib
 from ..context import RowGroup, get_context
-from .experts import linear_f32
+from .experts import linear_f32, project
 from .mixers import _DTYPE, _ptr, _stream, scratch
 
 
@@ -87,9 +86,9 @@ class Mlstm:
 
     def __call__(self, h: torch.Tensor) -> torch.Tensor:
         s, w = self.spec, self.weights
-        qkvg, gates = F.linear(h, w.qkvg), linear_f32(h, w.gates)
+        qkvg, gates = project(h, w.qkvg), linear_f32(h, w.gates)
         o = torch.empty((h.shape[0], s.heads * s.vdim), dtype=h.dtype, device=h.device)
         for group in get_context().groups:
             rows = slice(group.first, group.first + group.count)
             mlstm(qkvg[rows], gates[rows], w.gate_bias, w.norm, self.state, self.mass, self.top, group, o[rows], s.dim ** -0.5, s.gate_cap, self.eps)
-        return F.linear(o, w.o)
+        return project(o, w.o)

@@ -331,8 +331,9 @@ def test_latent_attention_validation_and_workspace():
         assert _with(ok, lib.nva_latent_prepare, **kw) == rc, kw
     ws = lib.nva_latent_attn_workspace_bytes
     assert ws(2000, 16, 512, 64, 16, 256, 4096, 0) == 0               # enough rows for the machine: one range of keys each
-    assert ws(1, 16, 512, 64, 16, 256, 1 << 20, 0) == 17 * 16 * 516 * 4   # 4096 keys and up to 63 before a multiple of 64, ranges of 256
-    assert ws(1, 16, 512, 64, 16, 256, 90, 0) == 0 and ws(1, 16, 512, 64, 16, 256, 4096, 1) == 0 and ws(1, 16, 516, 64, 16, 256, 4096, 0) == 0
+    assert ws(1, 16, 512, 64, 16, 256, 1 << 20, 0) == 33 * 16 * 516 * 4   # 4096 keys and up to 63 before a multiple of 64, ranges of 128
+    assert ws(40, 16, 512, 64, 16, 256, 1 << 20, 0) == 40 * 17 * 16 * 516 * 4
+    assert ws(1, 16, 512, 64, 16, 256, 60, 0) == 0 and ws(1, 16, 512, 64, 16, 256, 4096, 1) == 0 and ws(1, 16, 516, 64, 16, 256, 4096, 0) == 0
     ok = dict(ql=A, qr=A, qrs=3072, qrh=192, gate=A, gs=16, rope=A, cache=A, bt=A, bts=16, mb=16, cu=None, lens=A, tseq=None, out=A, ws=A, wsb=1 << 30,
               n=8, seqs=8, heads=16, rank=512, rot=64, bs=256, nb=64, window=4096, max_pos=4096, scale=0.1, dtype=0, stream=None)
     for kw, rc in ((dict(ql=None), _lib.ERR_NULL_POINTER), (dict(qr=None), _lib.ERR_NULL_POINTER), (dict(ws=None), _lib.ERR_NULL_POINTER),
