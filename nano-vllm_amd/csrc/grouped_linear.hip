@@ -160,23 +160,44 @@ __global__ __launch_bounds__(256) void linear_skinny_kernel(LinearArgs a) {
     }
 }
 
-// ---- bf16, many rows per expert: tiles of BM rows x 128 weight rows ---------------------------------
-// Routed only.  A workgroup of four wavefronts (2 x 2) takes BM assignments of one expert and 128 rows of its weights
-// (gated: 64 gates and the 64 ups that belong to them, side by side in every wavefront).  Both operands travel
-// global -> LDS without a register in between, in steps of 32 inner elements through three buffers: while one
-// step is multiplied the next one has landed or is about to and the one after it is on its way, and the wait
-// before the barrier leaves those loads in flight.  The LDS image is made of 1 KB blocks of 16 rows x 32 elements with the
-// 16-byte pieces of a row permuted so that operand reads spread over the banks.
-// Tiles are numbered expert by expert, weight tiles fastest, and dealt out so that each XCD walks one
-// stretch of that order: neighbours share rows or weights in its L2.
-constexpr int kTileN = 128;
+// ---- bf16, many rows per expert: tiles of BM rows x BN weight rows ----------------------------------
+// Routed only.  A workgroup of four wavefronts (2 x 2) takes BM assignments of one expert and BN rows of its weights
+// (gated: BN / 2 gates and the ups that belong to them, side by side in every wavefront).  Both operands travel
+// global -> LDS without a register in between, in steps of 32 inner elements, and the wait before a barrier leaves
+// later steps' loads in flight.  The LDS image is made of 1 KB blocks of 16 rows x 32 elements with the 16-byte pieces
+// of a row permuted so that operand reads spread over the banks.  A CU gets some 18 bytes a clock out of the L2 for
+// this, so the product per byte decides: 256 x 256 (one workgroup per CU, accumulators in accumulation registers, four
+// buffers, a step's operands read while the step before it is multiplied) where there are enough rows and steps;
+// otherwise 128 columns, three buffers and two or three workgroups per CU that cover for one another.
+// Tiles are numbered expert by expert, eight row tiles abreast, and dealt out so that each XCD walks one stretch of that
+// order: what runs together on it is about as many row tiles as weight tiles, which its L2 serves to all.
+constexpr int kGroup = 8;
 
-template <int BM, bool kGated>
-__global__ __launch_bounds__(256, 2) void linear_tile_kernel(const LinearArgs a, const int32_t n_tiles) {
-    constexpr int kTB = BM / 32;                         // blocks of 16 rows per wavefront
-    constexpr int kBlocksX = BM / 16, kBlocksW = kTileN / 16, kStage = (kBlocksX + kBlocksW) * 1024;
-    constexpr int kLX = kBlocksX / 4, kLW = kBlocksW / 4;                       // blocks a wavefront loads per step
-    __shared__ __attribute__((aligned(1024))) unsigned char smem[3 * kStage];
+// Products of large tiles: the accumulators are asked for in accumulation registers, where the compiler would move
+// them to and fro.  Nothing is known about the latency of these: products_done() before the results are read.
+__device__ __forceinline__ void mfma16_in_place(const u32x4_t &x, const u32x4_t &y, f32x4_t &c) {
+    asm("v_mfma_f32_16x16x32_bf16 %0, %1, %2, %0" : "+a"(c) : "v"(x), "v"(y));
+}
+template <int A, int B>
+__device__ __forceinline__ void products_done(f32x4_t (&c)[A][B]) {
+    auto tie = [&]() __attribute__((always_inline)) {        // neither products nor reads of their results cross it
+#pragma unroll
+        for (int i = 0; i < A; ++i)
+#pragma unroll
+            for (int j = 0; j < B; ++j) asm volatile("" : "+a"(c[i][j]));
+    };
+    tie();
+    asm volatile("s_nop 15\n\ts_nop 15" ::: "memory");
+    tie();
+}
+
+template <int BM, int BN, bool kGated>
+__global__ __launch_bounds__(256, BN > 128 ? 1 : 2) void linear_tile_kernel(const LinearArgs a, const int32_t n_tiles) {
+    constexpr bool kWide = BN > 128;
+    constexpr int kTM = BM / 32, kTN = BN / 32;          // blocks of 16 per wavefront
+    constexpr int kBlocksX = BM / 16, kBlocksW = BN / 16, kStage = (kBlocksX + kBlocksW) * 1024, kBuffers = kWide ? 4 : 3;
+    constexpr int kLX = kBlocksX / 4, kLW = kBlocksW / 4, kLoads = kLX + kLW;   // blocks a wavefront loads per step
+    __shared__ __attribute__((aligned(1024))) unsigned char smem[kBuffers * kStage];
     __shared__ int sh_row[BM];
     const int tid = threadIdx.x, lane = tid & 63, r = lane & 15, g = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -198,14 +219,14 @@ __global__ __launch_bounds__(256, 2) void linear_tile_kernel(const LinearArgs a,
     const int in_stretch = blockIdx.x / 8;
     const int tile = blockIdx.x % 8 * stretch + in_stretch;
     if (in_stretch >= stretch || tile >= total) return;
-    const int n_tile = tile % n_tiles;
-    int m_tile = tile / n_tiles, expert = 0;
+    int m_tile = tile / n_tiles, expert = 0, m_tiles = 0;        // (first as if weight tiles were fastest, to find the expert)
     for (int e0 = 0;;) {
         const unsigned long long here = __ballot(m_tile < upto);
         if (here != 0) {
             const int first = __ffsll(here) - 1;
             expert = e0 + first;
-            m_tile -= __shfl(upto, first, 64) - __shfl(own, first, 64);
+            m_tiles = __shfl(own, first, 64);
+            m_tile -= __shfl(upto, first, 64) - m_tiles;
             break;
         }
         m_tile -= __shfl(upto, 63, 64);
@@ -215,7 +236,13 @@ __global__ __launch_bounds__(256, 2) void linear_tile_kernel(const LinearArgs a,
         upto = up_to(own);
     }
     expert = __builtin_amdgcn_readfirstlane(expert);
-    m_tile = __builtin_amdgcn_readfirstlane(m_tile);
+    m_tiles = __builtin_amdgcn_readfirstlane(m_tiles);
+    // up to kGroup row tiles side by side, then the next weight tile
+    const int at_expert = __builtin_amdgcn_readfirstlane(m_tile) * n_tiles + tile % n_tiles;
+    const int group = at_expert / (kGroup * n_tiles), in_group = at_expert % (kGroup * n_tiles);
+    const int abreast = min(kGroup, m_tiles - group * kGroup);
+    const int n_tile = in_group / abreast;
+    m_tile = group * kGroup + in_group % abreast;
     const int count = group_rows(a, expert), m0 = m_tile * BM;
     if (tid < BM) sh_row[tid] = group_row(a, expert, min(m0 + tid, count - 1));       // (published by the barriers below)
 
@@ -227,10 +254,10 @@ __global__ __launch_bounds__(256, 2) void linear_tile_kernel(const LinearArgs a,
         xoff[i] = static_cast<uint32_t>(x_offset(a, expert, group_row(a, expert, min(m0 + 16 * (wave * kLX + i) + l16, count - 1))) + piece) * 2;
 #pragma unroll
     for (int i = 0; i < kLW; ++i) {
-        const int row = 16 * (wave * kLW + i) + l16;     // of the tile; gated: 32 gates, their 32 ups, twice
+        const int row = 16 * (wave * kLW + i) + l16;     // of the tile; gated: BN / 4 gates, their ups, twice
         int n;
-        if (kGated) n = min(n_tile * 64 + row / 64 * 32 + row % 32, a.n_out - 1) + (row % 64 < 32 ? 0 : a.n_out);
-        else n = min(n_tile * kTileN + row, a.n_out - 1);
+        if (kGated) n = min(n_tile * (BN / 2) + row / (BN / 2) * (BN / 4) + row % (BN / 4), a.n_out - 1) + (row % (BN / 2) < BN / 4 ? 0 : a.n_out);
+        else n = min(n_tile * BN + row, a.n_out - 1);
         woff[i] = static_cast<uint32_t>(n * static_cast<int64_t>(a.k) + piece) * 2;
     }
     const char *xb = static_cast<const char *>(a.x);
@@ -245,70 +272,113 @@ __global__ __launch_bounds__(256, 2) void linear_tile_kernel(const LinearArgs a,
 #pragma unroll
         for (int i = 0; i < kLW; ++i) load_to_lds_16(w, woff[i], at + (kBlocksX + wave * kLW + i) * 1024);
     };
-    // the loads above are ordinary instructions to the compiler: these two keep them on their side of a barrier
-    auto after_barrier = [&]() __attribute__((always_inline)) {
+    // the loads above are ordinary instructions to the compiler: this keeps them on their side of a barrier
+    auto fence_loads = [&]() __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < kLX; ++i) asm volatile("" : "+v"(xoff[i]));
 #pragma unroll
         for (int i = 0; i < kLW; ++i) asm volatile("" : "+v"(woff[i]));
     };
-
-    f32x4_t acc[4][kTB];
-#pragma unroll
-    for (int n = 0; n < 4; ++n)
-#pragma unroll
-        for (int m = 0; m < kTB; ++m) acc[n][m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    // what step + kBuffers - 2 and later steps have asked for may still be on its way
     const int steps = a.k / 32;
-    const lds_char_ptr frag = lds + 16 * (4 * r + (g ^ ((0 - (r >> 2)) & 3)));
-    fetch(0, 0);
-    after_barrier();
-    if (steps > 1) {
-        fetch(1, 1);
-        after_barrier();
-        asm volatile("s_waitcnt vmcnt(%0)" :: "i"(kLX + kLW) : "memory");
-    } else {
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    }
-    __syncthreads();
-    int buf = 0;
-    for (int step = 0; step < steps; ++step) {
-        after_barrier();
-        if (step + 2 < steps) fetch(step + 2, buf == 0 ? 2 : buf - 1);          // (the buffer of the step before this one)
-        const lds_char_ptr xl = frag + buf * kStage + wm * kTB * 1024, wl = frag + buf * kStage + (kBlocksX + wn * 4) * 1024;
-        u32x4_t wf[4];
-#pragma unroll
-        for (int n = 0; n < 4; ++n) wf[n] = *(lds_u32x4_ptr)(wl + n * 1024);
-#pragma unroll
-        for (int m = 0; m < kTB; ++m) {
-            const u32x4_t xf = *(lds_u32x4_ptr)(xl + m * 1024);
-#pragma unroll
-            for (int n = 0; n < 4; ++n) acc[n][m] = mfma16(wf[n], xf, acc[n][m]);
-        }
-        after_barrier();
-        if (step + 2 < steps) asm volatile("s_waitcnt vmcnt(%0)" :: "i"(kLX + kLW) : "memory");
+    auto landed = [&](int step) __attribute__((always_inline)) {
+        fence_loads();
+        if (step + 1 < steps) asm volatile("s_waitcnt vmcnt(%0)" :: "i"(kLoads) : "memory");
         else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         __syncthreads();
-        buf = buf == 2 ? 0 : buf + 1;
-    }
-    // ---- through LDS into whole pieces of rows (an accumulator holds four consecutive outputs of one row)
-    constexpr int kCols = kGated ? 64 : kTileN, kOutPitch = kCols * 2 + 16, kPer = kCols / 8;
-    static_assert(BM * kOutPitch <= 3 * kStage, "the tile fits the operands' buffers");
+        fence_loads();
+    };
+
+    f32x4_t acc[kTN][kTM];
 #pragma unroll
-    for (int m = 0; m < kTB; ++m)
+    for (int n = 0; n < kTN; ++n)
 #pragma unroll
-        for (int n = 0; n < (kGated ? 2 : 4); ++n) {
-            float y[4];
+        for (int m = 0; m < kTM; ++m) acc[n][m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    const lds_char_ptr frag = lds + 16 * (4 * r + (g ^ ((0 - (r >> 2)) & 3)));
+    const lds_char_ptr xl = frag + wm * kTM * 1024, wl = frag + (kBlocksX + wn * kTN) * 1024;
+    fetch(0, 0);
+    if (steps > 1) fetch(1, 1);
+    if constexpr (kWide) {
+        u32x4_t wf[2][kTN], xf[2][kTM];                  // operands of even and odd steps
+        auto read = [&](auto odd, int step) __attribute__((always_inline)) {
+            constexpr int p = decltype(odd)::value;
+            const int at = (step & 3) * kStage;
 #pragma unroll
-            for (int j = 0; j < 4; ++j) y[j] = kGated ? silu_of<bf16_t>(acc[n][m][j]) * acc[kGated ? n + 2 : n][m][j] : acc[n][m][j];
-            *(__attribute__((address_space(3))) u32x2_t *)(lds + (16 * (wm * kTB + m) + r) * kOutPitch + 2 * ((kGated ? 32 : 64) * wn + 16 * n + 4 * g)) =
-                u32x2_t{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
+            for (int n = 0; n < kTN; ++n) wf[p][n] = *(lds_u32x4_ptr)(wl + at + n * 1024);
+#pragma unroll
+            for (int m = 0; m < kTM; ++m) xf[p][m] = *(lds_u32x4_ptr)(xl + at + m * 1024);
+        };
+        // the next step's data is there on every wavefront, a buffer nobody reads any more is filled, the next step's
+        // operands are read, this step's are multiplied
+        auto advance = [&](auto odd, int step) __attribute__((always_inline)) {
+            constexpr int p = decltype(odd)::value;
+            if (step + 1 < steps) {
+                landed(step + 1);
+                if (step + 3 < steps) fetch(step + 3, (step + 3) & 3);
+                read(std::integral_constant<int, 1 - p>{}, step + 1);
+            }
+#pragma unroll
+            for (int m = 0; m < kTM; ++m)
+#pragma unroll
+                for (int n = 0; n < kTN; ++n) mfma16_in_place(wf[p][n], xf[p][m], acc[n][m]);
+        };
+        constexpr std::integral_constant<int, 0> kEven{};
+        constexpr std::integral_constant<int, 1> kOdd{};
+        landed(0);
+        if (steps > 2) fetch(2, 2);
+        read(kEven, 0);
+        int step = 0;
+        for (; step + 1 < steps; step += 2) {
+            advance(kEven, step);
+            advance(kOdd, step + 1);
         }
-    __syncthreads();
-    const int c = tid % kPer * 8, n0 = n_tile * kCols + c, end = min(BM, count - m0);
-    if (n0 < a.n_out)
+        if (step < steps) advance(kEven, step);
+        products_done(acc);
+    } else {
+        landed(0);
+        int buf = 0;
+        for (int step = 0; step < steps; ++step) {
+            if (step + 2 < steps) fetch(step + 2, buf == 0 ? 2 : buf - 1);      // (the buffer of the step before this one)
+            u32x4_t wf[kTN];
+#pragma unroll
+            for (int n = 0; n < kTN; ++n) wf[n] = *(lds_u32x4_ptr)(wl + buf * kStage + n * 1024);
+#pragma unroll
+            for (int m = 0; m < kTM; ++m) {
+                const u32x4_t xf = *(lds_u32x4_ptr)(xl + buf * kStage + m * 1024);
+#pragma unroll
+                for (int n = 0; n < kTN; ++n) acc[n][m] = mfma16(wf[n], xf, acc[n][m]);
+            }
+            if (step + 1 < steps) landed(step + 1);
+            buf = buf == 2 ? 0 : buf + 1;
+        }
+    }
+    __syncthreads();                                     // everything has been read
+    // ---- through LDS into whole pieces of rows (an accumulator holds four consecutive outputs of one row), the tile's
+    // two halves of rows one after the other where all of it would not fit
+    constexpr int kCols = kGated ? BN / 2 : BN, kOutPitch = kCols * 2 + 16, kPer = kCols / 8;
+    constexpr int kRounds = BM * kOutPitch <= kBuffers * kStage ? 1 : 2;
+    const int c = tid % kPer * 8, n0 = n_tile * kCols + c;
+#pragma unroll
+    for (int round = 0; round < kRounds; ++round) {
+        if (kRounds == 1 || wm == round)
+#pragma unroll
+            for (int m = 0; m < kTM; ++m)
+#pragma unroll
+                for (int n = 0; n < (kGated ? kTN / 2 : kTN); ++n) {
+                    float y[4];
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) y[j] = kGated ? silu_of<bf16_t>(acc[n][m][j]) * acc[kGated ? n + kTN / 2 : n][m][j] : acc[n][m][j];
+                    *(__attribute__((address_space(3))) u32x2_t *)(lds + (16 * ((kRounds == 1 ? wm * kTM : 0) + m) + r) * kOutPitch + 2 * (kCols / 2 * wn + 16 * n + 4 * g)) =
+                        u32x2_t{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
+                }
+        __syncthreads();
+        const int base = round * (BM / 2), end = min(base + BM / kRounds, count - m0);
+        if (n0 < a.n_out)
 #pragma unroll 4
-        for (int i = tid / kPer; i < end; i += 256 / kPer)               // (16-byte pieces)
-            *reinterpret_cast<u32x4_t *>(static_cast<bf16_t *>(a.out) + static_cast<int64_t>(sh_row[i]) * a.o_stride + n0) = *(lds_u32x4_ptr)(lds + i * kOutPitch + 2 * c);
+            for (int i = base + tid / kPer; i < end; i += 256 / kPer)            // (16-byte pieces)
+                *reinterpret_cast<u32x4_t *>(static_cast<bf16_t *>(a.out) + static_cast<int64_t>(sh_row[i]) * a.o_stride + n0) = *(lds_u32x4_ptr)(lds + (i - base) * kOutPitch + 2 * c);
+        if (kRounds > 1) __syncthreads();
+    }
 }
 
 // Sizes the tiled form is built for: whole steps, whole 16-byte stores, 32-bit offsets.
@@ -317,14 +387,14 @@ static bool tiles_ok(const LinearArgs &a, bool gated, int32_t x_rows) {
            static_cast<int64_t>(a.n_out) * (gated ? 2 : 1) * a.k < (1LL << 30);
 }
 
-template <int BM, bool kGated>
+template <int BM, int BN, bool kGated>
 static int launch_tiles(const LinearArgs &a, hipStream_t s) {
-    constexpr int kCols = kGated ? kTileN / 2 : kTileN;
+    constexpr int kCols = kGated ? BN / 2 : BN;
     const int32_t n_tiles = (a.n_out + kCols - 1) / kCols;
     const int64_t most = (static_cast<int64_t>(a.rows) / BM + a.groups) * n_tiles;      // row tiles there can be, whatever the counts are
     const int64_t grid = (most + 7) / 8 * 8 + 8;
     if (grid > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
-    hipLaunchKernelGGL((linear_tile_kernel<BM, kGated>), dim3(static_cast<uint32_t>(grid)), dim3(256), 0, s, a, n_tiles);
+    hipLaunchKernelGGL((linear_tile_kernel<BM, BN, kGated>), dim3(static_cast<uint32_t>(grid)), dim3(256), 0, s, a, n_tiles);
     return launch_status();
 }
 
@@ -569,8 +639,9 @@ extern "C" int nva_routed_linear(const void *x, int64_t x_row_stride, const void
     if (!linear_matrix_ok(a)) return gated ? launch_any_linear<bf16_t, bf16_t, true>(a, rows, s) : launch_any_linear<bf16_t, bf16_t, false>(a, rows, s);
     const int32_t average = static_cast<int32_t>(static_cast<int64_t>(rows) * terms / experts);
     if (average >= 48 && tiles_ok(a, gated, x_per_row ? rows : rows * terms)) {
-        if (average >= 512) return gated ? launch_tiles<256, true>(a, s) : launch_tiles<256, false>(a, s);
-        return gated ? launch_tiles<128, true>(a, s) : launch_tiles<128, false>(a, s);
+        if (average >= 512 && k_in >= 1536) return gated ? launch_tiles<256, 256, true>(a, s) : launch_tiles<256, 256, false>(a, s);
+        if (average >= 512) return gated ? launch_tiles<256, 128, true>(a, s) : launch_tiles<256, 128, false>(a, s);
+        return gated ? launch_tiles<128, 128, true>(a, s) : launch_tiles<128, 128, false>(a, s);
     }
     const int32_t busy = static_cast<int32_t>(std::min(static_cast<int64_t>(experts), static_cast<int64_t>(rows) * terms));
     return gated ? launch_skinny<true, bf16_t>(a, hint, rows, busy, s) : launch_skinny<false, bf16_t>(a, hint, rows, busy, s);

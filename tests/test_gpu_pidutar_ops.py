@@ -143,6 +143,34 @@ def test_experts(dev, dtype, shape, n):
         assert torch.isfinite(got).all() and float(err[clear].max()) < tol(dtype, 1.5e-2, 1e-5), (skewed, float(err[clear].max()))
 
 
+@pytest.mark.parametrize("shape", [  # experts, top, inner size, outputs, rows
+    (3, 2, 1536, 264, 1500), (2, 1, 1568, 96, 1100), (70, 2, 1600, 520, 20000), (4, 3, 96, 200, 900), (3, 2, 736, 72, 1300), (9, 2, 128, 520, 330)])
+@pytest.mark.parametrize("gated", [True, False])
+def test_tiles_of_experts(dev, shape, gated):
+    """Products with many rows per expert, whole and ragged tiles of every form, an expert without rows, against fp32 products."""
+    n_experts, top, k, n_out, n = shape
+    g = torch.Generator(device=dev).manual_seed(k)
+    rnd = lambda *s: torch.randn(*s, generator=g, device=dev)
+    x = rnd(n if gated else n * top, k).bfloat16()
+    w = rnd(n_experts, 2 * n_out if gated else n_out, k).mul(k ** -0.5).bfloat16()
+    router = rnd(n_experts, 64).bfloat16()
+    router[0] = 0.0                                          # (with all-positive rows below: never among the best)
+    h = rnd(n, 64).bfloat16()
+    h[:, 0], router[:, 0] = 8.0, 8.0
+    router[0, 0] = -8.0
+    a = experts.route(h, router, top, 1.0, torch.zeros(n_experts, dtype=torch.int32, device=dev))
+    assert n_experts == 1 or top == n_experts or int(a.counts[0]) == 0
+    got = experts.routed_linear(x, w, a, gated)
+    for e in range(n_experts):
+        rows = (a.choice.flatten() == e).nonzero()[:, 0]
+        y = x[rows // top if gated else rows].float() @ w[e].float().T
+        if gated:
+            y = torch.nn.functional.silu(y[:, :n_out]) * y[:, n_out:]
+        if len(rows):
+            err = (got[rows].float() - y).abs().max() / y.abs().max()
+            assert float(err) < 6e-3, (e, len(rows), float(err))
+
+
 # ---- latent attention --------------------------------------------------------------------------------------
 
 LATENT = [  # heads, unrotated, rotated, value size, query rank, latent rank
