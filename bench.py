@@ -1190,14 +1190,14 @@ def pidutar_kernels(dev, steps=60, only=None):
                 p.normal_(0.0, 0.03)
             counters = torch.zeros(n_exp, dtype=torch.int32, device=dev)
             a = experts.route(h, w.router, top, 1.0, counters)
-            runs.append((w, a, experts.routed_linear(h, w.gate_up, a, True), torch.zeros(n_exp, dtype=torch.int32, device=dev)))
+            runs.append((w, a, experts.routed_linear(h, w.gate_up, a, experts.SILU), torch.zeros(n_exp, dtype=torch.int32, device=dev)))
         hit = sum(int((r[1].counts > 0).sum()) for r in runs) / copies
         dense = [(rnd(2 * top * ff, width), rnd(width, top * ff)) for _ in range(copies)]
         mid, act = rnd(n, 2 * top * ff), rnd(n, top * ff)
         time = graph_us if n <= 512 else event_us
         n_calls = (200,) if n <= 512 else (steps,)
-        up = time([lambda r=r: experts.routed_linear(h, r[0].gate_up, r[1], True) for r in runs], *n_calls)
-        down = time([lambda r=r: experts.routed_linear(r[2], r[0].down, r[1], False) for r in runs], *n_calls)
+        up = time([lambda r=r: experts.routed_linear(h, r[0].gate_up, r[1], experts.SILU) for r in runs], *n_calls)
+        down = time([lambda r=r: experts.routed_linear(r[2], r[0].down, r[1], None) for r in runs], *n_calls)
         lup = time([lambda d=d: mixers.clamped_gate(F.linear(h, d[0]), 7.0, 1.702) for d in dense], *n_calls)
         ldown = time([lambda d=d: F.linear(act, d[1]) for d in dense], *n_calls)
         if n >= 512:

@@ -41,6 +41,9 @@ enum nva_status {
 /* Element type of the entry points that take bf16 or fp32 tensors. */
 enum nva_dtype { NVA_DTYPE_BF16 = 0, NVA_DTYPE_F32 = 1 };
 
+/* which keys the query at position p sees: [p / span * span, p], or the last `span` up to and with p */
+enum nva_mask { NVA_MASK_CHUNKS = 0, NVA_MASK_WINDOW = 1 };
+
 /* Library version, (major << 16) | minor. */
 int nva_version(void);
 
@@ -324,6 +327,13 @@ int nva_post_add_norm(const void *y, int64_t y_row_stride, float *residual, cons
 int nva_clamped_gate(const void *x, int64_t x_row_stride, void *out, int32_t rows, int32_t inter, float limit,
                      float alpha, int32_t dtype, void *stream);
 
+/* out = max(x, 0)^2; x: [rows, width] (row stride in elements), out dense, may be x. */
+int nva_squared_relu(const void *x, int64_t x_row_stride, void *out, int32_t rows, int32_t width, int32_t dtype,
+                     void *stream);
+
+/* x = cap * tanh(x / cap), in place; x: [rows, width] dense. */
+int nva_soft_cap(void *x, int32_t rows, int32_t width, float cap, int32_t dtype, void *stream);
+
 /* q, k and v of an attention layer: causal convolution over time on every channel, rotary embedding of
  * the first rot_dims elements of each q and k head (pairs i, i + rot_dims / 2), q to q_out, k and v to
  * their cache slots.
@@ -359,6 +369,30 @@ int nva_chunk_attn(const void *q, int64_t q_row_stride, const void *k_cache, con
                    int32_t num_blocks, int32_t chunk, float scale, float softcap, int32_t dtype,
                    void *stream);
 
+/* The same under any nva_mask (workspace: as above with chunk = span), with
+ * sinks (fp32 [num_heads], may be NULL): the sum of a head's weights also contains exp(sink), which has no key, and
+ * gate ([n_tokens, num_heads], row stride in elements, may be NULL): a head's result times sigmoid(gate). */
+int nva_masked_attn(const void *q, int64_t q_row_stride, const void *k_cache, const void *v_cache,
+                    const int32_t *block_tables, int64_t bt_row_stride, int32_t max_blocks,
+                    const int32_t *cu_seqlens_q, const int32_t *seq_lens, const int32_t *token_seq, void *out,
+                    void *workspace, size_t workspace_bytes,
+                    int32_t n_tokens, int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads,
+                    int32_t num_kv_heads, int32_t qk_dim, int32_t v_dim, int32_t block_size,
+                    int32_t num_blocks, int32_t mask, int32_t span, float scale, float softcap, const float *sinks,
+                    const void *gate, int64_t gate_row_stride, int32_t dtype, void *stream);
+
+/* q, k and v of an attention layer, between projection and attention.  x: [n_tokens, num_heads * qk_dim | num_kv_heads *
+ * qk_dim | num_kv_heads * v_dim] (row stride in elements) plus bias (as many elements, may be NULL); then RMS norms of q and
+ * k, of every head by itself (weights [qk_dim]) or, norm_whole, over all heads at once (weights [num_heads * qk_dim] and
+ * [num_kv_heads * qk_dim]; a NULL weight: no norm); then rotation of the first rot_dims elements of every head by the
+ * row's position (pairs i, i + rot_dims / 2; rope_cache as above).  q to q_out [n_tokens, num_heads * qk_dim], k and v to their
+ * cache slots.  Caches NULL: the queries only (x then has num_heads * qk_dim columns). */
+int nva_qkv_prepare(const void *x, int64_t x_row_stride, const void *bias, const void *q_norm_weight, const void *k_norm_weight,
+                    int32_t norm_whole, const float *rope_cache, void *q_out, void *k_cache, void *v_cache,
+                    const int32_t *slot_mapping, int64_t num_slots, const int32_t *cu_seqlens_q, const int32_t *seq_lens,
+                    const int32_t *token_seq, int32_t n_tokens, int32_t n_seqs, int32_t num_heads, int32_t num_kv_heads,
+                    int32_t qk_dim, int32_t v_dim, int32_t rot_dims, int32_t max_position, float eps, int32_t dtype, void *stream);
+
 /* Retention: S_t = decay S_{t-1} + k_t v_t^T, o_t = S_t^T q_t per head, with rotary q and k, k scaled by
  * k_scale; out = o / rms(o) * silu(gate).
  * qkvg: [n_tokens, 2 * num_heads * (qk_dim + v_dim)] (q | k | v | gate, row stride in elements);
@@ -383,7 +417,7 @@ int nva_retention(const void *qkvg, int64_t row_stride, float *state, const int3
  */
 
 /* residual[r] = table[ids[r]] * scale (fp32); out1[r] = residual[r] / rms * (weight_offset + weight1), out2 the
- * same with weight2 (weight2 may be NULL: one norm).  rms = sqrt(mean(x^2) + eps).  clear (may be NULL):
+ * same with weight2 (weight2 may be NULL: one norm; both NULL: out1 is the residual itself, rounded).  rms = sqrt(mean(x^2) + eps).  clear (may be NULL):
  * clear_count int32 counters set to zero, for a router that runs behind this. */
 int nva_embed_rms_norms(const int64_t *ids, const void *table, float scale, const void *weight1, const void *weight2,
                         float weight_offset, float *residual, void *out1, void *out2, int32_t *clear,
@@ -400,27 +434,51 @@ int nva_branches_rms_norms(const void *y1, int64_t y1_row_stride, const void *ga
                            const int32_t *rows_of, int32_t *clear, int32_t clear_count, int32_t rows,
                            int32_t src_rows, int32_t width, float eps, int32_t dtype, void *stream);
 
+/* Layers that norm what a sublayer gives: y[r] = y1_weight[r] * y1[r] + sum_k term_weight[r, k] * y2[r * terms + k];
+ * residual[r] += y[r] / rms * (weight_offset + post_weight), in place, fp32; out[r] = residual[r], rounded, or with
+ * next_weight residual[r] / rms * (weight_offset + next_weight).  y1_weight (one per row) and term_weight are fp32 with
+ * weight_row_stride elements between rows; either may be NULL (one).  The rest as above. */
+int nva_post_rms_norms(const void *y1, int64_t y1_row_stride, const float *y1_weight, const void *y2,
+                       const float *term_weight, int64_t weight_row_stride, int32_t terms, const void *post_weight,
+                       float *residual, const void *next_weight, float weight_offset, void *out, const int32_t *rows_of,
+                       int32_t *clear, int32_t clear_count, int32_t rows, int32_t src_rows, int32_t width, float eps,
+                       int32_t dtype, void *stream);
+
 /* out[r, g] = W_g x[r, g] for every row and group: x + r * x_row_stride + g * x_group_stride, weight [groups, n_out, k_in],
- * out + r * out_row_stride + g * out_group_stride (elements).  out_dtype fp32 keeps the fp32 sums of bf16 products. */
+ * out + r * out_row_stride + g * out_group_stride (elements).  out_dtype fp32 keeps the fp32 sums of bf16 products.
+ * squared_relu: out = max(., 0)^2. */
 int nva_grouped_linear(const void *x, int64_t x_row_stride, int64_t x_group_stride, const void *weight, void *out,
                        int64_t out_row_stride, int64_t out_group_stride, int32_t rows, int32_t groups, int32_t n_out,
-                       int32_t k_in, int32_t dtype, int32_t out_dtype, void *stream);
+                       int32_t k_in, int32_t squared_relu, int32_t dtype, int32_t out_dtype, void *stream);
 
-/* Router of a mixture of experts: logits = weight x (fp32), softmax over all experts, the `top` best (ties: the lower
+/* Router of a mixture of experts: logits = weight x + bias (fp32; bias may be NULL), softmax over all experts, the `top` best (ties: the lower
  * index) in descending order, their scores divided by their sum (+ 1e-20) and multiplied by scale.
- * choice int32, choice_weight fp32: [rows, top].  lists int32 [experts, list_stride], counts int32 [experts]: the
+ * (With scale 1 the weights are the softmax over the chosen logits.)  weight: [experts + gates, width]; the gates are outputs
+ * beside the experts' whose sigmoids follow the choices' weights in every row.
+ * choice int32 [rows, top], choice_weight fp32 [rows, top + gates].  lists int32 [experts, list_stride], counts int32 [experts]: the
  * assignments row * top + k of every expert, in no particular order; counts must be zero on entry;
- * list_stride >= rows.  experts <= 1024, top <= 128. */
-int nva_router(const void *x, int64_t x_row_stride, const void *weight, int32_t *choice, float *choice_weight,
-               int32_t *lists, int32_t *counts, int64_t list_stride, int32_t rows, int32_t width, int32_t experts,
-               int32_t top, float scale, int32_t dtype, void *stream);
+ * list_stride >= rows.  experts <= 1024, gates <= 64, top <= 128. */
+int nva_router(const void *x, int64_t x_row_stride, const void *weight, const float *bias, int32_t *choice,
+               float *choice_weight, int32_t *lists, int32_t *counts, int64_t list_stride, int32_t rows, int32_t width,
+               int32_t experts, int32_t gates, int32_t top, float scale, int32_t dtype, void *stream);
 
 /* out[p] = W_e x[p / terms] (x_per_row) or W_e x[p], for every assignment p of lists to its expert e.
- * weight: [experts, n_out, k_in], or gated: [experts, 2 n_out, k_in] (gate | up) and out = silu(gate) * up.
+ * weight: [experts, n_out, k_in], or gated: [experts, 2 n_out, k_in] (gate | up) and, with g = min(gate, gate_limit)
+ * and u = clamp(up, gate_limit), out = g * sigmoid(gate_slope * g) * (u + gate_shift) (infinity, 1, 0: silu(gate) * up).
  * out: [rows * terms, n_out] dense. */
 int nva_routed_linear(const void *x, int64_t x_row_stride, const void *weight, void *out, const int32_t *lists,
                       const int32_t *counts, int64_t list_stride, int32_t rows, int32_t terms, int32_t experts,
-                      int32_t n_out, int32_t k_in, int32_t x_per_row, int32_t gated, int32_t dtype, void *stream);
+                      int32_t n_out, int32_t k_in, int32_t x_per_row, int32_t gated, float gate_limit, float gate_slope,
+                      float gate_shift, int32_t dtype, void *stream);
+
+/* The same for few rows, bf16, and in the same launch the product of an expert that every row runs: shared_out[r] = W
+ * shared_x[r], shared_weight [shared_n_out, shared_k_in], or gated [2 shared_n_out, shared_k_in] in the same form with
+ * a limit of its own; shared_out [rows, shared_n_out] dense.  Inner sizes and row strides are multiples of 8. */
+int nva_routed_shared_linear(const void *x, int64_t x_row_stride, const void *weight, void *out, const int32_t *lists,
+                             const int32_t *counts, int64_t list_stride, int32_t rows, int32_t terms, int32_t experts,
+                             int32_t n_out, int32_t k_in, int32_t x_per_row, int32_t gated, float gate_limit, float gate_slope,
+                             float gate_shift, const void *shared_x, int64_t shared_x_row_stride, const void *shared_weight,
+                             void *shared_out, int32_t shared_n_out, int32_t shared_k_in, float shared_gate_limit, void *stream);
 
 /* Latent attention, what a row leaves behind and its query latent.
  * x: [n_tokens, q_rank | kv_rank | rot_dim] (row stride in elements).

@@ -1,6 +1,10 @@
-// Softmax attention over position chunks, keys and values in the paged cache: the query at position p
-// sees the keys [floor(p / chunk) * chunk, p] of its own sequence.  Scores may be capped
-// (cap * tanh(s / cap)); query/key and value sizes may differ; scores, weights and sums are fp32.
+// Softmax attention under a mask of positions, keys and values in the paged cache: the query at position p sees the
+// keys [first_key(p), p] of its own sequence, where
+//   chunks    first_key(p) = floor(p / span) * span
+//   window    first_key(p) = max(0, p - span + 1)     (a span no sequence reaches: all earlier keys)
+// Scores may be capped (cap * tanh(s / cap)); a head may have a sink, one more score that belongs to no key and only
+// enters the sum of the weights; a head's output may be multiplied by sigmoid(gate).  Query/key and value sizes may
+// differ; scores, weights and sums are fp32.
 #include "nva_elem.h"
 #include "nva_matrix.h"
 
@@ -21,9 +25,27 @@ struct ChunkAttnArgs {
     const int32_t *klen;             // tokens of every sequence, this step's included (decode: 0 = padded row)
     const int32_t *token_seq;        // portions: sequence of every row
     void *out;                       // [n, H, vdim] dense
-    int32_t n, n_seqs, heads, kv_heads, dim, vdim, block_shift, num_blocks, max_blocks, chunk;
+    int32_t n, n_seqs, heads, kv_heads, dim, vdim, block_shift, num_blocks, max_blocks, span, window;
     float scale, cap;                // cap <= 0: none
+    const float *sinks;              // [H] or null
+    const void *gate;                // [n, H] logits or null
+    int64_t gate_stride;
 };
+
+__device__ __forceinline__ int first_key(const ChunkAttnArgs &a, int pos) {
+    return a.window ? max(0, pos - a.span + 1) : pos / a.span * a.span;
+}
+// what a head's output is multiplied by
+template <typename T>
+__device__ __forceinline__ float head_gate(const ChunkAttnArgs &a, int64_t row, int head) {
+    if (a.gate == nullptr) return 1.0f;
+    return sigmoid_of<T>(Elem<T>::to_f32(static_cast<const T *>(a.gate)[row * a.gate_stride + head]));
+}
+constexpr float kLog2e = 1.4426950408889634f;
+// the sink's weight where weights are 2^(exponent - top)
+__device__ __forceinline__ float sink_weight(const ChunkAttnArgs &a, int head, float top) {
+    return a.sinks == nullptr ? 0.f : __builtin_amdgcn_exp2f(fmaf(a.sinks[head], kLog2e, -top));
+}
 
 // One wavefront per (row, head), any sizes, bf16 or fp32: lanes are keys for the scores and value
 // columns for the weighted sum; running maximum and sum per block of 64 keys.
@@ -52,7 +74,7 @@ __global__ __launch_bounds__(256) void chunk_attn_any_kernel(ChunkAttnArgs a) {
     __syncthreads();
     if (!live) return;
     const int g = head / (a.heads / a.kv_heads);
-    const int lo = pos < 0 ? 0 : pos / a.chunk * a.chunk;
+    const int lo = pos < 0 ? 0 : first_key(a, pos);
     float m = -INFINITY, sum = 0.f;
     float acc[kAnyMaxDim / 64];
 #pragma unroll
@@ -94,7 +116,8 @@ __global__ __launch_bounds__(256) void chunk_attn_any_kernel(ChunkAttnArgs a) {
         }
     }
     T *out = static_cast<T *>(a.out) + (t * a.heads + head) * a.vdim;
-    const float inv = sum > 0.f ? 1.0f / sum : 0.f;
+    if (a.sinks != nullptr && sum > 0.f) sum += exp_of<T>(a.sinks[head] - m);
+    const float inv = sum > 0.f ? head_gate<T>(a, t, head) / sum : 0.f;
 #pragma unroll
     for (int i = 0; i < kAnyMaxDim / 64; ++i)
         if (i * 64 + lane < a.vdim) out[i * 64 + lane] = Elem<T>::from_f32(acc[i] * inv);
@@ -118,7 +141,6 @@ struct Weighting {
     bool capped;
 };
 static Weighting weighting_of(float scale, float cap) {
-    constexpr float kLog2e = 1.4426950408889634f;
     if (cap > 0.f) return Weighting{2.0f * kLog2e * scale / cap, kLog2e * cap, true};
     return Weighting{kLog2e * scale, 0.f, false};
 }
@@ -127,8 +149,8 @@ __device__ __forceinline__ float exponent_of(const Weighting &w, bool capped, fl
     return w.in * s;
 }
 
-// Portions: a workgroup of four wavefronts takes 4 * 16 * NQ queries of one head and walks the keys of
-// their chunks in tiles of 64, double-buffered in LDS.  DK, DV: sizes the registers are laid out for.
+// Portions: a workgroup of four wavefronts takes 4 * 16 * NQ queries of one head and walks the keys that
+// any of them sees in tiles of 64, double-buffered in LDS.  DK, DV: sizes the registers are laid out for.
 // kDirect (the model's sizes are exactly these): tiles travel global -> LDS without a register in between,
 // the LDS image laid out in 1 KB blocks of 16 keys x 32 dims with the 16-byte pieces permuted so that
 // operand reads spread over the banks -- the scheme of the prefill kernel for whole contexts, whose
@@ -161,7 +183,7 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
     if (start < 0) return;
     const int last_row = min(row0 + kBM, lq) - 1;
     const int key_end = start + last_row;                            // last key any query of the tile sees
-    const int key_begin = (start + row0) / a.chunk * a.chunk & ~(kBN - 1);
+    const int key_begin = first_key(a, start + row0) & ~(kBN - 1);
     const int ntiles = (key_end - key_begin) / kBN + 1;
     const bf16_t *kc = static_cast<const bf16_t *>(a.k_cache) + static_cast<int64_t>(g_kv) * a.dim;
     const bf16_t *vc = static_cast<const bf16_t *>(a.v_cache) + static_cast<int64_t>(g_kv) * a.vdim;
@@ -175,7 +197,7 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
     for (int qa = 0; qa < NQ; ++qa) {
         const int row = row0 + wave * 16 * NQ + 16 * qa + r;
         pos[qa] = start + row;
-        lo[qa] = pos[qa] / a.chunk * a.chunk;
+        lo[qa] = first_key(a, pos[qa]);
         const bf16_t *q = static_cast<const bf16_t *>(a.q) + static_cast<int64_t>(t0 + min(row, lq - 1)) * a.q_stride +
                           static_cast<int64_t>(head) * a.dim + 8 * g;
 #pragma unroll
@@ -187,8 +209,8 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
     const int w_first = start + row0 + wave * 16 * NQ;               // the wavefront's queries: first and last position
     const int w_last = min(w_first + 16 * NQ - 1, key_end);
     const bool w_live = row0 + wave * 16 * NQ < lq;
-    const int w_lo = w_first / a.chunk * a.chunk;                    // oldest key one of them sees
-    const int w_lo_all = w_last / a.chunk * a.chunk;                 // keys from here to w_first are seen by all
+    const int w_lo = first_key(a, w_first);                          // oldest key one of them sees
+    const int w_lo_all = first_key(a, w_last);                       // keys from here to w_first are seen by all
 
     // ---- tiles into LDS.  Direct: a tile's block id is asked for one tile ahead (in a vector register, so
     // that nothing waits for it before it is used), its loads go out while the tile before it is multiplied.
@@ -380,9 +402,10 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
         float l = lsum[qa];
         l += __shfl_xor(l, 16, 64);
         l += __shfl_xor(l, 32, 64);
-        const float inv = l > 0.f ? 1.0f / l : 0.f;
         const int row = row0 + wave * 16 * NQ + 16 * qa + r;
         if (row >= lq) continue;
+        l += sink_weight(a, head, kBounded ? 0.f : m[qa]);
+        const float inv = l > 0.f ? head_gate<bf16_t>(a, t0 + row, head) / l : 0.f;
         bf16_t *out = static_cast<bf16_t *>(a.out) + (static_cast<int64_t>(t0 + row) * a.heads + head) * a.vdim + 4 * g;
 #pragma unroll
         for (int db = 0; db < DV / 16; ++db)
@@ -431,7 +454,7 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 3) void chunk_decode_kerne
             for (int i = tid; i < nheads * a.vdim; i += 256) out[i] = 0;
         return;
     }
-    const int lo = pos / a.chunk * a.chunk, first = (lo & ~31) + split * sp.keys;
+    const int lo = first_key(a, pos), first = (lo & ~31) + split * sp.keys;
     const int last = min(pos, first + sp.keys - 1);      // last key of this range
     if (first > last) return;
     const int ntiles = (last - first) / 32 + 1;
@@ -575,7 +598,8 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 3) void chunk_decode_kerne
             o = fmaf(reinterpret_cast<const float *>(&smem[v * kWaveBytes])[h * DV + c], f, o);
         }
         if (sp.splits == 1) {
-            out[i] = f32_to_bf16(l > 0.f ? o / l : 0.f);
+            l += sink_weight(a, head0 + h, top);
+            out[i] = f32_to_bf16(l > 0.f ? o * head_gate<bf16_t>(a, seq, head0 + h) / l : 0.f);
         } else {
             float *part = sp.partials + ((static_cast<int64_t>(seq) * sp.splits + split) * a.heads + head0 + h) * (a.vdim + 2);
             part[c] = o;
@@ -592,7 +616,7 @@ __global__ __launch_bounds__(256) void chunk_merge_kernel(const ChunkAttnArgs a,
     const int seq = static_cast<int>(item / a.heads), head = static_cast<int>(item % a.heads);
     const int pos = a.klen[seq] - 1;
     bf16_t *out = static_cast<bf16_t *>(a.out) + item * a.vdim;
-    const int lo = pos < 0 ? 0 : pos / a.chunk * a.chunk & ~31;
+    const int lo = pos < 0 ? 0 : first_key(a, pos) & ~31;
     const int count = pos < 0 ? 0 : min(sp.splits, (pos - lo) / sp.keys + 1);
     const int pitch = a.vdim + 2;
     const float *part = sp.partials + (static_cast<int64_t>(seq) * sp.splits * a.heads + head) * pitch;
@@ -602,8 +626,9 @@ __global__ __launch_bounds__(256) void chunk_merge_kernel(const ChunkAttnArgs a,
     const float my_m = lane < count ? part[lane * step + a.vdim + 1] : -INFINITY;
     const float top = wave_max(my_m);
     const float f = my_m == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(my_m - top);
-    const float l = wave_sum(my_l * f);
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    float l = wave_sum(my_l * f);
+    if (count > 0) l += sink_weight(a, head, top);
+    const float inv = l > 0.f ? head_gate<bf16_t>(a, seq, head) / l : 0.f;
     for (int c = lane; c < a.vdim; c += 64) {
         float o = 0.f;
         for (int j = 0; j < count; ++j) o = fmaf(part[j * step + c], __shfl(f, j, 64), o);
@@ -613,10 +638,10 @@ __global__ __launch_bounds__(256) void chunk_merge_kernel(const ChunkAttnArgs a,
 
 // How the keys of a decode step are split: ranges of 512 keys, longer ones where that would be more than 64.
 // Depends on shapes only.
-static SplitArgs plan_splits(int32_t heads, int32_t kv_heads, int32_t max_blocks, int32_t block_size, int32_t chunk) {
+static SplitArgs plan_splits(int32_t heads, int32_t kv_heads, int32_t max_blocks, int32_t block_size, int32_t span) {
     SplitArgs sp{};
     sp.head_groups = (heads / kv_heads + 15) / 16;
-    const int64_t most = std::min(static_cast<int64_t>(chunk), static_cast<int64_t>(max_blocks) * block_size) + 31;   // keys one query can see, from a multiple of 32 on
+    const int64_t most = std::min(static_cast<int64_t>(span), static_cast<int64_t>(max_blocks) * block_size) + 31;   // keys one query can see, from a multiple of 32 on
     int64_t keys = std::max(static_cast<int64_t>(512), (most + 63) / 64);
     keys = (keys + 127) / 128 * 128;
     sp.keys = static_cast<int32_t>(keys);
@@ -684,42 +709,42 @@ extern "C" size_t nva_chunk_attn_workspace_bytes(int32_t n_tokens, int32_t num_h
     return static_cast<size_t>(n_tokens) * sp.splits * num_heads * (v_dim + 2) * sizeof(float);
 }
 
-extern "C" int nva_chunk_attn(const void *q, int64_t q_row_stride, const void *k_cache, const void *v_cache,
+extern "C" int nva_masked_attn(const void *q, int64_t q_row_stride, const void *k_cache, const void *v_cache,
                               const int32_t *block_tables, int64_t bt_row_stride, int32_t max_blocks,
                               const int32_t *cu_seqlens_q, const int32_t *seq_lens, const int32_t *token_seq, void *out,
                               void *workspace, size_t workspace_bytes, int32_t n_tokens, int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads,
                               int32_t num_kv_heads, int32_t qk_dim, int32_t v_dim, int32_t block_size,
-                              int32_t num_blocks, int32_t chunk, float scale, float softcap, int32_t dtype,
-                              void *stream) {
+                              int32_t num_blocks, int32_t mask, int32_t span, float scale, float softcap, const float *sinks,
+                              const void *gate, int64_t gate_row_stride, int32_t dtype, void *stream) {
     using namespace nva;
     if (n_tokens < 0 || n_seqs < 0 || num_heads <= 0 || num_kv_heads <= 0 || qk_dim <= 0 || v_dim <= 0 || num_blocks < 0 ||
-        max_blocks < 0 || chunk <= 0 || max_seqlen_q < 0 || num_heads % num_kv_heads != 0)
+        max_blocks < 0 || span <= 0 || max_seqlen_q < 0 || num_heads % num_kv_heads != 0)
         return NVA_ERR_BAD_SHAPE;
     const int shift = block_shift_of(block_size);
-    if (shift < 0 || qk_dim > kAnyMaxDim || v_dim > kAnyMaxDim || !known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
+    if (shift < 0 || (mask != NVA_MASK_CHUNKS && mask != NVA_MASK_WINDOW) || qk_dim > kAnyMaxDim || v_dim > kAnyMaxDim || !known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     if (n_tokens == 0) return NVA_OK;
     if (!q || !k_cache || !v_cache || !block_tables || !seq_lens || !out) return NVA_ERR_NULL_POINTER;
     const bool decode = cu_seqlens_q == nullptr;
     if (!decode && (!token_seq || n_seqs == 0)) return NVA_ERR_NULL_POINTER;
     if (decode && n_seqs != n_tokens) return NVA_ERR_BAD_SHAPE;
-    if (q_row_stride < static_cast<int64_t>(num_heads) * qk_dim || bt_row_stride < max_blocks) return NVA_ERR_BAD_STRIDE;
+    if (q_row_stride < static_cast<int64_t>(num_heads) * qk_dim || bt_row_stride < max_blocks || (gate && gate_row_stride < num_heads)) return NVA_ERR_BAD_STRIDE;
     if (static_cast<int64_t>(n_tokens) * num_heads / 4 > 0x7ffffff0LL) return NVA_ERR_BAD_SHAPE;
     ChunkAttnArgs a{};
     a.q = q; a.q_stride = q_row_stride; a.k_cache = k_cache; a.v_cache = v_cache; a.block_tables = block_tables;
     a.bt_stride = bt_row_stride; a.cu = cu_seqlens_q; a.klen = seq_lens; a.token_seq = token_seq; a.out = out;
     a.n = n_tokens; a.n_seqs = n_seqs; a.heads = num_heads; a.kv_heads = num_kv_heads; a.dim = qk_dim; a.vdim = v_dim;
-    a.block_shift = shift; a.num_blocks = num_blocks; a.max_blocks = max_blocks; a.chunk = chunk; a.scale = scale;
-    a.cap = softcap;
+    a.block_shift = shift; a.num_blocks = num_blocks; a.max_blocks = max_blocks; a.span = span;
+    a.window = mask == NVA_MASK_WINDOW; a.scale = scale; a.cap = softcap; a.sinks = sinks; a.gate = gate; a.gate_stride = gate_row_stride;
     hipStream_t s = static_cast<hipStream_t>(stream);
     if (dtype == NVA_DTYPE_BF16 && matrix_ok(a)) {
         SplitArgs sp{};
         if (decode) {
-            sp = plan_splits(num_heads, num_kv_heads, max_blocks, block_size, chunk);
+            sp = plan_splits(num_heads, num_kv_heads, max_blocks, block_size, span);
             sp.partials = static_cast<float *>(workspace);
             if (sp.splits > 1) {
                 if (!workspace) return NVA_ERR_NULL_POINTER;
                 if (!aligned16(workspace)) return NVA_ERR_MISALIGNED;
-                if (workspace_bytes < nva_chunk_attn_workspace_bytes(n_tokens, num_heads, num_kv_heads, v_dim, max_blocks, block_size, chunk))
+                if (workspace_bytes < nva_chunk_attn_workspace_bytes(n_tokens, num_heads, num_kv_heads, v_dim, max_blocks, block_size, span))
                     return NVA_ERR_WORKSPACE_TOO_SMALL;
             }
         }
@@ -728,4 +753,16 @@ extern "C" int nva_chunk_attn(const void *q, int64_t q_row_stride, const void *k
         return launch_matrix_dk<256>(a, sp, max_seqlen_q, s);
     }
     return dtype == NVA_DTYPE_BF16 ? launch_any<bf16_t>(a, s) : launch_any<float>(a, s);
+}
+
+extern "C" int nva_chunk_attn(const void *q, int64_t q_row_stride, const void *k_cache, const void *v_cache,
+                              const int32_t *block_tables, int64_t bt_row_stride, int32_t max_blocks,
+                              const int32_t *cu_seqlens_q, const int32_t *seq_lens, const int32_t *token_seq, void *out,
+                              void *workspace, size_t workspace_bytes, int32_t n_tokens, int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads,
+                              int32_t num_kv_heads, int32_t qk_dim, int32_t v_dim, int32_t block_size,
+                              int32_t num_blocks, int32_t chunk, float scale, float softcap, int32_t dtype,
+                              void *stream) {
+    return nva_masked_attn(q, q_row_stride, k_cache, v_cache, block_tables, bt_row_stride, max_blocks, cu_seqlens_q, seq_lens, token_seq, out,
+                           workspace, workspace_bytes, n_tokens, n_seqs, max_seqlen_q, num_heads, num_kv_heads, qk_dim, v_dim, block_size,
+                           num_blocks, NVA_MASK_CHUNKS, chunk, scale, softcap, nullptr, nullptr, 0, dtype, stream);
 }

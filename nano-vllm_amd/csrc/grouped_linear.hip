@@ -3,8 +3,11 @@
 //                  product with few outputs, in fp32 where asked for)
 //   routed groups  out[p] = W_e x[p / terms] for every assignment p = row * terms + k of a row to an expert e;
 //                  lists[e] holds the assignments of expert e in any order, counts[e] their number
-//   gated          W has 2 n_out rows (gate | up): out = silu(gate) * up
-//   router         logits in fp32, softmax over all experts, the best `terms`, their normalised weights, lists
+//   gated          W has 2 n_out rows (gate | up): out = g sigmoid(slope g) (u + shift), g = min(gate, limit), u = clamp(up, limit)
+//                  (slope 1, shift 0, no limit: silu(gate) * up)
+//   squared relu   of a dense group's results, where asked for
+//   router         logits (with a bias) in fp32, softmax over all experts, the best `terms`, their normalised weights, lists;
+//                  and the sigmoids of further outputs, gates of what every row runs
 // bf16 tensors go through the matrix cores, fp32 ones and odd sizes through plain fp32 kernels.
 #include "nva_elem.h"
 #include "nva_matrix.h"
@@ -16,6 +19,10 @@
 
 namespace nva {
 
+struct GateForm {
+    float limit, slope, shift;
+};
+
 struct LinearArgs {
     const void *x;
     int64_t x_stride, x_group;       // elements between rows, between groups (dense)
@@ -26,6 +33,8 @@ struct LinearArgs {
     int64_t list_stride;
     int32_t rows, groups, n_out, k;  // rows: dense rows, or assignments in all
     int32_t x_div;                   // routed: x row = assignment / x_div
+    GateForm gate;                   // gated
+    int32_t squared_relu;            // of the results (not gated)
 };
 
 // number of rows of a group, and where its i-th row comes from and goes to
@@ -42,7 +51,15 @@ __device__ __forceinline__ int64_t out_offset(const LinearArgs &a, int g, int ro
     return row * a.o_stride + (a.lists == nullptr ? g * a.o_group : 0);
 }
 
-template <typename T> __device__ __forceinline__ float silu_of(float z) { return z * sigmoid_of<T>(z); }
+template <typename T> __device__ __forceinline__ float gated_value(const GateForm &f, float gate, float up) {
+    const float g = fminf(gate, f.limit), u = fminf(fmaxf(up, -f.limit), f.limit);
+    return g * sigmoid_of<T>(f.slope * g) * (u + f.shift);
+}
+__device__ __forceinline__ float result_of(const LinearArgs &a, float v) {
+    if (!a.squared_relu) return v;
+    v = fmaxf(v, 0.f);
+    return v * v;
+}
 
 // ---- any sizes, bf16 or fp32: tiles of 16 rows x 64 outputs in plain fp32 arithmetic ----------------
 template <typename T, typename O, bool kGated>
@@ -81,7 +98,7 @@ __global__ __launch_bounds__(256) void linear_any_kernel(LinearArgs a) {
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 const int n = n0 + c + 16 * j;
-                if (n < a.n_out) out[n] = Elem<O>::from_f32(kGated ? silu_of<T>(acc[0][j]) * acc[kParts - 1][j] : acc[0][j]);
+                if (n < a.n_out) out[n] = Elem<O>::from_f32(kGated ? gated_value<T>(a.gate, acc[0][j], acc[kParts - 1][j]) : result_of(a, acc[0][j]));
             }
         }
     }
@@ -91,11 +108,15 @@ __global__ __launch_bounds__(256) void linear_any_kernel(LinearArgs a) {
 // A workgroup takes 16 NB outputs of a group (NB blocks of 16 gates and the 16 ups that belong to them), its four
 // wavefronts a quarter of the inner dimension each, weights and rows straight from memory into operands
 // (weights first operand: an accumulator holds four consecutive outputs of one row).  The quarters meet in LDS.
+// Groups from all.groups on are those of `beside`: other, dense products of the same kind in the same launch.
 template <int MT, int NB, bool kGated, typename O>
-__global__ __launch_bounds__(256) void linear_skinny_kernel(LinearArgs a) {
+__global__ __launch_bounds__(256) void linear_skinny_kernel(const LinearArgs all, const LinearArgs beside) {
     constexpr int kParts = kGated ? 2 : 1, kBlocks = kParts * NB, kAhead = MT * NB == 1 ? 8 : 4;
     __shared__ __attribute__((aligned(16))) float part[4][MT * 16][kBlocks * 16 + 4];
-    const int g = blockIdx.y, n0 = blockIdx.x * 16 * NB;
+    const bool first = static_cast<int>(blockIdx.y) < all.groups;
+    const LinearArgs &a = first ? all : beside;
+    const int g = first ? blockIdx.y : blockIdx.y - all.groups, n0 = blockIdx.x * 16 * NB;
+    if (n0 >= a.n_out) return;                           // (the grid is as wide as the wider of the two)
     const int tid = threadIdx.x, lane = tid & 63, r = lane & 15, q = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int count = group_rows(a, g);
@@ -154,7 +175,7 @@ __global__ __launch_bounds__(256) void linear_skinny_kernel(LinearArgs a) {
                 v[p] = (part[0][m][c] + part[1][m][c]) + (part[2][m][c] + part[3][m][c]);
             }
             static_cast<O *>(a.out)[out_offset(a, g, group_row(a, g, m0 + m)) + n0 + n] =
-                Elem<O>::from_f32(kGated ? silu_of<bf16_t>(v[0]) * v[kParts - 1] : v[0]);
+                Elem<O>::from_f32(kGated ? gated_value<bf16_t>(a.gate, v[0], v[kParts - 1]) : result_of(a, v[0]));
         }
         __syncthreads();
     }
@@ -367,7 +388,7 @@ __global__ __launch_bounds__(256, BN > 128 ? 1 : 2) void linear_tile_kernel(cons
                 for (int n = 0; n < (kGated ? kTN / 2 : kTN); ++n) {
                     float y[4];
 #pragma unroll
-                    for (int j = 0; j < 4; ++j) y[j] = kGated ? silu_of<bf16_t>(acc[n][m][j]) * acc[kGated ? n + kTN / 2 : n][m][j] : acc[n][m][j];
+                    for (int j = 0; j < 4; ++j) y[j] = kGated ? gated_value<bf16_t>(a.gate, acc[n][m][j], acc[kGated ? n + kTN / 2 : n][m][j]) : acc[n][m][j];
                     *(__attribute__((address_space(3))) u32x2_t *)(lds + (16 * ((kRounds == 1 ? wm * kTM : 0) + m) + r) * kOutPitch + 2 * (kCols / 2 * wn + 16 * n + 4 * g)) =
                         u32x2_t{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
                 }
@@ -407,20 +428,21 @@ static int launch_any_linear(const LinearArgs &a, int32_t most_rows, hipStream_t
 
 // rows_hint: rows a group is expected to have
 template <int NB, bool kGated, typename O>
-static int launch_skinny_nb(const LinearArgs &a, int32_t rows_hint, int32_t most_rows, hipStream_t s) {
+static int launch_skinny_nb(const LinearArgs &a, const LinearArgs &beside, int32_t rows_hint, int32_t most_rows, hipStream_t s) {
     const int mt = rows_hint <= 16 ? 1 : rows_hint <= 32 ? 2 : 4;
     const int passes = std::max(1, (most_rows + 16 * mt - 1) / (16 * mt));
-    const dim3 grid((a.n_out + 16 * NB - 1) / (16 * NB), a.groups, a.lists ? 1 : std::min(passes, 65535)), block(256);
-    if (mt == 1) hipLaunchKernelGGL((linear_skinny_kernel<1, NB, kGated, O>), grid, block, 0, s, a);
-    else if (mt == 2) hipLaunchKernelGGL((linear_skinny_kernel<2, NB, kGated, O>), grid, block, 0, s, a);
-    else hipLaunchKernelGGL((linear_skinny_kernel<4, NB, kGated, O>), grid, block, 0, s, a);
+    const dim3 grid((std::max(a.n_out, beside.n_out) + 16 * NB - 1) / (16 * NB), a.groups + beside.groups, a.lists ? 1 : std::min(passes, 65535)), block(256);
+    if (mt == 1) hipLaunchKernelGGL((linear_skinny_kernel<1, NB, kGated, O>), grid, block, 0, s, a, beside);
+    else if (mt == 2) hipLaunchKernelGGL((linear_skinny_kernel<2, NB, kGated, O>), grid, block, 0, s, a, beside);
+    else hipLaunchKernelGGL((linear_skinny_kernel<4, NB, kGated, O>), grid, block, 0, s, a, beside);
     return launch_status();
 }
 template <bool kGated, typename O>
-static int launch_skinny(const LinearArgs &a, int32_t rows_hint, int32_t most_rows, int32_t busy_groups, hipStream_t s) {
+static int launch_skinny(const LinearArgs &a, int32_t rows_hint, int32_t most_rows, int32_t busy_groups, hipStream_t s,
+                         const LinearArgs &beside = LinearArgs{}) {
     // two blocks of outputs per workgroup where that leaves enough workgroups for the machine
-    if (static_cast<int64_t>(busy_groups) * ((a.n_out + 31) / 32) >= 512) return launch_skinny_nb<2, kGated, O>(a, rows_hint, most_rows, s);
-    return launch_skinny_nb<1, kGated, O>(a, rows_hint, most_rows, s);
+    if (static_cast<int64_t>(busy_groups) * ((a.n_out + 31) / 32) >= 512) return launch_skinny_nb<2, kGated, O>(a, beside, rows_hint, most_rows, s);
+    return launch_skinny_nb<1, kGated, O>(a, beside, rows_hint, most_rows, s);
 }
 
 static bool linear_matrix_ok(const LinearArgs &a) {
@@ -432,12 +454,13 @@ static bool linear_matrix_ok(const LinearArgs &a) {
 struct RouterArgs {
     const void *x;                   // [rows, width]
     int64_t x_stride;
-    const void *w;                   // [experts, width]
+    const void *w;                   // [experts + gates, width]
+    const float *bias;               // [experts + gates] or null
     int32_t *choice;                 // [rows, top]
-    float *weight;                   // [rows, top]
+    float *weight;                   // [rows, top + gates]: the choices' weights, the gates' sigmoids
     int32_t *lists, *counts;         // [experts, list_stride], [experts] (zero on entry)
     int64_t list_stride;
-    int32_t rows, width, experts, top;
+    int32_t rows, width, experts, gates, top;
     float scale;
 };
 
@@ -448,8 +471,9 @@ template <typename T, int TG, int NW, bool kMatrix>
 __global__ __launch_bounds__(64 * NW) void router_kernel(RouterArgs a) {
     constexpr int KS = NW / TG, kRows = 16 * TG, kThreads = 64 * NW;
     extern __shared__ __attribute__((aligned(16))) unsigned char router_smem[];
-    float *logits = reinterpret_cast<float *>(router_smem);                    // [kRows][experts]
-    float *partial = logits + kRows * a.experts;                               // [KS][kRows][64 + 4] (matrix form)
+    const int outs = a.experts + a.gates;
+    float *logits = reinterpret_cast<float *>(router_smem);                    // [kRows][outs]
+    float *partial = logits + kRows * outs;                                    // [KS][kRows][64 + 4] (matrix form)
     int *have = reinterpret_cast<int *>(partial + (kMatrix ? KS * kRows * 68 : 0)); // [experts]: this workgroup's assignments
     int *base = have + a.experts;                                              // [experts]
     int *mine = base + a.experts;                                              // [kRows * top]: expert, place among this workgroup's
@@ -463,14 +487,14 @@ __global__ __launch_bounds__(64 * NW) void router_kernel(RouterArgs a) {
         const int steps = (a.width + 31) / 32, per = (steps + KS - 1) / KS;
         const int s_begin = part * per, s_end = min(steps, s_begin + per);
         const bf16_t *x = static_cast<const bf16_t *>(a.x) + static_cast<int64_t>(row0 + min(16 * tg + r, rows - 1)) * a.x_stride;
-        for (int e0 = 0; e0 < a.experts; e0 += 64) {
-            const int blocks = min(4, (a.experts - e0 + 15) / 16);
+        for (int e0 = 0; e0 < outs; e0 += 64) {
+            const int blocks = min(4, (outs - e0 + 15) / 16);
             f32x4_t acc[4];
             const bf16_t *w[4];
 #pragma unroll
             for (int b = 0; b < 4; ++b) {
                 acc[b] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-                w[b] = static_cast<const bf16_t *>(a.w) + static_cast<int64_t>(min(e0 + 16 * b + r, a.experts - 1)) * a.width;
+                w[b] = static_cast<const bf16_t *>(a.w) + static_cast<int64_t>(min(e0 + 16 * b + r, outs - 1)) * a.width;
             }
             for (int s = s_begin; s < s_end; ++s) {
                 const int e = s * 32 + 8 * q;
@@ -489,20 +513,20 @@ __global__ __launch_bounds__(64 * NW) void router_kernel(RouterArgs a) {
             __syncthreads();
             for (int i = tid; i < kRows * 64; i += kThreads) {
                 const int row = i >> 6, e = i & 63;
-                if (e0 + e >= a.experts) continue;
-                float z = 0.f;
+                if (e0 + e >= outs) continue;
+                float z = a.bias != nullptr ? a.bias[e0 + e] : 0.f;
 #pragma unroll
                 for (int p = 0; p < KS; ++p) z += partial[(p * kRows + row) * 68 + e];
-                logits[row * a.experts + e0 + e] = z;
+                logits[row * outs + e0 + e] = z;
             }
             __syncthreads();
         }
     } else {
-        for (int i = tid; i < rows * a.experts; i += kThreads) {
-            const int row = i / a.experts, e = i % a.experts;
+        for (int i = tid; i < rows * outs; i += kThreads) {
+            const int row = i / outs, e = i % outs;
             const T *x = static_cast<const T *>(a.x) + static_cast<int64_t>(row0 + row) * a.x_stride;
             const T *w = static_cast<const T *>(a.w) + static_cast<int64_t>(e) * a.width;
-            float z = 0.f;
+            float z = a.bias != nullptr ? a.bias[e] : 0.f;
             for (int k = 0; k < a.width; ++k) z = fmaf(Elem<T>::to_f32(x[k]), Elem<T>::to_f32(w[k]), z);
             logits[i] = z;
         }
@@ -510,7 +534,7 @@ __global__ __launch_bounds__(64 * NW) void router_kernel(RouterArgs a) {
     }
     // one wavefront per row: softmax over the experts, then the best one `top` times (ties: the lower index)
     for (int row = wave; row < rows; row += NW) {
-        float *z = logits + row * a.experts;
+        float *z = logits + row * outs;
         float mine_z = -INFINITY, mx = -INFINITY;            // (up to 64 experts: one per lane)
         const bool narrow = a.experts <= 64;
         if (narrow) {
@@ -562,10 +586,12 @@ __global__ __launch_bounds__(64 * NW) void router_kernel(RouterArgs a) {
         __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
         const float f = a.scale / (chosen + kWeightGuard);
         const int64_t at = static_cast<int64_t>(row0 + row) * a.top;
+        float *out = a.weight + static_cast<int64_t>(row0 + row) * (a.top + a.gates);
+        for (int j = lane; j < a.gates; j += 64) out[a.top + j] = sigmoid_of<T>(z[a.experts + j]);
         for (int k = lane; k < a.top; k += 64) {
             const int who = mine[2 * (row * a.top + k)];
             a.choice[at + k] = who;
-            a.weight[at + k] = __int_as_float(mine[2 * (row * a.top + k) + 1]) * f;
+            out[k] = __int_as_float(mine[2 * (row * a.top + k) + 1]) * f;
             mine[2 * (row * a.top + k) + 1] = atomicAdd(&have[who], 1);
         }
     }
@@ -583,14 +609,14 @@ __global__ __launch_bounds__(64 * NW) void router_kernel(RouterArgs a) {
     }
 }
 
-static size_t router_lds(int32_t experts, int32_t top, int tg, int nw, bool matrix) {
+static size_t router_lds(int32_t experts, int32_t gates, int32_t top, int tg, int nw, bool matrix) {
     const size_t rows = 16 * static_cast<size_t>(tg);
-    return 4 * (rows * experts + (matrix ? nw / tg * rows * 68 : 0) + 2 * static_cast<size_t>(experts) + 2 * rows * top);
+    return 4 * (rows * (experts + gates) + (matrix ? nw / tg * rows * 68 : 0) + 2 * static_cast<size_t>(experts) + 2 * rows * top);
 }
 
 template <typename T, int TG, int NW, bool kMatrix>
 static int launch_router_tg(const RouterArgs &a, hipStream_t s) {
-    const size_t lds = router_lds(a.experts, a.top, TG, NW, kMatrix);
+    const size_t lds = router_lds(a.experts, a.gates, a.top, TG, NW, kMatrix);
     if (lds > 64 * 1024 &&
         hipFuncSetAttribute(reinterpret_cast<const void *>(&router_kernel<T, TG, NW, kMatrix>), hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds)) != hipSuccess)
         return NVA_ERR_LAUNCH_FAILED;
@@ -602,7 +628,7 @@ static int launch_router_tg(const RouterArgs &a, hipStream_t s) {
 
 extern "C" int nva_grouped_linear(const void *x, int64_t x_row_stride, int64_t x_group_stride, const void *weight, void *out,
                                   int64_t out_row_stride, int64_t out_group_stride, int32_t rows, int32_t groups, int32_t n_out,
-                                  int32_t k_in, int32_t dtype, int32_t out_dtype, void *stream) {
+                                  int32_t k_in, int32_t squared_relu, int32_t dtype, int32_t out_dtype, void *stream) {
     using namespace nva;
     if (rows < 0 || groups < 0 || n_out <= 0 || k_in <= 0) return NVA_ERR_BAD_SHAPE;
     if (!known_dtype(dtype) || !known_dtype(out_dtype) || (dtype == NVA_DTYPE_F32 && out_dtype != NVA_DTYPE_F32)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
@@ -612,7 +638,7 @@ extern "C" int nva_grouped_linear(const void *x, int64_t x_row_stride, int64_t x
     if (x_row_stride < k_in || out_row_stride < n_out || (groups > 1 && (x_group_stride < 0 || out_group_stride < n_out))) return NVA_ERR_BAD_STRIDE;
     LinearArgs a{};
     a.x = x; a.x_stride = x_row_stride; a.x_group = groups > 1 ? x_group_stride : 0; a.w = weight; a.out = out; a.o_stride = out_row_stride;
-    a.o_group = groups > 1 ? out_group_stride : 0; a.rows = rows; a.groups = groups; a.n_out = n_out; a.k = k_in; a.x_div = 1;
+    a.o_group = groups > 1 ? out_group_stride : 0; a.rows = rows; a.groups = groups; a.n_out = n_out; a.k = k_in; a.x_div = 1; a.squared_relu = squared_relu;
     hipStream_t s = static_cast<hipStream_t>(stream);
     if (dtype == NVA_DTYPE_F32) return launch_any_linear<float, float, false>(a, rows, s);
     if (!linear_matrix_ok(a))
@@ -620,21 +646,39 @@ extern "C" int nva_grouped_linear(const void *x, int64_t x_row_stride, int64_t x
     return out_dtype == NVA_DTYPE_F32 ? launch_skinny<false, float>(a, rows, rows, groups, s) : launch_skinny<false, bf16_t>(a, rows, rows, groups, s);
 }
 
-extern "C" int nva_routed_linear(const void *x, int64_t x_row_stride, const void *weight, void *out, const int32_t *lists,
-                                 const int32_t *counts, int64_t list_stride, int32_t rows, int32_t terms, int32_t experts,
-                                 int32_t n_out, int32_t k_in, int32_t x_per_row, int32_t gated, int32_t dtype, void *stream) {
-    using namespace nva;
+namespace nva {
+static int routed_args(LinearArgs &a, const void *x, int64_t x_row_stride, const void *weight, void *out, const int32_t *lists,
+                       const int32_t *counts, int64_t list_stride, int32_t rows, int32_t terms, int32_t experts, int32_t n_out,
+                       int32_t k_in, int32_t x_per_row, float gate_limit, float gate_slope, float gate_shift, int32_t dtype) {
     if (rows < 0 || terms <= 0 || experts <= 0 || n_out <= 0 || k_in <= 0 || list_stride < rows || terms > experts) return NVA_ERR_BAD_SHAPE;
     if (!known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     if (rows == 0) return NVA_OK;
     if (!x || !weight || !out || !lists || !counts) return NVA_ERR_NULL_POINTER;
     if (experts > 65535 || static_cast<int64_t>(rows) * terms > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
     if (x_row_stride < k_in) return NVA_ERR_BAD_STRIDE;
-    LinearArgs a{};
     a.x = x; a.x_stride = x_row_stride; a.w = weight; a.out = out; a.o_stride = n_out; a.lists = lists; a.counts = counts;
     a.list_stride = list_stride; a.rows = rows * terms; a.groups = experts; a.n_out = n_out; a.k = k_in; a.x_div = x_per_row ? terms : 1;
+    a.gate = GateForm{gate_limit, gate_slope, gate_shift};
+    return NVA_OK;
+}
+static int32_t rows_hint_of(int32_t rows, int32_t terms, int32_t experts) {
+    return static_cast<int32_t>((static_cast<int64_t>(rows) * terms * 3 / 2 + experts - 1) / experts);
+}
+static int32_t busy_experts(int32_t rows, int32_t terms, int32_t experts) {
+    return static_cast<int32_t>(std::min(static_cast<int64_t>(experts), static_cast<int64_t>(rows) * terms));
+}
+}  // namespace nva
+
+extern "C" int nva_routed_linear(const void *x, int64_t x_row_stride, const void *weight, void *out, const int32_t *lists,
+                                 const int32_t *counts, int64_t list_stride, int32_t rows, int32_t terms, int32_t experts,
+                                 int32_t n_out, int32_t k_in, int32_t x_per_row, int32_t gated, float gate_limit, float gate_slope, float gate_shift,
+                                 int32_t dtype, void *stream) {
+    using namespace nva;
+    LinearArgs a{};
+    const int rc = routed_args(a, x, x_row_stride, weight, out, lists, counts, list_stride, rows, terms, experts, n_out, k_in, x_per_row,
+                               gate_limit, gate_slope, gate_shift, dtype);
+    if (rc != NVA_OK || rows == 0) return rc;
     hipStream_t s = static_cast<hipStream_t>(stream);
-    const int32_t hint = static_cast<int32_t>((static_cast<int64_t>(rows) * terms * 3 / 2 + experts - 1) / experts);
     if (dtype == NVA_DTYPE_F32) return gated ? launch_any_linear<float, float, true>(a, rows, s) : launch_any_linear<float, float, false>(a, rows, s);
     if (!linear_matrix_ok(a)) return gated ? launch_any_linear<bf16_t, bf16_t, true>(a, rows, s) : launch_any_linear<bf16_t, bf16_t, false>(a, rows, s);
     const int32_t average = static_cast<int32_t>(static_cast<int64_t>(rows) * terms / experts);
@@ -643,23 +687,45 @@ extern "C" int nva_routed_linear(const void *x, int64_t x_row_stride, const void
         if (average >= 512) return gated ? launch_tiles<256, 128, true>(a, s) : launch_tiles<256, 128, false>(a, s);
         return gated ? launch_tiles<128, 128, true>(a, s) : launch_tiles<128, 128, false>(a, s);
     }
-    const int32_t busy = static_cast<int32_t>(std::min(static_cast<int64_t>(experts), static_cast<int64_t>(rows) * terms));
+    const int32_t hint = rows_hint_of(rows, terms, experts), busy = busy_experts(rows, terms, experts);
     return gated ? launch_skinny<true, bf16_t>(a, hint, rows, busy, s) : launch_skinny<false, bf16_t>(a, hint, rows, busy, s);
 }
 
-extern "C" int nva_router(const void *x, int64_t x_row_stride, const void *weight, int32_t *choice, float *choice_weight,
-                          int32_t *lists, int32_t *counts, int64_t list_stride, int32_t rows, int32_t width, int32_t experts,
-                          int32_t top, float scale, int32_t dtype, void *stream) {
+extern "C" int nva_routed_shared_linear(const void *x, int64_t x_row_stride, const void *weight, void *out, const int32_t *lists,
+                                        const int32_t *counts, int64_t list_stride, int32_t rows, int32_t terms, int32_t experts,
+                                        int32_t n_out, int32_t k_in, int32_t x_per_row, int32_t gated, float gate_limit, float gate_slope,
+                                        float gate_shift, const void *shared_x, int64_t shared_x_row_stride, const void *shared_weight,
+                                        void *shared_out, int32_t shared_n_out, int32_t shared_k_in, float shared_gate_limit, void *stream) {
     using namespace nva;
-    if (rows < 0 || width <= 0 || experts <= 0 || top <= 0 || top > experts || list_stride < rows) return NVA_ERR_BAD_SHAPE;
-    if (!known_dtype(dtype) || experts > 1024 || top > 128) return NVA_ERR_UNSUPPORTED_GEOMETRY;
+    LinearArgs a{}, b{};
+    const int rc = routed_args(a, x, x_row_stride, weight, out, lists, counts, list_stride, rows, terms, experts, n_out, k_in, x_per_row,
+                               gate_limit, gate_slope, gate_shift, NVA_DTYPE_BF16);
+    if (rc != NVA_OK) return rc;
+    if (shared_n_out <= 0 || shared_k_in <= 0) return NVA_ERR_BAD_SHAPE;
+    if (rows == 0) return NVA_OK;
+    if (!shared_x || !shared_weight || !shared_out) return NVA_ERR_NULL_POINTER;
+    if (shared_x_row_stride < shared_k_in) return NVA_ERR_BAD_STRIDE;
+    b.x = shared_x; b.x_stride = shared_x_row_stride; b.w = shared_weight; b.out = shared_out; b.o_stride = shared_n_out; b.rows = rows; b.groups = 1;
+    b.n_out = shared_n_out; b.k = shared_k_in; b.x_div = 1; b.gate = GateForm{shared_gate_limit, gate_slope, gate_shift};
+    if (!linear_matrix_ok(a) || !linear_matrix_ok(b)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    const int32_t hint = rows_hint_of(rows, terms, experts), busy = busy_experts(rows, terms, experts);
+    return gated ? launch_skinny<true, bf16_t>(a, hint, rows, busy, s, b) : launch_skinny<false, bf16_t>(a, hint, rows, busy, s, b);
+}
+
+extern "C" int nva_router(const void *x, int64_t x_row_stride, const void *weight, const float *bias, int32_t *choice,
+                          float *choice_weight, int32_t *lists, int32_t *counts, int64_t list_stride, int32_t rows, int32_t width,
+                          int32_t experts, int32_t gates, int32_t top, float scale, int32_t dtype, void *stream) {
+    using namespace nva;
+    if (rows < 0 || width <= 0 || experts <= 0 || gates < 0 || top <= 0 || top > experts || list_stride < rows) return NVA_ERR_BAD_SHAPE;
+    if (!known_dtype(dtype) || experts > 1024 || gates > 64 || top > 128) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     if (rows == 0) return NVA_OK;
     if (!x || !weight || !choice || !choice_weight || !lists || !counts) return NVA_ERR_NULL_POINTER;
     if (x_row_stride < width) return NVA_ERR_BAD_STRIDE;
     if (static_cast<int64_t>(rows) * top > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
     RouterArgs a{};
-    a.x = x; a.x_stride = x_row_stride; a.w = weight; a.choice = choice; a.weight = choice_weight; a.lists = lists; a.counts = counts;
-    a.list_stride = list_stride; a.rows = rows; a.width = width; a.experts = experts; a.top = top; a.scale = scale;
+    a.x = x; a.x_stride = x_row_stride; a.w = weight; a.bias = bias; a.choice = choice; a.weight = choice_weight; a.lists = lists; a.counts = counts;
+    a.list_stride = list_stride; a.rows = rows; a.width = width; a.experts = experts; a.gates = gates; a.top = top; a.scale = scale;
     hipStream_t s = static_cast<hipStream_t>(stream);
     const bool many = rows >= 4096 && experts <= 128 && top <= 32;       // more rows per workgroup: fewer additions to the counters
     if (dtype == NVA_DTYPE_F32) return launch_router_tg<float, 1, 8, false>(a, s);

@@ -2,7 +2,6 @@
 //   embed_norm        residual = embed[id] * scale; out = layer_norm(residual)
 //   post_add_norm     residual += layer_norm(y); out = layer_norm'(residual)     (the norm after a
 //                     sublayer, the residual add and the norm before the next one in one kernel)
-//   clamped_gate      out = g sigmoid(alpha g) (u + 1) with g capped and u clamped
 //   conv_rope_store   short causal convolution of q, k and v, rotary embedding of q and k, cache write
 //   conv_state_update the last taps - 1 projected rows of every portion, kept for the next one
 // Tensors are bf16 or fp32 (one template argument); every sum, norm and angle is fp32.
@@ -182,28 +181,6 @@ static void launch_norm(const NormArgs &a, bool vector, hipStream_t s) {
 static bool norm_vector_ok(const NormArgs &a) {
     return a.width % 8 == 0 && a.width <= 4096 && a.x_stride % 8 == 0 && aligned16(a.x) && aligned16(a.residual) &&
            aligned16(a.w_post) && aligned16(a.b_post) && aligned16(a.w_next) && aligned16(a.b_next) && aligned16(a.out);
-}
-
-// ---- gated feed-forward activation ---------------------------------------------------------------
-
-template <typename T, int V>
-__global__ __launch_bounds__(256) void clamped_gate_kernel(const T *__restrict__ x, int64_t stride, T *__restrict__ out,
-                                                           int64_t total, int32_t per_row, int32_t inter, float limit,
-                                                           float alpha) {
-    const int64_t idx = static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x;
-    if (idx >= total) return;
-    const int64_t row = idx / per_row;
-    const int e = static_cast<int>(idx % per_row) * V;
-    float g[V], u[V], y[V];
-    load_f32<T, V>(x + row * stride + e, g);
-    load_f32<T, V>(x + row * stride + inter + e, u);
-#pragma unroll
-    for (int i = 0; i < V; ++i) {
-        const float gc = fminf(g[i], limit);
-        const float uc = fminf(fmaxf(u[i], -limit), limit);
-        y[i] = gc * sigmoid_of<T>(alpha * gc) * (uc + 1.0f);
-    }
-    store_f32<T, V>(out + row * inter + e, y);
 }
 
 // ---- short convolution + rotary embedding + cache write ---------------------------------------------
@@ -498,34 +475,6 @@ extern "C" int nva_post_add_norm(const void *y, int64_t y_row_stride, float *res
     hipStream_t s = static_cast<hipStream_t>(stream);
     if (dtype == NVA_DTYPE_BF16) launch_norm<bf16_t, false>(a, norm_vector_ok(a), s);
     else launch_norm<float, false>(a, norm_vector_ok(a), s);
-    return launch_status();
-}
-
-extern "C" int nva_clamped_gate(const void *x, int64_t x_row_stride, void *out, int32_t rows, int32_t inter, float limit,
-                                float alpha, int32_t dtype, void *stream) {
-    using namespace nva;
-    if (rows < 0 || inter <= 0) return NVA_ERR_BAD_SHAPE;
-    if (!known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
-    if (rows == 0) return NVA_OK;
-    if (!x || !out) return NVA_ERR_NULL_POINTER;
-    if (x_row_stride < 2 * static_cast<int64_t>(inter)) return NVA_ERR_BAD_STRIDE;
-    const bool vector = inter % 8 == 0 && x_row_stride % 8 == 0 && aligned16(x) && aligned16(out);
-    const int32_t per_row = vector ? inter / 8 : inter;
-    const int64_t total = static_cast<int64_t>(rows) * per_row;
-    if ((total + 255) / 256 > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
-    const dim3 grid(static_cast<uint32_t>((total + 255) / 256)), block(256);
-    hipStream_t s = static_cast<hipStream_t>(stream);
-    if (dtype == NVA_DTYPE_BF16) {
-        const bf16_t *xp = static_cast<const bf16_t *>(x);
-        bf16_t *op = static_cast<bf16_t *>(out);
-        if (vector) hipLaunchKernelGGL((clamped_gate_kernel<bf16_t, 8>), grid, block, 0, s, xp, x_row_stride, op, total, per_row, inter, limit, alpha);
-        else hipLaunchKernelGGL((clamped_gate_kernel<bf16_t, 1>), grid, block, 0, s, xp, x_row_stride, op, total, per_row, inter, limit, alpha);
-    } else {
-        const float *xp = static_cast<const float *>(x);
-        float *op = static_cast<float *>(out);
-        if (vector) hipLaunchKernelGGL((clamped_gate_kernel<float, 8>), grid, block, 0, s, xp, x_row_stride, op, total, per_row, inter, limit, alpha);
-        else hipLaunchKernelGGL((clamped_gate_kernel<float, 1>), grid, block, 0, s, xp, x_row_stride, op, total, per_row, inter, limit, alpha);
-    }
     return launch_status();
 }
 

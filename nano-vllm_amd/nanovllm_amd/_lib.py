@@ -1,9 +1,11 @@
 """ctypes binding of the C ABI declared in include/nanovllm_amd.h.
 
 Shared libraries are built in-tree, next to this file, by ``csrc/Makefile``: ``libnanovllm_amd.so``
-(the attention hot path), ``libnanovllm_mixers.so`` (chunked attention and retention of layered models)
-and ``libnanovllm_latent.so`` (latent attention, matrix memory, routed experts).  Each is opened when one of its symbols is first used, so a model needs only its own.  There
-is no fallback: an op whose library is missing raises.
+(the attention hot path), ``libnanovllm_mixers.so`` (chunked attention and retention of layered models),
+``libnanovllm_latent.so`` (latent attention, matrix memory, routed experts) and ``libnanovllm_masked.so``
+(attention under masks with sinks and gates, routed experts).  Each is opened when one of its symbols is first
+used, so a model needs only its own; a kernel that several kinds of model need is in several, and comes from
+the first that is there.  There is no fallback: an op whose library is missing raises.
 """
 from __future__ import annotations
 
@@ -14,6 +16,7 @@ _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libnanovllm_amd.so")
 MIXERS_LIB_PATH = os.path.join(_HERE, "libnanovllm_mixers.so")
 LATENT_LIB_PATH = os.path.join(_HERE, "libnanovllm_latent.so")
+MASKED_LIB_PATH = os.path.join(_HERE, "libnanovllm_masked.so")
 
 # status codes of enum nva_status
 OK = 0
@@ -63,15 +66,25 @@ SIGNATURES = {
     "nva_chunk_attn_workspace_bytes": (_sz, [_i32, _i32, _i32, _i32, _i32, _i32, _i32]),
     "nva_chunk_attn": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _i64, _i32, _vp, _vp, _vp, _vp, _vp, _sz, _i32, _i32, _i32, _i32,
                                  _i32, _i32, _i32, _i32, _i32, _i32, _f32, _f32, _i32, _vp]),
+    "nva_masked_attn": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _i64, _i32, _vp, _vp, _vp, _vp, _vp, _sz, _i32, _i32, _i32, _i32,
+                                  _i32, _i32, _i32, _i32, _i32, _i32, _i32, _f32, _f32, _vp, _vp, _i64, _i32, _vp]),
+    "nva_qkv_prepare": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _i32, _vp, _vp, _vp, _vp, _vp, _i64, _vp, _vp, _vp, _i32, _i32, _i32,
+                                  _i32, _i32, _i32, _i32, _i32, _f32, _i32, _vp]),
+    "nva_squared_relu": (C.c_int, [_vp, _i64, _vp, _i32, _i32, _i32, _vp]),
+    "nva_soft_cap": (C.c_int, [_vp, _i32, _i32, _f32, _i32, _vp]),
     "nva_retention_workspace_bytes": (_sz, [_i32, _i32, _i32, _i32, _i32, _i32, _i32]),
     "nva_retention": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _sz, _i32, _i32, _i32, _i32, _i32,
                                 _i32, _i32, _i32, _i32, _f32, _f32, _i32, _vp]),
     "nva_embed_rms_norms": (C.c_int, [_vp, _vp, _f32, _vp, _vp, _f32, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _i32, _f32, _i32, _vp]),
     "nva_branches_rms_norms": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _i32, _vp, _f32, _vp, _vp, _vp, _f32, _vp, _vp, _vp, _vp, _i32,
                                          _i32, _i32, _i32, _f32, _i32, _vp]),
-    "nva_grouped_linear": (C.c_int, [_vp, _i64, _i64, _vp, _vp, _i64, _i64, _i32, _i32, _i32, _i32, _i32, _i32, _vp]),
-    "nva_router": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _f32, _i32, _vp]),
-    "nva_routed_linear": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _vp]),
+    "nva_grouped_linear": (C.c_int, [_vp, _i64, _i64, _vp, _vp, _i64, _i64, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _vp]),
+    "nva_router": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _i32, _f32, _i32, _vp]),
+    "nva_routed_linear": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _f32, _f32, _f32, _i32, _vp]),
+    "nva_routed_shared_linear": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _f32, _f32, _f32,
+                                           _vp, _i64, _vp, _vp, _i32, _i32, _f32, _vp]),
+    "nva_post_rms_norms": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _i64, _i32, _vp, _vp, _vp, _f32, _vp, _vp, _vp, _i32, _i32, _i32, _i32,
+                                     _f32, _i32, _vp]),
     "nva_latent_prepare": (C.c_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _vp, _vp, _vp, _i32, _i32, _i32, _i32, _i32,
                                      _i32, _f32, _i32, _vp]),
     "nva_latent_attn_workspace_bytes": (_sz, [_i32] * 8),
@@ -87,12 +100,16 @@ SIGNATURES = {
     "nva_probe_stream_read": (C.c_int, [_vp, _i64, _vp, _vp]),
 }
 
-# symbols of the libraries of layered models; the common ones are in every library, all others in libnanovllm_amd.so
-MIXER_SYMBOLS = {"nva_embed_norm", "nva_post_add_norm", "nva_clamped_gate", "nva_conv_rope_store", "nva_chunk_attn",
-                 "nva_chunk_attn_workspace_bytes", "nva_retention", "nva_retention_workspace_bytes"}
-LATENT_SYMBOLS = {"nva_embed_rms_norms", "nva_branches_rms_norms", "nva_grouped_linear", "nva_router", "nva_routed_linear",
-                  "nva_latent_prepare", "nva_latent_attn", "nva_latent_attn_workspace_bytes", "nva_latent_gather",
-                  "nva_latent_prefill", "nva_latent_prefill_supported", "nva_mlstm", "nva_mlstm_workspace_bytes"}
+# which libraries of layered models hold a symbol; the common ones are in every library, all others in libnanovllm_amd.so
+_NORM_SYMBOLS = {"nva_embed_rms_norms", "nva_branches_rms_norms", "nva_post_rms_norms"}
+_EXPERT_SYMBOLS = {"nva_grouped_linear", "nva_router", "nva_routed_linear", "nva_routed_shared_linear"}
+_ACTIVATION_SYMBOLS = {"nva_clamped_gate", "nva_squared_relu", "nva_soft_cap"}
+_ATTN_SYMBOLS = {"nva_chunk_attn", "nva_chunk_attn_workspace_bytes", "nva_masked_attn"}
+MIXER_SYMBOLS = {"nva_embed_norm", "nva_post_add_norm", "nva_conv_rope_store", "nva_retention",
+                 "nva_retention_workspace_bytes"} | _ATTN_SYMBOLS | _ACTIVATION_SYMBOLS
+LATENT_SYMBOLS = {"nva_latent_prepare", "nva_latent_attn", "nva_latent_attn_workspace_bytes", "nva_latent_gather",
+                  "nva_latent_prefill", "nva_latent_prefill_supported", "nva_mlstm", "nva_mlstm_workspace_bytes"} | _NORM_SYMBOLS | _EXPERT_SYMBOLS
+MASKED_SYMBOLS = {"nva_qkv_prepare"} | _ATTN_SYMBOLS | _ACTIVATION_SYMBOLS | _NORM_SYMBOLS | _EXPERT_SYMBOLS
 COMMON_SYMBOLS = {"nva_version", "nva_status_string", "nva_device_count", "nva_stage_decode_inputs"}
 
 
@@ -109,9 +126,11 @@ class _Symbols:
     def __getattr__(self, name: str):
         if name not in SIGNATURES:
             raise AttributeError(name)
-        paths = [MIXERS_LIB_PATH] if name in MIXER_SYMBOLS else [LATENT_LIB_PATH] if name in LATENT_SYMBOLS else [LIB_PATH]
+        layered = ((MIXER_SYMBOLS, MIXERS_LIB_PATH), (LATENT_SYMBOLS, LATENT_LIB_PATH), (MASKED_SYMBOLS, MASKED_LIB_PATH))
         if name in COMMON_SYMBOLS:
-            paths += [MIXERS_LIB_PATH, LATENT_LIB_PATH]
+            paths = [LIB_PATH] + [path for _, path in layered]
+        else:
+            paths = [path for names, path in layered if name in names] or [LIB_PATH]
         path = next((p for p in paths if os.path.exists(p)), None)
         if path is None:
             raise _missing(paths[0])
@@ -157,8 +176,21 @@ def load_latent():
     return _symbols
 
 
+def load_masked():
+    """The entry points of the library of masked attention and experts, and the common ones."""
+    if not os.path.exists(MASKED_LIB_PATH):
+        raise _missing(MASKED_LIB_PATH)
+    return _symbols
+
+
+def load_shared():
+    """Entry points that several libraries hold: each comes from the first that is there."""
+    return _symbols
+
+
 # kernel sets by name: the make target that builds one, its library and its loader
-LIBRARIES = {"path": (LIB_PATH, load), "mixers": (MIXERS_LIB_PATH, load_mixers), "latent": (LATENT_LIB_PATH, load_latent)}
+LIBRARIES = {"path": (LIB_PATH, load), "mixers": (MIXERS_LIB_PATH, load_mixers), "latent": (LATENT_LIB_PATH, load_latent),
+             "masked": (MASKED_LIB_PATH, load_masked)}
 
 
 def load_set(name: str):

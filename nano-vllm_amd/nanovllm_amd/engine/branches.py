@@ -1,5 +1,6 @@
 """The residual step of layers whose mixer and feed-forward read the same point of the stream: both branches'
-results are added at once and the next layer's two norms are taken in the same pass over the row."""
+results are added at once and the next layer's two norms are taken in the same pass over the row; and of layers
+that norm what a sublayer gives, where the next sublayer reads the stream itself."""
 from __future__ import annotations
 
 from typing import Optional, Tuple
@@ -16,18 +17,18 @@ def _outputs(rows: int, table: torch.Tensor, second: Optional[torch.Tensor]):
     return out1, None if second is None else torch.empty_like(out1)
 
 
-def embed_rms_norms(ids: torch.Tensor, table: torch.Tensor, scale: float, weights: Tuple[torch.Tensor, Optional[torch.Tensor]],
+def embed_rms_norms(ids: torch.Tensor, table: torch.Tensor, scale: float, weights: Tuple[Optional[torch.Tensor], Optional[torch.Tensor]],
                     eps: float, weight_offset: float = 0.0, clear: Optional[torch.Tensor] = None):
     """``residual = table[ids] * scale`` (fp32) and its RMS norms with one or two weights (stored as the
-    deviation from ``weight_offset``); ``clear``: int32 counters to zero.  Returns (residual, out1, out2)."""
+    deviation from ``weight_offset``; without weights: the residual itself, rounded); ``clear``: int32 counters to zero.  Returns (residual, out1, out2)."""
     vocab, width = table.shape
     assert ids.dtype == torch.int64 and ids.is_contiguous() and table.is_contiguous()
     _need_cuda(ids, table)
     n = ids.numel()
     residual = torch.empty((n, width), dtype=torch.float32, device=table.device)
     out1, out2 = _outputs(n, table, weights[1])
-    rc = _lib.load_latent().nva_embed_rms_norms(
-        ids.data_ptr(), table.data_ptr(), float(scale), weights[0].data_ptr(), _ptr(weights[1]), float(weight_offset),
+    rc = _lib.load_shared().nva_embed_rms_norms(
+        ids.data_ptr(), table.data_ptr(), float(scale), _ptr(weights[0]), _ptr(weights[1]), float(weight_offset),
         residual.data_ptr(), out1.data_ptr(), _ptr(out2), _ptr(clear), 0 if clear is None else clear.numel(), n, width, vocab,
         float(eps), _DTYPE[table.dtype], _stream())
     _lib.check(rc, "nva_embed_rms_norms")
@@ -54,9 +55,39 @@ def branches_rms_norms(residual: torch.Tensor, mult: float, y1: Optional[torch.T
     if rows is not None:
         assert rows.dtype == torch.int32 and rows.is_contiguous()
     out1, out2 = _outputs(count, weights[0], weights[1])
-    rc = _lib.load_latent().nva_branches_rms_norms(
+    rc = _lib.load_shared().nva_branches_rms_norms(
         _ptr(y1), 0 if y1 is None else y1.stride(0), _ptr(gain1), _ptr(y2), _ptr(term_weight), terms, _ptr(gain2), float(mult),
         residual.data_ptr(), weights[0].data_ptr(), _ptr(weights[1]), float(weight_offset), out1.data_ptr(), _ptr(out2), _ptr(rows),
         _ptr(clear), 0 if clear is None else clear.numel(), count, n, width, float(eps), _DTYPE[weights[0].dtype], _stream())
     _lib.check(rc, "nva_branches_rms_norms")
     return out1, out2
+
+
+def post_rms_norms(residual: torch.Tensor, y1: Optional[torch.Tensor], y1_weight: Optional[torch.Tensor], y2: Optional[torch.Tensor],
+                   term_weight: Optional[torch.Tensor], post: torch.Tensor, nxt: Optional[torch.Tensor], eps: float, weight_offset: float = 0.0,
+                   rows: Optional[torch.Tensor] = None, clear: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``residual += rms_norm(y1_weight * y1 + sum_k term_weight[:, k] * y2[:, k])`` in place; returns the residual, rounded, or with
+    ``nxt`` its norm.  ``y1_weight [n]`` and ``term_weight [n, terms]`` may be columns of one tensor.  With ``rows`` (int32) only
+    those rows are computed and the residual stays as it is."""
+    n, width = residual.shape
+    assert residual.dtype == torch.float32 and residual.is_contiguous() and (y1 is not None or y2 is not None)
+    _need_cuda(residual, post)
+    terms = stride = 0
+    if y1 is not None:
+        assert y1.shape == residual.shape and y1.stride(1) == 1 and y1.dtype == post.dtype
+    if y2 is not None:
+        terms = y2.shape[0] // max(n, 1)
+        assert y2.shape == (n * terms, width) and y2.is_contiguous() and y2.dtype == post.dtype
+    for w, shape in ((y1_weight, (n,)), (term_weight, (n, terms))):
+        if w is not None:
+            assert w.shape == shape and w.dtype == torch.float32 and stride in (0, w.stride(0)) and (w.dim() == 1 or w.stride(1) == 1)
+            stride = w.stride(0)
+    count = n if rows is None else rows.numel()
+    assert rows is None or (rows.dtype == torch.int32 and rows.is_contiguous())
+    out, _ = _outputs(count, post, None)
+    rc = _lib.load_shared().nva_post_rms_norms(
+        _ptr(y1), 0 if y1 is None else y1.stride(0), _ptr(y1_weight), _ptr(y2), _ptr(term_weight), stride, terms, post.data_ptr(),
+        residual.data_ptr(), _ptr(nxt), float(weight_offset), out.data_ptr(), _ptr(rows), _ptr(clear), 0 if clear is None else clear.numel(),
+        count, n, width, float(eps), _DTYPE[post.dtype], _stream())
+    _lib.check(rc, "nva_post_rms_norms")
+    return out

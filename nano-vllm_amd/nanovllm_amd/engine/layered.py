@@ -1,7 +1,7 @@
 """What layered model families share: a stack of layers whose mixers own their share of the paged cache and
 of the state slots, an fp32 residual stream, weights from safetensors.
 
-A layer has ``mixer`` (``mixers.py``, ``latent.py``, ``mlstm.py``: ``bind``, ``unbind``, ``kv_elements_per_token``,
+A layer has ``mixer`` (``mixers.py``, ``latent.py``, ``mlstm.py``, ``masked.py``: ``bind``, ``unbind``, ``kv_elements_per_token``,
 ``state_bytes_per_slot``); a family implements ``load_tensors`` and ``forward_layers``.
 """
 from __future__ import annotations
@@ -14,14 +14,14 @@ from .loader import TensorFolder
 
 class LayeredModel(nn.Module):
 
-    def __init__(self, cfg):
+    def __init__(self, cfg, tied: bool = False):
         super().__init__()
         # 32-bit accumulation in the library's matrix products, and full fp32 ones
         torch.backends.cuda.matmul.allow_bf16_reduced_precision_reduction = False
         torch.backends.cuda.matmul.allow_tf32 = False
         self.cfg = cfg
         self.embed = nn.Parameter(torch.empty(cfg.vocab_size, cfg.hidden_size))
-        self.head = nn.Parameter(torch.empty(cfg.vocab_size, cfg.hidden_size))
+        self.head = self.embed if tied else nn.Parameter(torch.empty(cfg.vocab_size, cfg.hidden_size))
         self.layers: list = []
 
     def random_weights(self, device, seed: int) -> None:
@@ -35,7 +35,8 @@ class LayeredModel(nn.Module):
     def load_weights(self, folder: str) -> None:
         tensors = TensorFolder(folder)
         self.embed.copy_(tensors.take("embed", self.embed.shape))
-        self.head.copy_(tensors.take("head", self.head.shape))
+        if self.head is not self.embed:
+            self.head.copy_(tensors.take("head", self.head.shape))
         self.load_tensors(tensors.take)
         if tensors.unused():
             raise ValueError(f"tensors without a place in the model: {', '.join(tensors.unused()[:5])}")

@@ -98,10 +98,28 @@ def clamped_gate(x: torch.Tensor, limit: float, alpha: float) -> torch.Tensor:
     _need_cuda(x)
     inter = x.shape[1] // 2
     out = torch.empty((x.shape[0], inter), dtype=x.dtype, device=x.device)
-    rc = _lib.load_mixers().nva_clamped_gate(x.data_ptr(), x.stride(0), out.data_ptr(), x.shape[0], inter, float(limit),
+    rc = _lib.load_shared().nva_clamped_gate(x.data_ptr(), x.stride(0), out.data_ptr(), x.shape[0], inter, float(limit),
                                       float(alpha), _DTYPE[x.dtype], _stream())
     _lib.check(rc, "nva_clamped_gate")
     return out
+
+
+def squared_relu_(x: torch.Tensor) -> torch.Tensor:
+    """``max(x, 0)^2`` in place."""
+    assert x.dim() == 2 and x.is_contiguous()
+    _need_cuda(x)
+    rc = _lib.load_shared().nva_squared_relu(x.data_ptr(), x.stride(0), x.data_ptr(), x.shape[0], x.shape[1], _DTYPE[x.dtype], _stream())
+    _lib.check(rc, "nva_squared_relu")
+    return x
+
+
+def soft_cap_(x: torch.Tensor, cap: float) -> torch.Tensor:
+    """``cap tanh(x / cap)`` in place."""
+    assert x.dim() == 2 and x.is_contiguous()
+    _need_cuda(x)
+    rc = _lib.load_shared().nva_soft_cap(x.data_ptr(), x.shape[0], x.shape[1], float(cap), _DTYPE[x.dtype], _stream())
+    _lib.check(rc, "nva_soft_cap")
+    return x
 
 
 def conv_rope_store(qkv: torch.Tensor, conv_weight: torch.Tensor, conv_state: Optional[torch.Tensor], group: RowGroup,
@@ -168,11 +186,27 @@ def retention(qkvg: torch.Tensor, state: torch.Tensor, group: RowGroup, rope: Op
 # ---- rotary tables -------------------------------------------------------------------------------
 
 @dataclass(frozen=True)
+class RotaryScaling:
+    """Frequencies stretched to longer contexts than ``original``: those that turn less than ``low`` times over it are
+    divided by ``factor``, those that turn more than ``high`` times stay, the ones between are blended."""
+    factor: float
+    low: float
+    high: float
+    original: float
+
+    def __call__(self, freq: torch.Tensor) -> torch.Tensor:
+        turns = self.original * freq / (2.0 * math.pi)
+        keep = ((turns - self.low) / (self.high - self.low) if self.high > self.low else (turns >= self.high).to(freq.dtype)).clamp(0.0, 1.0)
+        return freq * (keep + (1.0 - keep) / self.factor)
+
+
+@dataclass(frozen=True)
 class Rotary:
-    """Rotation of the first ``dims`` elements of a head by position * base^(-2i/dims); which elements make pair i
-    (i and i + dims / 2, or neighbours) is the mixer's affair."""
+    """Rotation of the first ``dims`` elements of a head by position * base^(-2i/dims), the frequencies possibly scaled;
+    which elements make pair i (i and i + dims / 2, or neighbours) is the mixer's affair."""
     base: float
     dims: int
+    scaling: Optional[RotaryScaling] = None
 
 
 class RopeTables:
@@ -189,6 +223,8 @@ class RopeTables:
             if rot.dims > 0:
                 i = torch.arange(rot.dims // 2, dtype=torch.float64)
                 freq = torch.exp(-2.0 * i / rot.dims * math.log(rot.base))
+                if rot.scaling is not None:
+                    freq = rot.scaling(freq)
                 angle = torch.outer(torch.arange(self.max_position, dtype=torch.float64), freq)
                 table = torch.cat([angle.cos(), angle.sin()], dim=-1).float().contiguous().to(self.device)
             self._tables[rot] = table

@@ -170,7 +170,7 @@ class Pidutar(LayeredModel):
         for i in range(first, last):
             layer, w = layers[i], layers[i].weights
             y1 = layer.mixer(hidden[0])
-            y2, weight = layer.mlp(hidden[1]) if layer.mlp is not None else (None, None)
+            y2, _, weight = layer.mlp(hidden[1]) if layer.mlp is not None else (None, None, None)
             step = (residual, cfg.residual_mult, y1, w.ls1, y2, weight, w.ls2)
             if i + 1 < len(layers):
                 nxt = layers[i + 1].weights

@@ -47,6 +47,7 @@ def register(architecture: str, config: str, model: str, kernels: str = "path") 
 register("Qwen3ForCausalLM", ".config:ModelConfig", ".model:Qwen3ForCausalLM")
 register("Kaparax", ".kaparax:KaparaxConfig", ".kaparax:Kaparax", "mixers")
 register("Pidutar", ".pidutar:PidutarConfig", ".pidutar:Pidutar", "latent")
+register("Sokolorn", ".sokolorn:SokolornConfig", ".sokolorn:Sokolorn", "masked")
 
 
 def family_of_raw(raw: dict) -> Family:

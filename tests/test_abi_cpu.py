@@ -304,21 +304,72 @@ def test_branches_and_experts_validation():
                    (dict(ys=63), _lib.ERR_BAD_STRIDE), (dict(terms=0), _lib.ERR_BAD_SHAPE), (dict(rows=3), _lib.ERR_BAD_SHAPE),
                    (dict(rows_of=A, src=0), _lib.ERR_BAD_SHAPE), (dict(rows=0, src=0), _lib.OK), (dict(dtype=-1), _lib.ERR_UNSUPPORTED_GEOMETRY)):
         assert _with(ok, lib.nva_branches_rms_norms, **kw) == rc, kw
-    ok = dict(x=A, xs=256, xg=64, w=A, out=A, os=256, og=64, rows=4, groups=4, n_out=64, k=64, dtype=0, odt=0, stream=None)
+    ok = dict(x=A, xs=256, xg=64, w=A, out=A, os=256, og=64, rows=4, groups=4, n_out=64, k=64, relu=0, dtype=0, odt=0, stream=None)
     for kw, rc in ((dict(x=None), _lib.ERR_NULL_POINTER), (dict(w=None), _lib.ERR_NULL_POINTER), (dict(xs=63), _lib.ERR_BAD_STRIDE),
                    (dict(og=63), _lib.ERR_BAD_STRIDE), (dict(k=0), _lib.ERR_BAD_SHAPE), (dict(groups=70000), _lib.ERR_BAD_SHAPE),
                    (dict(dtype=1, odt=0), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, x=None), _lib.OK), (dict(groups=0, x=None), _lib.OK)):
         assert _with(ok, lib.nva_grouped_linear, **kw) == rc, kw
-    ok = dict(x=A, xs=64, w=A, choice=A, cw=A, lists=A, counts=A, ls=16, rows=16, width=64, experts=8, top=2, scale=1.0, dtype=0, stream=None)
+    ok = dict(x=A, xs=64, w=A, b=None, choice=A, cw=A, lists=A, counts=A, ls=16, rows=16, width=64, experts=8, gates=0, top=2, scale=1.0, dtype=0, stream=None)
     for kw, rc in ((dict(counts=None), _lib.ERR_NULL_POINTER), (dict(cw=None), _lib.ERR_NULL_POINTER), (dict(top=9), _lib.ERR_BAD_SHAPE),
                    (dict(ls=15), _lib.ERR_BAD_SHAPE), (dict(xs=63), _lib.ERR_BAD_STRIDE), (dict(experts=1025), _lib.ERR_UNSUPPORTED_GEOMETRY),
-                   (dict(experts=512, top=129), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, x=None), _lib.OK)):
+                   (dict(experts=512, top=129), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(gates=-1), _lib.ERR_BAD_SHAPE),
+                   (dict(gates=65), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, x=None), _lib.OK)):
         assert _with(ok, lib.nva_router, **kw) == rc, kw
-    ok = dict(x=A, xs=64, w=A, out=A, lists=A, counts=A, ls=16, rows=16, terms=2, experts=8, n_out=32, k=64, per_row=1, gated=1, dtype=0, stream=None)
+    ok = dict(x=A, xs=64, w=A, out=A, lists=A, counts=A, ls=16, rows=16, terms=2, experts=8, n_out=32, k=64, per_row=1, gated=1, limit=1.0, slope=1.7, shift=1.0, dtype=0, stream=None)
     for kw, rc in ((dict(lists=None), _lib.ERR_NULL_POINTER), (dict(out=None), _lib.ERR_NULL_POINTER), (dict(terms=9), _lib.ERR_BAD_SHAPE),
                    (dict(ls=15), _lib.ERR_BAD_SHAPE), (dict(xs=63), _lib.ERR_BAD_STRIDE), (dict(dtype=5), _lib.ERR_UNSUPPORTED_GEOMETRY),
                    (dict(rows=0, x=None), _lib.OK)):
         assert _with(ok, lib.nva_routed_linear, **kw) == rc, kw
+    del ok["dtype"], ok["stream"]
+    ok.update(sx=A, sxs=64, sw=A, so=A, sn=24, sk=64, sl=1.0, stream=None)
+    for kw, rc in ((dict(lists=None), _lib.ERR_NULL_POINTER), (dict(so=None), _lib.ERR_NULL_POINTER), (dict(terms=9), _lib.ERR_BAD_SHAPE),
+                   (dict(sn=0), _lib.ERR_BAD_SHAPE), (dict(sxs=63), _lib.ERR_BAD_STRIDE), (dict(sk=60), _lib.ERR_UNSUPPORTED_GEOMETRY),
+                   (dict(k=60), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, sx=None), _lib.OK)):
+        assert _with(ok, lib.nva_routed_shared_linear, **kw) == rc, kw
+
+
+def test_post_norm_prepare_and_masks_validation():
+    lib = _lib.load_masked()
+    ok = dict(y1=A, ys=64, yw=A, y2=A, tw=A, ws=3, terms=2, post=A, res=A, nxt=None, off=1.0, out=A, rows_of=None, clear=None, nclear=0, rows=4, src=4,
+              width=64, eps=1e-5, dtype=0, stream=None)
+    for kw, rc in ((dict(post=None), _lib.ERR_NULL_POINTER), (dict(out=None), _lib.ERR_NULL_POINTER), (dict(y1=None, y2=None), _lib.ERR_NULL_POINTER),
+                   (dict(ys=63), _lib.ERR_BAD_STRIDE), (dict(ws=1), _lib.ERR_BAD_STRIDE), (dict(ws=0, tw=None), _lib.ERR_BAD_STRIDE),
+                   (dict(terms=0), _lib.ERR_BAD_SHAPE), (dict(rows=3), _lib.ERR_BAD_SHAPE), (dict(dtype=2), _lib.ERR_UNSUPPORTED_GEOMETRY),
+                   (dict(rows=0, src=0), _lib.OK)):
+        assert _with(ok, lib.nva_post_rms_norms, **kw) == rc, kw
+    ok = dict(x=A, xs=256, b=A, qn=A, kn=A, whole=1, rope=A, q=A, kc=A, vc=A, sm=A, slots=512, cu=A, lens=A, tseq=A, n=9, seqs=2, heads=4, kv=2, dim=32,
+              vdim=32, rot=16, maxp=64, eps=1e-5, dtype=0, stream=None)
+    for kw, rc in ((dict(x=None), _lib.ERR_NULL_POINTER), (dict(vc=None), _lib.ERR_NULL_POINTER), (dict(sm=None), _lib.ERR_NULL_POINTER),
+                   (dict(rope=None), _lib.ERR_NULL_POINTER), (dict(tseq=None), _lib.ERR_NULL_POINTER), (dict(xs=255), _lib.ERR_BAD_STRIDE),
+                   (dict(rot=15), _lib.ERR_BAD_SHAPE), (dict(rot=34), _lib.ERR_BAD_SHAPE), (dict(maxp=0), _lib.ERR_BAD_SHAPE), (dict(cu=None), _lib.ERR_BAD_SHAPE),
+                   (dict(dtype=7), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(heads=5000, kv=1, dim=9, vdim=9, rot=0, xs=1 << 20), _lib.ERR_UNSUPPORTED_GEOMETRY),
+                   (dict(n=0, x=None), _lib.OK)):
+        assert _with(ok, lib.nva_qkv_prepare, **kw) == rc, kw
+    ok = dict(q=A, qs=2048, kc=A, vc=A, bt=A, bts=16, mb=16, cu=None, lens=A, tseq=None, out=A, ws=A, wsb=1 << 30, n=8, seqs=8, mq=1, heads=16, kv=8,
+              dim=128, vdim=128, bs=256, nb=64, mask=1, span=8192, scale=0.1, cap=0.0, sinks=A, gate=A, gs=16, dtype=0, stream=None)
+    for kw, rc in ((dict(q=None), _lib.ERR_NULL_POINTER), (dict(ws=None), _lib.ERR_NULL_POINTER), (dict(mask=2), _lib.ERR_UNSUPPORTED_GEOMETRY),
+                   (dict(gs=15), _lib.ERR_BAD_STRIDE), (dict(span=0), _lib.ERR_BAD_SHAPE), (dict(wsb=100), _lib.ERR_WORKSPACE_TOO_SMALL),
+                   (dict(n=0, q=None), _lib.OK)):
+        assert _with(ok, lib.nva_masked_attn, **kw) == rc, kw
+    ok = dict(x=A, xs=64, out=A, rows=4, width=64, dtype=0, stream=None)
+    for kw, rc in ((dict(x=None), _lib.ERR_NULL_POINTER), (dict(xs=63), _lib.ERR_BAD_STRIDE), (dict(xs=72), _lib.ERR_BAD_STRIDE), (dict(width=0), _lib.ERR_BAD_SHAPE),
+                   (dict(dtype=3), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, x=None), _lib.OK)):
+        assert _with(ok, lib.nva_squared_relu, **kw) == rc, kw
+    ok = dict(x=A, rows=4, width=64, cap=30.0, dtype=0, stream=None)
+    for kw, rc in ((dict(x=None), _lib.ERR_NULL_POINTER), (dict(cap=0.0), _lib.ERR_BAD_SHAPE), (dict(cap=float("nan")), _lib.ERR_BAD_SHAPE),
+                   (dict(dtype=3), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, x=None), _lib.OK)):
+        assert _with(ok, lib.nva_soft_cap, **kw) == rc, kw
+
+
+def test_symbols_of_several_libraries_come_from_one_that_is_there(monkeypatch):
+    monkeypatch.setattr(_lib, "LATENT_LIB_PATH", "/nonexistent/libnanovllm_latent.so")
+    monkeypatch.setattr(_lib, "MIXERS_LIB_PATH", "/nonexistent/libnanovllm_mixers.so")
+    fresh = _lib._Symbols()
+    assert fresh.nva_chunk_attn_workspace_bytes(0, 16, 8, 128, 16, 256, 100) == 0 and fresh.nva_router is not None
+    with pytest.raises(_lib.HipLibraryMissing, match="no CPU fallback"):
+        fresh.nva_mlstm
+    with pytest.raises(_lib.HipLibraryMissing, match="no CPU fallback"):
+        fresh.nva_retention
 
 
 def test_latent_attention_validation_and_workspace():

@@ -133,7 +133,8 @@ def test_experts(dev, dtype, shape, n):
             weights = experts.ExpertWeights(spec, width).to(dtype).requires_grad_(False)
         weights.load(spec, width, lambda name, size: w[name], "")
         run = experts.Experts(spec, weights, dev)
-        y, weight = run(h.to(dev))
+        y, shared, weight = run(h.to(dev))
+        assert shared is None
         got = (y.double().view(n, top, width) * weight.double()[..., None]).sum(1)
         want = plain.expert_mixture(h.double(), lambda name: w[name].double(), dict(router=dict(experts=n_experts, top=top, scale=0.9)))
         err = ((got.cpu() - want).abs().amax(1) / want.abs().max())
@@ -160,7 +161,7 @@ def test_tiles_of_experts(dev, shape, gated):
     router[0, 0] = -8.0
     a = experts.route(h, router, top, 1.0, torch.zeros(n_experts, dtype=torch.int32, device=dev))
     assert n_experts == 1 or top == n_experts or int(a.counts[0]) == 0
-    got = experts.routed_linear(x, w, a, gated)
+    got = experts.routed_linear(x, w, a, experts.SILU if gated else None)
     for e in range(n_experts):
         rows = (a.choice.flatten() == e).nonzero()[:, 0]
         y = x[rows // top if gated else rows].float() @ w[e].float().T
