@@ -15,6 +15,7 @@ already resident in HBM.  Workloads (shapes are the five benchmark configuration
     glue      residual add + RMSNorm (--glue add-rms-norm) or SiLU(gate) * up (--glue silu-mul), 16,384 rows (--tokens N)
     decode-e2e-shape / decode-longctx-shape / copy   profiling helpers: the decode attention of configs 4 / 5
               alone (one layer); a plain copy of known size
+    sokolorn  the Sokolorn family beside Kaparax and Pidutar at equal size: engine prefill / decode tok/s and every kernel beside its like
     pidutar   the Pidutar family beside Kaparax at equal size: engine prefill / decode tok/s and every kernel beside its like
     kaparax   the Kaparax family beside Qwen3 at equal size: engine prefill / decode tok/s and every kernel beside its like
     read-probe    calibration: a bare streaming read at the sizes of the bandwidth-bound workloads
@@ -1247,6 +1248,180 @@ def pidutar_kernels(dev, steps=60, only=None):
     return rows
 
 
+def _sokolorn_config(layers, width, heads, kv_heads, dense_ff, experts, top, ff, shared_ff, window, vocab):
+    """Groups of four layers: one rotated with all keys (every second one reads the keys of the one before), three under a
+    window; dense and expert feed-forwards in turn."""
+    from nanovllm_amd.engine.sokolorn import SokolornConfig
+    out = []
+    for i in range(layers):
+        if i % 2 == 0:
+            mlp = dict(kind="dense", ff=dense_ff)
+        else:
+            mlp = dict(kind="moe", expert=dict(ff=ff, limit=7.0), router=dict(experts=experts, top=top), shared=dict(ff=shared_ff, limit=7.0))
+        m = dict(heads=heads, kv_heads=kv_heads, dim=128, vdim=128, scale=128 ** -0.5)
+        if i % 4:
+            out.append(dict(type="attention", mixer=dict(m, mask=dict(size=window)), mlp=mlp))
+            continue
+        m["rot"] = dict(base=1e6, dims=128, scaling=dict(factor=8.0, low=1.0, high=4.0, original=8192))
+        if i % 8 == 4:
+            m["kv_from"] = i - 4
+        out.append(dict(type="attention_2", mixer=m, mlp=mlp))
+    return SokolornConfig.from_raw(dict(architecture="Sokolorn", vocab=vocab, width=width, norm=dict(eps=1e-6), logit_softcap=30.0, layers=out))
+
+
+def sokolorn_kernels(dev, steps=60, only=None):
+    """Every kernel of the Sokolorn layers at sizes of a real layer (width 1024, 16 / 8 heads of 128; 4 of 32 experts of 576 and
+    a shared one of 768; dense feed-forward of 4608), each beside the like kernel of the closest model at equal size --
+    Kaparax's attention, convolution step, norms and gate, Pidutar's experts and residual step -- in one process."""
+    import torch
+    import torch.nn.functional as F
+    from nanovllm_amd import synthetic
+    from nanovllm_amd.context import RowGroup
+    from nanovllm_amd.engine import branches, experts, masked, mixers
+    bf = torch.bfloat16
+    rnd = lambda *shape: torch.randn(*shape, device=dev).to(bf)
+    i32 = lambda x: torch.as_tensor(x, dtype=torch.int32).to(dev)
+    rows = []
+    want = lambda name: only is None or only in name
+    heads, kv, d, width, dense_ff = 16, 8, 128, 1024, 4608
+    n_exp, top, ff, sff = 32, 4, 576, 768
+    rope = mixers.RopeTables(16384 + 256, dev).get(mixers.Rotary(1e6, d, mixers.RotaryScaling(8.0, 1.0, 4.0, 8192.0)))
+    graph_us = lambda fns, n=200: _graph_time_ms(fns, n, 10)[0] / n * 1e3
+    event_us = lambda fns, n=steps: _steady_time_ms(fns, n, max(3, n // 10))[0] / n * 1e3
+    sinks = torch.randn(heads, device=dev)
+
+    def lengths(count, lo, hi, seed=0):
+        return torch.randint(lo, hi + 1, (count,), generator=torch.Generator().manual_seed(seed)).tolist()
+
+    # ---- attention over portions
+    for what, lens, window, form in (("2x16384, all keys", [16384, 16384], 16384, (16, 8, 128)), ("2x16384, window 2048", [16384, 16384], 2048, (16, 8, 128)),
+                                     ("2x16384, window 128", [16384, 16384], 128, (16, 8, 128)), ("16 x U[100,1024], all keys", lengths(16, 100, 1024), 16384, (16, 8, 128)),
+                                     ("2x16384, window 1024, 16 heads of 64", [16384, 16384], 1024, (16, 16, 64)),
+                                     ("2x16384, window 1024, 16 / 8 heads of 96", [16384, 16384], 1024, (16, 8, 96))):
+        if not want("attention prefill"):
+            continue
+        h, g, e = form
+        group, blocks = _portions(dev, lens)
+        n = sum(lens)
+        q, out, gate = rnd(n, h * e), torch.empty(n, h * e, dtype=bf, device=dev), rnd(n, h)
+        kc, vc = rnd(blocks, 256, g, e), rnd(blocks, 256, g, e)
+        windowed = window < 16384
+        mine = event_us([lambda: masked.masked_attention(q, kc, vc, group, out, h, window if windowed else masked.ALL_KEYS, e ** -0.5, sinks if windowed else None, gate if windowed else None)])
+        seen = sum(sum(min(p + 1, window) for p in range(l)) for l in lens)
+        # the like kernel: chunks as long as the window, its own visible pairs
+        parts = window if max(lens) > window else max(lens)
+        theirs = event_us([lambda: mixers.chunk_attention(q, kc, vc, group, out, h, parts, e ** -0.5, 30.0)])
+        chunked = sum((l // parts) * (parts * (parts + 1) // 2) + (l % parts) * (l % parts + 1) // 2 for l in lens)
+        rows.append(_kernel_row("attention prefill, " + what, mine, 4 * e * h * seen, "mfma", ("chunk attention, capped", theirs, 4 * e * h * chunked, "mfma")))
+        del q, out, kc, vc
+
+    # ---- attention of single tokens
+    for what, batch, ctx, window, pools in (("batch 64, ctx U[100,2048]", 64, (100, 2048), 0, 4), ("batch 256, ctx U[300,1326]", 256, (300, 1326), 0, 2),
+                                            ("batch 16, ctx U[4096,8192]", 16, (4096, 8192), 0, 4), ("batch 64, ctx 8192, window 1024", 64, (8192, 8192), 1024, 2),
+                                            ("batch 64, ctx 2048, window 128", 64, (2048, 2048), 128, 4), ("batch 1, ctx 8192", 1, (8192, 8192), 0, 4)):
+        if not want("attention decode"):
+            continue
+        g = torch.Generator().manual_seed(1)
+        lens = torch.randint(ctx[0], ctx[1] + 1, (batch,), generator=g)
+        blocks = int(((lens + 255) // 256).sum())
+        tabs = synthetic.decode_tables(lens.tolist(), blocks, g).to(dev)
+        group = RowGroup(0, batch, batch, i32(lens), i32([0] * batch), tabs, i32([0] * batch))
+        q, out, gate = rnd(batch, heads * d), torch.empty(batch, heads * d, dtype=bf, device=dev), rnd(batch, heads)
+        caches = [(rnd(blocks, 256, kv, d), rnd(blocks, 256, kv, d)) for _ in range(pools)]
+        span = window or masked.ALL_KEYS
+        mine = graph_us([lambda c=c: masked.masked_attention(q, c[0], c[1], group, out, heads, span, d ** -0.5, sinks if window else None, gate if window else None) for c in caches], 56)
+        alg = int(torch.clamp(lens, max=span).sum()) * kv * d * 4 + 4 * q.numel()
+        theirs = graph_us([lambda c=c: mixers.chunk_attention(q, c[0], c[1], group, out, heads, span, d ** -0.5, 30.0) for c in caches], 56)
+        lalg = int(((lens - 1) % span + 1).sum()) * kv * d * 4 + 4 * q.numel()
+        rows.append(_kernel_row("attention decode, " + what, mine, alg, "hbm", ("chunk attention, capped", theirs, lalg, "hbm")))
+        del caches
+
+    # ---- what attention reads
+    for n in (16, 256, 16384):
+        if not want("prepare"):
+            continue
+        ch = (heads + 2 * kv) * d
+        x, q = rnd(n, ch + heads), torch.empty(n, heads * d, dtype=bf, device=dev)
+        kc, vc = (torch.empty(max(1, n // 256), 256, kv, d, dtype=bf, device=dev) for _ in range(2))
+        group = _portions(dev, [1024] * 16)[0] if n >= 16384 else RowGroup(0, n, n, i32([701] * n), i32(torch.randperm(n)), None, i32(list(range(n))))
+        conv, xc = rnd(1, ch), rnd(n, ch)
+        theirs = graph_us([lambda: mixers.conv_rope_store(xc, conv, None, group, rope, q, kc, vc, heads, d)])
+        like = ("conv_rope_store_kernel, one tap", theirs, n * ch * 4 + n * d * 4, "hbm")
+        bias, wq, wk, hq = rnd(ch), rnd(heads * d), rnd(kv * d), rnd(d)
+        mine = graph_us([lambda: masked.qkv_prepare(x, bias, hq, hq, False, rope, q, kc, vc, group, heads, kv, d, d, 1e-6)])
+        rows.append(_kernel_row("prepare: bias, head norms, rotation, cache, %d rows" % n, mine, n * ch * 4 + n * d * 4, "hbm", like))
+        mine = graph_us([lambda: masked.qkv_prepare(x, None, wq, wk, True, None, q, kc, vc, group, heads, kv, d, d, 1e-6)])
+        rows.append(_kernel_row("prepare: whole norms, cache, %d rows" % n, mine, n * ch * 4, "hbm", like))
+
+    # ---- feed-forwards
+    for n in (1, 16, 64, 512, 16384):
+        if want("dense"):
+            h, ws, wl = rnd(n, width), [rnd(dense_ff, width) for _ in range(8)], [rnd(dense_ff, width) for _ in range(8)]
+            time = graph_us if n <= 512 else event_us
+            mine = time([lambda w=w: experts.project(h, w, squared_relu=True) for w in ws])
+            theirs = time([lambda w=w: mixers.clamped_gate(F.linear(h, w), 7.0, 1.702) for w in wl])
+            alg = (2 * n * width * dense_ff, "mfma") if n >= 512 else (2 * (dense_ff * width + n * (width + dense_ff)), "hbm")
+            rows.append(_kernel_row("dense up + squared relu, %d rows" % n, mine, *alg, ("library product + clamped_gate_kernel", theirs, *alg)))
+    form = experts.GateForm(7.0, 1.702, 1.0)
+    for n in (1, 16, 64, 128, 512, 2048, 16384):
+        if not want("experts"):
+            continue
+        h = rnd(n, width)
+        spec = experts.ExpertsSpec(n_exp, top, ff, gate=form, bias=True, shared=experts.SharedExpertSpec(sff, form))
+        plain = experts.ExpertsSpec(n_exp, top, (top * ff + sff) // top)         # Pidutar's: as much arithmetic, all of it routed
+        copies = 6 if n <= 512 else 1
+        mine, like = [], []
+        for sp, made in ((spec, mine), (plain, like)):
+            for _ in range(copies):
+                with torch.device(dev):
+                    w = experts.ExpertWeights(sp, width).to(bf).requires_grad_(False)
+                for p in w.parameters():
+                    p.normal_(0.0, 0.03)
+                if sp.bias:
+                    w.bias = torch.nn.Parameter(torch.zeros(n_exp + 1, device=dev), requires_grad=False)
+                made.append(experts.Experts(sp, w, dev))
+        time = graph_us if n <= 512 else event_us
+
+        def run(e):
+            e.counters.zero_()
+            e(h)
+        us, lus = time([lambda e=e: run(e) for e in mine]), time([lambda e=e: run(e) for e in like])
+
+        def hit(made):
+            for e in made:
+                run(e)
+            return sum(int((e.counters > 0).sum()) for e in made) / copies
+        if n >= 512:
+            alg = lalg = 6 * n * width * (top * ff + sff)
+            bound = "mfma"
+        else:
+            io = 2 * n * (2 * width + 4 * (top * ff + sff))
+            alg, lalg = (hit(mine) * ff + sff) * 6 * width + io, hit(like) * plain.ff * 6 * width + io
+            bound = "hbm"
+        rows.append(_kernel_row("experts with a shared one (router and all), %d rows" % n, us, alg, bound, ("Pidutar's experts", lus, lalg, bound)))
+
+    # ---- steps around them
+    for n in (16, 256, 16384):
+        if want("post norm"):
+            y1, y2, r32 = rnd(n, width), rnd(n * top, width), torch.randn(n, width, device=dev)
+            tw, w = torch.rand(n, top + 1, device=dev), [rnd(width) for _ in range(4)]
+            cnt = torch.zeros(n_exp, dtype=torch.int32, device=dev)
+            mine = graph_us([lambda: branches.post_rms_norms(r32, y1, None, None, None, w[0], None, 1e-6, 1.0, clear=cnt)])
+            theirs = graph_us([lambda: mixers.post_add_norm(y1, r32, (w[0], w[1]), (w[2], w[3]), 1e-6)])
+            rows.append(_kernel_row("post norm of one branch, %d rows" % n, mine, n * width * 12, "hbm", ("norm_rows_kernel", theirs, n * width * 12, "hbm")))
+            mine = graph_us([lambda: branches.post_rms_norms(r32, y1, tw[:, top], y2, tw[:, :top], w[0], None, 1e-6, 1.0)])
+            tw4 = tw[:, :top].contiguous()
+            theirs = graph_us([lambda: branches.branches_rms_norms(r32, 0.5, y1, w[0], y2, tw4, w[1], (w[2], w[3]), 1e-6, 1.0, clear=cnt)])
+            rows.append(_kernel_row("post norm of experts, %d rows" % n, mine, n * width * (2 + 2 * top + 8 + 2), "hbm",
+                                    ("branch_norm_kernel, two norms", theirs, n * width * (2 + 2 * top + 8 + 4), "hbm")))
+    if want("soft cap"):
+        x, y = rnd(256, 151936), rnd(256, 2 * 75968)
+        mine = graph_us([lambda: mixers.soft_cap_(x, 30.0)], 50)
+        theirs = graph_us([lambda: mixers.clamped_gate(y, 7.0, 1.702)], 50)
+        rows.append(_kernel_row("soft cap of logits, 256 x 151936", mine, 4 * x.numel(), "hbm", ("clamped_gate_kernel", theirs, 3 * y.numel(), "hbm")))
+    return rows
+
+
 def _engine_rates(model, dev, batch, prompt_len, new_tokens, slots):
     """Prefill and decode tokens/s of the engine: ``batch`` prompts of ``prompt_len`` tokens, ``new_tokens`` each."""
     import gc
@@ -1333,9 +1508,35 @@ def bench_pidutar(args, dev):
     return result, lambda: None
 
 
-WORKLOADS = {"pidutar": bench_pidutar, "kaparax": bench_kaparax, "rope-scatter": bench_rope_scatter, "glue": bench_glue, "e2e": bench_e2e, "longctx": bench_longctx, "decode-e2e-shape": bench_decode_e2e_shape,
+def bench_sokolorn(args, dev):
+    """The Sokolorn family beside Kaparax (dense) and Pidutar (experts) at equal size: engine throughput (prompts of 1024
+    tokens, then 128 decoded tokens each) for two layer sizes and two batches, and every kernel beside its like (--part)."""
+    part = args.part
+    kernels = sokolorn_kernels(dev, only=args.kernel) if part in ("all", "kernels") else []
+    engines = {}
+    if part in ("all", "engine"):
+        sizes = {"28 layers, width 1024, 16/8 heads x 128, ff 4608 or 4 of 32 experts of 576 + 768": (
+                     _sokolorn_config(28, 1024, 16, 8, 4608, 32, 4, 576, 768, 1024, 151936), _kaparax_config(28, 1024, 16, 8, 128, 3072, 8, 128, 8192, 151936),
+                     _pidutar_config(28, 1024, 16, 512, 512, 8, 128, 32, 4, 768, 8192, 151936)),
+                 "8 layers, width 4096, 32/8 heads x 128, ff 18432 or 4 of 32 experts of 2304 + 3072": (
+                     _sokolorn_config(8, 4096, 32, 8, 18432, 32, 4, 2304, 3072, 1024, 151936), _kaparax_config(8, 4096, 32, 8, 128, 12288, 16, 128, 8192, 151936),
+                     _pidutar_config(8, 4096, 32, 1536, 512, 16, 128, 32, 4, 3072, 8192, 151936))}
+        for what, models in sizes.items():
+            for batch in (16, 128):
+                engines["%s; batch %d" % (what, batch)] = {name: _engine_rates(m, dev, batch, 1024, 128, 128)
+                                                           for name, m in zip(("sokolorn", "kaparax", "pidutar"), models)}
+    first = next(iter(engines.values()))["sokolorn"]["decode_tok_s"] if engines else None
+    result = {"metric": "Sokolorn decode tok/s (28 layers of width 1024, batch 16, prompts of 1024)", "value": first, "unit": "tok/s",
+              "ms_per_step": round(16e3 / first, 3) if first else None,
+              "config": {"workload": "random weights; one rotated layer in four, windows of 1024 in the others, dense and expert feed-forwards in turn",
+                         "engine": engines, "kernels": kernels},
+              "roofline": None}
+    return result, lambda: None
+
+
+WORKLOADS = {"sokolorn": bench_sokolorn, "pidutar": bench_pidutar, "kaparax": bench_kaparax, "rope-scatter": bench_rope_scatter, "glue": bench_glue, "e2e": bench_e2e, "longctx": bench_longctx, "decode-e2e-shape": bench_decode_e2e_shape,
              "decode-longctx-shape": bench_decode_longctx_shape, "copy": bench_copy, "read-probe": bench_read_probe, "decode": bench_decode, "scatter": bench_scatter, "prefill": bench_prefill, "sampler": bench_sampler}
-DEFAULT_STEPS = {"pidutar": 60, "kaparax": 60, "rope-scatter": 100, "glue": 100, "e2e": 1, "longctx": 1, "decode-e2e-shape": 1, "decode-longctx-shape": 1, "copy": 50, "read-probe": 60, "decode": 200, "scatter": 400, "prefill": 50, "sampler": 100}
+DEFAULT_STEPS = {"sokolorn": 60, "pidutar": 60, "kaparax": 60, "rope-scatter": 100, "glue": 100, "e2e": 1, "longctx": 1, "decode-e2e-shape": 1, "decode-longctx-shape": 1, "copy": 50, "read-probe": 60, "decode": 200, "scatter": 400, "prefill": 50, "sampler": 100}
 
 
 def main():
@@ -1356,8 +1557,8 @@ def main():
     ap.add_argument("--glue", choices=["add-rms-norm", "silu-mul", "last-token-norm"], default="add-rms-norm", help="glue: which elementwise kernel")
     ap.add_argument("--uniform", default=None, metavar="SxL", help="prefill: S packed sequences of L tokens each instead of config 3 (e.g. 2x16384)")
     ap.add_argument("--bucket-step", type=int, default=16, help="e2e only: spacing of the captured decode batch sizes")
-    ap.add_argument("--part", "--kaparax-part", choices=["all", "kernels", "engine"], default="all", help="kaparax / pidutar: which half of the workload")
-    ap.add_argument("--kernel", default=None, help="kaparax / pidutar: only kernels whose row name contains this")
+    ap.add_argument("--part", "--kaparax-part", choices=["all", "kernels", "engine"], default="all", help="sokolorn / kaparax / pidutar: which half of the workload")
+    ap.add_argument("--kernel", default=None, help="sokolorn / kaparax / pidutar: only kernels whose row name contains this")
     ap.add_argument("--no-extra", action="store_true", help="e2e only: skip the per-configuration rooflines and the eager pass")
     args = ap.parse_args()
     if args.gpus != 1:

@@ -133,7 +133,14 @@ __global__ __launch_bounds__(256) void chunk_attn_any_kernel(ChunkAttnArgs a) {
 // Where a score cap of at most kBoundedCap holds, weights need no running maximum: e^{+-cap} and its sums
 // stay inside fp32, so nothing is rescaled and partial results of different keys simply add up.
 
+// Otherwise weights need a reference.  For single tokens it is a running maximum.  For portions it is the maximum of the
+// first keys that a query meets, and stays: fp32 holds weights of up to 2^kHeadroom above it, so the accumulators are
+// never rescaled.  The maximum over all keys is kept beside it; where that passes the headroom the workgroup walks its
+// keys a second time with that maximum for the reference.
+
 constexpr float kBoundedCap = 60.0f;
+constexpr float kHeadroom = 64.0f;
+enum Cap { kNoCap, kBounded, kCapped };
 
 // Raw product -> base-2 exponent of the weight.
 struct Weighting {
@@ -156,7 +163,7 @@ __device__ __forceinline__ float exponent_of(const Weighting &w, bool capped, fl
 // operand reads spread over the banks -- the scheme of the prefill kernel for whole contexts, whose
 // description gives the permutations.  Otherwise (smaller sizes, multiples of 8) tiles go through registers
 // into padded rows, zero-filled to DK and DV.
-template <int DK, int DV, int NQ, bool kBounded, bool kDirect>
+template <int DK, int DV, int NQ, Cap kCap, bool kDirect>
 __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kernel(const ChunkAttnArgs a, const Weighting w,
                                                                                   const int32_t q_tiles) {
     constexpr int kBM = 64 * NQ, kBN = 64;
@@ -275,14 +282,10 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
     };
 
     f32x4_t oacc[DV / 16][NQ];
-    float lsum[NQ], m[NQ];
+    float lsum[NQ], m[NQ], top[NQ];
 #pragma unroll
-    for (int qa = 0; qa < NQ; ++qa) {
-        lsum[qa] = 0.f;
-        m[qa] = -INFINITY;
-#pragma unroll
-        for (int db = 0; db < DV / 16; ++db) oacc[db][qa] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    }
+    for (int qa = 0; qa < NQ; ++qa) m[qa] = top[qa] = -INFINITY;
+    const float to_exp2 = kCap == kCapped ? 1.0f : w.in;             // (not kBounded) of a score, capped already where it is
 
     auto attend = [&](auto masked_c, int key0, int buf) __attribute__((always_inline)) {
         constexpr bool kMasked = decltype(masked_c)::value;
@@ -295,65 +298,58 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
             return __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_ptr)(
                 vl + (kDirect ? (kb * (DV / 32) + (db >> 1)) * 1024 + 32 * ((g ^ db) & 1) : kb * 16 * kVPitch + 32 * db)));
         };
-        f32x4_t sacc[4][NQ];
+        f32x4_t sacc[2][NQ];
         auto scores = [&](int kb) __attribute__((always_inline)) {
 #pragma unroll
-            for (int qa = 0; qa < NQ; ++qa) sacc[kb][qa] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+            for (int qa = 0; qa < NQ; ++qa) sacc[kb & 1][qa] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int ks = 0; ks < DK / 32; ++ks) {
                 const u32x4_t kf = kpiece(kb, ks);
 #pragma unroll
-                for (int qa = 0; qa < NQ; ++qa) sacc[kb][qa] = mfma16(kf, qf[qa][ks], sacc[kb][qa]);
+                for (int qa = 0; qa < NQ; ++qa) sacc[kb & 1][qa] = mfma16(kf, qf[qa][ks], sacc[kb & 1][qa]);
             }
         };
-        if (!kBounded) {
-#pragma unroll
-            for (int kb = 0; kb < 4; ++kb) scores(kb);
-        }
         auto seen = [&](int qa, int kb, int i) __attribute__((always_inline)) -> bool {
             const int key = key0 + 16 * kb + 4 * g + i;
             return !kMasked || (key >= lo[qa] && key <= pos[qa]);
         };
-        if (!kBounded) {
 #pragma unroll
-            for (int qa = 0; qa < NQ; ++qa) {
-                float mx = -INFINITY;
+        for (int half = 0; half < 2; ++half) {           // half a tile at a time, and nothing moved across: fewer registers
+            __builtin_amdgcn_sched_barrier(0);
+            scores(2 * half);
+            scores(2 * half + 1);
+            if (kCap != kBounded) {
 #pragma unroll
-                for (int kb = 0; kb < 4; ++kb)
+                for (int qa = 0; qa < NQ; ++qa) {
+                    float mx = -INFINITY;
 #pragma unroll
-                    for (int i = 0; i < 4; ++i) {
-                        sacc[kb][qa][i] = exponent_of(w, w.capped, sacc[kb][qa][i]);
-                        if (seen(qa, kb, i)) mx = fmaxf(mx, sacc[kb][qa][i]);
+                    for (int kb2 = 0; kb2 < 2; ++kb2)
+#pragma unroll
+                        for (int i = 0; i < 4; ++i) {
+                            if (kCap == kCapped) sacc[kb2][qa][i] = exponent_of(w, true, sacc[kb2][qa][i]);
+                            if (seen(qa, 2 * half + kb2, i)) mx = fmaxf(mx, sacc[kb2][qa][i]);
+                        }
+                    mx *= to_exp2;
+                    top[qa] = fmaxf(top[qa], mx);
+                    if (__any(m[qa] == -INFINITY && mx > -INFINITY)) {
+                        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+                        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+                        if (m[qa] == -INFINITY) m[qa] = mx;
                     }
-                mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-                mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-                const float m_new = fmaxf(m[qa], mx);
-                const float keep = m[qa] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m[qa] - m_new);
-                m[qa] = m_new;
-                lsum[qa] *= keep;
-#pragma unroll
-                for (int db = 0; db < DV / 16; ++db)
-#pragma unroll
-                    for (int i = 0; i < 4; ++i) oacc[db][qa][i] *= keep;
-            }
-        }
-#pragma unroll
-        for (int half = 0; half < 2; ++half) {
-            if (kBounded) {                              // half a tile at a time: fewer registers
-                scores(2 * half);
-                scores(2 * half + 1);
+                }
             }
             u32x4_t ph[NQ], pl[NQ];
 #pragma unroll
-            for (int qa = 0; qa < NQ; ++qa)
+            for (int qa = 0; qa < NQ; ++qa) {
+                const float ref = kCap == kBounded || m[qa] == -INFINITY ? 0.f : m[qa];
 #pragma unroll
                 for (int kb2 = 0; kb2 < 2; ++kb2) {
                     float p[4];
 #pragma unroll
                     for (int i = 0; i < 4; ++i) {
-                        const float s = sacc[2 * half + kb2][qa][i];
+                        const float s = sacc[kb2][qa][i];
                         const bool vis = seen(qa, 2 * half + kb2, i);
-                        const float x = kBounded ? exponent_of(w, true, s) : s - m[qa];
+                        const float x = kCap == kBounded ? exponent_of(w, true, s) : fmaf(s, to_exp2, -ref);
                         p[i] = vis ? __builtin_amdgcn_exp2f(x) : 0.f;
                         lsum[qa] += p[i];
                     }
@@ -363,6 +359,7 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
                     ph[qa][2 * kb2] = h0; ph[qa][2 * kb2 + 1] = h1;
                     pl[qa][2 * kb2] = l0; pl[qa][2 * kb2 + 1] = l1;
                 }
+            }
 #pragma unroll
             for (int db = 0; db < DV / 16; ++db) {
                 const s16x4_t v0 = vpiece(2 * half, db), v1 = vpiece(2 * half + 1, db);
@@ -376,25 +373,43 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
         }
     };
 
-    int blk_next = block_of(1);
-    bool ok = fetch(0, block_of(0), 0);
-    put(0);
-    __syncthreads();
-    for (int tile = 0; tile < ntiles; ++tile) {
-        const int buf = tile & 1;
-        bool ok_next = false;
-        if (tile + 1 < ntiles) {
-            ok_next = fetch(tile + 1, blk_next, buf ^ 1);            // (that buffer was read one tile ago, a barrier lies between)
-            blk_next = block_of(tile + 2);
+    for (int pass = 0;; ++pass) {
+#pragma unroll
+        for (int qa = 0; qa < NQ; ++qa) {
+            lsum[qa] = 0.f;
+#pragma unroll
+            for (int db = 0; db < DV / 16; ++db) oacc[db][qa] = f32x4_t{0.f, 0.f, 0.f, 0.f};
         }
-        const int key0 = key_begin + tile * kBN;
-        if (ok && w_live && key0 <= w_last && key0 + kBN > w_lo) {
-            if (key0 >= w_lo_all && key0 + kBN - 1 <= w_first) attend(std::false_type{}, key0, buf);
-            else attend(std::true_type{}, key0, buf);
-        }
-        if (tile + 1 < ntiles) put(buf ^ 1);
-        ok = ok_next;
+        int blk_next = block_of(1);
+        bool ok = fetch(0, block_of(0), 0);
+        put(0);
         __syncthreads();
+        for (int tile = 0; tile < ntiles; ++tile) {
+            const int buf = tile & 1;
+            bool ok_next = false;
+            if (tile + 1 < ntiles) {
+                ok_next = fetch(tile + 1, blk_next, buf ^ 1);        // (that buffer was read one tile ago, a barrier lies between)
+                blk_next = block_of(tile + 2);
+            }
+            const int key0 = key_begin + tile * kBN;
+            if (ok && w_live && key0 <= w_last && key0 + kBN > w_lo) {
+                if (key0 >= w_lo_all && key0 + kBN - 1 <= w_first) attend(std::false_type{}, key0, buf);
+                else attend(std::true_type{}, key0, buf);
+            }
+            if (tile + 1 < ntiles) put(buf ^ 1);
+            ok = ok_next;
+            __syncthreads();
+        }
+        if (kCap == kBounded || pass > 0) break;
+        bool again = false;
+#pragma unroll
+        for (int qa = 0; qa < NQ; ++qa) again |= top[qa] > m[qa] + kHeadroom;
+        if (!__syncthreads_or(again)) break;
+#pragma unroll
+        for (int qa = 0; qa < NQ; ++qa) {
+            float mx = fmaxf(top[qa], __shfl_xor(top[qa], 16, 64));
+            m[qa] = fmaxf(mx, __shfl_xor(mx, 32, 64));
+        }
     }
     if (!w_live) return;
 #pragma unroll
@@ -404,7 +419,7 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
         l += __shfl_xor(l, 32, 64);
         const int row = row0 + wave * 16 * NQ + 16 * qa + r;
         if (row >= lq) continue;
-        l += sink_weight(a, head, kBounded ? 0.f : m[qa]);
+        l += sink_weight(a, head, kCap == kBounded ? 0.f : m[qa]);
         const float inv = l > 0.f ? head_gate<bf16_t>(a, t0 + row, head) / l : 0.f;
         bf16_t *out = static_cast<bf16_t *>(a.out) + (static_cast<int64_t>(t0 + row) * a.heads + head) * a.vdim + 4 * g;
 #pragma unroll
@@ -427,7 +442,7 @@ struct SplitArgs {
     int32_t head_groups;     // groups of 16 query heads per kv head
 };
 
-template <int DK, int DV, bool kBounded>
+template <int DK, int DV, bool kPlain>
 __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 3) void chunk_decode_kernel(const ChunkAttnArgs a, const Weighting w, const SplitArgs sp) {
     constexpr int kVPitch = DV * 2 + 32;
     constexpr int kWaveBytes = 32 * kVPitch > 16 * DV * 4 ? 32 * kVPitch : 16 * DV * 4;
@@ -537,11 +552,11 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 3) void chunk_decode_kerne
             for (int i = 0; i < 4; ++i) {
                 const int key = key0 + 16 * kb + 4 * g + i;
                 vis[kb][i] = ok && key >= lo && key <= last;
-                x[kb][i] = exponent_of(w, kBounded || w.capped, s[kb][i]);
+                x[kb][i] = exponent_of(w, kPlain || w.capped, s[kb][i]);
                 if (vis[kb][i]) mx = fmaxf(mx, x[kb][i]);
             }
         float ref = 0.f;
-        if (!kBounded) {
+        if (!kPlain) {
             mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
             mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
             const float m_new = fmaxf(m, mx);
@@ -590,10 +605,10 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 3) void chunk_decode_kerne
     for (int i = tid; i < nheads * a.vdim; i += 256) {
         const int h = i / a.vdim, c = i % a.vdim;
         float top = 0.f, l = 0.f, o = 0.f;
-        if (!kBounded) top = fmaxf(fmaxf(sh_m[0][h], sh_m[1][h]), fmaxf(sh_m[2][h], sh_m[3][h]));
+        if (!kPlain) top = fmaxf(fmaxf(sh_m[0][h], sh_m[1][h]), fmaxf(sh_m[2][h], sh_m[3][h]));
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
-            const float f = kBounded ? 1.0f : (sh_m[v][h] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(sh_m[v][h] - top));
+            const float f = kPlain ? 1.0f : (sh_m[v][h] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(sh_m[v][h] - top));
             l = fmaf(sh_l[v][h], f, l);
             o = fmaf(reinterpret_cast<const float *>(&smem[v * kWaveBytes])[h * DV + c], f, o);
         }
@@ -603,7 +618,7 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 3) void chunk_decode_kerne
         } else {
             float *part = sp.partials + ((static_cast<int64_t>(seq) * sp.splits + split) * a.heads + head0 + h) * (a.vdim + 2);
             part[c] = o;
-            if (c == 0) { part[a.vdim] = l; part[a.vdim + 1] = kBounded ? 0.f : top; }
+            if (c == 0) { part[a.vdim] = l; part[a.vdim + 1] = kPlain ? 0.f : top; }
         }
     }
 }
@@ -670,13 +685,12 @@ static int launch_matrix(const ChunkAttnArgs &a, const SplitArgs &sp, int32_t ma
     if (wgs > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
     if (wgs == 0) return NVA_OK;
     const dim3 grid(static_cast<uint32_t>(wgs)), block(256);
-    if (a.dim == DK && a.vdim == DV) {
-        if (bounded) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, true, true>), grid, block, 0, s, a, w, q_tiles);
-        else hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, false, true>), grid, block, 0, s, a, w, q_tiles);
-    } else {
-        if (bounded) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, true, false>), grid, block, 0, s, a, w, q_tiles);
-        else hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, false, false>), grid, block, 0, s, a, w, q_tiles);
-    }
+    const bool direct = a.dim == DK && a.vdim == DV;
+    if (a.cap > 0.f && !bounded) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, kCapped, false>), grid, block, 0, s, a, w, q_tiles);
+    else if (bounded && direct) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, kBounded, true>), grid, block, 0, s, a, w, q_tiles);
+    else if (bounded) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, kBounded, false>), grid, block, 0, s, a, w, q_tiles);
+    else if (direct) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, kNoCap, true>), grid, block, 0, s, a, w, q_tiles);
+    else hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, kNoCap, false>), grid, block, 0, s, a, w, q_tiles);
     return launch_status();
 }
 
@@ -688,7 +702,7 @@ static int launch_matrix_dk(const ChunkAttnArgs &a, const SplitArgs &sp, int32_t
 }
 
 static bool matrix_ok(const ChunkAttnArgs &a) {
-    return a.dim % 8 == 0 && a.vdim % 8 == 0 && a.dim <= 256 && a.vdim <= 256 && a.q_stride % 8 == 0 && aligned16(a.q) &&
+    return a.scale >= 0.f && a.dim % 8 == 0 && a.vdim % 8 == 0 && a.dim <= 256 && a.vdim <= 256 && a.q_stride % 8 == 0 && aligned16(a.q) &&
            aligned16(a.k_cache) && aligned16(a.v_cache) && aligned16(a.out);
 }
 
@@ -748,6 +762,7 @@ extern "C" int nva_masked_attn(const void *q, int64_t q_row_stride, const void *
                     return NVA_ERR_WORKSPACE_TOO_SMALL;
             }
         }
+        if (std::max(qk_dim, v_dim) > 64 && std::max(qk_dim, v_dim) <= 96) return launch_matrix<96, 96>(a, sp, max_seqlen_q, s);
         if (qk_dim <= 64) return launch_matrix_dk<64>(a, sp, max_seqlen_q, s);
         if (qk_dim <= 128) return launch_matrix_dk<128>(a, sp, max_seqlen_q, s);
         return launch_matrix_dk<256>(a, sp, max_seqlen_q, s);

@@ -431,7 +431,7 @@ template <int NB, bool kGated, typename O>
 static int launch_skinny_nb(const LinearArgs &a, const LinearArgs &beside, int32_t rows_hint, int32_t most_rows, hipStream_t s) {
     const int mt = rows_hint <= 16 ? 1 : rows_hint <= 32 ? 2 : 4;
     const int passes = std::max(1, (most_rows + 16 * mt - 1) / (16 * mt));
-    const dim3 grid((std::max(a.n_out, beside.n_out) + 16 * NB - 1) / (16 * NB), a.groups + beside.groups, a.lists ? 1 : std::min(passes, 65535)), block(256);
+    const dim3 grid((std::max(a.n_out, beside.n_out) + 16 * NB - 1) / (16 * NB), a.groups + beside.groups, a.lists && beside.groups == 0 ? 1 : std::min(passes, 65535)), block(256);
     if (mt == 1) hipLaunchKernelGGL((linear_skinny_kernel<1, NB, kGated, O>), grid, block, 0, s, a, beside);
     else if (mt == 2) hipLaunchKernelGGL((linear_skinny_kernel<2, NB, kGated, O>), grid, block, 0, s, a, beside);
     else hipLaunchKernelGGL((linear_skinny_kernel<4, NB, kGated, O>), grid, block, 0, s, a, beside);

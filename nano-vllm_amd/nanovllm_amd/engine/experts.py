@@ -26,7 +26,7 @@ class GateForm:
 
 
 SILU = GateForm()
-JOIN_ROWS = 64                   # rows up to which a shared expert runs in the launches of the routed ones
+JOIN_ROWS = 256                  # rows up to which a shared expert runs in the launches of the routed ones
 
 
 def grouped_linear(x: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, squared_relu: bool = False) -> torch.Tensor:
