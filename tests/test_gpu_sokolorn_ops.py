@@ -105,7 +105,7 @@ def test_router_with_bias_and_gate(dev, dtype, shape):
 
 @pytest.mark.parametrize("dtype", [BF16, F32])
 @pytest.mark.parametrize("shape", [  # experts, best, width, ff, the shared one's ff
-    (6, 2, 64, 40, 56), (3, 3, 50, 27, 13), (16, 4, 256, 128, 128), (1, 1, 16, 24, 8), (40, 6, 192, 48, 320), (4, 2, 520, 200, 8), (8, 2, 1024, 768, 1536), (5, 2, 256, 96, None)])
+    (6, 2, 64, 40, 56), (3, 3, 50, 27, 13), (16, 4, 256, 128, 128), (1, 1, 16, 24, 8), (40, 6, 192, 48, 320), (4, 2, 520, 200, 8), (8, 2, 1024, 768, 1536), (5, 2, 256, 88, None)])
 @pytest.mark.parametrize("n", [1, 7, 17, 64, 65, 700, 1500])
 def test_experts_with_a_shared_one(dev, dtype, shape, n):
     n_experts, top, width, ff, sff = shape
@@ -203,7 +203,7 @@ def test_bias_norms_rotation_and_cache_write(dev, dtype, shape, kind):
 # ---- attention --------------------------------------------------------------------------------------------------
 
 ATTN = [  # heads, key heads, key size, value size
-    (6, 2, 32, 48), (8, 8, 64, 64), (3, 1, 20, 9), (1, 1, 8, 8), (40, 2, 72, 96), (33, 1, 24, 16), (8, 2, 128, 128), (4, 4, 160, 32), (6, 3, 96, 96), (2, 1, 256, 200),
+    (6, 2, 32, 48), (8, 8, 64, 64), (3, 1, 20, 9), (1, 1, 8, 8), (40, 2, 72, 96), (33, 1, 24, 16), (8, 2, 128, 128), (4, 4, 160, 32), (10, 5, 96, 96), (2, 1, 256, 200),
     (2, 2, 64, 128), (2, 1, 128, 64), (4, 1, 128, 256), (5, 5, 17, 20)]
 
 
