@@ -1348,9 +1348,9 @@ def sokolorn_kernels(dev, steps=60, only=None):
         theirs = graph_us([lambda: mixers.conv_rope_store(xc, conv, None, group, rope, q, kc, vc, heads, d)])
         like = ("conv_rope_store_kernel, one tap", theirs, n * ch * 4 + n * d * 4, "hbm")
         bias, wq, wk, hq = rnd(ch), rnd(heads * d), rnd(kv * d), rnd(d)
-        mine = graph_us([lambda: masked.qkv_prepare(x, bias, hq, hq, False, rope, q, kc, vc, group, heads, kv, d, d, 1e-6)])
+        mine = graph_us([lambda: masked.qkv_prepare(x, bias, hq, hq, masked.HEAD, rope, q, kc, vc, group, heads, kv, d, d, 1e-6)])
         rows.append(_kernel_row("prepare: bias, head norms, rotation, cache, %d rows" % n, mine, n * ch * 4 + n * d * 4, "hbm", like))
-        mine = graph_us([lambda: masked.qkv_prepare(x, None, wq, wk, True, None, q, kc, vc, group, heads, kv, d, d, 1e-6)])
+        mine = graph_us([lambda: masked.qkv_prepare(x, None, wq, wk, masked.WHOLE, None, q, kc, vc, group, heads, kv, d, d, 1e-6)])
         rows.append(_kernel_row("prepare: whole norms, cache, %d rows" % n, mine, n * ch * 4, "hbm", like))
 
     # ---- feed-forwards

@@ -44,6 +44,13 @@ enum nva_dtype { NVA_DTYPE_BF16 = 0, NVA_DTYPE_F32 = 1 };
 /* which keys the query at position p sees: [p / span * span, p], or the last `span` up to and with p */
 enum nva_mask { NVA_MASK_CHUNKS = 0, NVA_MASK_WINDOW = 1 };
 
+/* norms of nva_qkv_prepare: over a whole projection instead of every head; q and k normed without a weight where theirs is
+ * NULL; every head's values normed, without a weight */
+enum nva_qkv_norms { NVA_QKV_NORM_WHOLE = 1, NVA_QKV_NORM_UNIT = 2, NVA_QKV_NORM_VALUES = 4 };
+
+/* weights of nva_router: softmax over all experts, normalised over the chosen ones, or the chosen logits' sigmoids as they are */
+enum nva_score { NVA_SCORE_SOFTMAX = 0, NVA_SCORE_SIGMOID = 1 };
+
 /* Library version, (major << 16) | minor. */
 int nva_version(void);
 
@@ -323,9 +330,10 @@ int nva_post_add_norm(const void *y, int64_t y_row_stride, float *residual, cons
                       int32_t dtype, void *stream);
 
 /* x: [rows, 2 * inter] (gate | up, row stride in elements).  g = min(gate, limit), u = clamp(up, -limit, limit),
- * out = g * sigmoid(alpha * g) * (u + 1). */
+ * out = g * sigmoid(alpha * (g + cubic * g^3)) * (u + shift).  (limit infinity, alpha 2 sqrt(2 / pi), cubic 0.044715, shift 0: the
+ * tanh form of gelu(gate), times up.) */
 int nva_clamped_gate(const void *x, int64_t x_row_stride, void *out, int32_t rows, int32_t inter, float limit,
-                     float alpha, int32_t dtype, void *stream);
+                     float alpha, float cubic, float shift, int32_t dtype, void *stream);
 
 /* out = max(x, 0)^2; x: [rows, width] (row stride in elements), out dense, may be x. */
 int nva_squared_relu(const void *x, int64_t x_row_stride, void *out, int32_t rows, int32_t width, int32_t dtype,
@@ -370,7 +378,9 @@ int nva_chunk_attn(const void *q, int64_t q_row_stride, const void *k_cache, con
                    void *stream);
 
 /* The same under any nva_mask (workspace: as above with chunk = span), with
- * sinks (fp32 [num_heads], may be NULL): the sum of a head's weights also contains exp(sink), which has no key, and
+ * sinks (fp32 [num_heads], may be NULL): the sum of a head's weights also contains exp(sink), which has no key,
+ * bias_slope, bias_rate (fp32 [num_heads], both or neither NULL; not beside a softcap): a key that lies d back has
+ * slope * ln(1 + rate * d) taken off its score, and
  * gate ([n_tokens, num_heads], row stride in elements, may be NULL): a head's result times sigmoid(gate). */
 int nva_masked_attn(const void *q, int64_t q_row_stride, const void *k_cache, const void *v_cache,
                     const int32_t *block_tables, int64_t bt_row_stride, int32_t max_blocks,
@@ -379,16 +389,18 @@ int nva_masked_attn(const void *q, int64_t q_row_stride, const void *k_cache, co
                     int32_t n_tokens, int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads,
                     int32_t num_kv_heads, int32_t qk_dim, int32_t v_dim, int32_t block_size,
                     int32_t num_blocks, int32_t mask, int32_t span, float scale, float softcap, const float *sinks,
-                    const void *gate, int64_t gate_row_stride, int32_t dtype, void *stream);
+                    const float *bias_slope, const float *bias_rate, const void *gate, int64_t gate_row_stride, int32_t dtype,
+                    void *stream);
 
 /* q, k and v of an attention layer, between projection and attention.  x: [n_tokens, num_heads * qk_dim | num_kv_heads *
  * qk_dim | num_kv_heads * v_dim] (row stride in elements) plus bias (as many elements, may be NULL); then RMS norms of q and
- * k, of every head by itself (weights [qk_dim]) or, norm_whole, over all heads at once (weights [num_heads * qk_dim] and
- * [num_kv_heads * qk_dim]; a NULL weight: no norm); then rotation of the first rot_dims elements of every head by the
+ * k, of every head by itself (weights [qk_dim]) or over all heads at once (weights [num_heads * qk_dim] and
+ * [num_kv_heads * qk_dim]; a NULL weight: no norm, unless norms, of enum nva_qkv_norms, asks for one without a weight), and of
+ * every head's values where norms asks for it; then rotation of the first rot_dims elements of every head by the
  * row's position (pairs i, i + rot_dims / 2; rope_cache as above).  q to q_out [n_tokens, num_heads * qk_dim], k and v to their
  * cache slots.  Caches NULL: the queries only (x then has num_heads * qk_dim columns). */
 int nva_qkv_prepare(const void *x, int64_t x_row_stride, const void *bias, const void *q_norm_weight, const void *k_norm_weight,
-                    int32_t norm_whole, const float *rope_cache, void *q_out, void *k_cache, void *v_cache,
+                    int32_t norms, const float *rope_cache, void *q_out, void *k_cache, void *v_cache,
                     const int32_t *slot_mapping, int64_t num_slots, const int32_t *cu_seqlens_q, const int32_t *seq_lens,
                     const int32_t *token_seq, int32_t n_tokens, int32_t n_seqs, int32_t num_heads, int32_t num_kv_heads,
                     int32_t qk_dim, int32_t v_dim, int32_t rot_dims, int32_t max_position, float eps, int32_t dtype, void *stream);
@@ -417,12 +429,13 @@ int nva_retention(const void *qkvg, int64_t row_stride, float *state, const int3
  */
 
 /* residual[r] = table[ids[r]] * scale (fp32); out1[r] = residual[r] / rms * (weight_offset + weight1), out2 the
- * same with weight2 (weight2 may be NULL: one norm; both NULL: out1 is the residual itself, rounded).  rms = sqrt(mean(x^2) + eps).  clear (may be NULL):
+ * same with weight2 (weight2 may be NULL: one norm; both NULL: out1 is the residual itself, rounded).  rms = sqrt(mean(x^2) + eps).  out1 has a row stride in elements; copy (may be
+ * NULL, row stride likewise): the residual itself, rounded, as well.  clear (may be NULL):
  * clear_count int32 counters set to zero, for a router that runs behind this. */
 int nva_embed_rms_norms(const int64_t *ids, const void *table, float scale, const void *weight1, const void *weight2,
-                        float weight_offset, float *residual, void *out1, void *out2, int32_t *clear,
-                        int32_t clear_count, int32_t rows, int32_t width, int32_t vocab, float eps, int32_t dtype,
-                        void *stream);
+                        float weight_offset, float *residual, void *out1, int64_t out1_row_stride, void *out2, void *copy,
+                        int64_t copy_row_stride, int32_t *clear, int32_t clear_count, int32_t rows, int32_t width, int32_t vocab,
+                        float eps, int32_t dtype, void *stream);
 
 /* residual[r] += mult * (gain1 * y1[r] + gain2 * sum_k term_weight[r, k] * y2[r * terms + k]), in place, fp32; then
  * the norms as above.  y1 or y2, either gain ([width]) and term_weight (fp32) may be NULL (absent; one; one).
@@ -444,6 +457,19 @@ int nva_post_rms_norms(const void *y1, int64_t y1_row_stride, const float *y1_we
                        int32_t *clear, int32_t clear_count, int32_t rows, int32_t src_rows, int32_t width, float eps,
                        int32_t dtype, void *stream);
 
+/* Branches behind gates of every element: residual[r] += sigmoid(gate[r, :width] + gate_bias[:width]) * y1[r] + sigmoid(gate[r, width:] +
+ * gate_bias[width:]) * sum_k y2[r * terms + k], in place, fp32 (y2 may be NULL; gate and gate_bias then need their first width
+ * elements only); out[r] = residual[r] / rms * (weight_offset + weight), or, weight NULL, the residual itself, rounded.  gate
+ * and out have row strides in elements.  The rest as above. */
+int nva_gated_rms_norm(const void *y1, int64_t y1_row_stride, const void *y2, int32_t terms, const void *gate,
+                       int64_t gate_row_stride, const void *gate_bias, float *residual, const void *weight, float weight_offset,
+                       void *out, int64_t out_row_stride, const int32_t *rows_of, int32_t *clear, int32_t clear_count,
+                       int32_t rows, int32_t src_rows, int32_t width, float eps, int32_t dtype, void *stream);
+
+/* A stream that begins anew: residual[r] = product[r] (fp32, dense) + step; out[r] = residual[r] / rms * (weight_offset + weight). */
+int nva_entry_rms_norm(const float *product, const void *step, float *residual, const void *weight, float weight_offset, void *out,
+                       int32_t *clear, int32_t clear_count, int32_t rows, int32_t width, float eps, int32_t dtype, void *stream);
+
 /* out[r, g] = W_g x[r, g] for every row and group: x + r * x_row_stride + g * x_group_stride, weight [groups, n_out, k_in],
  * out + r * out_row_stride + g * out_group_stride (elements).  out_dtype fp32 keeps the fp32 sums of bf16 products.
  * squared_relu: out = max(., 0)^2. */
@@ -453,23 +479,25 @@ int nva_grouped_linear(const void *x, int64_t x_row_stride, int64_t x_group_stri
 
 /* Router of a mixture of experts: logits = weight x + bias (fp32; bias may be NULL), softmax over all experts, the `top` best (ties: the lower
  * index) in descending order, their scores divided by their sum (+ 1e-20) and multiplied by scale.
- * (With scale 1 the weights are the softmax over the chosen logits.)  weight: [experts + gates, width]; the gates are outputs
+ * (With scale 1 the weights are the softmax over the chosen logits.)  score (enum nva_score) sigmoid: the chosen logits' sigmoids times
+ * scale instead.  weight: [experts + gates, width]; the gates are outputs
  * beside the experts' whose sigmoids follow the choices' weights in every row.
  * choice int32 [rows, top], choice_weight fp32 [rows, top + gates].  lists int32 [experts, list_stride], counts int32 [experts]: the
  * assignments row * top + k of every expert, in no particular order; counts must be zero on entry;
  * list_stride >= rows.  experts <= 1024, gates <= 64, top <= 128. */
 int nva_router(const void *x, int64_t x_row_stride, const void *weight, const float *bias, int32_t *choice,
                float *choice_weight, int32_t *lists, int32_t *counts, int64_t list_stride, int32_t rows, int32_t width,
-               int32_t experts, int32_t gates, int32_t top, float scale, int32_t dtype, void *stream);
+               int32_t experts, int32_t gates, int32_t top, int32_t score, float scale, int32_t dtype, void *stream);
 
 /* out[p] = W_e x[p / terms] (x_per_row) or W_e x[p], for every assignment p of lists to its expert e.
  * weight: [experts, n_out, k_in], or gated: [experts, 2 n_out, k_in] (gate | up) and, with g = min(gate, gate_limit)
  * and u = clamp(up, gate_limit), out = g * sigmoid(gate_slope * g) * (u + gate_shift) (infinity, 1, 0: silu(gate) * up).
- * out: [rows * terms, n_out] dense. */
+ * in_weight (gated only; fp32 [rows, terms], row stride in elements, may be NULL): of what an assignment's expert reads; the products
+ * are multiplied by it ahead of the form.  out: [rows * terms, n_out] dense. */
 int nva_routed_linear(const void *x, int64_t x_row_stride, const void *weight, void *out, const int32_t *lists,
                       const int32_t *counts, int64_t list_stride, int32_t rows, int32_t terms, int32_t experts,
                       int32_t n_out, int32_t k_in, int32_t x_per_row, int32_t gated, float gate_limit, float gate_slope,
-                      float gate_shift, int32_t dtype, void *stream);
+                      float gate_shift, const float *in_weight, int64_t in_weight_row_stride, int32_t dtype, void *stream);
 
 /* The same for few rows, bf16, and in the same launch the product of an expert that every row runs: shared_out[r] = W
  * shared_x[r], shared_weight [shared_n_out, shared_k_in], or gated [2 shared_n_out, shared_k_in] in the same form with
@@ -484,7 +512,7 @@ int nva_routed_shared_linear(const void *x, int64_t x_row_stride, const void *we
  * x: [n_tokens, q_rank | kv_rank | rot_dim] (row stride in elements).
  * q_out [n_tokens, q_rank] = first part / rms * q_norm_weight; cache row slot_mapping[i] of [num_slots, kv_rank + rot_dim] =
  * (second part / rms * kv_norm_weight | third part, neighbours (2i, 2i + 1) rotated by the row's position).
- * cache NULL: the queries only (x then has q_rank columns).  rope_cache: fp32 [max_position, rot_dim], cos in the
+ * q_rank 0: no query latent (q_out and its weight are not used).  cache NULL: the queries only (x then has q_rank columns).  rope_cache: fp32 [max_position, rot_dim], cos in the
  * first half of a row, sin in the second. */
 int nva_latent_prepare(const void *x, int64_t x_row_stride, const void *q_norm_weight, const void *kv_norm_weight,
                        const float *rope_cache, void *q_out, void *cache, const int32_t *slot_mapping, int64_t num_slots,
@@ -494,6 +522,7 @@ int nva_latent_prepare(const void *x, int64_t x_row_stride, const void *q_norm_w
 
 /* Absorbed form: the query at position p meets the cached rows (p - window, p] of its sequence,
  *   score = (q_latent . c + rotate(q_rot) . k_rot) * scale,  out = sigmoid(gate) * sum softmax(score) c.
+ * gate may be NULL (one); sinks (fp32 [num_heads], may be NULL): the sum of a head's weights also contains exp(sink).
  * q_latent [n_tokens, num_heads, kv_rank] dense; q_rot [n_tokens, num_heads, rot_dim], not yet rotated; gate
  * [n_tokens, num_heads] logits; cache [num_blocks, block_size, kv_rank + rot_dim]; out [n_tokens, num_heads, kv_rank] dense.
  * A key behind a table entry outside [0, num_blocks) is not seen.  kv_rank + rot_dim <= 1024.
@@ -501,7 +530,7 @@ int nva_latent_prepare(const void *x, int64_t x_row_stride, const void *q_norm_w
 size_t nva_latent_attn_workspace_bytes(int32_t n_tokens, int32_t num_heads, int32_t kv_rank, int32_t rot_dim,
                                        int32_t max_blocks, int32_t block_size, int32_t window, int32_t dtype);
 int nva_latent_attn(const void *q_latent, const void *q_rot, int64_t qr_row_stride, int64_t qr_head_stride, const void *gate,
-                    int64_t gate_row_stride, const float *rope_cache, const void *cache, const int32_t *block_tables,
+                    int64_t gate_row_stride, const float *sinks, const float *rope_cache, const void *cache, const int32_t *block_tables,
                     int64_t bt_row_stride, int32_t max_blocks, const int32_t *cu_seqlens_q, const int32_t *seq_lens,
                     const int32_t *token_seq, void *out, void *workspace, size_t workspace_bytes, int32_t n_tokens,
                     int32_t n_seqs, int32_t num_heads, int32_t kv_rank, int32_t rot_dim, int32_t block_size,
@@ -511,14 +540,14 @@ int nva_latent_attn(const void *q_latent, const void *q_rot, int64_t qr_row_stri
  * every sequence s to out [n_keys, row_width]; the caller multiplies the latents out to kv [n_keys, num_heads * dim |
  * num_heads * v_dim]; nva_latent_prefill attends:
  *   score = (q[:dim] . k + rotate(q[dim:]) . k_rot) * scale,  out = sigmoid(gate) * sum softmax(score) v
- * over the positions (p - window, p] that were gathered.  q [n_tokens, num_heads, dim + rot_dim], bf16 only, sizes
+ * over the positions (p - window, p] that were gathered, gate and sinks as above.  q [n_tokens, num_heads, dim + rot_dim], bf16 only, sizes
  * multiples of 8 (nva_latent_prefill_supported). */
 int nva_latent_gather(const void *cache, const int32_t *block_tables, int64_t bt_row_stride, int32_t max_blocks,
                       const int32_t *key_cu, const int32_t *seq_lens, void *out, int32_t n_keys, int32_t n_seqs,
                       int32_t row_width, int32_t block_size, int32_t num_blocks, int32_t dtype, void *stream);
 int nva_latent_prefill_supported(int32_t dim, int32_t rot_dim, int32_t v_dim, int32_t dtype);
 int nva_latent_prefill(const void *q, int64_t q_row_stride, const void *kv, int64_t kv_row_stride, const void *k_rot,
-                       int64_t kr_row_stride, const void *gate, int64_t gate_row_stride, const float *rope_cache,
+                       int64_t kr_row_stride, const void *gate, int64_t gate_row_stride, const float *sinks, const float *rope_cache,
                        const int32_t *cu_seqlens_q, const int32_t *seq_lens, const int32_t *key_cu, void *out,
                        int32_t n_tokens, int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads, int32_t dim, int32_t rot_dim,
                        int32_t v_dim, int32_t window, int32_t max_position, float scale, int32_t dtype, void *stream);

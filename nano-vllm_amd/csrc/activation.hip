@@ -1,5 +1,6 @@
 // Element-wise steps behind matrix products:
-//   clamped_gate   out = g sigmoid(alpha g) (u + 1) of a (gate | up) projection, g capped and u clamped
+//   clamped_gate   out = g sigmoid(alpha (g + cubic g^3)) (u + shift) of a (gate | up) projection, g capped and u clamped
+//                  (the tanh form of gelu(g) u is alpha = 2 sqrt(2 / pi), cubic = 0.044715, shift = 0: (1 + tanh y) / 2 = sigmoid(2 y))
 //   squared_relu   out = max(x, 0)^2
 //   soft_cap       x = cap tanh(x / cap), in place
 // Tensors are bf16 or fp32, arithmetic fp32.  V elements per thread: 8, or 1 where sizes or addresses do not allow it.
@@ -10,7 +11,7 @@ namespace nva {
 template <typename T, int V>
 __global__ __launch_bounds__(256) void clamped_gate_kernel(const T *__restrict__ x, int64_t stride, T *__restrict__ out,
                                                            int64_t total, int32_t per_row, int32_t inter, float limit,
-                                                           float alpha) {
+                                                           float alpha, float cubic, float shift) {
     const int64_t idx = static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x;
     if (idx >= total) return;
     const int64_t row = idx / per_row;
@@ -22,7 +23,7 @@ __global__ __launch_bounds__(256) void clamped_gate_kernel(const T *__restrict__
     for (int i = 0; i < V; ++i) {
         const float gc = fminf(g[i], limit);
         const float uc = fminf(fmaxf(u[i], -limit), limit);
-        y[i] = gc * sigmoid_of<T>(alpha * gc) * (uc + 1.0f);
+        y[i] = gc * sigmoid_of<T>(alpha * fmaf(cubic * gc, gc * gc, gc)) * (uc + shift);
     }
     store_f32<T, V>(out + row * inter + e, y);
 }
@@ -69,7 +70,7 @@ static int launch_unary(const void *x, int64_t stride, void *out, int32_t rows, 
 }  // namespace nva
 
 extern "C" int nva_clamped_gate(const void *x, int64_t x_row_stride, void *out, int32_t rows, int32_t inter, float limit,
-                                float alpha, int32_t dtype, void *stream) {
+                                float alpha, float cubic, float shift, int32_t dtype, void *stream) {
     using namespace nva;
     if (rows < 0 || inter <= 0) return NVA_ERR_BAD_SHAPE;
     if (!known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
@@ -85,13 +86,13 @@ extern "C" int nva_clamped_gate(const void *x, int64_t x_row_stride, void *out, 
     if (dtype == NVA_DTYPE_BF16) {
         const bf16_t *xp = static_cast<const bf16_t *>(x);
         bf16_t *op = static_cast<bf16_t *>(out);
-        if (vector) hipLaunchKernelGGL((clamped_gate_kernel<bf16_t, 8>), grid, block, 0, s, xp, x_row_stride, op, total, per_row, inter, limit, alpha);
-        else hipLaunchKernelGGL((clamped_gate_kernel<bf16_t, 1>), grid, block, 0, s, xp, x_row_stride, op, total, per_row, inter, limit, alpha);
+        if (vector) hipLaunchKernelGGL((clamped_gate_kernel<bf16_t, 8>), grid, block, 0, s, xp, x_row_stride, op, total, per_row, inter, limit, alpha, cubic, shift);
+        else hipLaunchKernelGGL((clamped_gate_kernel<bf16_t, 1>), grid, block, 0, s, xp, x_row_stride, op, total, per_row, inter, limit, alpha, cubic, shift);
     } else {
         const float *xp = static_cast<const float *>(x);
         float *op = static_cast<float *>(out);
-        if (vector) hipLaunchKernelGGL((clamped_gate_kernel<float, 8>), grid, block, 0, s, xp, x_row_stride, op, total, per_row, inter, limit, alpha);
-        else hipLaunchKernelGGL((clamped_gate_kernel<float, 1>), grid, block, 0, s, xp, x_row_stride, op, total, per_row, inter, limit, alpha);
+        if (vector) hipLaunchKernelGGL((clamped_gate_kernel<float, 8>), grid, block, 0, s, xp, x_row_stride, op, total, per_row, inter, limit, alpha, cubic, shift);
+        else hipLaunchKernelGGL((clamped_gate_kernel<float, 1>), grid, block, 0, s, xp, x_row_stride, op, total, per_row, inter, limit, alpha, cubic, shift);
     }
     return launch_status();
 }

@@ -2,7 +2,8 @@
 // keys [first_key(p), p] of its own sequence, where
 //   chunks    first_key(p) = floor(p / span) * span
 //   window    first_key(p) = max(0, p - span + 1)     (a span no sequence reaches: all earlier keys)
-// Scores may be capped (cap * tanh(s / cap)); a head may have a sink, one more score that belongs to no key and only
+// Scores may be capped (cap * tanh(s / cap)), or lose a bias that grows with the logarithm of the distance (slope
+// ln(1 + rate (p - j)), two numbers per head); a head may have a sink, one more score that belongs to no key and only
 // enters the sum of the weights; a head's output may be multiplied by sigmoid(gate).  Query/key and value sizes may
 // differ; scores, weights and sums are fp32.
 #include "nva_elem.h"
@@ -28,6 +29,7 @@ struct ChunkAttnArgs {
     int32_t n, n_seqs, heads, kv_heads, dim, vdim, block_shift, num_blocks, max_blocks, span, window;
     float scale, cap;                // cap <= 0: none
     const float *sinks;              // [H] or null
+    const float *slope, *rate;       // [H] each or null: distance bias (excludes a cap)
     const void *gate;                // [n, H] logits or null
     int64_t gate_stride;
 };
@@ -95,6 +97,7 @@ __global__ __launch_bounds__(256) void chunk_attn_any_kernel(ChunkAttnArgs a) {
             for (int i = 0; i < a.dim; ++i) d = fmaf(sh_q[wave][i], Elem<T>::to_f32(k[i]), d);
             s = d * a.scale;
             if (a.cap > 0.f) s = a.cap * tanh_of<T>(s / a.cap);
+            if (a.slope != nullptr) s -= a.slope[head] * log1p_of<T>(a.rate[head] * static_cast<float>(pos - j));
         }
         const float m_new = fmaxf(m, wave_max(s));
         if (m_new == -INFINITY) continue;
@@ -140,7 +143,7 @@ __global__ __launch_bounds__(256) void chunk_attn_any_kernel(ChunkAttnArgs a) {
 
 constexpr float kBoundedCap = 60.0f;
 constexpr float kHeadroom = 64.0f;
-enum Cap { kNoCap, kBounded, kCapped };
+enum Cap { kNoCap, kBounded, kCapped, kBiased };
 
 // Raw product -> base-2 exponent of the weight.
 struct Weighting {
@@ -154,6 +157,10 @@ static Weighting weighting_of(float scale, float cap) {
 __device__ __forceinline__ float exponent_of(const Weighting &w, bool capped, float s) {
     if (capped) return fmaf(-2.0f * w.out, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(w.in * s)), w.out);
     return w.in * s;
+}
+// ... minus a distance bias: ahead = 1 + rate * distance
+__device__ __forceinline__ float biased_exponent(float in, float s, float slope, float ahead) {
+    return fmaf(-slope, __builtin_amdgcn_logf(ahead), in * s);
 }
 
 // Portions: a workgroup of four wavefronts takes 4 * 16 * NQ queries of one head and walks the keys that
@@ -285,7 +292,8 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
     float lsum[NQ], m[NQ], top[NQ];
 #pragma unroll
     for (int qa = 0; qa < NQ; ++qa) m[qa] = top[qa] = -INFINITY;
-    const float to_exp2 = kCap == kCapped ? 1.0f : w.in;             // (not kBounded) of a score, capped already where it is
+    const float to_exp2 = kCap == kCapped || kCap == kBiased ? 1.0f : w.in;      // (not kBounded) of a score, capped or biased already where it is
+    const float slope = kCap == kBiased ? a.slope[head] : 0.f, rate = kCap == kBiased ? a.rate[head] : 0.f;
 
     auto attend = [&](auto masked_c, int key0, int buf) __attribute__((always_inline)) {
         constexpr bool kMasked = decltype(masked_c)::value;
@@ -322,10 +330,14 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 2) void chunk_prefill_kern
 #pragma unroll
                 for (int qa = 0; qa < NQ; ++qa) {
                     float mx = -INFINITY;
+                    // 1 + rate * distance of the half tile's first key of this lane; later keys are nearer (unseen ones may
+                    // give no number, which nothing reads)
+                    const float ahead = fmaf(rate, static_cast<float>(pos[qa] - key0 - 32 * half - 4 * g), 1.0f);
 #pragma unroll
                     for (int kb2 = 0; kb2 < 2; ++kb2)
 #pragma unroll
                         for (int i = 0; i < 4; ++i) {
+                            if (kCap == kBiased) sacc[kb2][qa][i] = biased_exponent(w.in, sacc[kb2][qa][i], slope, fmaf(rate, static_cast<float>(-16 * kb2 - i), ahead));
                             if (kCap == kCapped) sacc[kb2][qa][i] = exponent_of(w, true, sacc[kb2][qa][i]);
                             if (seen(qa, 2 * half + kb2, i)) mx = fmaxf(mx, sacc[kb2][qa][i]);
                         }
@@ -442,8 +454,9 @@ struct SplitArgs {
     int32_t head_groups;     // groups of 16 query heads per kv head
 };
 
-template <int DK, int DV, bool kPlain>
+template <int DK, int DV, Cap kCap>
 __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 3) void chunk_decode_kernel(const ChunkAttnArgs a, const Weighting w, const SplitArgs sp) {
+    constexpr bool kPlain = kCap == kBounded;            // (kCapped: with or without a cap)
     constexpr int kVPitch = DV * 2 + 32;
     constexpr int kWaveBytes = 32 * kVPitch > 16 * DV * 4 ? 32 * kVPitch : 16 * DV * 4;
     constexpr int kVPieces = DV / 16;                    // 16-byte pieces of a 32-key V tile per lane
@@ -524,6 +537,7 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 3) void chunk_decode_kerne
 #pragma unroll
     for (int db = 0; db < DV / 16; ++db) oacc[db] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     float lsum = 0.f, m = -INFINITY;
+    const float slope = kCap == kBiased ? a.slope[head0 + min(r, nheads - 1)] : 0.f, rate = kCap == kBiased ? a.rate[head0 + min(r, nheads - 1)] : 0.f;
     const lds_char_ptr vl = vlds + (4 * g + (r >> 2)) * kVPitch + 8 * (r & 3);
     for (; tile < ntiles; tile += 4) {
         const int key0 = first + tile * 32;
@@ -552,7 +566,8 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 3) void chunk_decode_kerne
             for (int i = 0; i < 4; ++i) {
                 const int key = key0 + 16 * kb + 4 * g + i;
                 vis[kb][i] = ok && key >= lo && key <= last;
-                x[kb][i] = exponent_of(w, kPlain || w.capped, s[kb][i]);
+                if (kCap == kBiased) x[kb][i] = biased_exponent(w.in, s[kb][i], slope, fmaf(rate, static_cast<float>(pos - key), 1.0f));
+                else x[kb][i] = exponent_of(w, kPlain || w.capped, s[kb][i]);
                 if (vis[kb][i]) mx = fmaxf(mx, x[kb][i]);
             }
         float ref = 0.f;
@@ -672,8 +687,9 @@ static int launch_matrix(const ChunkAttnArgs &a, const SplitArgs &sp, int32_t ma
         const int64_t wgs = static_cast<int64_t>(a.n) * sp.splits * sp.head_groups * a.kv_heads;
         if (wgs > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
         const dim3 grid(static_cast<uint32_t>(wgs)), block(256);
-        if (bounded) hipLaunchKernelGGL((chunk_decode_kernel<DK, DV, true>), grid, block, 0, s, a, w, sp);
-        else hipLaunchKernelGGL((chunk_decode_kernel<DK, DV, false>), grid, block, 0, s, a, w, sp);
+        if (a.slope) hipLaunchKernelGGL((chunk_decode_kernel<DK, DV, kBiased>), grid, block, 0, s, a, w, sp);
+        else if (bounded) hipLaunchKernelGGL((chunk_decode_kernel<DK, DV, kBounded>), grid, block, 0, s, a, w, sp);
+        else hipLaunchKernelGGL((chunk_decode_kernel<DK, DV, kCapped>), grid, block, 0, s, a, w, sp);
         const int rc = launch_status();
         if (rc != NVA_OK || sp.splits == 1) return rc;
         hipLaunchKernelGGL(chunk_merge_kernel, dim3(static_cast<uint32_t>((static_cast<int64_t>(a.n) * a.heads + 3) / 4)), block, 0, s, a, sp);
@@ -686,7 +702,9 @@ static int launch_matrix(const ChunkAttnArgs &a, const SplitArgs &sp, int32_t ma
     if (wgs == 0) return NVA_OK;
     const dim3 grid(static_cast<uint32_t>(wgs)), block(256);
     const bool direct = a.dim == DK && a.vdim == DV;
-    if (a.cap > 0.f && !bounded) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, kCapped, false>), grid, block, 0, s, a, w, q_tiles);
+    if (a.slope && direct) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, kBiased, true>), grid, block, 0, s, a, w, q_tiles);
+    else if (a.slope) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, kBiased, false>), grid, block, 0, s, a, w, q_tiles);
+    else if (a.cap > 0.f && !bounded) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, kCapped, false>), grid, block, 0, s, a, w, q_tiles);
     else if (bounded && direct) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, kBounded, true>), grid, block, 0, s, a, w, q_tiles);
     else if (bounded) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, kBounded, false>), grid, block, 0, s, a, w, q_tiles);
     else if (direct) hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NQ, kNoCap, true>), grid, block, 0, s, a, w, q_tiles);
@@ -729,15 +747,17 @@ extern "C" int nva_masked_attn(const void *q, int64_t q_row_stride, const void *
                               void *workspace, size_t workspace_bytes, int32_t n_tokens, int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads,
                               int32_t num_kv_heads, int32_t qk_dim, int32_t v_dim, int32_t block_size,
                               int32_t num_blocks, int32_t mask, int32_t span, float scale, float softcap, const float *sinks,
-                              const void *gate, int64_t gate_row_stride, int32_t dtype, void *stream) {
+                              const float *bias_slope, const float *bias_rate, const void *gate, int64_t gate_row_stride, int32_t dtype,
+                              void *stream) {
     using namespace nva;
     if (n_tokens < 0 || n_seqs < 0 || num_heads <= 0 || num_kv_heads <= 0 || qk_dim <= 0 || v_dim <= 0 || num_blocks < 0 ||
         max_blocks < 0 || span <= 0 || max_seqlen_q < 0 || num_heads % num_kv_heads != 0)
         return NVA_ERR_BAD_SHAPE;
     const int shift = block_shift_of(block_size);
     if (shift < 0 || (mask != NVA_MASK_CHUNKS && mask != NVA_MASK_WINDOW) || qk_dim > kAnyMaxDim || v_dim > kAnyMaxDim || !known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
+    if (bias_slope && softcap > 0.f) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     if (n_tokens == 0) return NVA_OK;
-    if (!q || !k_cache || !v_cache || !block_tables || !seq_lens || !out) return NVA_ERR_NULL_POINTER;
+    if (!q || !k_cache || !v_cache || !block_tables || !seq_lens || !out || (bias_slope == nullptr) != (bias_rate == nullptr)) return NVA_ERR_NULL_POINTER;
     const bool decode = cu_seqlens_q == nullptr;
     if (!decode && (!token_seq || n_seqs == 0)) return NVA_ERR_NULL_POINTER;
     if (decode && n_seqs != n_tokens) return NVA_ERR_BAD_SHAPE;
@@ -748,7 +768,7 @@ extern "C" int nva_masked_attn(const void *q, int64_t q_row_stride, const void *
     a.bt_stride = bt_row_stride; a.cu = cu_seqlens_q; a.klen = seq_lens; a.token_seq = token_seq; a.out = out;
     a.n = n_tokens; a.n_seqs = n_seqs; a.heads = num_heads; a.kv_heads = num_kv_heads; a.dim = qk_dim; a.vdim = v_dim;
     a.block_shift = shift; a.num_blocks = num_blocks; a.max_blocks = max_blocks; a.span = span;
-    a.window = mask == NVA_MASK_WINDOW; a.scale = scale; a.cap = softcap; a.sinks = sinks; a.gate = gate; a.gate_stride = gate_row_stride;
+    a.window = mask == NVA_MASK_WINDOW; a.scale = scale; a.cap = softcap; a.sinks = sinks; a.slope = bias_slope; a.rate = bias_rate; a.gate = gate; a.gate_stride = gate_row_stride;
     hipStream_t s = static_cast<hipStream_t>(stream);
     if (dtype == NVA_DTYPE_BF16 && matrix_ok(a)) {
         SplitArgs sp{};
@@ -779,5 +799,5 @@ extern "C" int nva_chunk_attn(const void *q, int64_t q_row_stride, const void *k
                               void *stream) {
     return nva_masked_attn(q, q_row_stride, k_cache, v_cache, block_tables, bt_row_stride, max_blocks, cu_seqlens_q, seq_lens, token_seq, out,
                            workspace, workspace_bytes, n_tokens, n_seqs, max_seqlen_q, num_heads, num_kv_heads, qk_dim, v_dim, block_size,
-                           num_blocks, NVA_MASK_CHUNKS, chunk, scale, softcap, nullptr, nullptr, 0, dtype, stream);
+                           num_blocks, NVA_MASK_CHUNKS, chunk, scale, softcap, nullptr, nullptr, nullptr, nullptr, 0, dtype, stream);
 }

@@ -5,8 +5,10 @@
 //                  lists[e] holds the assignments of expert e in any order, counts[e] their number
 //   gated          W has 2 n_out rows (gate | up): out = g sigmoid(slope g) (u + shift), g = min(gate, limit), u = clamp(up, limit)
 //                  (slope 1, shift 0, no limit: silu(gate) * up)
+//                  (routed: an assignment's weight may belong to what its expert reads; it then multiplies gate and up)
 //   squared relu   of a dense group's results, where asked for
-//   router         logits (with a bias) in fp32, softmax over all experts, the best `terms`, their normalised weights, lists;
+//   router         logits (with a bias) in fp32, the best `terms`, their weights (from a softmax over all experts, normalised, or
+//                  their sigmoids as they are), lists;
 //                  and the sigmoids of further outputs, gates of what every row runs
 // bf16 tensors go through the matrix cores, fp32 ones and odd sizes through plain fp32 kernels.
 #include "nva_elem.h"
@@ -35,7 +37,15 @@ struct LinearArgs {
     int32_t x_div;                   // routed: x row = assignment / x_div
     GateForm gate;                   // gated
     int32_t squared_relu;            // of the results (not gated)
+    const float *in_weight;          // gated, routed: of assignment p at p / terms * in_stride + p % terms, or null
+    int64_t in_stride;
+    int32_t terms;
 };
+
+// what the rows a group reads are multiplied by
+__device__ __forceinline__ float input_weight(const LinearArgs &a, int row) {
+    return a.in_weight == nullptr ? 1.0f : a.in_weight[row / a.terms * a.in_stride + row % a.terms];
+}
 
 // number of rows of a group, and where its i-th row comes from and goes to
 __device__ __forceinline__ int group_rows(const LinearArgs &a, int g) {
@@ -95,10 +105,11 @@ __global__ __launch_bounds__(256) void linear_any_kernel(LinearArgs a) {
         }
         if (m0 + r < count) {
             O *out = static_cast<O *>(a.out) + out_offset(a, g, row);
+            const float f = kGated ? input_weight(a, row) : 1.0f;
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 const int n = n0 + c + 16 * j;
-                if (n < a.n_out) out[n] = Elem<O>::from_f32(kGated ? gated_value<T>(a.gate, acc[0][j], acc[kParts - 1][j]) : result_of(a, acc[0][j]));
+                if (n < a.n_out) out[n] = Elem<O>::from_f32(kGated ? gated_value<T>(a.gate, f * acc[0][j], f * acc[kParts - 1][j]) : result_of(a, acc[0][j]));
             }
         }
     }
@@ -174,8 +185,10 @@ __global__ __launch_bounds__(256) void linear_skinny_kernel(const LinearArgs all
                 const int c = 16 * NB * p + n;
                 v[p] = (part[0][m][c] + part[1][m][c]) + (part[2][m][c] + part[3][m][c]);
             }
-            static_cast<O *>(a.out)[out_offset(a, g, group_row(a, g, m0 + m)) + n0 + n] =
-                Elem<O>::from_f32(kGated ? gated_value<bf16_t>(a.gate, v[0], v[kParts - 1]) : result_of(a, v[0]));
+            const int row = group_row(a, g, m0 + m);
+            const float f = kGated ? input_weight(a, row) : 1.0f;
+            static_cast<O *>(a.out)[out_offset(a, g, row) + n0 + n] =
+                Elem<O>::from_f32(kGated ? gated_value<bf16_t>(a.gate, f * v[0], f * v[kParts - 1]) : result_of(a, v[0]));
         }
         __syncthreads();
     }
@@ -220,6 +233,7 @@ __global__ __launch_bounds__(256, BN > 128 ? 1 : 2) void linear_tile_kernel(cons
     constexpr int kLX = kBlocksX / 4, kLW = kBlocksW / 4, kLoads = kLX + kLW;   // blocks a wavefront loads per step
     __shared__ __attribute__((aligned(1024))) unsigned char smem[kBuffers * kStage];
     __shared__ int sh_row[BM];
+    __shared__ float sh_weight[kGated ? BM : 1];
     const int tid = threadIdx.x, lane = tid & 63, r = lane & 15, g = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int wm = wave & 1, wn = wave >> 1;
@@ -265,7 +279,10 @@ __global__ __launch_bounds__(256, BN > 128 ? 1 : 2) void linear_tile_kernel(cons
     const int n_tile = in_group / abreast;
     m_tile = group * kGroup + in_group % abreast;
     const int count = group_rows(a, expert), m0 = m_tile * BM;
-    if (tid < BM) sh_row[tid] = group_row(a, expert, min(m0 + tid, count - 1));       // (published by the barriers below)
+    if (tid < BM) {                                      // (published by the barriers below)
+        sh_row[tid] = group_row(a, expert, min(m0 + tid, count - 1));
+        if constexpr (kGated) sh_weight[tid] = input_weight(a, sh_row[tid]);
+    }
 
     // ---- what this wavefront loads: byte offsets of its lanes' pieces in the first step
     const int l16 = lane >> 2, piece = ((lane & 3) ^ ((0 - (l16 >> 2)) & 3)) * 8;
@@ -383,15 +400,17 @@ __global__ __launch_bounds__(256, BN > 128 ? 1 : 2) void linear_tile_kernel(cons
     for (int round = 0; round < kRounds; ++round) {
         if (kRounds == 1 || wm == round)
 #pragma unroll
-            for (int m = 0; m < kTM; ++m)
+            for (int m = 0; m < kTM; ++m) {
+                const float f = kGated ? sh_weight[16 * (wm * kTM + m) + r] : 1.0f;
 #pragma unroll
                 for (int n = 0; n < (kGated ? kTN / 2 : kTN); ++n) {
                     float y[4];
 #pragma unroll
-                    for (int j = 0; j < 4; ++j) y[j] = kGated ? gated_value<bf16_t>(a.gate, acc[n][m][j], acc[kGated ? n + kTN / 2 : n][m][j]) : acc[n][m][j];
+                    for (int j = 0; j < 4; ++j) y[j] = kGated ? gated_value<bf16_t>(a.gate, f * acc[n][m][j], f * acc[kGated ? n + kTN / 2 : n][m][j]) : acc[n][m][j];
                     *(__attribute__((address_space(3))) u32x2_t *)(lds + (16 * ((kRounds == 1 ? wm * kTM : 0) + m) + r) * kOutPitch + 2 * (kCols / 2 * wn + 16 * n + 4 * g)) =
                         u32x2_t{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
                 }
+            }
         __syncthreads();
         const int base = round * (BM / 2), end = min(base + BM / kRounds, count - m0);
         if (n0 < a.n_out)
@@ -461,6 +480,7 @@ struct RouterArgs {
     int32_t *lists, *counts;         // [experts, list_stride], [experts] (zero on entry)
     int64_t list_stride;
     int32_t rows, width, experts, gates, top;
+    int32_t sigmoid;                 // weights: the chosen logits' sigmoids
     float scale;
 };
 
@@ -532,7 +552,8 @@ __global__ __launch_bounds__(64 * NW) void router_kernel(RouterArgs a) {
         }
         __syncthreads();
     }
-    // one wavefront per row: softmax over the experts, then the best one `top` times (ties: the lower index)
+    // one wavefront per row: softmax over the experts (or their sigmoids; both rise with the logit), then the best one `top`
+    // times (ties: the lower index)
     for (int row = wave; row < rows; row += NW) {
         float *z = logits + row * outs;
         float mine_z = -INFINITY, mx = -INFINITY;            // (up to 64 experts: one per lane)
@@ -564,7 +585,7 @@ __global__ __launch_bounds__(64 * NW) void router_kernel(RouterArgs a) {
             if (narrow) win = at != 0 ? __ffsll(at) - 1 : 0;
             else win = 1023 - static_cast<int>(wave_max(best == best_now ? static_cast<float>(1023 - who) : 0.f));
             if (win >= a.experts) win = 0;                   // (only where logits are not numbers)
-            const float s = exp_of<T>(best_now - mx) * inv;
+            const float s = a.sigmoid ? sigmoid_of<T>(best_now) : exp_of<T>(best_now - mx) * inv;
             chosen += s;
             if (lane == k % 64) {
                 my_s = s;
@@ -584,7 +605,7 @@ __global__ __launch_bounds__(64 * NW) void router_kernel(RouterArgs a) {
             }
         }
         __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-        const float f = a.scale / (chosen + kWeightGuard);
+        const float f = a.sigmoid ? a.scale : a.scale / (chosen + kWeightGuard);
         const int64_t at = static_cast<int64_t>(row0 + row) * a.top;
         float *out = a.weight + static_cast<int64_t>(row0 + row) * (a.top + a.gates);
         for (int j = lane; j < a.gates; j += 64) out[a.top + j] = sigmoid_of<T>(z[a.experts + j]);
@@ -649,13 +670,15 @@ extern "C" int nva_grouped_linear(const void *x, int64_t x_row_stride, int64_t x
 namespace nva {
 static int routed_args(LinearArgs &a, const void *x, int64_t x_row_stride, const void *weight, void *out, const int32_t *lists,
                        const int32_t *counts, int64_t list_stride, int32_t rows, int32_t terms, int32_t experts, int32_t n_out,
-                       int32_t k_in, int32_t x_per_row, float gate_limit, float gate_slope, float gate_shift, int32_t dtype) {
+                       int32_t k_in, int32_t x_per_row, float gate_limit, float gate_slope, float gate_shift, const float *in_weight,
+                       int64_t in_weight_row_stride, int32_t dtype) {
     if (rows < 0 || terms <= 0 || experts <= 0 || n_out <= 0 || k_in <= 0 || list_stride < rows || terms > experts) return NVA_ERR_BAD_SHAPE;
     if (!known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     if (rows == 0) return NVA_OK;
     if (!x || !weight || !out || !lists || !counts) return NVA_ERR_NULL_POINTER;
     if (experts > 65535 || static_cast<int64_t>(rows) * terms > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
-    if (x_row_stride < k_in) return NVA_ERR_BAD_STRIDE;
+    if (x_row_stride < k_in || (in_weight && in_weight_row_stride < terms)) return NVA_ERR_BAD_STRIDE;
+    a.in_weight = in_weight; a.in_stride = in_weight_row_stride; a.terms = terms;
     a.x = x; a.x_stride = x_row_stride; a.w = weight; a.out = out; a.o_stride = n_out; a.lists = lists; a.counts = counts;
     a.list_stride = list_stride; a.rows = rows * terms; a.groups = experts; a.n_out = n_out; a.k = k_in; a.x_div = x_per_row ? terms : 1;
     a.gate = GateForm{gate_limit, gate_slope, gate_shift};
@@ -672,11 +695,12 @@ static int32_t busy_experts(int32_t rows, int32_t terms, int32_t experts) {
 extern "C" int nva_routed_linear(const void *x, int64_t x_row_stride, const void *weight, void *out, const int32_t *lists,
                                  const int32_t *counts, int64_t list_stride, int32_t rows, int32_t terms, int32_t experts,
                                  int32_t n_out, int32_t k_in, int32_t x_per_row, int32_t gated, float gate_limit, float gate_slope, float gate_shift,
-                                 int32_t dtype, void *stream) {
+                                 const float *in_weight, int64_t in_weight_row_stride, int32_t dtype, void *stream) {
     using namespace nva;
+    if (in_weight && !gated) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     LinearArgs a{};
     const int rc = routed_args(a, x, x_row_stride, weight, out, lists, counts, list_stride, rows, terms, experts, n_out, k_in, x_per_row,
-                               gate_limit, gate_slope, gate_shift, dtype);
+                               gate_limit, gate_slope, gate_shift, in_weight, in_weight_row_stride, dtype);
     if (rc != NVA_OK || rows == 0) return rc;
     hipStream_t s = static_cast<hipStream_t>(stream);
     if (dtype == NVA_DTYPE_F32) return gated ? launch_any_linear<float, float, true>(a, rows, s) : launch_any_linear<float, float, false>(a, rows, s);
@@ -699,7 +723,7 @@ extern "C" int nva_routed_shared_linear(const void *x, int64_t x_row_stride, con
     using namespace nva;
     LinearArgs a{}, b{};
     const int rc = routed_args(a, x, x_row_stride, weight, out, lists, counts, list_stride, rows, terms, experts, n_out, k_in, x_per_row,
-                               gate_limit, gate_slope, gate_shift, NVA_DTYPE_BF16);
+                               gate_limit, gate_slope, gate_shift, nullptr, 0, NVA_DTYPE_BF16);
     if (rc != NVA_OK) return rc;
     if (shared_n_out <= 0 || shared_k_in <= 0) return NVA_ERR_BAD_SHAPE;
     if (rows == 0) return NVA_OK;
@@ -715,8 +739,9 @@ extern "C" int nva_routed_shared_linear(const void *x, int64_t x_row_stride, con
 
 extern "C" int nva_router(const void *x, int64_t x_row_stride, const void *weight, const float *bias, int32_t *choice,
                           float *choice_weight, int32_t *lists, int32_t *counts, int64_t list_stride, int32_t rows, int32_t width,
-                          int32_t experts, int32_t gates, int32_t top, float scale, int32_t dtype, void *stream) {
+                          int32_t experts, int32_t gates, int32_t top, int32_t score, float scale, int32_t dtype, void *stream) {
     using namespace nva;
+    if (score != NVA_SCORE_SOFTMAX && score != NVA_SCORE_SIGMOID) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     if (rows < 0 || width <= 0 || experts <= 0 || gates < 0 || top <= 0 || top > experts || list_stride < rows) return NVA_ERR_BAD_SHAPE;
     if (!known_dtype(dtype) || experts > 1024 || gates > 64 || top > 128) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     if (rows == 0) return NVA_OK;
@@ -725,7 +750,7 @@ extern "C" int nva_router(const void *x, int64_t x_row_stride, const void *weigh
     if (static_cast<int64_t>(rows) * top > 0x7fffffffLL) return NVA_ERR_BAD_SHAPE;
     RouterArgs a{};
     a.x = x; a.x_stride = x_row_stride; a.w = weight; a.bias = bias; a.choice = choice; a.weight = choice_weight; a.lists = lists; a.counts = counts;
-    a.list_stride = list_stride; a.rows = rows; a.width = width; a.experts = experts; a.gates = gates; a.top = top; a.scale = scale;
+    a.list_stride = list_stride; a.rows = rows; a.width = width; a.experts = experts; a.gates = gates; a.top = top; a.sigmoid = score == NVA_SCORE_SIGMOID; a.scale = scale;
     hipStream_t s = static_cast<hipStream_t>(stream);
     const bool many = rows >= 4096 && experts <= 128 && top <= 32;       // more rows per workgroup: fewer additions to the counters
     if (dtype == NVA_DTYPE_F32) return launch_router_tg<float, 1, 8, false>(a, s);

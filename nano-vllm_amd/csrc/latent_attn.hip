@@ -1,7 +1,8 @@
 // Latent attention: a token leaves one normed latent c (rank R) and one rotated key part (rot elements), shared
 // by all heads, in the paged cache.  Head h's key is [W_uk,h c | rotated part], its value W_uv,h c; the query at
-// position p sees the keys (p - window, p].  Scores, weights and sums are fp32; a head's result is multiplied by
-// the sigmoid of a gate projection.  Two forms:
+// position p sees the keys (p - window, p].  Scores, weights and sums are fp32; a head may have a
+// sink, one more score that belongs to no key and only enters the sum of the weights, and its result may be multiplied
+// by the sigmoid of a gate projection.  Two forms:
 //   absorbed   the query goes through W_uk,h^T first and meets the latents as they lie in the cache; the result
 //              is a weighted latent, which goes through W_uv,h afterwards (single tokens, short portions)
 //   expanded   the visible latents are gathered and multiplied out into keys and values (longer portions)
@@ -32,6 +33,15 @@ __device__ __forceinline__ void place_of(const RowsOf &w, int64_t t, int &seq, i
     }
 }
 
+// what a head's sum of weights 2^(exponent - top) gets for its sink, and what its result is multiplied by
+__device__ __forceinline__ float latent_sink(const float *sinks, int head, float top) {
+    return sinks == nullptr ? 0.f : __builtin_amdgcn_exp2f(fmaf(sinks[head], 1.4426950408889634f, -top));
+}
+template <typename T>
+__device__ __forceinline__ float latent_gate(const void *gate, int64_t stride, int64_t row, int head) {
+    return gate == nullptr ? 1.0f : sigmoid_of<T>(Elem<T>::to_f32(static_cast<const T *>(gate)[row * stride + head]));
+}
+
 // V elements at e (a multiple of V, V even) of a vector whose neighbours (2i, 2i + 1) turn; table row: cos | sin
 template <int V>
 __device__ __forceinline__ void turn_pairs(float (&x)[V], const float *cs, int half, int e) {
@@ -47,7 +57,7 @@ __device__ __forceinline__ void turn_pairs(float (&x)[V], const float *cs, int h
 // ---- what a token leaves behind, and its query latent ------------------------------------------------
 
 struct LatentPrepareArgs {
-    const void *x;                   // [n, q_rank + (R + rot)], row stride in elements
+    const void *x;                   // [n, q_rank + (R + rot)], row stride in elements (q_rank 0: no query latent)
     int64_t stride;
     const void *wq, *wkv;            // norm weights [q_rank], [R]
     const float *rope;               // [max_position, rot]
@@ -83,7 +93,7 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(LatentPrepareArgs a
             store_f32<T, V>(dst + e, v);
         }
     };
-    normed(x, static_cast<const T *>(a.wq), a.q_rank, static_cast<T *>(a.q_out) + t * a.q_rank);
+    if (a.q_rank > 0) normed(x, static_cast<const T *>(a.wq), a.q_rank, static_cast<T *>(a.q_out) + t * a.q_rank);
     if (a.cache == nullptr) return;
     const int64_t slot = a.slot_mapping[t];
     if (slot < 0 || slot >= a.num_slots) return;
@@ -117,8 +127,9 @@ struct LatentAttnArgs {
     const void *q_lat;               // [n, H, R] dense
     const void *q_rot;               // [n, H, rot]: not yet rotated; strides in elements
     int64_t qr_row, qr_head;
-    const void *gate;                // [n, H] logits, row stride in elements
+    const void *gate;                // [n, H] logits, row stride in elements, or null
     int64_t gate_stride;
+    const float *sinks;              // [H] or null
     const float *rope;
     const void *cache;               // [num_blocks, block, R + rot]
     const int32_t *block_tables;     // [n_seqs, >= max_blocks]
@@ -198,8 +209,8 @@ __global__ __launch_bounds__(256) void latent_attn_any_kernel(LatentAttnArgs a) 
         }
     }
     T *out = static_cast<T *>(a.out) + item * a.rank;
-    const float z = Elem<T>::to_f32(static_cast<const T *>(a.gate)[t * a.gate_stride + head]);
-    const float f = sum > 0.f ? sigmoid_of<T>(z) / sum : 0.f;
+    if (a.sinks != nullptr && sum > 0.f) sum += exp_of<T>(a.sinks[head] - m);
+    const float f = sum > 0.f ? latent_gate<T>(a.gate, a.gate_stride, t, head) / sum : 0.f;
 #pragma unroll
     for (int i = 0; i < kLatentMax / 64; ++i)
         if (i * 64 + lane < a.rank) out[i * 64 + lane] = Elem<T>::from_f32(acc[i] * f);
@@ -414,8 +425,7 @@ __global__ __launch_bounds__(256, 2) void latent_rows_kernel(const LatentAttnArg
         if (hh >= nheads) continue;
         const float l = (sh_l[h][0][r] + sh_l[h][1][r]) + (sh_l[h][2][r] + sh_l[h][3][r]);
         if (sp.splits == 1) {
-            const float z = bf16_to_f32(static_cast<const bf16_t *>(a.gate)[t * a.gate_stride + head0 + hh]);
-            const float f = l > 0.f ? sigmoid_of<bf16_t>(z) / l : 0.f;
+            const float f = l > 0.f ? latent_gate<bf16_t>(a.gate, a.gate_stride, t, head0 + hh) / (l + latent_sink(a.sinks, head0 + hh, m[h])) : 0.f;
 #pragma unroll
             for (int db = 0; db < kDB; ++db) {
                 const int c = wave * (RK / 4) + 16 * db + 4 * g;
@@ -454,7 +464,7 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const LatentAttnArgs 
     // lane j holds sum and reference of range j
     const float my_l = lane < count ? part[lane * step + a.rank] : 0.f;
     const float my_m = lane < count ? part[lane * step + a.rank + 1] : -INFINITY;
-    const float z = bf16_to_f32(static_cast<const bf16_t *>(a.gate)[t * a.gate_stride + head]);
+    const float gate = latent_gate<bf16_t>(a.gate, a.gate_stride, t, head);
     constexpr int kAhead = 8;
     f32x4_t p[kAhead], o = {0.f, 0.f, 0.f, 0.f};
     const bool in = c < a.rank;                          // (the rank is a multiple of 8)
@@ -467,7 +477,7 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const LatentAttnArgs 
     const float top = wave_max(my_m);
     const float f = my_m == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(my_m - top);
     const float l = wave_sum(my_l * f);
-    const float inv = l > 0.f ? sigmoid_of<bf16_t>(z) / l : 0.f;
+    const float inv = l > 0.f ? gate / (l + latent_sink(a.sinks, head, top)) : 0.f;
     for (int j0 = 0; j0 < count; j0 += kAhead) {
 #pragma unroll
         for (int j = 0; j < kAhead; ++j) {
@@ -551,8 +561,9 @@ struct LatentPrefillArgs {
     int64_t kv_stride;
     const bf16_t *k_rot;             // [n_keys, rot], row stride in elements
     int64_t kr_stride;
-    const bf16_t *gate;
+    const bf16_t *gate;              // or null
     int64_t gate_stride;
+    const float *sinks;              // [H] or null
     const float *rope;
     const int32_t *cu, *klen, *key_cu;
     bf16_t *out;                     // [n, H, vdim] dense
@@ -808,8 +819,7 @@ __global__ __launch_bounds__(256, DN + DR + DV > 384 ? 1 : 2) void latent_prefil
         l += __shfl_xor(l, 32, 64);
         const int row = row0 + wave * 16 * NQ + 16 * qa + r;
         if (row >= lq) continue;
-        const float z = bf16_to_f32(a.gate[static_cast<int64_t>(t0 + row) * a.gate_stride + head]);
-        const float inv = l > 0.f ? sigmoid_of<bf16_t>(z) / l : 0.f;
+        const float inv = l > 0.f ? latent_gate<bf16_t>(a.gate, a.gate_stride, t0 + row, head) / (l + latent_sink(a.sinks, head, m[qa])) : 0.f;
         bf16_t *out = a.out + (static_cast<int64_t>(t0 + row) * a.heads + head) * a.vdim + 4 * g;
 #pragma unroll
         for (int db = 0; db < DV / 16; ++db)
@@ -838,10 +848,10 @@ extern "C" int nva_latent_prepare(const void *x, int64_t x_row_stride, const voi
                                   int32_t n_seqs, int32_t q_rank, int32_t kv_rank, int32_t rot_dim, int32_t max_position, float eps,
                                   int32_t dtype, void *stream) {
     using namespace nva;
-    if (n_tokens < 0 || n_seqs < 0 || q_rank <= 0 || max_position <= 0 || (cache && (kv_rank <= 0 || rot_dim < 0 || num_slots < 0))) return NVA_ERR_BAD_SHAPE;
+    if (n_tokens < 0 || n_seqs < 0 || q_rank < 0 || max_position <= 0 || (cache && (kv_rank <= 0 || rot_dim < 0 || num_slots < 0))) return NVA_ERR_BAD_SHAPE;
     if (!known_dtype(dtype) || (cache && rot_dim % 2 != 0)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     if (n_tokens == 0) return NVA_OK;
-    if (!x || !q_norm_weight || !q_out || !seq_lens || (cache && (!kv_norm_weight || !slot_mapping || (rot_dim > 0 && !rope_cache)))) return NVA_ERR_NULL_POINTER;
+    if (!x || (q_rank > 0 && (!q_norm_weight || !q_out)) || !seq_lens || (cache && (!kv_norm_weight || !slot_mapping || (rot_dim > 0 && !rope_cache)))) return NVA_ERR_NULL_POINTER;
     if (cu_seqlens_q && (!token_seq || n_seqs == 0)) return NVA_ERR_NULL_POINTER;
     if (!cu_seqlens_q && n_seqs != n_tokens) return NVA_ERR_BAD_SHAPE;
     if (x_row_stride < static_cast<int64_t>(q_rank) + (cache ? kv_rank + rot_dim : 0)) return NVA_ERR_BAD_STRIDE;
@@ -873,7 +883,7 @@ extern "C" size_t nva_latent_attn_workspace_bytes(int32_t n_tokens, int32_t num_
 }
 
 extern "C" int nva_latent_attn(const void *q_latent, const void *q_rot, int64_t qr_row_stride, int64_t qr_head_stride, const void *gate,
-                               int64_t gate_row_stride, const float *rope_cache, const void *cache, const int32_t *block_tables,
+                               int64_t gate_row_stride, const float *sinks, const float *rope_cache, const void *cache, const int32_t *block_tables,
                                int64_t bt_row_stride, int32_t max_blocks, const int32_t *cu_seqlens_q, const int32_t *seq_lens,
                                const int32_t *token_seq, void *out, void *workspace, size_t workspace_bytes, int32_t n_tokens,
                                int32_t n_seqs, int32_t num_heads, int32_t kv_rank, int32_t rot_dim, int32_t block_size,
@@ -884,14 +894,14 @@ extern "C" int nva_latent_attn(const void *q_latent, const void *q_rot, int64_t 
     const int shift = block_shift_of(block_size);
     if (shift < 0 || kv_rank + rot_dim > kLatentMax || rot_dim % 2 != 0 || !known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     if (n_tokens == 0) return NVA_OK;
-    if (!q_latent || !gate || !cache || !block_tables || !seq_lens || !out || (rot_dim > 0 && (!q_rot || !rope_cache))) return NVA_ERR_NULL_POINTER;
+    if (!q_latent || !cache || !block_tables || !seq_lens || !out || (rot_dim > 0 && (!q_rot || !rope_cache))) return NVA_ERR_NULL_POINTER;
     if (cu_seqlens_q && (!token_seq || n_seqs == 0)) return NVA_ERR_NULL_POINTER;
     if (!cu_seqlens_q && n_seqs != n_tokens) return NVA_ERR_BAD_SHAPE;
-    if (bt_row_stride < max_blocks || gate_row_stride < num_heads || qr_head_stride < rot_dim || qr_row_stride < static_cast<int64_t>(num_heads - 1) * qr_head_stride + rot_dim)
+    if (bt_row_stride < max_blocks || (gate && gate_row_stride < num_heads) || qr_head_stride < rot_dim || qr_row_stride < static_cast<int64_t>(num_heads - 1) * qr_head_stride + rot_dim)
         return NVA_ERR_BAD_STRIDE;
     if (static_cast<int64_t>(n_tokens) * num_heads / 4 > 0x7ffffff0LL) return NVA_ERR_BAD_SHAPE;
     LatentAttnArgs a{};
-    a.q_lat = q_latent; a.q_rot = q_rot; a.qr_row = qr_row_stride; a.qr_head = qr_head_stride; a.gate = gate; a.gate_stride = gate_row_stride;
+    a.q_lat = q_latent; a.q_rot = q_rot; a.qr_row = qr_row_stride; a.qr_head = qr_head_stride; a.gate = gate; a.gate_stride = gate_row_stride; a.sinks = sinks;
     a.rope = rope_cache; a.cache = cache; a.block_tables = block_tables; a.bt_stride = bt_row_stride; a.out = out;
     a.rows = RowsOf{cu_seqlens_q, seq_lens, token_seq, n_tokens, n_seqs}; a.heads = num_heads; a.rank = kv_rank; a.rot = rot_dim;
     a.block_shift = shift; a.num_blocks = num_blocks; a.max_blocks = max_blocks; a.window = window; a.max_position = max_position; a.scale = scale;
@@ -952,7 +962,7 @@ extern "C" int nva_latent_prefill_supported(int32_t dim, int32_t rot_dim, int32_
 }
 
 extern "C" int nva_latent_prefill(const void *q, int64_t q_row_stride, const void *kv, int64_t kv_row_stride, const void *k_rot,
-                                  int64_t kr_row_stride, const void *gate, int64_t gate_row_stride, const float *rope_cache,
+                                  int64_t kr_row_stride, const void *gate, int64_t gate_row_stride, const float *sinks, const float *rope_cache,
                                   const int32_t *cu_seqlens_q, const int32_t *seq_lens, const int32_t *key_cu, void *out,
                                   int32_t n_tokens, int32_t n_seqs, int32_t max_seqlen_q, int32_t num_heads, int32_t dim, int32_t rot_dim,
                                   int32_t v_dim, int32_t window, int32_t max_position, float scale, int32_t dtype, void *stream) {
@@ -960,15 +970,15 @@ extern "C" int nva_latent_prefill(const void *q, int64_t q_row_stride, const voi
     if (n_tokens < 0 || n_seqs < 0 || max_seqlen_q < 0 || num_heads <= 0 || dim <= 0 || rot_dim < 0 || v_dim <= 0 || window <= 0 || max_position <= 0) return NVA_ERR_BAD_SHAPE;
     if (!nva_latent_prefill_supported(dim, rot_dim, v_dim, dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     if (n_tokens == 0 || n_seqs == 0) return NVA_OK;
-    if (!q || !kv || !gate || !cu_seqlens_q || !seq_lens || !key_cu || !out || (rot_dim > 0 && (!k_rot || !rope_cache))) return NVA_ERR_NULL_POINTER;
+    if (!q || !kv || !cu_seqlens_q || !seq_lens || !key_cu || !out || (rot_dim > 0 && (!k_rot || !rope_cache))) return NVA_ERR_NULL_POINTER;
     if (q_row_stride < static_cast<int64_t>(num_heads) * (dim + rot_dim) || kv_row_stride < static_cast<int64_t>(num_heads) * (dim + v_dim) ||
-        kr_row_stride < rot_dim || gate_row_stride < num_heads || q_row_stride % 8 != 0 || kv_row_stride % 8 != 0 || kr_row_stride % 8 != 0)
+        kr_row_stride < rot_dim || (gate && gate_row_stride < num_heads) || q_row_stride % 8 != 0 || kv_row_stride % 8 != 0 || kr_row_stride % 8 != 0)
         return NVA_ERR_BAD_STRIDE;
     if (kv_row_stride > (1 << 24) || kr_row_stride > (1 << 24)) return NVA_ERR_BAD_STRIDE;      // offsets inside a tile are 32-bit
     if (!aligned16(q) || !aligned16(kv) || !aligned16(k_rot) || !aligned16(out)) return NVA_ERR_MISALIGNED;
     LatentPrefillArgs a{};
     a.q = static_cast<const bf16_t *>(q); a.q_stride = q_row_stride; a.kv = static_cast<const bf16_t *>(kv); a.kv_stride = kv_row_stride;
-    a.k_rot = static_cast<const bf16_t *>(k_rot); a.kr_stride = kr_row_stride; a.gate = static_cast<const bf16_t *>(gate); a.gate_stride = gate_row_stride;
+    a.k_rot = static_cast<const bf16_t *>(k_rot); a.kr_stride = kr_row_stride; a.gate = static_cast<const bf16_t *>(gate); a.gate_stride = gate_row_stride; a.sinks = sinks;
     a.rope = rope_cache; a.cu = cu_seqlens_q; a.klen = seq_lens; a.key_cu = key_cu; a.out = static_cast<bf16_t *>(out);
     a.heads = num_heads; a.dim = dim; a.rot = rot_dim; a.vdim = v_dim; a.window = window; a.max_position = max_position; a.scale = scale;
     hipStream_t s = static_cast<hipStream_t>(stream);

@@ -65,6 +65,12 @@ template <typename T> __device__ __forceinline__ float tanh_of(float x) {
     }
 }
 
+// ln(1 + x): the hardware's base-2 logarithm of the rounded sum in the bf16 kernels
+template <typename T> __device__ __forceinline__ float log1p_of(float x) {
+    if constexpr (sizeof(T) == 2) return 0.6931471805599453f * __builtin_amdgcn_logf(1.0f + x);
+    else return log1pf(x);
+}
+
 inline bool known_dtype(int32_t dtype) { return dtype == NVA_DTYPE_BF16 || dtype == NVA_DTYPE_F32; }
 inline int elem_bytes(int32_t dtype) { return dtype == NVA_DTYPE_F32 ? 4 : 2; }
 

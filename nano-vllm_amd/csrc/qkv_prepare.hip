@@ -1,5 +1,5 @@
 // What an attention layer does with its projections before it attends: bias, norm of queries and keys (of every head by
-// itself, or over all of a projection's rows at once), rotation, queries out, keys and values into the paged cache.
+// itself, or over all of a projection's rows at once; with a weight or without), norm of every head's values, rotation, queries out, keys and values into the paged cache.
 // One pass over the row; tensors are bf16 or fp32, arithmetic fp32.
 #include "nva_elem.h"
 
@@ -11,7 +11,7 @@ struct QkvArgs {
     const void *x;                  // [n, H * dim | G * dim | G * vdim], row stride in elements (without cache: H * dim)
     int64_t stride;
     const void *bias;               // as many, or null
-    const void *q_norm, *k_norm;    // per head [dim]; whole [H * dim], [G * dim]; null: no norm
+    const void *q_norm, *k_norm;    // per head [dim]; whole [H * dim], [G * dim]; null: no norm, or one without a weight
     const float *rope;              // [max_position, 2 * half]: cos | sin
     void *q_out;                    // [n, H * dim]
     void *k_cache, *v_cache;        // flat [num_slots, G * dim], [num_slots, G * vdim]; null: queries only
@@ -22,6 +22,7 @@ struct QkvArgs {
     int64_t num_slots;
     int32_t n, n_seqs, heads, kv_heads, dim, vdim, half, max_position;
     int32_t whole;                  // norms over whole projections
+    int32_t unit, unit_values;      // norms without weights: of queries and keys, of every head's values
     float eps;
 };
 
@@ -34,7 +35,7 @@ __device__ __forceinline__ int row_position(const QkvArgs &a, int t) {
 // A workgroup per row, 8 elements per lane; a head takes `lanes` lanes (a power of two, dim / 8 of them at work), a thread
 // NP heads' pieces, all kept in registers until the norms are known.
 template <typename T, int NP>
-__global__ __launch_bounds__(256) void qkv_prepare_kernel(QkvArgs a, int32_t log_lanes) {
+__global__ __launch_bounds__(256) void qkv_prepare_kernel(QkvArgs a, int32_t log_lanes, int32_t log_vlanes) {
     __shared__ float sh[2][4];
     const int t = blockIdx.x, tid = threadIdx.x;
     const int pos = row_position(a, t);
@@ -67,8 +68,30 @@ __global__ __launch_bounds__(256) void qkv_prepare_kernel(QkvArgs a, int32_t log
             }
         }
     }
-    // values: a plain copy
-    if (store) {
+    if (store && a.unit_values) {                            // values, head by head
+        const int first = (a.heads + a.kv_heads) * a.dim, vlanes = 1 << log_vlanes, e = (tid & (vlanes - 1)) * 8;
+        for (int h = tid >> log_vlanes; h < a.kv_heads; h += 256 >> log_vlanes) {
+            float y[8], s = 0.f;
+#pragma unroll
+            for (int i = 0; i < 8; ++i) y[i] = 0.f;
+            if (e < a.vdim) {
+                load_f32<T, 8>(x + first + h * a.vdim + e, y);
+                if (bias != nullptr) {
+                    float b[8];
+                    load_f32<T, 8>(bias + first + h * a.vdim + e, b);
+#pragma unroll
+                    for (int i = 0; i < 8; ++i) y[i] += b[i];
+                }
+            }
+#pragma unroll
+            for (int i = 0; i < 8; ++i) s = fmaf(y[i], y[i], s);
+            for (int d = 1; d < vlanes; d <<= 1) s += __shfl_xor(s, d, 64);      // (a head's lanes are here together)
+            const float rstd = rsqrtf(s / static_cast<float>(a.vdim) + a.eps);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) y[i] *= rstd;
+            if (e < a.vdim) store_f32<T, 8>(static_cast<T *>(a.v_cache) + (slot * a.kv_heads + h) * a.vdim + e, y);
+        }
+    } else if (store) {                                      // values: a plain copy
         const int first = (a.heads + a.kv_heads) * a.dim, count = a.kv_heads * a.vdim;
         for (int e = tid * 8; e < count; e += 2048) {
             float y[8];
@@ -112,7 +135,7 @@ __global__ __launch_bounds__(256) void qkv_prepare_kernel(QkvArgs a, int32_t log
         const int h = head0 + p * step;
         const bool is_q = h < a.heads, mine = h < qk_heads && at < a.dim;
         const T *w = static_cast<const T *>(is_q ? a.q_norm : a.k_norm);
-        if (w != nullptr) {
+        if (w != nullptr || a.unit) {
             float rstd = is_q ? rstd_q : rstd_k;
             if (!a.whole) {
                 float s = 0.f;
@@ -121,7 +144,10 @@ __global__ __launch_bounds__(256) void qkv_prepare_kernel(QkvArgs a, int32_t log
                 for (int d = 1; d < lanes; d <<= 1) s += __shfl_xor(s, d, 64);
                 rstd = rsqrtf(s / static_cast<float>(a.dim) + a.eps);
             }
-            if (mine) {
+            if (w == nullptr) {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) v[p][i] *= rstd;
+            } else if (mine) {
                 float g[8];
                 load_f32<T, 8>(w + (a.whole ? (is_q ? h : h - a.heads) * a.dim : 0) + at, g);
 #pragma unroll
@@ -169,7 +195,15 @@ __global__ __launch_bounds__(256) void qkv_prepare_any_kernel(QkvArgs a) {
         if (e < queries) sq_q = fmaf(v, v, sq_q);
         else sq_k = fmaf(v, v, sq_k);
     }
-    if (store)
+    if (store && a.unit_values)
+        for (int h = wave; h < a.kv_heads; h += 4) {
+            float s = 0.f;
+            for (int e = lane; e < a.vdim; e += 64) s = fmaf(value(total + h * a.vdim + e), value(total + h * a.vdim + e), s);
+            const float rstd = rsqrtf(wave_sum(s) / static_cast<float>(a.vdim) + a.eps);
+            for (int e = lane; e < a.vdim; e += 64)
+                static_cast<T *>(a.v_cache)[(slot * a.kv_heads + h) * a.vdim + e] = Elem<T>::from_f32(value(total + h * a.vdim + e) * rstd);
+        }
+    else if (store)
         for (int e = tid; e < a.kv_heads * a.vdim; e += 256)
             static_cast<T *>(a.v_cache)[slot * a.kv_heads * a.vdim + e] = Elem<T>::from_f32(value(total + e));
     sq_q = wave_sum(sq_q);
@@ -194,7 +228,7 @@ __global__ __launch_bounds__(256) void qkv_prepare_any_kernel(QkvArgs a) {
         const bool is_q = h < a.heads;
         const T *w = static_cast<const T *>(is_q ? a.q_norm : a.k_norm);
         const float v = qkv_smem[h * a.dim + e];
-        if (w == nullptr) return v;
+        if (w == nullptr) return a.unit ? v * rstd_of[h] : v;
         return v * (rstd_of[h] * Elem<T>::to_f32(w[(a.whole ? (is_q ? h : h - a.heads) * a.dim : 0) + e]));
     };
     const float *angle = a.half > 0 ? a.rope + static_cast<int64_t>(min(pos, a.max_position - 1)) * (2 * a.half) : nullptr;
@@ -217,18 +251,20 @@ constexpr size_t kMaxLds = 150 * 1024;
 template <typename T>
 static int launch_qkv_prepare(const QkvArgs &a, hipStream_t s) {
     const int qk_heads = a.heads + (a.k_cache ? a.kv_heads : 0);
-    int log_lanes = 0;
+    int log_lanes = 0, log_vlanes = 0;
     while ((8 << log_lanes) < a.dim) ++log_lanes;
+    while ((8 << log_vlanes) < a.vdim) ++log_vlanes;
     const int pieces = log_lanes <= 6 ? ((qk_heads << log_lanes) + 255) / 256 : kMaxPieces + 1;
-    const bool vector = a.dim % 8 == 0 && a.vdim % 8 == 0 && a.half % 8 == 0 && a.stride % 8 == 0 && pieces <= kMaxPieces && aligned16(a.x) &&
+    const bool vector = a.dim % 8 == 0 && a.vdim % 8 == 0 && a.half % 8 == 0 && a.stride % 8 == 0 && pieces <= kMaxPieces &&
+                        (!a.unit_values || log_vlanes <= 6) && aligned16(a.x) &&
                         aligned16(a.bias) && aligned16(a.q_norm) && aligned16(a.k_norm) && aligned16(a.rope) && aligned16(a.q_out) &&
                         aligned16(a.k_cache) && aligned16(a.v_cache);
     const dim3 grid(a.n), block(256);
     if (vector) {
-        if (pieces <= 1) hipLaunchKernelGGL((qkv_prepare_kernel<T, 1>), grid, block, 0, s, a, log_lanes);
-        else if (pieces <= 2) hipLaunchKernelGGL((qkv_prepare_kernel<T, 2>), grid, block, 0, s, a, log_lanes);
-        else if (pieces <= 4) hipLaunchKernelGGL((qkv_prepare_kernel<T, 4>), grid, block, 0, s, a, log_lanes);
-        else hipLaunchKernelGGL((qkv_prepare_kernel<T, kMaxPieces>), grid, block, 0, s, a, log_lanes);
+        if (pieces <= 1) hipLaunchKernelGGL((qkv_prepare_kernel<T, 1>), grid, block, 0, s, a, log_lanes, log_vlanes);
+        else if (pieces <= 2) hipLaunchKernelGGL((qkv_prepare_kernel<T, 2>), grid, block, 0, s, a, log_lanes, log_vlanes);
+        else if (pieces <= 4) hipLaunchKernelGGL((qkv_prepare_kernel<T, 4>), grid, block, 0, s, a, log_lanes, log_vlanes);
+        else hipLaunchKernelGGL((qkv_prepare_kernel<T, kMaxPieces>), grid, block, 0, s, a, log_lanes, log_vlanes);
         return launch_status();
     }
     const size_t lds = (static_cast<size_t>(qk_heads) * a.dim + qk_heads) * sizeof(float);
@@ -243,7 +279,7 @@ static int launch_qkv_prepare(const QkvArgs &a, hipStream_t s) {
 }  // namespace nva
 
 extern "C" int nva_qkv_prepare(const void *x, int64_t x_row_stride, const void *bias, const void *q_norm_weight, const void *k_norm_weight,
-                               int32_t norm_whole, const float *rope_cache, void *q_out, void *k_cache, void *v_cache,
+                               int32_t norms, const float *rope_cache, void *q_out, void *k_cache, void *v_cache,
                                const int32_t *slot_mapping, int64_t num_slots, const int32_t *cu_seqlens_q, const int32_t *seq_lens,
                                const int32_t *token_seq, int32_t n_tokens, int32_t n_seqs, int32_t num_heads, int32_t num_kv_heads,
                                int32_t qk_dim, int32_t v_dim, int32_t rot_dims, int32_t max_position, float eps, int32_t dtype, void *stream) {
@@ -251,7 +287,7 @@ extern "C" int nva_qkv_prepare(const void *x, int64_t x_row_stride, const void *
     if (n_tokens < 0 || n_seqs < 0 || num_heads <= 0 || num_kv_heads <= 0 || qk_dim <= 0 || v_dim <= 0 || num_slots < 0 || rot_dims < 0 ||
         rot_dims % 2 != 0 || rot_dims > qk_dim || (rot_dims > 0 && max_position <= 0))
         return NVA_ERR_BAD_SHAPE;
-    if (!known_dtype(dtype)) return NVA_ERR_UNSUPPORTED_GEOMETRY;
+    if (!known_dtype(dtype) || (norms & ~(NVA_QKV_NORM_WHOLE | NVA_QKV_NORM_UNIT | NVA_QKV_NORM_VALUES)) != 0) return NVA_ERR_UNSUPPORTED_GEOMETRY;
     if (n_tokens == 0) return NVA_OK;
     if (!x || !q_out || !seq_lens || (rot_dims > 0 && !rope_cache) || (k_cache == nullptr) != (v_cache == nullptr) || (k_cache && !slot_mapping))
         return NVA_ERR_NULL_POINTER;
@@ -264,7 +300,8 @@ extern "C" int nva_qkv_prepare(const void *x, int64_t x_row_stride, const void *
     a.x = x; a.stride = x_row_stride; a.bias = bias; a.q_norm = q_norm_weight; a.k_norm = k_norm_weight; a.rope = rope_cache; a.q_out = q_out;
     a.k_cache = k_cache; a.v_cache = v_cache; a.slot_mapping = slot_mapping; a.cu = cu_seqlens_q; a.klen = seq_lens; a.token_seq = token_seq;
     a.num_slots = num_slots; a.n = n_tokens; a.n_seqs = n_seqs; a.heads = num_heads; a.kv_heads = num_kv_heads; a.dim = qk_dim; a.vdim = v_dim;
-    a.half = rot_dims / 2; a.max_position = max_position; a.whole = norm_whole; a.eps = eps;
+    a.half = rot_dims / 2; a.max_position = max_position; a.whole = (norms & NVA_QKV_NORM_WHOLE) != 0; a.unit = (norms & NVA_QKV_NORM_UNIT) != 0;
+    a.unit_values = (norms & NVA_QKV_NORM_VALUES) != 0; a.eps = eps;
     hipStream_t s = static_cast<hipStream_t>(stream);
     return dtype == NVA_DTYPE_BF16 ? launch_qkv_prepare<bf16_t>(a, s) : launch_qkv_prepare<float>(a, s);
 }

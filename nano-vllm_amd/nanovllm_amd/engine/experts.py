@@ -1,5 +1,5 @@
-"""Mixture of experts: a softmax router in fp32 and small gated feed-forwards of which every row uses the best few;
-optionally a shared expert that every row runs, behind a gate of its own.
+"""Mixture of experts: a router in fp32 (softmax or sigmoids) and small gated feed-forwards of which every row uses the best
+few, weighted on their results or on what they read; optionally a shared expert that every row runs, behind a gate of its own.
 
 Nothing depends on the host knowing how many rows an expert has: the router leaves lists of assignments, and the
 products walk them, so a step with experts is captured into a graph like any other."""
@@ -26,6 +26,8 @@ class GateForm:
 
 
 SILU = GateForm()
+SOFTMAX, SIGMOID = "softmax", "sigmoid"       # weights: softmax over the chosen logits; their sigmoids as they are
+_SCORES = {SOFTMAX: _lib.SCORE_SOFTMAX, SIGMOID: _lib.SCORE_SIGMOID}
 JOIN_ROWS = 256                  # rows up to which a shared expert runs in the launches of the routed ones
 
 
@@ -64,6 +66,15 @@ def project(x: torch.Tensor, weight: torch.Tensor, squared_relu: bool = False) -
     return out
 
 
+def project_f32(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """``x @ weight.T`` whose fp32 sums are kept."""
+    if x.dtype == torch.float32:
+        return F.linear(x, weight)
+    if streams(x, weight):
+        return linear_f32(x, weight)
+    return torch.mm(x, weight.t(), out_dtype=torch.float32)
+
+
 @dataclass
 class Assignments:
     choice: torch.Tensor         # int32 [n, top], best first
@@ -73,7 +84,7 @@ class Assignments:
 
 
 def route(h: torch.Tensor, router: torch.Tensor, top: int, scale: float, counts: torch.Tensor, bias: Optional[torch.Tensor] = None,
-          gates: int = 0) -> Assignments:
+          gates: int = 0, score: str = SOFTMAX) -> Assignments:
     """Router of ``h [n, width]``, ``router [experts + gates, width]``; ``counts`` (int32 ``[experts]``) must be zero."""
     n, width = h.shape
     experts = router.shape[0] - gates
@@ -84,15 +95,16 @@ def route(h: torch.Tensor, router: torch.Tensor, top: int, scale: float, counts:
     i32 = lambda *shape: torch.empty(shape, dtype=torch.int32, device=h.device)
     a = Assignments(i32(n, top), torch.empty((n, top + gates), dtype=torch.float32, device=h.device), i32(experts, n), counts)
     rc = _lib.load_shared().nva_router(h.data_ptr(), h.stride(0), router.data_ptr(), _ptr(bias), a.choice.data_ptr(), a.weight.data_ptr(),
-                                       a.lists.data_ptr(), counts.data_ptr(), n, n, width, experts, gates, top, float(scale),
+                                       a.lists.data_ptr(), counts.data_ptr(), n, n, width, experts, gates, top, _SCORES[score], float(scale),
                                        _DTYPE[h.dtype], _stream())
     _lib.check(rc, "nva_router")
     return a
 
 
-def routed_linear(x: torch.Tensor, weight: torch.Tensor, a: Assignments, gate: Optional[GateForm], shared=None):
+def routed_linear(x: torch.Tensor, weight: torch.Tensor, a: Assignments, gate: Optional[GateForm], shared=None, weigh_input: bool = False):
     """One product per assignment, ``[n * top, n_out]``: of row ``p // top`` of ``x [n, k]``, or of row ``p`` of
     ``x [n * top, k]``.  With ``gate`` the weights are (gate | up) and the result has its form.
+    ``weigh_input``: as if every assignment's row were multiplied by its weight first (with ``gate``).
     ``shared = (x [n, k'], weight, limit)``: a product of every row with a weight of its own in the same launch (few rows);
     then both results are returned."""
     experts, rows, k = weight.shape
@@ -103,8 +115,10 @@ def routed_linear(x: torch.Tensor, weight: torch.Tensor, a: Assignments, gate: O
     form = gate or SILU
     args = (x.data_ptr(), x.stride(0), weight.data_ptr(), out.data_ptr(), a.lists.data_ptr(), a.counts.data_ptr(), a.lists.stride(0), n, top,
             experts, n_out, k, int(x.shape[0] == n), int(gate is not None), form.limit, form.slope, form.shift)
+    assert not weigh_input or (gate is not None and shared is None)
     if shared is None:
-        _lib.check(_lib.load_shared().nva_routed_linear(*args, _DTYPE[x.dtype], _stream()), "nva_routed_linear")
+        weigh = (a.weight.data_ptr(), a.weight.stride(0)) if weigh_input else (None, 0)
+        _lib.check(_lib.load_shared().nva_routed_linear(*args, *weigh, _DTYPE[x.dtype], _stream()), "nva_routed_linear")
         return out
     xs, ws, limit = shared
     assert xs.shape == (n, ws.shape[1]) and xs.stride(1) == 1 and ws.is_contiguous() and xs.dtype == ws.dtype == x.dtype == torch.bfloat16
@@ -130,6 +144,8 @@ class ExpertsSpec:
     gate: GateForm = SILU
     bias: bool = False                            # of the router
     shared: Optional[SharedExpertSpec] = None
+    score: str = SOFTMAX
+    weigh_input: bool = False                     # the weights belong to what the experts read
 
 
 class ExpertWeights(nn.Module):
@@ -171,12 +187,13 @@ class Experts:
 
     def __call__(self, h: torch.Tensor):
         """The chosen experts' outputs ``[n * top, width]``, the shared one's ``[n, width]`` (or None), and their weights: ``[n, top]``
-        and, as one more column, the shared expert's."""
+        and, as one more column, the shared expert's.  (With ``weigh_input`` the outputs are only to be added.)"""
         s, w = self.spec, self.weights
-        a = route(h, w.router, s.top, s.scale, self.counters, w.bias, w.router.shape[0] - s.experts)
+        a = route(h, w.router, s.top, s.scale, self.counters, w.bias, w.router.shape[0] - s.experts, s.score)
         if s.shared is None:
-            return routed_linear(routed_linear(h, w.gate_up, a, s.gate), w.down, a, None), None, a.weight
+            return routed_linear(routed_linear(h, w.gate_up, a, s.gate, weigh_input=s.weigh_input), w.down, a, None), None, a.weight
         form = s.shared.gate
+        assert not s.weigh_input
         assert (form.slope, form.shift) == (s.gate.slope, s.gate.shift) and form.shift == 1.0
         if self._joins(h):
             mid, shared = routed_linear(h, w.gate_up, a, s.gate, (h, w.shared_gate_up, form.limit))

@@ -12,6 +12,13 @@ from torch import nn
 from .loader import TensorFolder
 
 
+def load_rows(param: torch.Tensor, first: int, parts) -> None:
+    """Copies tensors into consecutive rows of a fused weight, from row ``first`` on."""
+    for t in parts:
+        param[first: first + t.shape[0]].copy_(t)
+        first += t.shape[0]
+
+
 class LayeredModel(nn.Module):
 
     def __init__(self, cfg, tied: bool = False):

@@ -92,16 +92,24 @@ def post_add_norm(y: torch.Tensor, residual: torch.Tensor, post: Tuple[torch.Ten
     return out
 
 
-def clamped_gate(x: torch.Tensor, limit: float, alpha: float) -> torch.Tensor:
-    """``g sigmoid(alpha g) (u + 1)`` of a fused ``[gate | up]`` projection, g capped and u clamped at ``limit``."""
+def clamped_gate(x: torch.Tensor, limit: float, alpha: float, cubic: float = 0.0, shift: float = 1.0) -> torch.Tensor:
+    """``g sigmoid(alpha (g + cubic g^3)) (u + shift)`` of a fused ``[gate | up]`` projection, g capped and u clamped at ``limit``."""
     assert x.dim() == 2 and x.stride(1) == 1 and x.shape[1] % 2 == 0
     _need_cuda(x)
     inter = x.shape[1] // 2
     out = torch.empty((x.shape[0], inter), dtype=x.dtype, device=x.device)
     rc = _lib.load_shared().nva_clamped_gate(x.data_ptr(), x.stride(0), out.data_ptr(), x.shape[0], inter, float(limit),
-                                      float(alpha), _DTYPE[x.dtype], _stream())
+                                      float(alpha), float(cubic), float(shift), _DTYPE[x.dtype], _stream())
     _lib.check(rc, "nva_clamped_gate")
     return out
+
+
+GELU_SLOPE, GELU_CUBIC = 2.0 * math.sqrt(2.0 / math.pi), 0.044715      # the tanh form: (1 + tanh y) / 2 = sigmoid(2 y)
+
+
+def gelu_gate(x: torch.Tensor) -> torch.Tensor:
+    """``gelu(gate) up`` of a fused ``[gate | up]`` projection, the tanh form of gelu."""
+    return clamped_gate(x, math.inf, GELU_SLOPE, GELU_CUBIC, 0.0)
 
 
 def squared_relu_(x: torch.Tensor) -> torch.Tensor:

@@ -48,6 +48,7 @@ register("Qwen3ForCausalLM", ".config:ModelConfig", ".model:Qwen3ForCausalLM")
 register("Kaparax", ".kaparax:KaparaxConfig", ".kaparax:Kaparax", "mixers")
 register("Pidutar", ".pidutar:PidutarConfig", ".pidutar:Pidutar", "latent")
 register("Sokolorn", ".sokolorn:SokolornConfig", ".sokolorn:Sokolorn", "masked")
+register("Bedenex", ".bedenex:BedenexConfig", ".bedenex:Bedenex", "parallel")
 
 
 def family_of_raw(raw: dict) -> Family:

@@ -242,7 +242,7 @@ def test_norms_and_gate_of_layered_models_validation():
                    (dict(rows=3), _lib.ERR_BAD_SHAPE), (dict(rows_of=A, src=0), _lib.ERR_BAD_SHAPE), (dict(rows=0, src=0), _lib.OK),
                    (dict(dtype=-1), _lib.ERR_UNSUPPORTED_GEOMETRY)):
         assert _with(ok, lib.nva_post_add_norm, **kw) == rc, kw
-    ok = dict(x=A, xs=128, out=A, rows=4, inter=64, limit=1.0, alpha=1.7, dtype=0, stream=None)
+    ok = dict(x=A, xs=128, out=A, rows=4, inter=64, limit=1.0, alpha=1.7, cubic=0.0, shift=1.0, dtype=0, stream=None)
     for kw, rc in ((dict(x=None), _lib.ERR_NULL_POINTER), (dict(xs=127), _lib.ERR_BAD_STRIDE), (dict(inter=0), _lib.ERR_BAD_SHAPE),
                    (dict(rows=-1), _lib.ERR_BAD_SHAPE), (dict(rows=0, x=None), _lib.OK)):
         assert _with(ok, lib.nva_clamped_gate, **kw) == rc, kw
@@ -294,10 +294,23 @@ def test_retention_validation_and_workspace():
 
 def test_branches_and_experts_validation():
     lib = _lib.load()
-    ok = dict(ids=A, table=A, scale=1.0, w1=A, w2=A, off=1.0, res=A, o1=A, o2=A, clear=None, nclear=0, rows=4, width=64, vocab=10, eps=1e-5, dtype=0, stream=None)
+    ok = dict(ids=A, table=A, scale=1.0, w1=A, w2=A, off=1.0, res=A, o1=A, o1s=64, o2=A, copy=A, cs=128, clear=None, nclear=0, rows=4, width=64, vocab=10, eps=1e-5, dtype=0, stream=None)
     for kw, rc in ((dict(ids=None), _lib.ERR_NULL_POINTER), (dict(o2=None), _lib.ERR_NULL_POINTER), (dict(width=0), _lib.ERR_BAD_SHAPE),
-                   (dict(nclear=-1), _lib.ERR_BAD_SHAPE), (dict(dtype=2), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, ids=None), _lib.OK)):
+                   (dict(nclear=-1), _lib.ERR_BAD_SHAPE), (dict(o1s=63), _lib.ERR_BAD_STRIDE), (dict(cs=63), _lib.ERR_BAD_STRIDE),
+                   (dict(dtype=2), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, ids=None), _lib.OK)):
         assert _with(ok, lib.nva_embed_rms_norms, **kw) == rc, kw
+    ok = dict(y1=A, ys=64, y2=A, terms=2, gate=A, gs=128, gb=A, res=A, w=A, off=0.0, out=A, os=64, rows_of=None, clear=None, nclear=0, rows=4, src=4, width=64,
+              eps=1e-5, dtype=0, stream=None)
+    for kw, rc in ((dict(y1=None), _lib.ERR_NULL_POINTER), (dict(gate=None), _lib.ERR_NULL_POINTER), (dict(gb=None), _lib.ERR_NULL_POINTER),
+                   (dict(out=None), _lib.ERR_NULL_POINTER), (dict(ys=63), _lib.ERR_BAD_STRIDE), (dict(gs=127), _lib.ERR_BAD_STRIDE),
+                   (dict(y2=None, gs=63), _lib.ERR_BAD_STRIDE), (dict(os=63), _lib.ERR_BAD_STRIDE), (dict(terms=0), _lib.ERR_BAD_SHAPE),
+                   (dict(rows=3), _lib.ERR_BAD_SHAPE), (dict(rows_of=A, src=0), _lib.ERR_BAD_SHAPE), (dict(dtype=2), _lib.ERR_UNSUPPORTED_GEOMETRY),
+                   (dict(rows=0, src=0), _lib.OK)):
+        assert _with(ok, lib.nva_gated_rms_norm, **kw) == rc, kw
+    ok = dict(p=A, step=A, res=A, w=A, off=0.0, out=A, clear=None, nclear=0, rows=4, width=64, eps=1e-5, dtype=0, stream=None)
+    for kw, rc in ((dict(p=None), _lib.ERR_NULL_POINTER), (dict(step=None), _lib.ERR_NULL_POINTER), (dict(w=None), _lib.ERR_NULL_POINTER),
+                   (dict(width=0), _lib.ERR_BAD_SHAPE), (dict(dtype=2), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, p=None), _lib.OK)):
+        assert _with(ok, lib.nva_entry_rms_norm, **kw) == rc, kw
     ok = dict(y1=A, ys=64, g1=A, y2=A, tw=A, terms=2, g2=A, mult=1.0, res=A, w1=A, w2=A, off=1.0, o1=A, o2=A, rows_of=None, clear=None, nclear=0,
               rows=4, src=4, width=64, eps=1e-5, dtype=1, stream=None)
     for kw, rc in ((dict(res=None), _lib.ERR_NULL_POINTER), (dict(w1=None), _lib.ERR_NULL_POINTER), (dict(o2=None), _lib.ERR_NULL_POINTER),
@@ -309,18 +322,18 @@ def test_branches_and_experts_validation():
                    (dict(og=63), _lib.ERR_BAD_STRIDE), (dict(k=0), _lib.ERR_BAD_SHAPE), (dict(groups=70000), _lib.ERR_BAD_SHAPE),
                    (dict(dtype=1, odt=0), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, x=None), _lib.OK), (dict(groups=0, x=None), _lib.OK)):
         assert _with(ok, lib.nva_grouped_linear, **kw) == rc, kw
-    ok = dict(x=A, xs=64, w=A, b=None, choice=A, cw=A, lists=A, counts=A, ls=16, rows=16, width=64, experts=8, gates=0, top=2, scale=1.0, dtype=0, stream=None)
+    ok = dict(x=A, xs=64, w=A, b=None, choice=A, cw=A, lists=A, counts=A, ls=16, rows=16, width=64, experts=8, gates=0, top=2, score=1, scale=1.0, dtype=0, stream=None)
     for kw, rc in ((dict(counts=None), _lib.ERR_NULL_POINTER), (dict(cw=None), _lib.ERR_NULL_POINTER), (dict(top=9), _lib.ERR_BAD_SHAPE),
                    (dict(ls=15), _lib.ERR_BAD_SHAPE), (dict(xs=63), _lib.ERR_BAD_STRIDE), (dict(experts=1025), _lib.ERR_UNSUPPORTED_GEOMETRY),
                    (dict(experts=512, top=129), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(gates=-1), _lib.ERR_BAD_SHAPE),
-                   (dict(gates=65), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, x=None), _lib.OK)):
+                   (dict(gates=65), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(score=2), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, x=None), _lib.OK)):
         assert _with(ok, lib.nva_router, **kw) == rc, kw
-    ok = dict(x=A, xs=64, w=A, out=A, lists=A, counts=A, ls=16, rows=16, terms=2, experts=8, n_out=32, k=64, per_row=1, gated=1, limit=1.0, slope=1.7, shift=1.0, dtype=0, stream=None)
+    ok = dict(x=A, xs=64, w=A, out=A, lists=A, counts=A, ls=16, rows=16, terms=2, experts=8, n_out=32, k=64, per_row=1, gated=1, limit=1.0, slope=1.7, shift=1.0, iw=A, iws=2, dtype=0, stream=None)
     for kw, rc in ((dict(lists=None), _lib.ERR_NULL_POINTER), (dict(out=None), _lib.ERR_NULL_POINTER), (dict(terms=9), _lib.ERR_BAD_SHAPE),
                    (dict(ls=15), _lib.ERR_BAD_SHAPE), (dict(xs=63), _lib.ERR_BAD_STRIDE), (dict(dtype=5), _lib.ERR_UNSUPPORTED_GEOMETRY),
-                   (dict(rows=0, x=None), _lib.OK)):
+                   (dict(iws=1), _lib.ERR_BAD_STRIDE), (dict(gated=0), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rows=0, x=None), _lib.OK)):
         assert _with(ok, lib.nva_routed_linear, **kw) == rc, kw
-    del ok["dtype"], ok["stream"]
+    del ok["dtype"], ok["stream"], ok["iw"], ok["iws"]
     ok.update(sx=A, sxs=64, sw=A, so=A, sn=24, sk=64, sl=1.0, stream=None)
     for kw, rc in ((dict(lists=None), _lib.ERR_NULL_POINTER), (dict(so=None), _lib.ERR_NULL_POINTER), (dict(terms=9), _lib.ERR_BAD_SHAPE),
                    (dict(sn=0), _lib.ERR_BAD_SHAPE), (dict(sxs=63), _lib.ERR_BAD_STRIDE), (dict(sk=60), _lib.ERR_UNSUPPORTED_GEOMETRY),
@@ -337,17 +350,18 @@ def test_post_norm_prepare_and_masks_validation():
                    (dict(terms=0), _lib.ERR_BAD_SHAPE), (dict(rows=3), _lib.ERR_BAD_SHAPE), (dict(dtype=2), _lib.ERR_UNSUPPORTED_GEOMETRY),
                    (dict(rows=0, src=0), _lib.OK)):
         assert _with(ok, lib.nva_post_rms_norms, **kw) == rc, kw
-    ok = dict(x=A, xs=256, b=A, qn=A, kn=A, whole=1, rope=A, q=A, kc=A, vc=A, sm=A, slots=512, cu=A, lens=A, tseq=A, n=9, seqs=2, heads=4, kv=2, dim=32,
+    ok = dict(x=A, xs=256, b=A, qn=A, kn=A, norms=5, rope=A, q=A, kc=A, vc=A, sm=A, slots=512, cu=A, lens=A, tseq=A, n=9, seqs=2, heads=4, kv=2, dim=32,
               vdim=32, rot=16, maxp=64, eps=1e-5, dtype=0, stream=None)
     for kw, rc in ((dict(x=None), _lib.ERR_NULL_POINTER), (dict(vc=None), _lib.ERR_NULL_POINTER), (dict(sm=None), _lib.ERR_NULL_POINTER),
                    (dict(rope=None), _lib.ERR_NULL_POINTER), (dict(tseq=None), _lib.ERR_NULL_POINTER), (dict(xs=255), _lib.ERR_BAD_STRIDE),
                    (dict(rot=15), _lib.ERR_BAD_SHAPE), (dict(rot=34), _lib.ERR_BAD_SHAPE), (dict(maxp=0), _lib.ERR_BAD_SHAPE), (dict(cu=None), _lib.ERR_BAD_SHAPE),
                    (dict(dtype=7), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(heads=5000, kv=1, dim=9, vdim=9, rot=0, xs=1 << 20), _lib.ERR_UNSUPPORTED_GEOMETRY),
-                   (dict(n=0, x=None), _lib.OK)):
+                   (dict(norms=8), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(n=0, x=None), _lib.OK)):
         assert _with(ok, lib.nva_qkv_prepare, **kw) == rc, kw
     ok = dict(q=A, qs=2048, kc=A, vc=A, bt=A, bts=16, mb=16, cu=None, lens=A, tseq=None, out=A, ws=A, wsb=1 << 30, n=8, seqs=8, mq=1, heads=16, kv=8,
-              dim=128, vdim=128, bs=256, nb=64, mask=1, span=8192, scale=0.1, cap=0.0, sinks=A, gate=A, gs=16, dtype=0, stream=None)
+              dim=128, vdim=128, bs=256, nb=64, mask=1, span=8192, scale=0.1, cap=0.0, sinks=A, slope=A, rate=A, gate=A, gs=16, dtype=0, stream=None)
     for kw, rc in ((dict(q=None), _lib.ERR_NULL_POINTER), (dict(ws=None), _lib.ERR_NULL_POINTER), (dict(mask=2), _lib.ERR_UNSUPPORTED_GEOMETRY),
+                   (dict(slope=None), _lib.ERR_NULL_POINTER), (dict(rate=None), _lib.ERR_NULL_POINTER), (dict(cap=1.0), _lib.ERR_UNSUPPORTED_GEOMETRY),
                    (dict(gs=15), _lib.ERR_BAD_STRIDE), (dict(span=0), _lib.ERR_BAD_SHAPE), (dict(wsb=100), _lib.ERR_WORKSPACE_TOO_SMALL),
                    (dict(n=0, q=None), _lib.OK)):
         assert _with(ok, lib.nva_masked_attn, **kw) == rc, kw
@@ -366,6 +380,7 @@ def test_symbols_of_several_libraries_come_from_one_that_is_there(monkeypatch):
     monkeypatch.setattr(_lib, "MIXERS_LIB_PATH", "/nonexistent/libnanovllm_mixers.so")
     fresh = _lib._Symbols()
     assert fresh.nva_chunk_attn_workspace_bytes(0, 16, 8, 128, 16, 256, 100) == 0 and fresh.nva_router is not None
+    assert fresh.nva_latent_prefill_supported(128, 64, 128, 0) == 1
     with pytest.raises(_lib.HipLibraryMissing, match="no CPU fallback"):
         fresh.nva_mlstm
     with pytest.raises(_lib.HipLibraryMissing, match="no CPU fallback"):
@@ -378,14 +393,15 @@ def test_latent_attention_validation_and_workspace():
               eps=1e-5, dtype=0, stream=None)
     for kw, rc in ((dict(x=None), _lib.ERR_NULL_POINTER), (dict(wkv=None), _lib.ERR_NULL_POINTER), (dict(rope=None), _lib.ERR_NULL_POINTER),
                    (dict(tseq=None), _lib.ERR_NULL_POINTER), (dict(cu=None), _lib.ERR_BAD_SHAPE), (dict(xs=255), _lib.ERR_BAD_STRIDE),
-                   (dict(rot=31), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rank=0), _lib.ERR_BAD_SHAPE), (dict(n=0, x=None), _lib.OK)):
+                   (dict(rot=31), _lib.ERR_UNSUPPORTED_GEOMETRY), (dict(rank=0), _lib.ERR_BAD_SHAPE), (dict(q_rank=-1), _lib.ERR_BAD_SHAPE),
+                   (dict(q=None), _lib.ERR_NULL_POINTER), (dict(n=0, x=None), _lib.OK)):
         assert _with(ok, lib.nva_latent_prepare, **kw) == rc, kw
     ws = lib.nva_latent_attn_workspace_bytes
     assert ws(2000, 16, 512, 64, 16, 256, 4096, 0) == 0               # enough rows for the machine: one range of keys each
     assert ws(1, 16, 512, 64, 16, 256, 1 << 20, 0) == 33 * 16 * 516 * 4   # 4096 keys and up to 63 before a multiple of 64, ranges of 128
     assert ws(40, 16, 512, 64, 16, 256, 1 << 20, 0) == 40 * 17 * 16 * 516 * 4
     assert ws(1, 16, 512, 64, 16, 256, 60, 0) == 0 and ws(1, 16, 512, 64, 16, 256, 4096, 1) == 0 and ws(1, 16, 516, 64, 16, 256, 4096, 0) == 0
-    ok = dict(ql=A, qr=A, qrs=3072, qrh=192, gate=A, gs=16, rope=A, cache=A, bt=A, bts=16, mb=16, cu=None, lens=A, tseq=None, out=A, ws=A, wsb=1 << 30,
+    ok = dict(ql=A, qr=A, qrs=3072, qrh=192, gate=A, gs=16, sinks=A, rope=A, cache=A, bt=A, bts=16, mb=16, cu=None, lens=A, tseq=None, out=A, ws=A, wsb=1 << 30,
               n=8, seqs=8, heads=16, rank=512, rot=64, bs=256, nb=64, window=4096, max_pos=4096, scale=0.1, dtype=0, stream=None)
     for kw, rc in ((dict(ql=None), _lib.ERR_NULL_POINTER), (dict(qr=None), _lib.ERR_NULL_POINTER), (dict(ws=None), _lib.ERR_NULL_POINTER),
                    (dict(ws=A + 8), _lib.ERR_MISALIGNED), (dict(wsb=100), _lib.ERR_WORKSPACE_TOO_SMALL), (dict(window=0), _lib.ERR_BAD_SHAPE),
@@ -399,7 +415,7 @@ def test_latent_attention_validation_and_workspace():
         assert _with(ok, lib.nva_latent_gather, **kw) == rc, kw
     fits = lib.nva_latent_prefill_supported
     assert fits(128, 64, 128, 0) == 1 and fits(128, 64, 128, 1) == 0 and fits(100, 64, 128, 0) == 0 and fits(264, 64, 128, 0) == 0 and fits(8, 136, 8, 0) == 0
-    ok = dict(q=A, qs=3072, kv=A, kvs=4096, kr=A, krs=576, gate=A, gs=16, rope=A, cu=A, lens=A, kcu=A, out=A, n=9, seqs=2, mq=7, heads=16, dim=128, rot=64,
+    ok = dict(q=A, qs=3072, kv=A, kvs=4096, kr=A, krs=576, gate=A, gs=16, sinks=A, rope=A, cu=A, lens=A, kcu=A, out=A, n=9, seqs=2, mq=7, heads=16, dim=128, rot=64,
               vdim=128, window=100, max_pos=4096, scale=0.1, dtype=0, stream=None)
     for kw, rc in ((dict(q=None), _lib.ERR_NULL_POINTER), (dict(kr=None), _lib.ERR_NULL_POINTER), (dict(kcu=None), _lib.ERR_NULL_POINTER),
                    (dict(kvs=4088), _lib.ERR_BAD_STRIDE), (dict(qs=3076), _lib.ERR_BAD_STRIDE), (dict(kv=A + 2), _lib.ERR_MISALIGNED),

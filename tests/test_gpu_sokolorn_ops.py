@@ -171,7 +171,7 @@ def test_bias_norms_rotation_and_cache_write(dev, dtype, shape, kind):
         kc = torch.full((batch.num_blocks, BLOCK, kv, dim), 7.0, dtype=dtype, device=dev)
         vc = torch.full((batch.num_blocks, BLOCK, kv, vdim), 7.0, dtype=dtype, device=dev)
         q = torch.full((x.shape[0], queries), 9.0, dtype=dtype, device=dev)
-        masked.qkv_prepare(x, on(bias), on(wq), on(wk), whole, rope, q, kc, vc, batch.group, heads, kv, dim, vdim, 1e-5)
+        masked.qkv_prepare(x, on(bias), on(wq), on(wk), masked.WHOLE if whole else masked.HEAD, rope, q, kc, vc, batch.group, heads, kv, dim, vdim, 1e-5)
 
         def normed(t, w):
             if w is None:
@@ -195,7 +195,7 @@ def test_bias_norms_rotation_and_cache_write(dev, dtype, shape, kind):
         untouched[slots[slots >= 0]] = False
         assert bool((kc.view(-1, keys).cpu()[untouched] == 7).all()) and bool((vc.view(-1, kv * vdim).cpu()[untouched] == 7).all())
         again = torch.full_like(q, 9.0)                       # a layer that reads another one's keys: queries only
-        masked.qkv_prepare(wide(batch.rows(full)[:, :queries]), on(None if bias is None else bias[:queries]), on(wq), None, whole, rope, again, None, None,
+        masked.qkv_prepare(wide(batch.rows(full)[:, :queries]), on(None if bias is None else bias[:queries]), on(wq), None, masked.WHOLE if whole else masked.HEAD, rope, again, None, None,
                            batch.group, heads, kv, dim, vdim, 1e-5)
         close(again, q, tol(dtype, 8e-3, 1e-6), "queries alone")
 
@@ -315,7 +315,7 @@ def test_chunks_with_sinks_gates_and_caps(dev):
             rc = _lib.load_masked().nva_masked_attn(
                 qs.data_ptr(), qs.stride(0), kc.data_ptr(), vc.data_ptr(), grp.block_tables.data_ptr(), grp.block_tables.stride(0), grp.block_tables.shape[1],
                 ptr(grp.cu), grp.seq_lens.data_ptr(), ptr(grp.token_seq), out.data_ptr(), None, 0, grp.count, grp.num_seqs, grp.max_q, heads, kv, dim, dim,
-                BLOCK, batch.num_blocks, 0, chunk, 0.3, cap, sk.data_ptr(), gs.data_ptr(), heads, _lib.DTYPE_BF16 if dtype is BF16 else _lib.DTYPE_F32,
+                BLOCK, batch.num_blocks, 0, chunk, 0.3, cap, sk.data_ptr(), None, None, gs.data_ptr(), heads, _lib.DTYPE_BF16 if dtype is BF16 else _lib.DTYPE_F32,
                 torch.cuda.current_stream().cuda_stream)
             _lib.check(rc, "nva_masked_attn")
             want = []

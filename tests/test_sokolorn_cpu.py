@@ -127,7 +127,7 @@ def test_weights_land_where_they_belong(tmp_path):
     assert torch.equal(moe.gate_up[4], torch.cat([f["l0.mlp.e4.gate"], f["l0.mlp.e4.up"]])) and torch.equal(moe.down[2], f["l0.mlp.e2.down"])
     assert torch.equal(moe.shared_gate_up, torch.cat([f["l0.mlp.shared.gate"], f["l0.mlp.shared.up"]])) and torch.equal(moe.shared_down, f["l0.mlp.shared.down"])
     assert m.layer_weights[3].mlp.router.shape[0] == 5 and m.layer_weights[3].mlp.shared_down is None and m.layer_weights[2].norm2 is None
-    assert m.layers[3].mixer.source is m.layers[1].mixer and m.layers[6].mixer.source is m.layers[1].mixer and m.layers[1].mixer.window == ALL_KEYS
+    assert m.layers[3].mixer.source is m.layers[1].mixer and m.layers[6].mixer.source is m.layers[1].mixer and m.layers[1].mixer.span == ALL_KEYS
     del w["l3.norm1"]
     with pytest.raises(KeyError, match="l3.norm1"):
         m.load_weights(cases.write_model(tmp_path / "b", raw, w))
