@@ -73,6 +73,15 @@ def latent_attention(h: torch.Tensor, w, m: dict, eps: float) -> torch.Tensor:
     return out.reshape(t, -1) @ w("o").T
 
 
+def head_norm(x: torch.Tensor, eps: float) -> torch.Tensor:
+    """Queries and keys, every head by itself."""
+    return unit_rms(x, eps)
+
+
+def value_norm(v: torch.Tensor, eps: float) -> torch.Tensor:
+    return unit_rms(v, eps)
+
+
 def head_gates(h: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     return torch.sigmoid(h @ w.T)
 
@@ -81,8 +90,8 @@ def biased_attention(h: torch.Tensor, w, m: dict, eps: float) -> torch.Tensor:
     """Queries, keys and values of unit root mean square, a bias that grows with the logarithm of the distance, chunks,
     a gate per head."""
     t, heads, groups = h.shape[0], m["heads"], m["kv_heads"]
-    q = unit_rms((h @ w("q").T).view(t, heads, m["dim"]), eps)
-    k = unit_rms((h @ w("k").T).view(t, groups, m["dim"]), eps)
+    q = head_norm((h @ w("q").T).view(t, heads, m["dim"]), eps)
+    k = head_norm((h @ w("k").T).view(t, groups, m["dim"]), eps)
     v = value_norm((h @ w("v").T).view(t, groups, m["vdim"]), eps)
     out = torch.zeros(t, heads, m["vdim"], dtype=h.dtype)
     for n in range(heads):
@@ -90,10 +99,6 @@ def biased_attention(h: torch.Tensor, w, m: dict, eps: float) -> torch.Tensor:
         s = q[:, n] @ k[:, g].T * m["scale"] - distance_bias(t, w("r1")[n], w("r2")[n])
         out[:, n] = torch.softmax(s.masked_fill(~in_chunk(t, m["mask"]["size"]), -math.inf), -1) @ v[:, g]
     return (out * head_gates(h, w("g"))[..., None]).reshape(t, -1) @ w("o").T
-
-
-def value_norm(v: torch.Tensor, eps: float) -> torch.Tensor:
-    return unit_rms(v, eps)
 
 
 def gelu(z: torch.Tensor) -> torch.Tensor:
