@@ -1422,6 +1422,208 @@ def sokolorn_kernels(dev, steps=60, only=None):
     return rows
 
 
+def _bedenex_config(layers, loop, width, heads, kv_heads, kv_rank, dense_ff, experts, top, ff, chunk, vocab):
+    """Chunked and latent attention in turn (heads of 128; 128 + 64 key elements over latents), beside a dense feed-forward and
+    routed experts in turn; ``loop`` (start, stop, times) of the layers runs again."""
+    from nanovllm_amd.engine.bedenex import BedenexConfig
+    out = []
+    for i in range(layers):
+        mlp = dict(kind="dense", ff=dense_ff) if i // 2 % 2 == 0 else dict(kind="moe", expert=dict(ff=ff), router=dict(experts=experts, top=top))
+        if i % 2 == 0:
+            out.append(dict(type="attention", mixer=dict(heads=heads, kv_heads=kv_heads, dim=128, vdim=128, mask=dict(size=chunk), scale=128 ** -0.5), mlp=mlp))
+        else:
+            out.append(dict(type="latent_attention", mixer=dict(heads=heads, dim=128, rot_dim=64, vdim=128, kv_rank=kv_rank, scale=192 ** -0.5,
+                                                                rot=dict(base=1e4, dims=64)), mlp=mlp))
+    return BedenexConfig.from_raw(dict(architecture="Bedenex", vocab=vocab, width=width, norm=dict(eps=1e-6), layers=out,
+                                       loop=dict(zip(("start", "stop", "times"), loop))))
+
+
+def bedenex_kernels(dev, steps=60, only=None):
+    """Every kernel of the Bedenex layers at sizes of a real layer (width 1024; 16 / 8 heads of 128; 16 heads of 128 + 64 / 128 over
+    latents of 512; dense feed-forward of 3072; 4 of 32 experts of 768), each beside the like kernel of the closest model at equal
+    size -- Kaparax's attention in chunks, gate and norms, Pidutar's latent attention, experts and residual step, Sokolorn's
+    preparation -- in one process."""
+    import torch
+    import torch.nn.functional as F
+    from nanovllm_amd import synthetic
+    from nanovllm_amd.context import RowGroup
+    from nanovllm_amd.engine import branches, experts, latent, masked, mixers
+    bf = torch.bfloat16
+    rnd = lambda *shape: torch.randn(*shape, device=dev).to(bf)
+    i32 = lambda x: torch.as_tensor(x, dtype=torch.int32).to(dev)
+    rows = []
+    want = lambda name: only is None or only in name
+    heads, kv, d, rot, rank, width, dense_ff = 16, 8, 128, 64, 512, 1024, 3072
+    n_exp, top, ff = 32, 4, 768
+    rope = mixers.RopeTables(16384 + 256, dev).get(mixers.Rotary(1e4, rot))
+    graph_us = lambda fns, n=200: _graph_time_ms(fns, n, 10)[0] / n * 1e3
+    event_us = lambda fns, n=steps: _steady_time_ms(fns, n, max(3, n // 10))[0] / n * 1e3
+    sinks, bias = torch.randn(heads, device=dev), (torch.rand(heads, device=dev) + 0.5, torch.rand(heads, device=dev))
+
+    def lengths(count, lo, hi, seed=0):
+        return torch.randint(lo, hi + 1, (count,), generator=torch.Generator().manual_seed(seed)).tolist()
+
+    def unit(x, e):                                           # heads of unit root mean square, as the layers attend with
+        return (x.float().unflatten(-1, (-1, e)) / x.float().unflatten(-1, (-1, e)).pow(2).mean(-1, keepdim=True).sqrt()).flatten(-2).to(bf).view(x.shape)
+
+    def singles(batch, lo, hi):
+        g = torch.Generator().manual_seed(1)
+        lens = torch.randint(lo, hi + 1, (batch,), generator=g)
+        blocks = int(((lens + 255) // 256).sum())
+        tabs = synthetic.decode_tables(lens.tolist(), blocks, g).to(dev)
+        return RowGroup(0, batch, batch, i32(lens), i32([0] * batch), tabs, i32([0] * batch)), lens, blocks
+
+    # ---- attention over portions
+    for what, lens, chunk, form in (("2x16384, one chunk", [16384, 16384], 16384, (16, 8, 128)), ("2x16384, chunks of 2048", [16384, 16384], 2048, (16, 8, 128)),
+                                    ("2x16384, chunks of 128", [16384, 16384], 128, (16, 8, 128)), ("16 x U[100,1024], one chunk", lengths(16, 100, 1024), 16384, (16, 8, 128)),
+                                    ("2x16384, chunks of 1024, 16 heads of 64", [16384, 16384], 1024, (16, 16, 64)),
+                                    ("2x16384, chunks of 1024, 16 / 8 heads of 96", [16384, 16384], 1024, (16, 8, 96))):
+        if not want("chunked attention prefill"):
+            continue
+        h, g, e = form
+        group, blocks = _portions(dev, lens)
+        n = sum(lens)
+        q, out, gate = unit(rnd(n, h * e), e), torch.empty(n, h * e, dtype=bf, device=dev), rnd(n, h)
+        kc, vc = unit(rnd(blocks, 256, g, e), e), rnd(blocks, 256, g, e)
+        b = (bias[0][:h], bias[1][:h])
+        mine = event_us([lambda: masked.masked_attention(q, kc, vc, group, out, h, chunk, e ** -0.5, None, gate, chunks=True, bias=b)])
+        theirs = event_us([lambda: mixers.chunk_attention(q, kc, vc, group, out, h, chunk, e ** -0.5, 30.0)])
+        parts = min(chunk, max(lens))
+        seen = sum((l // parts) * (parts * (parts + 1) // 2) + (l % parts) * (l % parts + 1) // 2 for l in lens)
+        rows.append(_kernel_row("chunked attention prefill, " + what, mine, 4 * e * h * seen, "mfma", ("chunk attention, capped", theirs, 4 * e * h * seen, "mfma")))
+        del q, out, kc, vc
+    for what, lens in (("2x16384", [16384, 16384]), ("16 x U[100,1024]", lengths(16, 100, 1024))):
+        if not want("latent attention prefill"):
+            continue
+        group, blocks = _portions(dev, lens)
+        n = sum(lens)
+        x, kvs, keys, gate = rnd(n, heads * (d + rot) + rank + rot + 2 * width), rnd(n, heads * 2 * d), rnd(n, rank + rot), rnd(n, heads)
+        q, out = x[:, : heads * (d + rot)], torch.empty(n, heads * d, dtype=bf, device=dev)
+        qd = q.contiguous()
+        mine = event_us([lambda: latent.latent_prefill(q, kvs, keys[:, rank:], None, rope, group, group.cu, out, d, d, 1 << 30, 192 ** -0.5, sinks)])
+        theirs = event_us([lambda: latent.latent_prefill(qd, kvs, keys[:, rank:], gate, rope, group, group.cu, out, d, d, 16384, 192 ** -0.5)])
+        alg = 2 * heads * sum(l * (l + 1) // 2 for l in lens) * (2 * d + rot)
+        rows.append(_kernel_row("latent attention prefill, " + what, mine, alg, "mfma", ("Pidutar's", theirs, alg, "mfma")))
+        del x, kvs, keys, q, qd, out
+
+    # ---- attention of single tokens
+    for what, batch, ctx, chunk, pools in (("batch 64, ctx U[100,2048]", 64, (100, 2048), 16384, 4), ("batch 256, ctx U[300,1326]", 256, (300, 1326), 16384, 2),
+                                           ("batch 16, ctx U[4096,8192]", 16, (4096, 8192), 16384, 4), ("batch 64, ctx 8192, chunks of 1024", 64, (8192, 8192), 1024, 2),
+                                           ("batch 64, ctx 2000, chunks of 128", 64, (2000, 2000), 128, 4), ("batch 1, ctx 8192", 1, (8192, 8192), 16384, 4)):
+        if not want("chunked attention decode"):
+            continue
+        group, lens, blocks = singles(batch, *ctx)
+        q, out, gate = unit(rnd(batch, heads * d), d), torch.empty(batch, heads * d, dtype=bf, device=dev), rnd(batch, heads)
+        caches = [(unit(rnd(blocks, 256, kv, d), d), rnd(blocks, 256, kv, d)) for _ in range(pools)]
+        mine = graph_us([lambda c=c: masked.masked_attention(q, c[0], c[1], group, out, heads, chunk, d ** -0.5, None, gate, chunks=True, bias=bias) for c in caches], 56)
+        theirs = graph_us([lambda c=c: mixers.chunk_attention(q, c[0], c[1], group, out, heads, chunk, d ** -0.5, 30.0) for c in caches], 56)
+        alg = int(((lens - 1) % chunk + 1).sum()) * kv * d * 4 + 4 * q.numel()
+        rows.append(_kernel_row("chunked attention decode, " + what, mine, alg, "hbm", ("chunk attention, capped", theirs, alg, "hbm")))
+        del caches
+    for what, batch, ctx, pools in (("batch 64, ctx U[100,2048]", 64, (100, 2048), 4), ("batch 256, ctx U[300,1326]", 256, (300, 1326), 3),
+                                    ("batch 16, ctx U[4096,8192]", 16, (4096, 8192), 4), ("batch 1, ctx 8192", 1, (8192, 8192), 8)):
+        if not want("latent attention decode"):
+            continue
+        group, lens, blocks = singles(batch, *ctx)
+        met, x, gate, out = rnd(batch, heads, rank), rnd(batch, heads * (d + rot) + rank + rot + 2 * width), rnd(batch, heads), torch.empty(batch, heads, rank, dtype=bf, device=dev)
+        qr = x[:, : heads * (d + rot)].unflatten(1, (heads, d + rot))[..., d:]
+        caches = [rnd(blocks, 256, rank + rot) for _ in range(pools)]
+        mine = graph_us([lambda c=c: latent.latent_attention(met, qr, None, rope, c, group, out, 1 << 30, 192 ** -0.5, sinks) for c in caches], 56)
+        theirs = graph_us([lambda c=c: latent.latent_attention(met, qr, gate, rope, c, group, out, 8192, 192 ** -0.5) for c in caches], 56)
+        alg = int(lens.sum()) * (rank + rot) * 2 + 4 * met.numel()
+        rows.append(_kernel_row("latent attention decode, " + what, mine, alg, "hbm", ("Pidutar's", theirs, alg, "hbm")))
+        del caches
+
+    # ---- what attention reads
+    for n in (16, 256, 16384):
+        group = _portions(dev, [1024] * 16)[0] if n >= 16384 else RowGroup(0, n, n, i32([701] * n), i32(torch.randperm(n)), None, i32(list(range(n))))
+        beside = 2 * width + 2 * dense_ff                     # columns of the same product that others read
+        if want("prepare"):
+            ch = (heads + 2 * kv) * d
+            x, xs, q = rnd(n, ch + heads + beside), rnd(n, ch + heads), torch.empty(n, heads * d, dtype=bf, device=dev)
+            kc, vc = (torch.empty(max(1, n // 256), 256, kv, d, dtype=bf, device=dev) for _ in range(2))
+            wq, wk = rnd(heads * d), rnd(kv * d)
+            mine = graph_us([lambda: masked.qkv_prepare(x, None, None, None, masked.UNIT, None, q, kc, vc, group, heads, kv, d, d, 1e-6, True)])
+            theirs = graph_us([lambda: masked.qkv_prepare(xs, None, wq, wk, masked.WHOLE, None, q, kc, vc, group, heads, kv, d, d, 1e-6)])
+            rows.append(_kernel_row("prepare: norms of q, k and v, cache, %d rows" % n, mine, n * ch * 4, "hbm", ("Sokolorn's, whole norms", theirs, n * ch * 4, "hbm")))
+            x, xs, qo = rnd(n, heads * (d + rot) + rank + rot + beside), rnd(n, 512 + rank + rot + heads), torch.empty(n, 512, dtype=bf, device=dev)
+            wkv, cache = rnd(rank), torch.empty(max(1, n // 256), 256, rank + rot, dtype=bf, device=dev)
+            mine = graph_us([lambda: latent.latent_prepare(x[:, heads * (d + rot):], None, wkv, rope, None, cache, group, rot, 1e-6)])
+            theirs = graph_us([lambda: latent.latent_prepare(xs, wkv, wkv, rope, qo, cache, group, rot, 1e-6)])
+            rows.append(_kernel_row("prepare: latent, rotation, cache, %d rows" % n, mine, n * (rank + rot) * 4 + n * rot * 4, "hbm",
+                                    ("Pidutar's, query latents too", theirs, n * (512 + rank + rot) * 4 + n * rot * 4, "hbm")))
+        if want("one product"):
+            cols = [(heads + 2 * kv) * d + 16, 2 * width, 2 * dense_ff]
+            h, ws = rnd(n, width), [[rnd(c, width) for c in cols] for _ in range(6 if n < 16384 else 1)]
+            wf = [torch.cat(w) for w in ws]
+            time = graph_us if n < 16384 else event_us
+            mine, theirs = time([lambda w=w: experts.project(h, w) for w in wf]), time([lambda w=w: [experts.project(h, x) for x in w] for w in ws])
+            alg = (2 * n * width * sum(cols), "mfma") if n >= 512 else (2 * (sum(cols) * width + n * (width + sum(cols))), "hbm")
+            rows.append(_kernel_row("one product for mixer, gates and feed-forward, %d rows" % n, mine, *alg, ("three products", theirs, *alg)))
+
+    # ---- feed-forwards
+    for n in (1, 16, 256, 16384):
+        if want("gelu"):
+            x = rnd(n, 4096 + 2 * dense_ff)[:, 4096:]
+            xd = x.contiguous()
+            mine, theirs = graph_us([lambda: mixers.gelu_gate(x)]), graph_us([lambda: mixers.clamped_gate(xd, 7.0, 1.702)])
+            rows.append(_kernel_row("gelu gate, %d rows" % n, mine, n * dense_ff * 6, "hbm", ("clamped_gate_kernel, as Kaparax calls it", theirs, n * dense_ff * 6, "hbm")))
+    for n in (1, 16, 64, 128, 512, 2048, 16384):
+        if not want("experts"):
+            continue
+        h, copies = rnd(n, width), 6 if n <= 512 else 1
+        made = []
+        for sp in (experts.ExpertsSpec(n_exp, top, ff, score=experts.SIGMOID, weigh_input=True), experts.ExpertsSpec(n_exp, top, ff)):
+            made.append([])
+            for _ in range(copies):
+                with torch.device(dev):
+                    w = experts.ExpertWeights(sp, width).to(bf).requires_grad_(False)
+                for p in w.parameters():
+                    p.normal_(0.0, 0.03)
+                made[-1].append(experts.Experts(sp, w, dev))
+        time = graph_us if n <= 512 else event_us
+
+        def run(e):
+            e.counters.zero_()
+            e(h)
+
+        def alg_of(es):
+            if n >= 512:
+                return 6 * n * width * top * ff, "mfma"
+            for e in es:
+                run(e)
+            return sum(int((e.counters > 0).sum()) for e in es) / copies * ff * 6 * width + 2 * n * (width + 3 * top * ff + top * width), "hbm"
+        mine, theirs = (time([lambda e=e: run(e) for e in es]) for es in made)
+        rows.append(_kernel_row("experts (router and all), %d rows" % n, mine, *alg_of(made[0]), ("Pidutar's experts", theirs, *alg_of(made[1]))))
+        del made
+
+    # ---- the stream
+    for n in (16, 256, 16384):
+        y1, y2, r32, z = rnd(n, width), rnd(n * top, width), torch.randn(n, width, device=dev), rnd(n, 4096 + 2 * width)[:, 4096:]
+        tw, w, gb = torch.rand(n, top, device=dev), [rnd(width) for _ in range(4)], rnd(2 * width)
+        cnt, both = torch.zeros(n_exp, dtype=torch.int32, device=dev), rnd(n, 2 * width)
+        if want("gated step"):
+            theirs = graph_us([lambda: mixers.post_add_norm(y1, r32, (w[0], w[1]), (w[2], w[3]), 1e-6)])
+            like = ("norm_rows_kernel", theirs, n * width * 12, "hbm")
+            mine = graph_us([lambda: branches.gated_rms_norm(r32, y1, y2[:n], z, gb, w[2], 1e-6, clear=cnt)])
+            rows.append(_kernel_row("gated step of two branches + norm, %d rows" % n, mine, n * width * (2 + 2 + 4 + 8 + 2), "hbm", like))
+            mine = graph_us([lambda: branches.gated_rms_norm(r32, y1, y2, z, gb, w[2], 1e-6, clear=cnt)])
+            theirs = graph_us([lambda: branches.branches_rms_norms(r32, 0.5, y1, w[0], y2, tw, w[1], (w[2], w[3]), 1e-6, 1.0, clear=cnt)])
+            rows.append(_kernel_row("gated step of experts + norm, %d rows" % n, mine, n * width * (2 + 2 * top + 4 + 8 + 2), "hbm",
+                                    ("branch_norm_kernel, Pidutar's step", theirs, n * width * (2 + 2 * top + 8 + 4), "hbm")))
+        if want("pass"):
+            wi = [rnd(width, 2 * width) for _ in range(6 if n < 16384 else 1)]
+            time = graph_us if n < 16384 else event_us
+            mine, theirs = time([lambda x=x: experts.project_f32(both, x) for x in wi]), time([lambda x=x: F.linear(both, x) for x in wi])
+            alg = (4 * n * width * width, "mfma") if n >= 512 else (4 * width * width + n * width * 8, "hbm")
+            rows.append(_kernel_row("begin of a pass: product with fp32 sums, %d rows" % n, mine, *alg, ("library product, bf16 sums", theirs, *alg)))
+            p32 = torch.randn(n, width, device=dev)
+            mine = graph_us([lambda: branches.entry_rms_norm(p32, w[0], r32, w[1], 1e-6, clear=cnt)])
+            theirs = graph_us([lambda: mixers.post_add_norm(y1, r32, (w[0], w[1]), (w[2], w[3]), 1e-6)])
+            rows.append(_kernel_row("begin of a pass: vector + norm, %d rows" % n, mine, n * width * 10, "hbm", ("norm_rows_kernel", theirs, n * width * 12, "hbm")))
+    return rows
+
+
 def _engine_rates(model, dev, batch, prompt_len, new_tokens, slots):
     """Prefill and decode tokens/s of the engine: ``batch`` prompts of ``prompt_len`` tokens, ``new_tokens`` each."""
     import gc
@@ -1534,9 +1736,36 @@ def bench_sokolorn(args, dev):
     return result, lambda: None
 
 
-WORKLOADS = {"sokolorn": bench_sokolorn, "pidutar": bench_pidutar, "kaparax": bench_kaparax, "rope-scatter": bench_rope_scatter, "glue": bench_glue, "e2e": bench_e2e, "longctx": bench_longctx, "decode-e2e-shape": bench_decode_e2e_shape,
+def bench_bedenex(args, dev):
+    """The Bedenex family beside Pidutar and Sokolorn at equal size: engine throughput (prompts of 1024 tokens, then 128 decoded
+    tokens each) for two layer sizes and two batches, and every kernel beside its like (--part)."""
+    part = args.part
+    kernels = bedenex_kernels(dev, only=args.kernel) if part in ("all", "kernels") else []
+    engines = {}
+    if part in ("all", "engine"):
+        sizes = {"28 runs of 16 layers, width 1024, 16/8 heads x 128, ff 3072 or 4 of 32 experts of 768": (
+                     _bedenex_config(16, (4, 16, 2), 1024, 16, 8, 512, 3072, 32, 4, 768, 1024, 151936), _pidutar_config(28, 1024, 16, 512, 512, 8, 128, 32, 4, 768, 8192, 151936),
+                     _sokolorn_config(28, 1024, 16, 8, 4608, 32, 4, 576, 768, 1024, 151936)),
+                 "8 runs of 6 layers, width 4096, 32/8 heads x 128, ff 12288 or 4 of 32 experts of 3072": (
+                     _bedenex_config(6, (2, 4, 2), 4096, 32, 8, 512, 12288, 32, 4, 3072, 1024, 151936), _pidutar_config(8, 4096, 32, 1536, 512, 16, 128, 32, 4, 3072, 8192, 151936),
+                     _sokolorn_config(8, 4096, 32, 8, 18432, 32, 4, 2304, 3072, 1024, 151936))}
+        for what, models in sizes.items():
+            for batch in (16, 128):
+                engines["%s; batch %d" % (what, batch)] = {name: _engine_rates(m, dev, batch, 1024, 128, 128)
+                                                           for name, m in zip(("bedenex", "pidutar", "sokolorn"), models)}
+                print(what, batch, engines["%s; batch %d" % (what, batch)], file=sys.stderr, flush=True)
+    first = next(iter(engines.values()))["bedenex"]["decode_tok_s"] if engines else None
+    result = {"metric": "Bedenex decode tok/s (28 runs of 16 layers of width 1024, batch 16, prompts of 1024)", "value": first, "unit": "tok/s",
+              "ms_per_step": round(16e3 / first, 3) if first else None,
+              "config": {"workload": "random weights; chunked (1024) and latent attention in turn, dense and expert feed-forwards in turn, most layers run twice",
+                         "engine": engines, "kernels": kernels},
+              "roofline": None}
+    return result, lambda: None
+
+
+WORKLOADS = {"bedenex": bench_bedenex, "sokolorn": bench_sokolorn, "pidutar": bench_pidutar, "kaparax": bench_kaparax, "rope-scatter": bench_rope_scatter, "glue": bench_glue, "e2e": bench_e2e, "longctx": bench_longctx, "decode-e2e-shape": bench_decode_e2e_shape,
              "decode-longctx-shape": bench_decode_longctx_shape, "copy": bench_copy, "read-probe": bench_read_probe, "decode": bench_decode, "scatter": bench_scatter, "prefill": bench_prefill, "sampler": bench_sampler}
-DEFAULT_STEPS = {"sokolorn": 60, "pidutar": 60, "kaparax": 60, "rope-scatter": 100, "glue": 100, "e2e": 1, "longctx": 1, "decode-e2e-shape": 1, "decode-longctx-shape": 1, "copy": 50, "read-probe": 60, "decode": 200, "scatter": 400, "prefill": 50, "sampler": 100}
+DEFAULT_STEPS = {"bedenex": 60, "sokolorn": 60, "pidutar": 60, "kaparax": 60, "rope-scatter": 100, "glue": 100, "e2e": 1, "longctx": 1, "decode-e2e-shape": 1, "decode-longctx-shape": 1, "copy": 50, "read-probe": 60, "decode": 200, "scatter": 400, "prefill": 50, "sampler": 100}
 
 
 def main():
@@ -1557,8 +1786,8 @@ def main():
     ap.add_argument("--glue", choices=["add-rms-norm", "silu-mul", "last-token-norm"], default="add-rms-norm", help="glue: which elementwise kernel")
     ap.add_argument("--uniform", default=None, metavar="SxL", help="prefill: S packed sequences of L tokens each instead of config 3 (e.g. 2x16384)")
     ap.add_argument("--bucket-step", type=int, default=16, help="e2e only: spacing of the captured decode batch sizes")
-    ap.add_argument("--part", "--kaparax-part", choices=["all", "kernels", "engine"], default="all", help="sokolorn / kaparax / pidutar: which half of the workload")
-    ap.add_argument("--kernel", default=None, help="sokolorn / kaparax / pidutar: only kernels whose row name contains this")
+    ap.add_argument("--part", "--kaparax-part", choices=["all", "kernels", "engine"], default="all", help="bedenex / sokolorn / kaparax / pidutar: which half of the workload")
+    ap.add_argument("--kernel", default=None, help="bedenex / sokolorn / kaparax / pidutar: only kernels whose row name contains this")
     ap.add_argument("--no-extra", action="store_true", help="e2e only: skip the per-configuration rooflines and the eager pass")
     args = ap.parse_args()
     if args.gpus != 1:

@@ -560,13 +560,14 @@ __global__ __launch_bounds__(256, DK + DV > 256 ? 1 : 3) void chunk_decode_kerne
         blk = blk_this;
         float x[2][4], mx = -INFINITY;
         bool vis[2][4];
+        const float ahead = fmaf(rate, static_cast<float>(pos - key0 - 4 * g), 1.0f);      // of this lane's first key, as in the other kernel
 #pragma unroll
         for (int kb = 0; kb < 2; ++kb)
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int key = key0 + 16 * kb + 4 * g + i;
                 vis[kb][i] = ok && key >= lo && key <= last;
-                if (kCap == kBiased) x[kb][i] = biased_exponent(w.in, s[kb][i], slope, fmaf(rate, static_cast<float>(pos - key), 1.0f));
+                if (kCap == kBiased) x[kb][i] = biased_exponent(w.in, s[kb][i], slope, fmaf(rate, static_cast<float>(-16 * kb - i), ahead));
                 else x[kb][i] = exponent_of(w, kPlain || w.capped, s[kb][i]);
                 if (vis[kb][i]) mx = fmaxf(mx, x[kb][i]);
             }
